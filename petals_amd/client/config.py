@@ -13,6 +13,7 @@ MAX_RETRIES = int(os.environ.get("PETALS_AMD_MAX_RETRIES", "10"))
 class ClientConfig:
     initial_peers: Sequence[Tuple[str, int]] = ()
     dht_prefix: Optional[str] = None
+    standalone: bool = False  # only the client's own modules, no swarm behind them
 
     show_route: str | bool = "inference"  # False / "inference" / True
     allowed_servers: Optional[Sequence[str]] = None

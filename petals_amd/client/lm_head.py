@@ -34,6 +34,11 @@ class LMHead(nn.Module):
             and self.use_chunked_forward
         ):
             return self.chunked_forward(hidden_states)
+        if hidden_states.is_cuda and hidden_states.dtype == torch.float32 and self.weight.dtype == torch.bfloat16:
+            # families with a 32-bit residual stream: bf16 product, 32-bit logits
+            from petals_amd import ops
+
+            return ops.linear_f32(hidden_states, self.weight)
         return F.linear(hidden_states, self.weight.to(hidden_states.dtype))
 
     def chunked_forward(self, hidden_states: torch.Tensor) -> torch.Tensor:

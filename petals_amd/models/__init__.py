@@ -35,6 +35,7 @@ def _ensure_families():
         import petals_amd.models.bloom  # noqa: F401
         import petals_amd.models.falcon  # noqa: F401
         import petals_amd.models.mixtral  # noqa: F401
+        import petals_amd.models.tulezen  # noqa: F401
 
         _loaded = True
 

@@ -23,6 +23,9 @@ class BloomConfig(ModelConfig):
             self.intermediate_size = 4 * self.hidden_size
         super().__post_init__()
 
+    def client_tensor_names(self):
+        return "transformer.word_embeddings.weight", "transformer.ln_f.weight", "lm_head.weight"
+
     def default_dht_prefix(self) -> str:
         base = self.name_or_path.split("/")[-1] if self.name_or_path else "bloom"
         return f"{base.replace('.', '-')}-petals-amd"

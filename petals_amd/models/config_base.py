@@ -13,18 +13,35 @@ from __future__ import annotations
 import dataclasses
 import json
 import os
-from typing import Any, ClassVar, Dict, Optional, Type
+from typing import Any, ClassVar, Dict, FrozenSet, Optional, Tuple, Type
+
+import torch
 
 _MODEL_CONFIG_REGISTRY: Dict[str, Type["ModelConfig"]] = {}
+_ARCHITECTURES: Dict[str, str] = {}  # config.json "architecture" -> model_type
 
 
-def register_config(model_type: str):
+def register_config(model_type: str, architecture: Optional[str] = None):
+    """`architecture`: value of the config.json key of that name by which
+    checkpoints without a `model_type` identify the family."""
+
     def deco(cls):
         _MODEL_CONFIG_REGISTRY[model_type] = cls
         cls.model_type = model_type
+        if architecture is not None:
+            _ARCHITECTURES[architecture] = model_type
         return cls
 
     return deco
+
+
+def resolve_model_type(d: Dict[str, Any]) -> str:
+    """The registered family of a config.json dict."""
+    model_type = d.get("model_type") or _ARCHITECTURES.get(d.get("architecture"))
+    if model_type not in _MODEL_CONFIG_REGISTRY:
+        named = d.get("model_type") or d.get("architecture")
+        raise ValueError(f"unsupported model_type {named!r}; known: {sorted(_MODEL_CONFIG_REGISTRY)}")
+    return model_type
 
 
 @dataclasses.dataclass
@@ -76,6 +93,36 @@ class ModelConfig:
         base = self.name_or_path.split("/")[-1] if self.name_or_path else self.model_type
         base = base.replace(".", "-") or self.model_type or "model"
         return f"{base}-petals-amd"
+
+    # ------------------------------------------- checkpoint and span layout
+
+    def block_tensor_prefix(self, block_index: int) -> str:
+        """Checkpoint prefix of one block's tensors."""
+        return f"{self.block_prefix}.{block_index}."
+
+    def client_tensor_names(self) -> Tuple[str, str, str]:
+        """(embeddings, final norm, lm head) names in the checkpoint."""
+        return "model.embed_tokens.weight", "model.norm.weight", "lm_head.weight"
+
+    def stream_dtype(self, dtype: torch.dtype) -> torch.dtype:
+        """dtype of the hidden states that travel between blocks served in `dtype`."""
+        return dtype
+
+    def valid_cuts(self) -> Optional[FrozenSet[int]]:
+        """Block indices at which the chain may be split between servers
+        (None: anywhere). Families whose blocks read another block's cache
+        restrict this so that reader and owner are always served together."""
+        return None
+
+    def block_param_count(self) -> int:
+        """Parameters of one (the largest) block."""
+        h = self.hidden_size
+        kv = self.n_kv_heads * self.head_dim
+        return 2 * h * h + 2 * h * kv + 3 * h * self.intermediate_size * getattr(self, "num_local_experts", 1)
+
+    def cache_values_per_token(self, block_index: int = 0) -> int:
+        """Elements that one token occupies in one block's attention cache."""
+        return 2 * self.n_kv_heads * self.head_dim
 
     # ------------------------------------------------------- HF conversion
 
@@ -129,7 +176,4 @@ def load_model_config(path_or_preset: str) -> ModelConfig:
         with open(p) as f:
             d = json.load(f)
         name = path_or_preset
-    model_type = d.get("model_type")
-    if model_type not in _MODEL_CONFIG_REGISTRY:
-        raise ValueError(f"unsupported model_type {model_type!r}; known: {sorted(_MODEL_CONFIG_REGISTRY)}")
-    return _MODEL_CONFIG_REGISTRY[model_type].from_hf_dict(d, name_or_path=name)
+    return _MODEL_CONFIG_REGISTRY[resolve_model_type(d)].from_hf_dict(d, name_or_path=name)

@@ -31,6 +31,9 @@ class FalconConfig(ModelConfig):
         else:
             self.num_key_value_heads = self.num_attention_heads
 
+    def client_tensor_names(self):
+        return "transformer.word_embeddings.weight", "transformer.ln_f.weight", "lm_head.weight"
+
     def default_dht_prefix(self) -> str:
         base = self.name_or_path.split("/")[-1] if self.name_or_path else "falcon"
         return f"{base.replace('.', '-')}-petals-amd"

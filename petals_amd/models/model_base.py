@@ -75,7 +75,8 @@ class DistributedModelBase(nn.Module, PTuneMixin):
         super().__init__()
         self.config = config
         self.embed_tokens = nn.Embedding(config.vocab_size, config.hidden_size)
-        self.h = RemoteSequential(config, dht=dht)
+        # standalone: the caller runs the blocks itself (server/local_engine.py)
+        self.h = None if config.client.standalone else RemoteSequential(config, dht=dht)
         self.norm = self._make_final_norm(config)
         self.init_prompts(config)
         self.requires_grad_(False)
@@ -224,24 +225,12 @@ class DistributedForSequenceClassificationBase(nn.Module):
 # ------------------------------------------------------------------ weights
 
 
-def _client_side_names(config):
-    """(embeddings name, final norm name, lm head name) in HF state dicts."""
-    mt = config.model_type
-    if mt in ("llama", "mixtral"):
-        return "model.embed_tokens.weight", "model.norm.weight", "lm_head.weight"
-    if mt == "bloom":
-        return "transformer.word_embeddings.weight", "transformer.ln_f.weight", "lm_head.weight"
-    if mt == "falcon":
-        return "transformer.word_embeddings.weight", "transformer.ln_f.weight", "lm_head.weight"
-    raise ValueError(mt)
-
-
 def _load_client_side_weights(model, model_dir: str, config):
     """Load ONLY embeddings/norm/head shards (parity: client/from_pretrained.py —
     shards for block layers are skipped)."""
     from safetensors import safe_open
 
-    emb_name, norm_name, head_name = _client_side_names(config)
+    emb_name, norm_name, head_name = config.client_tensor_names()
     wanted = {emb_name, norm_name, head_name}
     if config.model_type == "bloom":
         wanted |= {"transformer.ln_f.bias", "transformer.word_embeddings_layernorm.weight",

@@ -181,6 +181,24 @@ def swiglu(gate, up):
     return reference.swiglu(gate, up)
 
 
+def zero_centered_rms_norm(x, weight, eps: float):
+    """x / sqrt(mean(x^2) + eps) * (1 + weight) over the last axis, 32-bit."""
+    if x.is_cuda and not _grad_mode(x, weight):
+        from petals_amd.ops import latent
+
+        return latent.zero_centered_rms_norm(x, weight, eps)
+    return reference.zero_centered_rms_norm(x, weight, eps)
+
+
+def linear_f32(x, weight):
+    """x @ weight.T with a 32-bit result, the product in the weight's dtype."""
+    if x.is_cuda:
+        from petals_amd.ops import latent
+
+        return latent.linear_f32(x, weight)
+    return (x.to(weight.dtype) @ weight.t()).float()
+
+
 # re-exports used by blocks
 build_rope_cache = reference.build_rope_cache
 build_alibi_bias = reference.build_alibi_bias

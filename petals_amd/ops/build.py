@@ -1,7 +1,11 @@
-"""Build the HIP extension IN-TREE (the .so must travel with the repo snapshot
-to GPU boxes): `python -m petals_amd.ops.build`.
+"""Build the HIP extensions IN-TREE (the .so files must travel with the source
+tree to GPU boxes): `python -m petals_amd.ops.build [name ...]`.
 
-Cross-compiles for gfx950 (no GPU needed at build time).
+Cross-compiles for gfx950 (no GPU needed at build time). Two libraries:
+
+  core    the kernels of the llama / bloom / falcon / mixtral families
+  latent  latent attention, output norms and routed experts (tulezen); it is
+          all that a process serving such a model needs
 """
 
 from __future__ import annotations
@@ -12,18 +16,33 @@ import sys
 
 PKG_DIR = os.path.dirname(os.path.abspath(__file__))
 SRC_DIR = os.path.join(PKG_DIR, "csrc")
-BUILD_DIR = os.path.join(PKG_DIR, "_build")
-SO_PATH = os.path.join(PKG_DIR, "_hip_ops.so")
 
-SOURCES = ["bindings.cpp", "elementwise.hip", "gemv.hip", "attention.hip", "nf4.hip", "int8.hip", "prefill_attn.hip", "moe.hip"]
+# name -> (.so next to this file, torch extension name, build folder, sources)
+EXTENSIONS = {
+    "core": (
+        "_hip_ops.so", "petals_amd_hip_ops", "_build",
+        ["bindings.cpp", "elementwise.hip", "gemv.hip", "attention.hip", "nf4.hip", "int8.hip", "prefill_attn.hip",
+         "moe.hip"],
+    ),
+    "latent": (
+        "_hip_latent.so", "petals_amd_hip_latent", os.path.join("_build", "latent"),
+        ["latent_bindings.cpp", "latent_attn.hip", "sublayer.hip", "gemv.hip", "moe.hip"],
+    ),
+}
 
 
-def build(verbose: bool = False) -> str:
+def so_path(name: str = "core") -> str:
+    return os.path.join(PKG_DIR, EXTENSIONS[name][0])
+
+
+def build(verbose: bool = False, name: str = "core") -> str:
     os.environ.setdefault("PYTORCH_ROCM_ARCH", "gfx950")
     os.environ.setdefault("MAX_JOBS", str(min(8, os.cpu_count() or 4)))
     from torch.utils.cpp_extension import load
 
-    os.makedirs(BUILD_DIR, exist_ok=True)
+    _, ext_name, folder, files = EXTENSIONS[name]
+    build_dir = os.path.join(PKG_DIR, folder)
+    os.makedirs(build_dir, exist_ok=True)
     # torch's hipify writes `<name>_hip.<ext>` next to each source and skips
     # regeneration based on mtimes; a repo snapshot (gpurun) can scramble those
     # and leave a stale artifact compiling instead of the real source. Purge
@@ -32,25 +51,26 @@ def build(verbose: bool = False) -> str:
 
     for stale in glob.glob(os.path.join(SRC_DIR, "*_hip.*")):
         os.unlink(stale)
-    sources = [os.path.join(SRC_DIR, s) for s in SOURCES if os.path.exists(os.path.join(SRC_DIR, s))]
-    module = load(
-        name="petals_amd_hip_ops",
-        sources=sources,
-        build_directory=BUILD_DIR,
+    load(
+        name=ext_name,
+        sources=[os.path.join(SRC_DIR, s) for s in files],
+        build_directory=build_dir,
         extra_cflags=["-O3", "-std=c++17"],
-        extra_cuda_cflags=["-O3", "-std=c++17", "-ffast-math"],
+        # packed FP32 instructions stay off: some of their forms have given
+        # wrong results on these machines
+        extra_cuda_cflags=["-O3", "-std=c++17", "-ffast-math", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"],
         verbose=verbose,
         is_python_module=False,
         is_standalone=False,
         keep_intermediates=True,
     )
     # copy the built .so in-tree under a stable name
-    built = os.path.join(BUILD_DIR, "petals_amd_hip_ops.so")
+    built = os.path.join(build_dir, ext_name + ".so")
     if os.path.exists(built):
-        shutil.copy2(built, SO_PATH)
-    return SO_PATH
+        shutil.copy2(built, so_path(name))
+    return so_path(name)
 
 
 if __name__ == "__main__":
-    path = build(verbose="-v" in sys.argv)
-    print(f"built {path}")
+    for which in [a for a in sys.argv[1:] if not a.startswith("-")] or list(EXTENSIONS):
+        print(f"built {build(verbose='-v' in sys.argv, name=which)}", flush=True)

@@ -47,7 +47,7 @@ torch::Tensor gemv_nf4(
 torch::Tensor sumsq_rows(torch::Tensor x);
 torch::Tensor gemv_bf16_moe(
     torch::Tensor wt_all, torch::Tensor x, torch::Tensor sel, int64_t k_per_tok,
-    torch::Tensor workspace, int64_t epilogue, int64_t splits_override);
+    torch::Tensor workspace, int64_t epilogue, int64_t splits_override, double limit, double alpha);
 torch::Tensor gemv_nf4_moe(
     torch::Tensor packed_all, torch::Tensor absmax_all, torch::Tensor x, torch::Tensor sel,
     int64_t k_per_tok, torch::Tensor workspace, int64_t epilogue, int64_t splits_override);
@@ -96,7 +96,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gemv_bf16_moe", &gemv_bf16_moe,
         "device-routed MoE gemv: stacked bf16 expert weights, expert ids from a device tensor",
         py::arg("wt_all"), py::arg("x"), py::arg("sel"), py::arg("k_per_tok"),
-        py::arg("workspace"), py::arg("epilogue"), py::arg("splits") = 0);
+        py::arg("workspace"), py::arg("epilogue"), py::arg("splits") = 0,
+        py::arg("limit") = 0.0, py::arg("alpha") = 0.0);
   m.def("gemv_nf4_moe", &gemv_nf4_moe,
         "device-routed MoE gemv: stacked NF4 expert weights, expert ids from a device tensor",
         py::arg("packed_all"), py::arg("absmax_all"), py::arg("x"), py::arg("sel"),

@@ -10,9 +10,7 @@
 // (plain / +residual / SwiGLU-pair) and dtype conversion.
 //
 // Replaces (capability-wise) the per-token GEMMs the reference runs through
-// torch/CUDA inside HF blocks (reference models/llama/block.py:44-127); the
-// design follows /opt/skills/guides/cdna_hip_programming.md Appendix B
-// ("Element-wise"/"GEMM" vectorization rules; G13).
+// torch/CUDA inside HF blocks (reference models/llama/block.py:44-127).
 
 #include "common.h"
 #include "gemv_reduce.h"

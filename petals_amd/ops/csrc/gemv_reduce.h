@@ -16,6 +16,14 @@ enum GemvEpilogue : int {
   EPI_RESIDUAL_BF16 = 2, // y_bf16 = residual_bf16 + sum
   EPI_SWIGLU_F32 = 3,    // out = silu(sum[:half]) * sum[half:], y_f32[b, half]
   EPI_GELU_F32 = 4,      // y_f32[b, out] = gelu_tanh(sum) (BLOOM/Falcon MLPs)
+  EPI_CLAMPED_SWIGLU_F32 = 5,  // g = min(sum[:half], limit), u = clamp(sum[half:], +-limit):
+                               // g * sigmoid(alpha g) * (u + 1), y_f32[b, half]
+};
+
+// constants of EPI_CLAMPED_SWIGLU_F32
+struct ClampedGate {
+  float limit = 0.f;
+  float alpha = 0.f;
 };
 
 // deterministic split sum with 4 independent accumulators so the loads
@@ -66,11 +74,13 @@ static __global__ __launch_bounds__(64 * G) void gemv_reduce_kernel_impl(
     int n_splits,
     int batch,
     int out_dim,
-    int epilogue) {
+    int epilogue,
+    ClampedGate gate) {
   __shared__ float acc_g[G][64];
   __shared__ float acc_u[G][64];
   const int half = out_dim >> 1;
-  const int n_out = (epilogue == EPI_SWIGLU_F32) ? half : out_dim;
+  const bool pair = epilogue == EPI_SWIGLU_F32 || epilogue == EPI_CLAMPED_SWIGLU_F32;
+  const int n_out = pair ? half : out_dim;
   const int total = batch * n_out;
   const int ol = threadIdx.x & 63;
   const int sg = threadIdx.x >> 6;
@@ -84,7 +94,7 @@ static __global__ __launch_bounds__(64 * G) void gemv_reduce_kernel_impl(
   float g = 0.f, u = 0.f;
   if (live) {
     for (int s = sg; s < n_splits; s += G) g += partials[(size_t)s * stride + row + o];
-    if (epilogue == EPI_SWIGLU_F32)
+    if (pair)
       for (int s = sg; s < n_splits; s += G) u += partials[(size_t)s * stride + row + o + half];
   }
   acc_g[sg][ol] = g;
@@ -97,12 +107,19 @@ static __global__ __launch_bounds__(64 * G) void gemv_reduce_kernel_impl(
     sum += acc_g[k][ol];
     usum += acc_u[k][ol];
   }
-  if (epilogue == EPI_SWIGLU_F32) {
+  if (pair) {
     if (bias) {
       sum += bf16_to_f32(bias[o]);
       usum += bf16_to_f32(bias[o + half]);
     }
-    const float act = sum / (1.f + __expf(-sum)) * usum;
+    float act;
+    if (epilogue == EPI_SWIGLU_F32) {
+      act = sum / (1.f + __expf(-sum)) * usum;
+    } else {
+      const float g = fminf(sum, gate.limit);
+      const float u = fmaxf(fminf(usum, gate.limit), -gate.limit);
+      act = g / (1.f + __expf(-gate.alpha * g)) * (u + 1.f);
+    }
     reinterpret_cast<float*>(y)[(size_t)b * half + o] = act;
   } else {
     if (bias) sum += bf16_to_f32(bias[o]);
@@ -136,13 +153,15 @@ static inline torch::Tensor launch_gemv_reduce(
     int epilogue,
     const torch::TensorOptions& f32_opts,
     const torch::TensorOptions& bf16_opts,
-    c10::optional<torch::Tensor> sumsq_out = c10::nullopt) {
+    c10::optional<torch::Tensor> sumsq_out = c10::nullopt,
+    ClampedGate gate = ClampedGate()) {
   const int half = out_dim / 2;
-  const int n_out = (epilogue == EPI_SWIGLU_F32) ? half : out_dim;
+  const bool pair = epilogue == EPI_SWIGLU_F32 || epilogue == EPI_CLAMPED_SWIGLU_F32;
+  const int n_out = pair ? half : out_dim;
   torch::Tensor y;
   if (epilogue == EPI_PLAIN_F32 || epilogue == EPI_GELU_F32)
     y = torch::empty({batch, out_dim}, f32_opts);
-  else if (epilogue == EPI_SWIGLU_F32)
+  else if (pair)
     y = torch::empty({batch, half}, f32_opts);
   else
     y = torch::empty({batch, out_dim}, bf16_opts);
@@ -175,10 +194,10 @@ static inline torch::Tensor launch_gemv_reduce(
   auto stream = c10::hip::getCurrentHIPStream().stream();
   if (red_g == 16)
     gemv_reduce_kernel_impl<16><<<rblocks, 64 * 16, 0, stream>>>(
-        partials.data_ptr<float>(), res_p, bias_p, y.data_ptr(), ss_p, n_splits, batch, out_dim, epilogue);
+        partials.data_ptr<float>(), res_p, bias_p, y.data_ptr(), ss_p, n_splits, batch, out_dim, epilogue, gate);
   else
     gemv_reduce_kernel_impl<8><<<rblocks, 64 * 8, 0, stream>>>(
-        partials.data_ptr<float>(), res_p, bias_p, y.data_ptr(), ss_p, n_splits, batch, out_dim, epilogue);
+        partials.data_ptr<float>(), res_p, bias_p, y.data_ptr(), ss_p, n_splits, batch, out_dim, epilogue, gate);
   HIP_CHECK_LAST();
   return y;
 }

@@ -1,0 +1,474 @@
+// Latent (MLA-style) attention over a paged cache for CDNA4 (gfx950).
+//
+// The cache holds one latent row c (RP values) per token and nothing per head.
+// Queries arrive already carried into latent space (q' = W_uk^T q), so a score
+// is q'.c and the weighted sum of c is carried to value space afterwards: all
+// heads of a token attend over ONE shared key/value row, i.e. multi-query
+// attention with head size RP. (token, head) pairs of a run of tokens are the
+// rows of an mfma_f32_16x16x32_bf16 tile, so a staged latent tile serves every
+// head and every token of the run.
+//
+//   latent_attn_kernel     MFMA flash kernel, prompts and decoding, ragged
+//                          batches, sliding window, optional key split
+//   latent_attn_combine    merges key splits
+//   latent_attn_simple     any latent size, 32-bit or bf16 storage
+//   latent_write           RMS-normalises new latents into their pages
+//
+// Rows, positions and page tables come from device memory; every page index is
+// checked against the pool before it is used.
+
+#include "common.h"
+#include <torch/extension.h>
+#include <ATen/cuda/CUDAContext.h>
+
+using bf16x8 = __attribute__((ext_vector_type(8))) short;
+using f32x4 = __attribute__((ext_vector_type(4))) float;
+
+#define PAGE 64   // tokens per page
+#define LKVT 32   // keys per staged tile
+#define LPAD 8    // LDS row padding (elements)
+
+// transposed tile addressing: XOR swizzle on the dim group (see prefill_attn.hip)
+#define LVT_BYTE(dim, key_byte) \
+  ((((unsigned)(dim)) * ((LKVT + LPAD) * 2) + (unsigned)(key_byte)) ^ ((((unsigned)(dim) >> 3) & 7u) << 4))
+
+struct PagedRows {
+  const int* pos;     // [T] position of each row
+  const int* owner;   // [T] sequence of each row
+  const int* tables;  // [S, width] pages of each sequence
+  int width;
+  int num_pages;
+};
+
+// start of the cache row of (sequence, key) in tokens, -1 if there is none
+__device__ __forceinline__ long cache_row(const PagedRows& b, int seq, int key) {
+  const int slot = key / PAGE;
+  if (key < 0 || slot >= b.width) return -1;
+  const int page = b.tables[(size_t)seq * b.width + slot];
+  if (page < 0 || page >= b.num_pages) return -1;
+  return (long)page * PAGE + (key - slot * PAGE);
+}
+
+template <typename T> __device__ __forceinline__ float load_f32(const T* p);
+template <> __device__ __forceinline__ float load_f32<float>(const float* p) { return *p; }
+template <> __device__ __forceinline__ float load_f32<unsigned short>(const unsigned short* p) { return bf16_to_f32(*p); }
+template <typename T> __device__ __forceinline__ void store_f32(T* p, float v);
+template <> __device__ __forceinline__ void store_f32<float>(float* p, float v) { *p = v; }
+template <> __device__ __forceinline__ void store_f32<unsigned short>(unsigned short* p, float v) { *p = f32_to_bf16(v); }
+
+// ------------------------------------------------------------ MFMA kernel
+
+// RC = latent size in 32-wide MFMA k-chunks (columns past RP read as zero).
+// Grid: (token runs, groups of 16*NW rows, key splits); NW = blockDim.x / 64.
+template <int RC>
+__global__ __launch_bounds__(256) void latent_attn_kernel(
+    const unsigned short* __restrict__ q,      // [T, H, RP]
+    const unsigned short* __restrict__ cache,  // [num_pages, PAGE, RP]
+    unsigned short* __restrict__ out,          // [T, H, RP] (n_splits == 1)
+    float* __restrict__ part_o,                // [n_splits, T*H, RP]
+    float* __restrict__ part_ml,               // [n_splits, T*H, 2]
+    const int* __restrict__ tiles,             // [n, 2] first token, token count
+    PagedRows b,
+    int total_tokens,
+    int heads,
+    int rp,
+    int window,
+    float scale_log2e,
+    int n_splits) {
+  constexpr int R = RC * 32;
+  const int nw = blockDim.x / WAVE;
+  const int tok0 = tiles[2 * blockIdx.x];
+  const int ntok = tiles[2 * blockIdx.x + 1];
+  const int rows = ntok * heads;
+  const int g0 = blockIdx.y * 16 * nw;  // first row of this workgroup
+  if (g0 >= rows) return;               // uniform over the workgroup
+  const int g1 = min(g0 + 16 * nw, rows);
+
+  const int tid = threadIdx.x;
+  const int wave = tid / WAVE;
+  const int lane = tid & (WAVE - 1);
+  const int col = lane & 15;
+  const int hi = lane >> 4;
+  const int r0 = g0 + wave * 16;  // first row of this wave
+
+  extern __shared__ unsigned char smem[];
+  unsigned short* k_lds = reinterpret_cast<unsigned short*>(smem);  // [LKVT][R + LPAD]
+  unsigned char* vt_raw = smem + LKVT * (R + LPAD) * 2;             // [R][LKVT + LPAD] swizzled
+  unsigned short* p_lds =
+      reinterpret_cast<unsigned short*>(vt_raw + R * (LKVT + LPAD) * 2) + wave * 16 * (LKVT + LPAD);
+
+  const int seq = b.owner[tok0];
+  const int first_pos = b.pos[tok0 + g0 / heads];
+  const int last_pos = b.pos[tok0 + (g1 - 1) / heads];
+  const int key_lo = window > 0 ? max(0, first_pos - window + 1) : 0;
+  const int key_hi = last_pos + 1;
+  const int n_tiles = (key_hi - key_lo + LKVT - 1) / LKVT;
+  const int per_split = (n_tiles + n_splits - 1) / n_splits;
+  const int j_begin = key_lo + blockIdx.z * per_split * LKVT;
+  const int j_end = min(key_hi, j_begin + per_split * LKVT);
+
+  bf16x8 q_frag[RC];
+  {
+    const int row = r0 + col;
+    const unsigned short* src = q + ((size_t)tok0 * heads + row) * rp;
+#pragma unroll
+    for (int kc = 0; kc < RC; ++kc) {
+      const int c0 = kc * 32 + hi * 8;
+      if (row < rows && c0 < rp)
+        q_frag[kc] = *reinterpret_cast<const bf16x8*>(src + c0);
+      else
+        q_frag[kc] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    }
+  }
+
+  f32x4 acc_o[R / 16];
+  float m_row[4], l_row[4];
+  int row_pos[4], row_lo[4];
+#pragma unroll
+  for (int d = 0; d < R / 16; ++d) acc_o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    m_row[r] = NEG_SENTINEL;
+    l_row[r] = 0.f;
+    const int row = r0 + hi * 4 + r;
+    row_pos[r] = row < rows ? b.pos[tok0 + row / heads] : -1;  // -1: sees nothing
+    row_lo[r] = window > 0 ? row_pos[r] - window + 1 : 0;
+  }
+  // keys that every row of this wave sees: [all_lo, all_hi]
+  const int wave_last = min(r0 + 15, rows - 1);
+  const bool full_wave = r0 + 16 <= rows;
+  const int all_hi = full_wave ? b.pos[tok0 + r0 / heads] : -1;
+  const int all_lo = full_wave && window > 0 ? b.pos[tok0 + wave_last / heads] - window + 1 : 0;
+
+  for (int j0 = j_begin; j0 < j_end; j0 += LKVT) {
+    __syncthreads();
+    for (int idx = tid; idx < LKVT * (R / 8); idx += blockDim.x) {
+      const int row = idx / (R / 8);
+      const int c8 = (idx - row * (R / 8)) * 8;
+      bf16x8 v8 = {0, 0, 0, 0, 0, 0, 0, 0};
+      if (j0 + row < j_end && c8 < rp) {
+        const long at = cache_row(b, seq, j0 + row);
+        if (at >= 0) v8 = *reinterpret_cast<const bf16x8*>(cache + (size_t)at * rp + c8);
+      }
+      *reinterpret_cast<bf16x8*>(&k_lds[row * (R + LPAD) + c8]) = v8;
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        *reinterpret_cast<unsigned short*>(&vt_raw[LVT_BYTE(c8 + e, row * 2)]) = (unsigned short)v8[e];
+    }
+    __syncthreads();
+
+    f32x4 s_acc[2];
+#pragma unroll
+    for (int nb = 0; nb < 2; ++nb) {
+      s_acc[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int kc = 0; kc < RC; ++kc) {
+        const bf16x8 kt =
+            *reinterpret_cast<const bf16x8*>(&k_lds[(nb * 16 + col) * (R + LPAD) + kc * 32 + hi * 8]);
+        s_acc[nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q_frag[kc], kt, s_acc[nb], 0, 0, 0);
+      }
+    }
+
+    const bool interior = j0 >= all_lo && j0 + LKVT - 1 <= all_hi && j0 + LKVT <= j_end;
+    float corr[4], p[2][4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      // masking and the running max stay in separate loops (see prefill_attn.hip)
+      float s[2];
+#pragma unroll
+      for (int nb = 0; nb < 2; ++nb) s[nb] = s_acc[nb][r] * scale_log2e;
+      if (!interior) {
+#pragma unroll
+        for (int nb = 0; nb < 2; ++nb) {
+          const int key = j0 + nb * 16 + col;
+          if (key >= j_end || key > row_pos[r] || key < row_lo[r]) s[nb] = NEG_SENTINEL;
+        }
+      }
+      float mx = fmaxf(s[0], s[1]);
+#pragma unroll
+      for (int off = 8; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, WAVE));
+      const float m_new = fmaxf(m_row[r], mx);
+      corr[r] = (m_row[r] <= NEG_THRESHOLD) ? 0.f : exp2f(m_row[r] - m_new);
+      float lsum = 0.f;
+#pragma unroll
+      for (int nb = 0; nb < 2; ++nb) {
+        p[nb][r] = (s[nb] <= NEG_THRESHOLD) ? 0.f : exp2f(s[nb] - m_new);
+        lsum += p[nb][r];
+      }
+#pragma unroll
+      for (int off = 8; off > 0; off >>= 1) lsum += __shfl_xor(lsum, off, WAVE);
+      l_row[r] = l_row[r] * corr[r] + lsum;
+      m_row[r] = m_new;
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+#pragma unroll
+      for (int nb = 0; nb < 2; ++nb)
+        p_lds[(hi * 4 + r) * (LKVT + LPAD) + nb * 16 + col] = f32_to_bf16(p[nb][r]);
+    __syncthreads();
+
+    const bf16x8 p_frag = *reinterpret_cast<const bf16x8*>(&p_lds[col * (LKVT + LPAD) + hi * 8]);
+#pragma unroll
+    for (int d = 0; d < R / 16; ++d) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) acc_o[d][r] *= corr[r];
+      const bf16x8 vfrag = *reinterpret_cast<const bf16x8*>(&vt_raw[LVT_BYTE(d * 16 + col, hi * 16)]);
+      acc_o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p_frag, vfrag, acc_o[d], 0, 0, 0);
+    }
+  }
+
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int row = r0 + hi * 4 + r;
+    if (row >= rows) continue;
+    const size_t flat = (size_t)tok0 * heads + row;
+    if (n_splits == 1) {
+      const float inv_l = l_row[r] > 0.f ? 1.0f / l_row[r] : 0.f;
+#pragma unroll
+      for (int d = 0; d < R / 16; ++d)
+        if (d * 16 + col < rp) out[flat * rp + d * 16 + col] = f32_to_bf16(acc_o[d][r] * inv_l);
+    } else {
+      const size_t at = (size_t)blockIdx.z * total_tokens * heads + flat;
+#pragma unroll
+      for (int d = 0; d < R / 16; ++d)
+        if (d * 16 + col < rp) part_o[at * rp + d * 16 + col] = acc_o[d][r];
+      if (col == 0) {
+        part_ml[at * 2] = m_row[r];
+        part_ml[at * 2 + 1] = l_row[r];
+      }
+    }
+  }
+}
+
+// one workgroup per (token, head) row
+__global__ __launch_bounds__(128) void latent_attn_combine(
+    const float* __restrict__ part_o, const float* __restrict__ part_ml,
+    unsigned short* __restrict__ out, int n_rows, int rp, int n_splits) {
+  const int row = blockIdx.x;
+  float m = NEG_SENTINEL;
+  for (int s = 0; s < n_splits; ++s) m = fmaxf(m, part_ml[((size_t)s * n_rows + row) * 2]);
+  float l = 0.f;
+  for (int s = 0; s < n_splits; ++s) {
+    const float* ml = part_ml + ((size_t)s * n_rows + row) * 2;
+    if (ml[0] > NEG_THRESHOLD) l += ml[1] * exp2f(ml[0] - m);
+  }
+  const float inv_l = l > 0.f ? 1.f / l : 0.f;
+  for (int d = threadIdx.x; d < rp; d += blockDim.x) {
+    float o = 0.f;
+    for (int s = 0; s < n_splits; ++s) {
+      const float ms = part_ml[((size_t)s * n_rows + row) * 2];
+      if (ms > NEG_THRESHOLD) o += part_o[((size_t)s * n_rows + row) * rp + d] * exp2f(ms - m);
+    }
+    out[(size_t)row * rp + d] = f32_to_bf16(o * inv_l);
+  }
+}
+
+// ---------------------------------------------------------- simple kernel
+
+// one workgroup of 256 per (token, head): a key per thread for the scores, a
+// latent dimension per thread for the sum
+template <typename T>
+__global__ __launch_bounds__(256) void latent_attn_simple(
+    const T* __restrict__ q,      // [T, H, RP]
+    const T* __restrict__ cache,  // [num_pages, PAGE, RP]
+    T* __restrict__ out,          // [T, H, RP]
+    PagedRows b, int heads, int rp, int window, float scale) {
+  extern __shared__ float sm[];
+  float* qs = sm;           // [rp]
+  float* acc = qs + rp;     // [rp]
+  float* p = acc + rp;      // [256]
+  long* at = reinterpret_cast<long*>(p + 256);  // [256]
+  __shared__ float red[4];
+  const int tid = threadIdx.x;
+  const int tok = blockIdx.x / heads;
+  const int seq = b.owner[tok];
+  const int pos = b.pos[tok];
+  const int lo = window > 0 ? max(0, pos - window + 1) : 0;
+  for (int d = tid; d < rp; d += 256) {
+    qs[d] = load_f32(q + (size_t)blockIdx.x * rp + d);
+    acc[d] = 0.f;
+  }
+  float m = NEG_SENTINEL, l = 0.f;
+  for (int j0 = lo; j0 <= pos; j0 += 256) {
+    __syncthreads();
+    const int key = j0 + tid;
+    float s = NEG_SENTINEL;
+    long row = -1;
+    if (key <= pos) row = cache_row(b, seq, key);
+    if (row >= 0) {
+      float dot = 0.f;
+      for (int d = 0; d < rp; ++d) dot = fmaf(qs[d], load_f32(cache + (size_t)row * rp + d), dot);
+      s = dot * scale;
+    }
+    at[tid] = row;
+    float mx = wave_reduce_max(s);
+    if ((tid & 63) == 0) red[tid >> 6] = mx;
+    __syncthreads();
+    const float m_new = fmaxf(m, fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])));
+    const float corr = m <= NEG_THRESHOLD ? 0.f : expf(m - m_new);
+    const float e = s <= NEG_THRESHOLD ? 0.f : expf(s - m_new);
+    p[tid] = e;
+    __syncthreads();  // red is read, p and at are written
+    const float sum = wave_reduce_sum(e);
+    if ((tid & 63) == 0) red[tid >> 6] = sum;
+    __syncthreads();
+    l = l * corr + ((red[0] + red[1]) + (red[2] + red[3]));
+    m = m_new;
+    const int n = min(256, pos - j0 + 1);
+    for (int d = tid; d < rp; d += 256) {
+      float o = acc[d] * corr;
+      for (int j = 0; j < n; ++j)
+        if (at[j] >= 0) o = fmaf(p[j], load_f32(cache + (size_t)at[j] * rp + d), o);
+      acc[d] = o;
+    }
+  }
+  const float inv_l = l > 0.f ? 1.f / l : 0.f;
+  for (int d = tid; d < rp; d += 256) store_f32(out + (size_t)blockIdx.x * rp + d, acc[d] * inv_l);
+}
+
+// ---------------------------------------------------------- latent writing
+
+// c = y / sqrt(mean(y^2) + eps) * w of one token, stored at its place
+template <typename TY, typename TC>
+__global__ __launch_bounds__(256) void latent_write_kernel(
+    const TY* __restrict__ y, int y_stride,  // [T, y_stride], rank values each
+    const float* __restrict__ w,             // [rank]
+    TC* __restrict__ cache, PagedRows b, int rank, int rp, float eps) {
+  __shared__ float red[4];
+  const int tid = threadIdx.x;
+  const TY* row = y + (size_t)blockIdx.x * y_stride;
+  float ss = 0.f;
+  for (int d = tid; d < rank; d += 256) {
+    const float v = load_f32(row + d);
+    ss = fmaf(v, v, ss);
+  }
+  ss = wave_reduce_sum(ss);
+  if ((tid & 63) == 0) red[tid >> 6] = ss;
+  __syncthreads();
+  const float inv = 1.f / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / rank + eps);
+  const long at = cache_row(b, b.owner[blockIdx.x], b.pos[blockIdx.x]);
+  if (at < 0) return;
+  for (int d = tid; d < rp; d += 256)
+    store_f32(cache + (size_t)at * rp + d, d < rank ? load_f32(row + d) * inv * w[d] : 0.f);
+}
+
+// ------------------------------------------------------------------- host
+
+static PagedRows paged_rows(const torch::Tensor& pos, const torch::Tensor& owner, const torch::Tensor& tables,
+                            const torch::Tensor& cache, int64_t tokens) {
+  TORCH_CHECK(cache.is_cuda() && cache.dim() == 3 && cache.size(1) == PAGE && cache.is_contiguous(),
+              "the cache must be [pages, ", PAGE, ", width]");
+  for (const auto& t : {pos, owner, tables})
+    TORCH_CHECK(t.is_cuda() && t.dtype() == torch::kInt32 && t.is_contiguous(), "int32 device metadata expected");
+  TORCH_CHECK(pos.numel() == tokens && owner.numel() == tokens && tables.dim() == 2, "metadata does not fit the rows");
+  return PagedRows{pos.data_ptr<int>(), owner.data_ptr<int>(), tables.data_ptr<int>(),
+                   (int)tables.size(1), (int)cache.size(0)};
+}
+
+#define BF16P(t) reinterpret_cast<unsigned short*>((t).data_ptr())
+
+template <int RC>
+static void launch_mfma(dim3 grid, int nw, const torch::Tensor& q, const torch::Tensor& cache, torch::Tensor& out,
+                        torch::Tensor& part_o, torch::Tensor& part_ml, const torch::Tensor& tiles, PagedRows b,
+                        int heads, int rp, int window, float scale, int n_splits) {
+  const size_t lds = LKVT * (RC * 32 + LPAD) * 2 + RC * 32 * (LKVT + LPAD) * 2 + (size_t)nw * 16 * (LKVT + LPAD) * 2;
+  static bool allowed = false;
+  if (!allowed) {
+    const size_t most = LKVT * (RC * 32 + LPAD) * 2 + RC * 32 * (LKVT + LPAD) * 2 + 4 * 16 * (LKVT + LPAD) * 2;
+    if (most > 65536) {
+      hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<RC>),
+                                         hipFuncAttributeMaxDynamicSharedMemorySize, (int)most);
+      TORCH_CHECK(e == hipSuccess, "LDS request refused: ", hipGetErrorString(e));
+    }
+    allowed = true;
+  }
+  latent_attn_kernel<RC><<<grid, nw * WAVE, lds, at::cuda::getCurrentCUDAStream()>>>(
+      BF16P(q), BF16P(cache), BF16P(out), part_o.numel() ? part_o.data_ptr<float>() : nullptr,
+      part_ml.numel() ? part_ml.data_ptr<float>() : nullptr, tiles.data_ptr<int>(), b, (int)q.size(0), heads, rp,
+      window, scale * 1.4426950408889634f, n_splits);
+}
+
+torch::Tensor latent_attention(
+    torch::Tensor q,       // [T, H, RP] bf16 or f32
+    torch::Tensor cache,   // [pages, PAGE, RP], dtype of q
+    torch::Tensor pos, torch::Tensor owner, torch::Tensor tables,
+    torch::Tensor tiles,   // [n, 2] int32 runs of at most run_tokens tokens
+    int64_t run_tokens,
+    int64_t max_keys,      // most keys that any row sees
+    int64_t window, double scale, int64_t splits) {
+  TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() && q.dtype() == cache.dtype());
+  const int t = q.size(0), heads = q.size(1), rp = q.size(2);
+  TORCH_CHECK(cache.size(2) == rp && rp % 32 == 0, "latent width mismatch");
+  const PagedRows b = paged_rows(pos, owner, tables, cache, t);
+  auto out = torch::empty_like(q);
+  auto stream = at::cuda::getCurrentCUDAStream();
+  const bool f32 = q.dtype() == torch::kFloat32;
+  TORCH_CHECK(f32 || q.dtype() == torch::kBFloat16);
+  if (f32 || rp > 512) {
+    const size_t lds = (2 * (size_t)rp + 256) * 4 + 256 * 8;
+    TORCH_CHECK(lds <= 65536, "latent size ", rp, " is not supported");
+    if (f32)
+      latent_attn_simple<float><<<t * heads, 256, lds, stream>>>(
+          q.data_ptr<float>(), cache.data_ptr<float>(), out.data_ptr<float>(), b, heads, rp, (int)window, (float)scale);
+    else
+      latent_attn_simple<unsigned short><<<t * heads, 256, lds, stream>>>(
+          BF16P(q), BF16P(cache), BF16P(out), b, heads, rp, (int)window, (float)scale);
+    HIP_CHECK_LAST();
+    return out;
+  }
+  TORCH_CHECK(tiles.is_cuda() && tiles.dtype() == torch::kInt32 && tiles.is_contiguous() && tiles.dim() == 2);
+  const int rows = (int)run_tokens * heads;
+  const int nw = std::min(4, (rows + 15) / 16);
+  dim3 grid(tiles.size(0), (rows + 16 * nw - 1) / (16 * nw), 1);
+  int n_splits = (int)splits;
+  if (n_splits <= 0) {
+    // enough workgroups for the chip, at least two key tiles each
+    const long wgs = (long)grid.x * grid.y;
+    n_splits = (int)std::max(1L, std::min({(long)((max_keys + 63) / 64), 512 / std::max(1L, wgs), 64L}));
+  }
+  grid.z = n_splits;
+  auto f32o = q.options().dtype(torch::kFloat32);
+  auto part_o = torch::empty({n_splits > 1 ? (long)n_splits * t * heads * rp : 0}, f32o);
+  auto part_ml = torch::empty({n_splits > 1 ? (long)n_splits * t * heads * 2 : 0}, f32o);
+#define LA(RC) launch_mfma<RC>(grid, nw, q, cache, out, part_o, part_ml, tiles, b, heads, rp, (int)window, (float)scale, n_splits)
+  const int rc = rp / 32;
+  if (rc <= 1) LA(1);
+  else if (rc <= 2) LA(2);
+  else if (rc <= 3) LA(3);
+  else if (rc <= 4) LA(4);
+  else if (rc <= 6) LA(6);
+  else if (rc <= 8) LA(8);
+  else if (rc <= 12) LA(12);
+  else LA(16);
+#undef LA
+  HIP_CHECK_LAST();
+  if (n_splits > 1) {
+    latent_attn_combine<<<t * heads, 128, 0, stream>>>(
+        part_o.data_ptr<float>(), part_ml.data_ptr<float>(), BF16P(out), t * heads, rp, n_splits);
+    HIP_CHECK_LAST();
+  }
+  return out;
+}
+
+void latent_write(
+    torch::Tensor y,      // [T, >= offset + rank] f32 or bf16; columns [offset, offset + rank)
+    int64_t offset,
+    torch::Tensor w,      // [rank] f32
+    torch::Tensor cache, torch::Tensor pos, torch::Tensor owner, torch::Tensor tables, double eps) {
+  TORCH_CHECK(y.is_cuda() && y.dim() == 2 && y.is_contiguous());
+  TORCH_CHECK(w.is_cuda() && w.dtype() == torch::kFloat32 && w.is_contiguous());
+  const int rank = w.numel(), rp = cache.size(2), stride = y.size(1), t = y.size(0);
+  TORCH_CHECK(rank <= rp && offset + rank <= stride, "latent sizes do not fit");
+  const PagedRows b = paged_rows(pos, owner, tables, cache, t);
+  auto stream = at::cuda::getCurrentCUDAStream();
+  const bool yf = y.dtype() == torch::kFloat32, cf = cache.dtype() == torch::kFloat32;
+  TORCH_CHECK((yf || y.dtype() == torch::kBFloat16) && (cf || cache.dtype() == torch::kBFloat16));
+#define LW(TY, TC, YP, CP) \
+  latent_write_kernel<TY, TC><<<t, 256, 0, stream>>>(YP + offset, stride, w.data_ptr<float>(), CP, b, rank, rp, (float)eps)
+  if (yf && cf) LW(float, float, y.data_ptr<float>(), cache.data_ptr<float>());
+  else if (yf) LW(float, unsigned short, y.data_ptr<float>(), BF16P(cache));
+  else if (cf) LW(unsigned short, float, BF16P(y), cache.data_ptr<float>());
+  else LW(unsigned short, unsigned short, BF16P(y), BF16P(cache));
+#undef LW
+  HIP_CHECK_LAST();
+}

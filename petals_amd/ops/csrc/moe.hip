@@ -443,14 +443,16 @@ torch::Tensor gemv_bf16_moe(
     int64_t k_per_tok,
     torch::Tensor workspace,
     int64_t epilogue,
-    int64_t splits_override) {
+    int64_t splits_override,
+    double limit,            // EPI_CLAMPED_SWIGLU_F32 only
+    double alpha) {
   TORCH_CHECK(wt_all.is_cuda() && wt_all.dtype() == torch::kBFloat16 && wt_all.dim() == 3);
   TORCH_CHECK(x.dtype() == torch::kFloat32 && x.dim() == 2);
   TORCH_CHECK(sel.dtype() == torch::kInt32 && sel.is_contiguous());
   const int in_dim = wt_all.size(1), out_dim = wt_all.size(2);
   const int rows = sel.size(0);
   TORCH_CHECK(x.size(1) == in_dim && rows == x.size(0) * k_per_tok);
-  TORCH_CHECK(rows <= 16, "moe gemv supports batch*k <= 16");
+  TORCH_CHECK(rows <= 64, "moe gemv supports batch*k <= 64");
 
   const long out_waves = (out_dim + GEMV_OUT_PER_WAVE - 1) / GEMV_OUT_PER_WAVE;
   long splits = splits_override > 0 ? splits_override : (768 + out_waves * rows - 1) / (out_waves * rows);
@@ -474,7 +476,7 @@ torch::Tensor gemv_bf16_moe(
   HIP_CHECK_LAST();
   return launch_gemv_reduce(
       partials, c10::nullopt, c10::nullopt, (int)splits, rows, out_dim, (int)epilogue,
-      x.options(), wt_all.options());
+      x.options(), wt_all.options(), c10::nullopt, ClampedGate{(float)limit, (float)alpha});
 }
 
 torch::Tensor gemv_nf4_moe(

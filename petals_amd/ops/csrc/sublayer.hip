@@ -1,0 +1,462 @@
+// Sublayer kernels for blocks that norm each sublayer's OUTPUT and keep the
+// residual stream in 32-bit (CDNA4, gfx950).
+//
+//   sublayer_out      sum of a token's (weighted) sublayer rows -> RMS norm with
+//                     a zero-centered weight -> + residual, and, for a sublayer
+//                     that is followed by routed experts, the 32-bit router:
+//                     logits, softmax over all experts, top-k
+//   batched_linear    out[t, h, n] = sum_k a[t, h, k] w[h, n, k]: the per-head
+//                     projections of latent attention, MFMA for bf16 weights
+//   clamped_swiglu    g * sigmoid(alpha g) * (u + 1), g and u clamped
+//   moe_group         expert-sorted, tile-padded (token, slot) pairs for moe_gemm
+//   moe_linear_f32    expert products in 32-bit
+
+#include "common.h"
+#include <torch/extension.h>
+#include <ATen/cuda/CUDAContext.h>
+
+using bf16x8 = __attribute__((ext_vector_type(8))) short;
+using f32x4 = __attribute__((ext_vector_type(4))) float;
+
+#define BF16P(t) reinterpret_cast<unsigned short*>((t).data_ptr())
+
+__device__ __forceinline__ float ld(const float* p) { return *p; }
+__device__ __forceinline__ float ld(const unsigned short* p) { return bf16_to_f32(*p); }
+__device__ __forceinline__ void st(float* p, float v) { *p = v; }
+__device__ __forceinline__ void st(unsigned short* p, float v) { *p = f32_to_bf16(v); }
+
+// sum over the workgroup, the same value in every thread; red holds one float
+// per wave and is free again on return
+__device__ __forceinline__ float block_sum(float v, float* red) {
+  v = wave_reduce_sum(v);
+  if ((threadIdx.x & (WAVE - 1)) == 0) red[threadIdx.x / WAVE] = v;
+  __syncthreads();
+  float s = 0.f;
+  for (int i = 0; i < (int)blockDim.x / WAVE; ++i) s += red[i];
+  __syncthreads();
+  return s;
+}
+
+// ---------------------------------------------------------- sublayer output
+
+// One workgroup per token.
+//   y [T*k, ys]     sublayer rows; a token's k rows are summed with slot_w
+//   x [T, dp]       residual before, xo after (null: the norm alone is written)
+//   xb              bf16 copy of xo or null
+//   router [E, dp]  or null; sel/sel_w [T, top] get the experts and their scores
+template <typename TY, typename TW>
+__global__ __launch_bounds__(1024) void sublayer_out_kernel(
+    const TY* __restrict__ y, int ys, int k, const float* __restrict__ slot_w,
+    const float* __restrict__ norm_w, float eps,
+    const float* __restrict__ x, float* __restrict__ xo, unsigned short* __restrict__ xb,
+    const TW* __restrict__ router, int experts, int top, int* __restrict__ sel, float* __restrict__ sel_w,
+    int d, int dp) {
+  extern __shared__ float sm[];
+  float* row = sm;          // [dp]
+  float* logit = row + dp;  // [experts]
+  __shared__ float red[16];
+  const int tid = threadIdx.x, nt = blockDim.x;
+  const size_t t = blockIdx.x;
+
+  float ss = 0.f;
+  for (int c = tid; c < d; c += nt) {
+    float v;
+    if (slot_w) {
+      v = 0.f;
+      for (int j = 0; j < k; ++j) v = fmaf(slot_w[t * k + j], ld(y + (t * k + j) * ys + c), v);
+    } else {
+      v = ld(y + t * ys + c);
+    }
+    row[c] = v;
+    ss = fmaf(v, v, ss);
+  }
+  const float inv = 1.f / sqrtf(block_sum(ss, red) / d + eps);
+  for (int c = tid; c < dp; c += nt) {
+    float v = 0.f;
+    if (c < d) {
+      v = row[c] * inv * (1.f + norm_w[c]);
+      if (x) v += x[t * dp + c];
+    }
+    xo[t * dp + c] = v;
+    if (xb) xb[t * dp + c] = f32_to_bf16(v);
+    row[c] = v;
+  }
+  if (!router) return;
+  __syncthreads();
+  const int wave = tid / WAVE, lane = tid & (WAVE - 1);
+  for (int e = wave; e < experts; e += nt / WAVE) {
+    float z = 0.f;
+    for (int c = lane; c < d; c += WAVE) z = fmaf(row[c], ld(router + (size_t)e * dp + c), z);
+    z = wave_reduce_sum(z);
+    if (lane == 0) logit[e] = z;
+  }
+  __syncthreads();
+  if (wave != 0) return;
+  float mx = NEG_SENTINEL;
+  for (int e = lane; e < experts; e += WAVE) mx = fmaxf(mx, logit[e]);
+  mx = wave_reduce_max(mx);
+  float sum = 0.f;
+  for (int e = lane; e < experts; e += WAVE) sum += expf(logit[e] - mx);
+  sum = wave_reduce_sum(sum);
+  for (int j = 0; j < top; ++j) {
+    float best = NEG_SENTINEL * 2.f;
+    int arg = experts;
+    for (int e = lane; e < experts; e += WAVE)
+      if (logit[e] > best) {
+        best = logit[e];
+        arg = e;
+      }
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) {
+      const float ob = __shfl_xor(best, off, WAVE);
+      const int oa = __shfl_xor(arg, off, WAVE);
+      if (ob > best || (ob == best && oa < arg)) {
+        best = ob;
+        arg = oa;
+      }
+    }
+    if (arg >= experts) arg = 0;  // logits that compare with nothing (NaN)
+    if (lane == 0) {
+      sel[t * top + j] = arg;
+      sel_w[t * top + j] = expf(best - mx) / sum;
+    }
+    if ((arg & (WAVE - 1)) == lane) logit[arg] = NEG_SENTINEL * 3.f;  // taken; this lane alone reads it
+  }
+}
+
+// ----------------------------------------------------------- batched linear
+
+__device__ __forceinline__ bf16x8 frag8(const unsigned short* p, int k, int k_dim, bool wide) {
+  if (wide && k + 8 <= k_dim) return *reinterpret_cast<const bf16x8*>(p + k);
+  short v[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = k + e < k_dim ? (short)p[k + e] : (short)0;
+  return bf16x8{v[0], v[1], v[2], v[3], v[4], v[5], v[6], v[7]};
+}
+__device__ __forceinline__ bf16x8 frag8(const float* p, int k, int k_dim, bool wide) {
+  short v[8];
+  if (wide && k + 8 <= k_dim) {
+    const f32x4 a = *reinterpret_cast<const f32x4*>(p + k), b = *reinterpret_cast<const f32x4*>(p + k + 4);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      v[e] = (short)f32_to_bf16(a[e]);
+      v[4 + e] = (short)f32_to_bf16(b[e]);
+    }
+  } else {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[e] = k + e < k_dim ? (short)f32_to_bf16(p[k + e]) : (short)0;
+  }
+  return bf16x8{v[0], v[1], v[2], v[3], v[4], v[5], v[6], v[7]};
+}
+
+// A wave computes 16*MT rows x 16*NT columns of one head; 4 waves side by side
+// in n. Fragments come straight from global memory (the weights are read once
+// per 16*MT rows; k is short or the rows are few wherever this runs).
+template <typename TA, typename TO, int MT, int NT>
+__global__ __launch_bounds__(256) void batched_linear_kernel(
+    const TA* __restrict__ a, long a_t, long a_h,   // strides of rows and heads
+    const unsigned short* __restrict__ w,           // [H, N, K]
+    TO* __restrict__ out, long o_t, long o_h, int t_dim, int n_dim, int k_dim, bool a_wide, bool w_wide) {
+  const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;
+  const int col = lane & 15, hi = lane >> 4;
+  const int n0 = (blockIdx.x * 4 + wave) * 16 * NT;
+  const int t0 = blockIdx.y * 16 * MT;
+  const size_t h = blockIdx.z;
+  if (n0 >= n_dim) return;
+  const TA* ap[MT];
+  const unsigned short* wp[NT];
+  bool a_ok[MT], w_ok[NT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    const int t = t0 + m * 16 + col;
+    a_ok[m] = t < t_dim;
+    ap[m] = a + (size_t)(a_ok[m] ? t : 0) * a_t + h * a_h;
+  }
+#pragma unroll
+  for (int n = 0; n < NT; ++n) {
+    const int c = n0 + n * 16 + col;
+    w_ok[n] = c < n_dim;
+    wp[n] = w + (h * n_dim + (w_ok[n] ? c : 0)) * (size_t)k_dim;
+  }
+  f32x4 acc[MT][NT];
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int n = 0; n < NT; ++n) acc[m][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k0 = 0; k0 < k_dim; k0 += 32) {
+    bf16x8 af[MT], wf[NT];
+#pragma unroll
+    for (int n = 0; n < NT; ++n)
+      wf[n] = w_ok[n] ? frag8(wp[n], k0 + hi * 8, k_dim, w_wide) : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+      af[m] = a_ok[m] ? frag8(ap[m], k0 + hi * 8, k_dim, a_wide) : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int n = 0; n < NT; ++n)
+        acc[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af[m], wf[n], acc[m][n], 0, 0, 0);
+  }
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = t0 + m * 16 + hi * 4 + r;
+      if (t >= t_dim) continue;
+#pragma unroll
+      for (int n = 0; n < NT; ++n) {
+        const int c = n0 + n * 16 + col;
+        if (c < n_dim) st(out + (size_t)t * o_t + h * o_h + c, acc[m][n][r]);
+      }
+    }
+}
+
+__global__ __launch_bounds__(256) void batched_linear_f32_kernel(
+    const float* __restrict__ a, long a_t, long a_h, const float* __restrict__ w,
+    float* __restrict__ out, long o_t, long o_h, int n_dim, int k_dim) {
+  const int n = blockIdx.x * 4 + threadIdx.x / WAVE;  // a wave per output
+  if (n >= n_dim) return;
+  const int lane = threadIdx.x & (WAVE - 1);
+  const float* ap = a + (size_t)blockIdx.y * a_t + blockIdx.z * a_h;
+  const float* wp = w + ((size_t)blockIdx.z * n_dim + n) * k_dim;
+  float s = 0.f;
+  for (int k = lane; k < k_dim; k += WAVE) s = fmaf(ap[k], wp[k], s);
+  s = wave_reduce_sum(s);
+  if (lane == 0) out[(size_t)blockIdx.y * o_t + blockIdx.z * o_h + n] = s;
+}
+
+// -------------------------------------------------------------- activation
+
+template <typename T>
+__global__ __launch_bounds__(256) void clamped_swiglu_kernel(
+    const T* __restrict__ gu, T* __restrict__ out, int half, long total, float limit, float alpha) {
+  const long i = ((long)blockIdx.x * 256 + threadIdx.x) * 8;
+  if (i >= total) return;  // half % 8 == 0: a group of 8 never crosses a row
+  const long r = i / half;
+  const T* g = gu + r * 2 * half + (i - r * half);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float gv = fminf(ld(g + e), limit);
+    const float uv = fmaxf(fminf(ld(g + half + e), limit), -limit);
+    st(out + i + e, gv / (1.f + expf(-alpha * gv)) * (uv + 1.f));
+  }
+}
+
+// ------------------------------------------------------------ expert groups
+
+// One workgroup. counts -> padded offsets -> scatter; every sorted slot and
+// every tile is written. The order of an expert's pairs is not fixed, which no
+// result depends on (each pair is a row of its own).
+__global__ __launch_bounds__(1024) void moe_group_kernel(
+    const int* __restrict__ sel, int pairs, int experts, int mt, int slots,
+    int* __restrict__ sorted_pairs, int* __restrict__ tile_expert) {
+  extern __shared__ int cnt[];  // [experts] counts, then next free slot
+  int* end = cnt + experts;     // [experts] end of the padded segment
+  const int tid = threadIdx.x;
+  for (int e = tid; e < experts; e += blockDim.x) cnt[e] = 0;
+  for (int i = tid; i < slots; i += blockDim.x) sorted_pairs[i] = -1;
+  for (int i = tid; i < slots / mt; i += blockDim.x) tile_expert[i] = -1;
+  __syncthreads();
+  for (int i = tid; i < pairs; i += blockDim.x) {
+    const int e = sel[i];
+    if (e >= 0 && e < experts) atomicAdd(&cnt[e], 1);
+  }
+  __syncthreads();
+  if (tid == 0) {
+    int at = 0;
+    for (int e = 0; e < experts; ++e) {
+      const int padded = (cnt[e] + mt - 1) / mt * mt;
+      cnt[e] = at;
+      at += padded;
+      end[e] = at;
+    }
+  }
+  __syncthreads();
+  for (int e = tid; e < experts; e += blockDim.x)
+    for (int i = cnt[e]; i < end[e]; i += mt) tile_expert[i / mt] = e;
+  __syncthreads();
+  for (int i = tid; i < pairs; i += blockDim.x) {
+    const int e = sel[i];
+    if (e >= 0 && e < experts) sorted_pairs[atomicAdd(&cnt[e], 1)] = i;
+  }
+}
+
+__global__ __launch_bounds__(64) void moe_linear_f32_kernel(
+    const float* __restrict__ w,  // [E, in, out]
+    const float* __restrict__ x,  // [rows / k, in]
+    const int* __restrict__ sel,  // [rows]
+    float* __restrict__ out,      // [rows, out]
+    int experts, int k, int in_dim, int out_dim) {
+  const int c = blockIdx.x * 64 + threadIdx.x;
+  const int e = sel[blockIdx.y];
+  if (c >= out_dim || e < 0 || e >= experts) return;
+  const float* wp = w + (size_t)e * in_dim * out_dim + c;
+  const float* xr = x + (size_t)(blockIdx.y / k) * in_dim;
+  float s = 0.f;
+  for (int i = 0; i < in_dim; ++i) s = fmaf(xr[i], wp[(size_t)i * out_dim], s);
+  out[(size_t)blockIdx.y * out_dim + c] = s;
+}
+
+// -------------------------------------------------------------------- host
+
+static bool is_f32(const torch::Tensor& t) {
+  TORCH_CHECK(t.is_cuda() && (t.dtype() == torch::kFloat32 || t.dtype() == torch::kBFloat16));
+  return t.dtype() == torch::kFloat32;
+}
+
+// Returns (xo [T, dp] f32, xb [T, dp] bf16 or empty, sel [T, top], sel_w [T, top])
+std::vector<torch::Tensor> sublayer_out(
+    torch::Tensor y,                       // [T*k, ys]
+    c10::optional<torch::Tensor> slot_w,   // [T, k] f32
+    torch::Tensor norm_w,                  // [d] f32
+    double eps,
+    c10::optional<torch::Tensor> x,        // [T, dp] f32
+    int64_t dp,
+    bool want_bf16,
+    c10::optional<torch::Tensor> router,   // [E, dp]
+    int64_t top) {
+  const bool yf = is_f32(y);
+  TORCH_CHECK(y.dim() == 2 && y.is_contiguous() && norm_w.is_contiguous() && norm_w.dtype() == torch::kFloat32);
+  const int d = norm_w.numel();
+  int k = 1;
+  long t = y.size(0);
+  const float* sw = nullptr;
+  if (slot_w.has_value()) {
+    TORCH_CHECK(slot_w->is_contiguous() && slot_w->dtype() == torch::kFloat32 && slot_w->dim() == 2);
+    k = slot_w->size(1);
+    t = slot_w->size(0);
+    sw = slot_w->data_ptr<float>();
+  }
+  TORCH_CHECK(y.size(0) == t * k && y.size(1) >= d && dp >= d, "sublayer rows do not fit");
+  auto f32o = y.options().dtype(torch::kFloat32);
+  auto xo = torch::empty({t, (long)dp}, f32o);
+  auto xb = torch::empty({want_bf16 ? t : 0, (long)dp}, y.options().dtype(torch::kBFloat16));
+  const float* xp = nullptr;
+  if (x.has_value()) {
+    TORCH_CHECK(x->is_contiguous() && x->dtype() == torch::kFloat32 && x->size(0) == t && x->size(1) == dp);
+    xp = x->data_ptr<float>();
+  }
+  int experts = 0;
+  bool rf = false;
+  const void* rp = nullptr;
+  if (router.has_value()) {
+    rf = is_f32(*router);
+    TORCH_CHECK(router->is_contiguous() && router->dim() == 2 && router->size(1) == dp);
+    experts = router->size(0);
+    TORCH_CHECK(top >= 1 && top <= experts);
+    rp = router->data_ptr();
+  }
+  auto sel = torch::empty({experts ? t : 0, (long)top}, y.options().dtype(torch::kInt32));
+  auto sel_w = torch::empty({experts ? t : 0, (long)top}, f32o);
+  const size_t lds = ((size_t)dp + experts) * 4;
+  TORCH_CHECK(lds <= 65536 - 64, "width ", d, " with ", experts, " experts is not supported");
+  const int threads = t < 64 ? 1024 : 256;
+  auto stream = at::cuda::getCurrentCUDAStream();
+  unsigned short* xbp = want_bf16 ? BF16P(xb) : nullptr;
+  int* selp = experts ? sel.data_ptr<int>() : nullptr;
+  float* selwp = experts ? sel_w.data_ptr<float>() : nullptr;
+  if (t > 0) {
+#define SO(TY, TW, YP)                                                                                     \
+  sublayer_out_kernel<TY, TW><<<t, threads, lds, stream>>>(                                                \
+      YP, (int)y.size(1), k, sw, norm_w.data_ptr<float>(), (float)eps, xp, xo.data_ptr<float>(), xbp,      \
+      reinterpret_cast<const TW*>(rp), experts, (int)top, selp, selwp, d, (int)dp)
+    if (yf && rf) SO(float, float, y.data_ptr<float>());
+    else if (yf) SO(float, unsigned short, y.data_ptr<float>());
+    else if (rf) SO(unsigned short, float, BF16P(y));
+    else SO(unsigned short, unsigned short, BF16P(y));
+#undef SO
+    HIP_CHECK_LAST();
+  }
+  return {xo, xb, sel, sel_w};
+}
+
+// a: [T, H, K] view (any row and head stride, unit k stride); w: [H, N, K]
+torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32) {
+  const bool af = is_f32(a), wf = is_f32(w);
+  TORCH_CHECK(a.dim() == 3 && w.dim() == 3 && w.is_contiguous() && a.stride(2) == 1);
+  const long t = a.size(0), h = a.size(1), k = a.size(2), n = w.size(1);
+  TORCH_CHECK(w.size(0) == h && w.size(2) == k, "batched_linear shapes");
+  TORCH_CHECK(!wf || (af && out_f32), "32-bit weights need 32-bit rows");
+  auto out = torch::empty({t, h, n}, a.options().dtype(out_f32 ? torch::kFloat32 : torch::kBFloat16));
+  if (t == 0) return out;
+  auto stream = at::cuda::getCurrentCUDAStream();
+  const long at_ = a.stride(0), ah = a.stride(1), ot = h * n, oh = n;
+  if (wf) {
+    TORCH_CHECK(t <= 65535 && h <= 65535);
+    batched_linear_f32_kernel<<<dim3((n + 3) / 4, t, h), 256, 0, stream>>>(
+        a.data_ptr<float>(), at_, ah, w.data_ptr<float>(), out.data_ptr<float>(), ot, oh, n, k);
+    HIP_CHECK_LAST();
+    return out;
+  }
+  const size_t ab = af ? 4 : 2;
+  const bool a_wide = (reinterpret_cast<uintptr_t>(a.data_ptr()) % 16 == 0) && (at_ * ab) % 16 == 0 && (ah * ab) % 16 == 0;
+  const bool w_wide = k % 8 == 0;
+#define BL(TA, TO, MT, NT, AP, OP)                                                                          \
+  batched_linear_kernel<TA, TO, MT, NT><<<dim3((n + 64 * NT - 1) / (64 * NT), (t + 16 * MT - 1) / (16 * MT), h), \
+                                          256, 0, stream>>>(AP, at_, ah, BF16P(w), OP, ot, oh, t, n, k, a_wide, w_wide)
+#define BLO(TA, MT, NT, AP)                                         \
+  do {                                                              \
+    if (out_f32) BL(TA, float, MT, NT, AP, out.data_ptr<float>());  \
+    else BL(TA, unsigned short, MT, NT, AP, BF16P(out));            \
+  } while (0)
+  if (af) {
+    if (t <= 16) BLO(float, 1, 1, a.data_ptr<float>()); else BLO(float, 4, 2, a.data_ptr<float>());
+  } else {
+    if (t <= 16) BLO(unsigned short, 1, 1, BF16P(a)); else BLO(unsigned short, 4, 2, BF16P(a));
+  }
+#undef BLO
+#undef BL
+  HIP_CHECK_LAST();
+  return out;
+}
+
+torch::Tensor clamped_swiglu(torch::Tensor gu, double limit, double alpha) {
+  const bool f = is_f32(gu);
+  TORCH_CHECK(gu.dim() == 2 && gu.is_contiguous() && gu.size(1) % 16 == 0, "gate|up rows of 2 x (a multiple of 8)");
+  const int half = gu.size(1) / 2;
+  auto out = torch::empty({gu.size(0), half}, gu.options());
+  const long total = out.numel();
+  if (total == 0) return out;
+  const long blocks = (total / 8 + 255) / 256;
+  auto stream = at::cuda::getCurrentCUDAStream();
+  if (f)
+    clamped_swiglu_kernel<float><<<blocks, 256, 0, stream>>>(
+        gu.data_ptr<float>(), out.data_ptr<float>(), half, total, (float)limit, (float)alpha);
+  else
+    clamped_swiglu_kernel<unsigned short><<<blocks, 256, 0, stream>>>(
+        BF16P(gu), BF16P(out), half, total, (float)limit, (float)alpha);
+  HIP_CHECK_LAST();
+  return out;
+}
+
+// sel [R] expert of each (token, slot) pair -> (sorted_pairs, tile_expert), see moe.hip
+std::vector<torch::Tensor> moe_group(torch::Tensor sel, int64_t experts, int64_t mt) {
+  TORCH_CHECK(sel.is_cuda() && sel.dtype() == torch::kInt32 && sel.is_contiguous());
+  TORCH_CHECK(experts >= 1 && experts <= 4096 && mt >= 1);
+  const long r = sel.numel();
+  // at most min(r, experts) segments end in a partly filled tile
+  const long slots = (r + std::min(r, (long)experts) * (mt - 1) + mt - 1) / mt * mt;
+  auto pairs = torch::empty({slots}, sel.options());
+  auto tiles = torch::empty({slots / mt}, sel.options());
+  moe_group_kernel<<<1, 1024, experts * 8, at::cuda::getCurrentCUDAStream()>>>(
+      sel.data_ptr<int>(), r, experts, mt, slots, pairs.data_ptr<int>(), tiles.data_ptr<int>());
+  HIP_CHECK_LAST();
+  return {pairs, tiles};
+}
+
+torch::Tensor moe_linear_f32(torch::Tensor w, torch::Tensor x, torch::Tensor sel, int64_t k) {
+  TORCH_CHECK(is_f32(w) && is_f32(x) && w.dim() == 3 && x.dim() == 2 && w.is_contiguous() && x.is_contiguous());
+  TORCH_CHECK(sel.is_cuda() && sel.dtype() == torch::kInt32 && sel.is_contiguous());
+  const long rows = sel.numel();
+  TORCH_CHECK(x.size(1) == w.size(1) && x.size(0) * k == rows);
+  auto out = torch::empty({rows, w.size(2)}, x.options());
+  const long step = std::max(1L, 32768 / k) * k;  // rows per launch (grid.y), whole tokens
+  for (long r = 0; r < rows; r += step)
+    moe_linear_f32_kernel<<<dim3((w.size(2) + 63) / 64, std::min(step, rows - r)), 64, 0,
+                            at::cuda::getCurrentCUDAStream()>>>(
+        w.data_ptr<float>(), x.data_ptr<float>() + r / k * w.size(1), sel.data_ptr<int>() + r,
+        out.data_ptr<float>() + r * w.size(2), (int)w.size(0), (int)k, (int)w.size(1), (int)w.size(2));
+  HIP_CHECK_LAST();
+  return out;
+}

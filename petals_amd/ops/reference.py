@@ -157,3 +157,67 @@ def build_alibi_bias(
     # bloom-style: bias depends only on key position distance from the last axis
     bias = slopes[:, None, None] * k_pos[None, None, :]  # [heads, 1, kv_len]
     return bias.unsqueeze(0).to(dtype).expand(1, n_heads, q_len, kv_len)
+
+
+# ------------------------------------------- latent attention, routed experts
+
+
+def zero_centered_rms_norm(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
+    """x / sqrt(mean(x^2) + eps) * (1 + weight), 32-bit in and out."""
+    x = x.float()
+    return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * (1.0 + weight.float())
+
+
+def clamped_swiglu(gate: torch.Tensor, up: torch.Tensor, limit: float, alpha: float = 1.702) -> torch.Tensor:
+    """g * sigmoid(alpha g) * (u + 1) with g = min(gate, limit), |u| <= limit."""
+    g = gate.float().clamp(max=limit)
+    u = up.float().clamp(min=-limit, max=limit)
+    return g * torch.sigmoid(alpha * g) * (u + 1.0)
+
+
+def softmax_topk(x: torch.Tensor, w_router: torch.Tensor, top: int):
+    """32-bit router: (scores [T, top], experts [T, top]); the scores are the
+    softmax over ALL experts, not renormalized over the chosen ones."""
+    return torch.topk(torch.softmax(x.float() @ w_router.float().T, dim=-1), top, dim=-1)
+
+
+def sliding_window_mask(q_len: int, kv_len: int, kv_offset: int, window: int, device=None) -> torch.Tensor:
+    """[q_len, kv_len] visibility: query i stands at kv_offset + i among the keys
+    and sees itself and the window - 1 keys before it (window 0: all before)."""
+    gap = (torch.arange(q_len, device=device) + kv_offset)[:, None] - torch.arange(kv_len, device=device)[None, :]
+    return (gap >= 0) & (gap < window) if window > 0 else gap >= 0
+
+
+def masked_attention(q, k, v, mask, scale: float) -> torch.Tensor:
+    """q [..., Sq, H, d], k/v [..., Sk, H, d]; 32-bit scores, weights and output."""
+    q, k, v = (t.transpose(-3, -2).float() for t in (q, k, v))
+    scores = (q @ k.transpose(-1, -2)) * scale
+    p = torch.softmax(scores.masked_fill(~mask, float("-inf")), dim=-1)
+    return (p @ v).transpose(-3, -2)
+
+
+def paged_write(cache: torch.Tensor, batch, rows: torch.Tensor) -> None:
+    """Store one row per token of the batch in the paged cache [pages, page, width]."""
+    page = cache.shape[1]
+    for s, (lo, hi) in enumerate(batch.row_ranges()):
+        pos = torch.arange(batch.starts[s], batch.starts[s] + hi - lo)
+        pages = torch.as_tensor(batch.pages[s])[pos // page]
+        cache[pages, pos % page, : rows.shape[1]] = rows[lo:hi]
+
+
+def latent_attention_paged(q, cache, batch, w_uk, w_uv, *, scale: float, window: int) -> torch.Tensor:
+    """q [T, H, dim] of the batch's rows against the latents in the paged cache;
+    returns [T, H, vdim], 32-bit."""
+    t, heads, dim = q.shape
+    rank, page = w_uk.shape[1], cache.shape[1]
+    out = torch.empty(t, heads, w_uv.shape[0] // heads, dtype=torch.float32)
+    for s, (lo, hi) in enumerate(batch.row_ranges()):
+        start, n = batch.starts[s], hi - lo
+        first = max(0, start - window + 1) if window > 0 else 0
+        pos = torch.arange(first, start + n)
+        c = cache[torch.as_tensor(batch.pages[s])[pos // page], pos % page, :rank].to(w_uk.dtype)
+        k = (c @ w_uk.T).view(-1, heads, dim)
+        v = (c @ w_uv.T).view(c.shape[0], heads, -1)
+        mask = sliding_window_mask(n, len(pos), start - first, window)
+        out[lo:hi] = masked_attention(q[lo:hi], k, v, mask, scale)
+    return out

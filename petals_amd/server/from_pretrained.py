@@ -40,7 +40,7 @@ def _find_block_tensors(model_dir: str, prefix: str) -> Dict[str, str]:
 
 
 def load_block_state_dict(model_dir: str, config: ModelConfig, block_index: int) -> Dict[str, torch.Tensor]:
-    prefix = f"{config.block_prefix}.{block_index}."
+    prefix = config.block_tensor_prefix(block_index)
     tensor_map = _find_block_tensors(model_dir, prefix)
     if not tensor_map:
         # fall back to alternate prefixes used by some checkpoints
@@ -111,6 +111,8 @@ def load_pretrained_block(
     block = build_empty_block(config, block_index, device, torch_dtype)
     if os.path.isdir(model_name_or_dir):
         sd = load_block_state_dict(model_name_or_dir, config, block_index)
+        if hasattr(block, "convert_state_dict"):
+            sd = block.convert_state_dict(sd)
         sd = {k: v.to(device=device, dtype=torch_dtype if v.is_floating_point() else None) for k, v in sd.items()}
         report = block.load_state_dict(sd, strict=False, assign=True)
         if report.missing_keys:
@@ -136,7 +138,7 @@ def init_random_block_(block: torch.nn.Module, config: ModelConfig, block_index:
         for name, p in sorted(block.named_parameters()):
             if p.dim() >= 2:
                 p.normal_(0.0, 0.02, generator=gen)
-            elif "bias" in name:
+            elif "bias" in name or name in getattr(block, "neutral_at_zero", ()):
                 p.zero_()
             else:  # norm weights
                 p.fill_(1.0)

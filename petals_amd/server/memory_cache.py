@@ -51,9 +51,16 @@ class TensorDescriptor:
     def nbytes(self) -> int:
         return self.numel * get_size_in_bytes(self.dtype)
 
+    def allocate(self, device: torch.device) -> torch.Tensor:
+        return torch.zeros(self.shape, dtype=self.dtype, device=device)
+
+    def release(self, tensor: torch.Tensor) -> None:
+        """Nothing to give back beyond the bytes."""
+
 
 class MemoryCache:
-    """Byte-budgeted allocator of per-session KV tensors on one device."""
+    """Byte-budgeted allocator of per-session attention state on one device: KV
+    tensors (TensorDescriptor) or page lists (paged_cache.PageDescriptor)."""
 
     def __init__(self, max_size_bytes: Optional[int], device: torch.device, alloc_timeout: float = 600.0):
         self.max_size_bytes = max_size_bytes if max_size_bytes is not None else (1 << 62)
@@ -100,7 +107,7 @@ class MemoryCache:
                         handles = []
                         for d in descriptors:
                             handle = next(self._handle_counter)
-                            self._tensors[handle] = torch.zeros(d.shape, dtype=d.dtype, device=self.device)
+                            self._tensors[handle] = d.allocate(self.device)
                             handles.append(handle)
                         self._current_size += total_bytes
                         self._alloc_queue.remove(ticket)
@@ -122,10 +129,11 @@ class MemoryCache:
                 self._alloc_queue.remove(ticket)
             if handles is not None:
                 with self._lock:
-                    for handle in handles:
+                    for handle, d in zip(handles, descriptors):
                         t = self._tensors.pop(handle, None)
                         if t is not None:
-                            self._current_size -= t.numel() * get_size_in_bytes(t.dtype)
+                            d.release(t)
+                            self._current_size -= d.nbytes
                 self._freed_event.set()
 
     @contextlib.contextmanager

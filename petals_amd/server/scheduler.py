@@ -8,9 +8,12 @@ asyncio handlers and the runtime thread share one process, so a task is just
 a closure and an asyncio future. Priority and task-size accounting semantics
 are preserved (`server/task_pool.py:29-177`).
 
-On GPU, inference tasks run on a dedicated high-priority HIP stream and
-training tasks on a second stream, so a long training forward does not add
-latency to token decoding beyond the kernel in flight.
+On GPU, inference tasks and training tasks run on two HIP streams of the same
+(default) priority; inference is favoured by the queue order.
+
+Steps of different sessions that may run as one ragged batch are submitted with
+`submit_merged`: whatever has queued up under one key when the runtime gets to
+it is executed by a single call.
 """
 
 from __future__ import annotations
@@ -21,7 +24,7 @@ import itertools
 import logging
 import threading
 import time
-from typing import Any, Callable, Optional
+from typing import Any, Callable, Dict, List, Optional, Tuple
 
 import torch
 
@@ -54,6 +57,7 @@ class PriorityRuntime:
         self._shutdown = False
         self._thread: Optional[threading.Thread] = None
         self._streams = {}
+        self._merged: Dict[Any, List[Tuple[Any, Any, Any]]] = {}  # key -> [(item, loop, future)]
         self.stats = {"tasks": 0, "busy_time": 0.0}
         # keep-warm (opt-in, PETALS_AMD_KEEP_WARM=<seconds>): for a short
         # window after each task, keep the device queue non-empty while idle.
@@ -76,9 +80,7 @@ class PriorityRuntime:
             return None
         key = "inference" if priority <= 1.0 else "training"
         if key not in self._streams:
-            self._streams[key] = torch.cuda.Stream(
-                device=self.device, priority=-1 if key == "inference" else 0
-            )
+            self._streams[key] = torch.cuda.Stream(device=self.device)
         return self._streams[key]
 
     def _run(self):
@@ -153,6 +155,38 @@ class PriorityRuntime:
             heapq.heappush(self._queue, (priority, next(self._counter), fn, args, kwargs, loop, future))
             self._cv.notify()
         return await future
+
+    async def submit_merged(self, priority: float, key: Any, fn: Callable[[List[Any]], List[Any]], item: Any) -> Any:
+        """Like submit(priority, fn, item), except that all items waiting under
+        `key` are passed to ONE call of `fn`, which returns a result (or an
+        exception instance) for each. Callers of one key pass the same `fn`."""
+        loop = asyncio.get_event_loop()
+        future: asyncio.Future = loop.create_future()
+        with self._cv:
+            if self._shutdown:
+                raise RuntimeError("runtime is shut down")
+            waiting = self._merged.setdefault(key, [])
+            waiting.append((item, loop, future))
+            if len(waiting) == 1:
+                heapq.heappush(
+                    self._queue,
+                    (priority, next(self._counter), self._run_merged, (key, fn), {}, _DummyLoop(), _DummyFuture()),
+                )
+                self._cv.notify()
+        return await future
+
+    def _run_merged(self, key: Any, fn: Callable) -> None:
+        with self._cv:
+            waiting = self._merged.pop(key, [])
+        try:
+            results = fn([item for item, _, _ in waiting])
+            if self.device is not None and self.device.type == "cuda":
+                torch.cuda.current_stream(self.device).synchronize()
+        except BaseException as e:  # noqa: BLE001
+            results = [e] * len(waiting)
+        for (_, loop, future), result in zip(waiting, results):
+            deliver = _set_exception_safe if isinstance(result, BaseException) else _set_result_safe
+            loop.call_soon_threadsafe(deliver, future, result)
 
     def submit_sync(self, priority: float, fn: Callable, *args, timeout: float = 600.0, **kwargs) -> Any:
         """Blocking submit from a non-asyncio thread."""

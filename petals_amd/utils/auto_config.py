@@ -21,7 +21,7 @@ def _ensure_registered():
     import petals_amd.models as m
 
     m._ensure_families()
-    for family in ("llama", "bloom", "falcon", "mixtral"):
+    for family in ("llama", "bloom", "falcon", "mixtral", "tulezen"):
         if family not in _REGISTRY:
             mod = getattr(__import__(f"petals_amd.models.{family}", fromlist=["_register_models"]), "_register_models")
             mod()
@@ -50,10 +50,9 @@ class _AutoDistributedBase:
     def from_pretrained(cls, model_name_or_path: str, **kwargs):
         _ensure_registered()
         d, name = _resolve_config_dict(model_name_or_path)
-        model_type = d.get("model_type")
-        if model_type not in _REGISTRY:
-            raise ValueError(f"unsupported model_type {model_type!r}; known: {sorted(_REGISTRY)}")
-        classes = _REGISTRY[model_type]
+        from petals_amd.models.config_base import resolve_model_type
+
+        classes = _REGISTRY[resolve_model_type(d)]
         config_cls = classes["config"]
         # build the *distributed* config (family config + client knobs)
         from petals_amd.models.model_base import make_distributed_config
