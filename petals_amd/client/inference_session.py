@@ -189,6 +189,7 @@ class InferenceSession:
             self._manager.config.use_server_to_server
             and len(self._sessions) > 1
             and is_dummy(prompts)
+            and is_dummy(hypo_ids)  # a push carries activations only: every server must reorder
             and all(s.position == self._position and s.stepped for s in self._sessions)
         )
         if use_push:

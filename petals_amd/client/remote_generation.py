@@ -352,5 +352,6 @@ class RemoteGenerationMixin:
                 self._next_hypo_ids = beam_idx.to(torch.int64)
                 if eos_token_id is not None and (token_idx == eos_token_id).all():
                     break
+            self._next_hypo_ids = None  # the last reorder has no step to go with
             best = beam_scores.argmax()
             return sequences[best : best + 1]

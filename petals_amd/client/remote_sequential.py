@@ -38,7 +38,10 @@ class RemoteSequential(nn.Module):
             if end_block is None:
                 end_block = config.num_blocks
             block_uids = tuple(f"{config.dht_prefix}{UID_DELIMITER}{i}" for i in range(start_block, end_block))
-            sequence_manager = RemoteSequenceManager(config.client, block_uids, dht=dht)
+            cuts = config.valid_cuts()
+            if cuts is not None:
+                cuts = frozenset(c - start_block for c in cuts if start_block <= c <= end_block)
+            sequence_manager = RemoteSequenceManager(config.client, block_uids, dht=dht, cuts=cuts)
         self.sequence_manager = sequence_manager
 
     def forward(self, inputs: torch.Tensor, prompts: torch.Tensor = DUMMY, **kwargs) -> torch.Tensor:
@@ -75,7 +78,12 @@ class RemoteSequential(nn.Module):
         assert isinstance(ix, slice) and (ix.step is None or ix.step == 1)
         start, stop = ix.indices(len(self))[:2]
         sub_uids = self.sequence_manager.block_uids[start:stop]
-        sub_manager = RemoteSequenceManager(self.sequence_manager.config, sub_uids, dht=self.sequence_manager.dht)
+        cuts = self.sequence_manager.state.cuts
+        if cuts is not None:
+            cuts = frozenset(c - start for c in cuts if start <= c <= stop)
+        sub_manager = RemoteSequenceManager(
+            self.sequence_manager.config, sub_uids, dht=self.sequence_manager.dht, cuts=cuts
+        )
         return RemoteSequential(self.config, sequence_manager=sub_manager)
 
     def __len__(self):

@@ -4,7 +4,7 @@ from __future__ import annotations
 
 import dataclasses
 import time
-from typing import Dict, List, Optional, Sequence, Tuple
+from typing import Dict, FrozenSet, List, Optional, Sequence, Tuple
 
 from petals_amd.data_structures import ModuleUID, RemoteModuleInfo, RemoteSpanInfo, ServerState
 
@@ -16,12 +16,16 @@ class RemoteSequenceInfo:
     spans_by_priority: List[RemoteSpanInfo]  # sorted by length, longest first
     spans_containing_block: Tuple[List[RemoteSpanInfo], ...]
     last_updated_time: float
+    # block indices at which the chain may change servers (None: anywhere)
+    cuts: Optional[FrozenSet[int]] = None
 
     @classmethod
-    def make_empty(cls, block_uids: Sequence[ModuleUID]) -> "RemoteSequenceInfo":
+    def make_empty(
+        cls, block_uids: Sequence[ModuleUID], cuts: Optional[FrozenSet[int]] = None
+    ) -> "RemoteSequenceInfo":
         block_uids = tuple(block_uids)
         empty = tuple([] for _ in block_uids)
-        return cls(block_uids, [None] * len(block_uids), [], empty, last_updated_time=-float("inf"))
+        return cls(block_uids, [None] * len(block_uids), [], empty, last_updated_time=-float("inf"), cuts=cuts)
 
     def __len__(self):
         return len(self.block_uids)
@@ -29,11 +33,11 @@ class RemoteSequenceInfo:
     def update_(self, new_block_infos: List[Optional[RemoteModuleInfo]]):
         assert len(new_block_infos) == len(self.block_uids)
         self.block_infos = list(new_block_infos)
-        self.spans_by_priority, self.spans_containing_block = self.compute_spans(self.block_infos)
+        self.spans_by_priority, self.spans_containing_block = self.compute_spans(self.block_infos, self.cuts)
         self.last_updated_time = time.monotonic()
 
     @staticmethod
-    def compute_spans(block_infos: List[Optional[RemoteModuleInfo]]):
+    def compute_spans(block_infos: List[Optional[RemoteModuleInfo]], cuts: Optional[FrozenSet[int]] = None):
         num_blocks = len(block_infos)
         spans: Dict[str, RemoteSpanInfo] = {}
         active: Dict[str, RemoteSpanInfo] = {}
@@ -55,6 +59,13 @@ class RemoteSequenceInfo:
                 if active[peer_id].end <= block_idx:
                     del active[peer_id]
 
+        if cuts is not None:
+            # a server's blocks are usable from the first to the last place
+            # where the chain may be cut
+            for span in all_spans:
+                inside = [c for c in cuts if span.start <= c <= span.end]
+                span.start, span.end = (min(inside), max(inside)) if inside else (span.start, span.start)
+            all_spans = [s for s in all_spans if s.length > 0]
         spans_by_priority = sorted(all_spans, key=lambda s: s.length, reverse=True)
         spans_containing_block = tuple([] for _ in range(num_blocks))
         for span in all_spans:

@@ -15,7 +15,7 @@ import math
 import random
 import threading
 import time
-from typing import Any, Dict, List, Optional, Sequence, Tuple
+from typing import Any, Dict, FrozenSet, List, Optional, Sequence, Tuple
 
 from petals_amd.client.config import ClientConfig
 from petals_amd.client.routing.sequence_info import RemoteSequenceInfo
@@ -47,6 +47,7 @@ class RemoteSequenceManager:
         block_uids: Sequence[ModuleUID],
         *,
         dht: Optional[DHT] = None,
+        cuts: Optional[FrozenSet[int]] = None,  # see ModelConfig.valid_cuts
     ):
         self.config = config
         if config.secure is not None:
@@ -56,7 +57,7 @@ class RemoteSequenceManager:
         self.block_uids = tuple(block_uids)
         self.dht = dht or DHT(initial_peers=config.initial_peers, client_mode=True)
         self._owns_dht = dht is None
-        self.state = RemoteSequenceInfo.make_empty(self.block_uids)
+        self.state = RemoteSequenceInfo.make_empty(self.block_uids, cuts)
         self.addrs: Dict[str, Tuple[str, int]] = {}
         self._lock = threading.Lock()
         self._bans: Dict[str, _Ban] = {}

@@ -61,6 +61,8 @@ class ModelConfig:
     name_or_path: str = ""
 
     model_type: ClassVar[str] = ""  # set by @register_config
+    # server options that the family's blocks do not have
+    unsupported: ClassVar[FrozenSet[str]] = frozenset()
     # dht_prefix identifies the block namespace in the swarm: "{prefix}.{i}"
     dht_prefix: str = ""
     # block_prefix is the state-dict path of the block list, e.g. "model.layers"

@@ -10,7 +10,7 @@ rank, window and experts.
 from __future__ import annotations
 
 import dataclasses
-from typing import Any, Dict, FrozenSet, List, Optional, Tuple
+from typing import Any, ClassVar, Dict, FrozenSet, List, Optional, Tuple
 
 import torch
 
@@ -77,6 +77,8 @@ def _parse_layer(index: int, entry: Dict[str, Any]) -> LayerSpec:
 class TulezenConfig(ModelConfig):
     layers: List[Dict[str, Any]] = dataclasses.field(default_factory=list)
     block_prefix: str = "l"
+
+    unsupported: ClassVar[FrozenSet[str]] = frozenset({"adapters", "quantization", "tensor parallelism"})
 
     def __post_init__(self):
         super().__post_init__()

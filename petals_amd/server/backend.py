@@ -45,11 +45,18 @@ class TransformerBackend:
     def device(self) -> torch.device:
         return next(self.block.parameters()).device
 
+    @property
+    def stream_dtype(self) -> torch.dtype:
+        """dtype of the hidden states this block takes and returns."""
+        return self.config.stream_dtype(self.dtype)
+
     def get_inference_cache_descriptors(self, batch_size: int, max_length: int) -> Sequence[TensorDescriptor]:
         k_shape, v_shape = self.block.kv_cache_shape(batch_size, max_length)
         return [TensorDescriptor(k_shape, self.dtype), TensorDescriptor(v_shape, self.dtype)]
 
     def cache_bytes_per_token(self, batch_size: int = 1) -> int:
+        if getattr(self.block, "paged", False):
+            return batch_size * self.config.cache_values_per_token(self.block.layer_idx) * self.dtype_bytes
         descs = self.get_inference_cache_descriptors(batch_size, 1)
         return sum(d.nbytes for d in descs)
 

@@ -9,7 +9,7 @@ re-placement of every server (eps guards against oscillation).
 
 from __future__ import annotations
 
-from typing import Dict, List, Optional
+from typing import Dict, FrozenSet, List, Optional
 
 import numpy as np
 
@@ -28,20 +28,44 @@ def compute_throughputs(spans: Dict[str, RemoteSpanInfo], *, total_blocks: int) 
     return throughputs
 
 
-def _choose_best_start(throughputs: np.ndarray, num_blocks: int) -> int:
+def _starts(total: int, num_blocks: int, cuts: Optional[FrozenSet[int]]) -> List[int]:
+    """Starts of windows of `num_blocks` whose both ends are valid cuts (all
+    windows if the cuts admit none: the caller's span is what it is)."""
+    starts = list(range(0, total - num_blocks + 1))
+    if cuts is None:
+        return starts
+    return [i for i in starts if i in cuts and i + num_blocks in cuts] or starts
+
+
+def _choose_best_start(throughputs: np.ndarray, num_blocks: int, cuts: Optional[FrozenSet[int]] = None) -> int:
     options = (
         (sorted(throughputs[i : i + num_blocks]), i)
-        for i in range(0, len(throughputs) - num_blocks + 1)
+        for i in _starts(len(throughputs), num_blocks, cuts)
     )
     return min(options)[-1]
 
 
-def choose_best_blocks(num_blocks: int, module_infos: List[Optional[RemoteModuleInfo]]) -> List[int]:
+def servable_length(num_blocks: int, total: int, cuts: Optional[FrozenSet[int]]) -> int:
+    """Length of the longest span of at most `num_blocks` blocks between valid
+    cuts; the shortest one if even that needs more."""
+    if cuts is None:
+        return num_blocks
+    lengths = {b - a for a in cuts for b in cuts if 0 <= a < b <= total}
+    fitting = [n for n in lengths if n <= num_blocks]
+    return max(fitting) if fitting else min(lengths)
+
+
+def choose_best_blocks(
+    num_blocks: int,
+    module_infos: List[Optional[RemoteModuleInfo]],
+    cuts: Optional[FrozenSet[int]] = None,
+) -> List[int]:
     from petals_amd.data_structures import compute_spans
 
     spans = compute_spans(module_infos)
     throughputs = compute_throughputs(spans, total_blocks=len(module_infos))
-    start = _choose_best_start(throughputs, num_blocks)
+    num_blocks = servable_length(num_blocks, len(module_infos), cuts)
+    start = _choose_best_start(throughputs, num_blocks, cuts)
     return list(range(start, start + num_blocks))
 
 
@@ -49,6 +73,7 @@ def should_choose_other_blocks(
     local_peer_id: str,
     module_infos: List[Optional[RemoteModuleInfo]],
     balance_quality: float,
+    cuts: Optional[FrozenSet[int]] = None,
 ) -> bool:
     if balance_quality > 1.0:
         return True  # forces rebalancing on each check (for tests)
@@ -65,7 +90,7 @@ def should_choose_other_blocks(
     throughputs = compute_throughputs(spans, total_blocks=len(module_infos))
     throughputs[local_span.start : local_span.end] -= local_span.throughput * (1 + eps)
 
-    new_start = _choose_best_start(throughputs, local_span.length)
+    new_start = _choose_best_start(throughputs, local_span.length, cuts)
     if local_span.start == new_start:
         return False  # already in the best place
 
@@ -80,7 +105,7 @@ def should_choose_other_blocks(
         for peer_id in servers:
             span = spans[peer_id]
             throughputs[span.start : span.end] -= span.throughput * (1 + eps)
-            new_start = _choose_best_start(throughputs, span.length)
+            new_start = _choose_best_start(throughputs, span.length, cuts)
             if span.start != new_start:
                 span.start, span.end = new_start, new_start + span.length
                 moved = True

@@ -13,6 +13,8 @@ from __future__ import annotations
 
 import asyncio
 import contextlib
+import dataclasses
+import functools
 import logging
 import os
 import time
@@ -25,7 +27,9 @@ from petals_amd.p2p.streaming import receive_tensors_streamed, send_tensors_stre
 from petals_amd.p2p.transport import P2PNode, RpcError, RpcMessage, RpcStream
 from petals_amd.server.backend import TransformerBackend
 from petals_amd.server.memory_cache import MemoryCache, TensorDescriptor
+from petals_amd.server.paged_cache import PageDescriptor
 from petals_amd.server.scheduler import PriorityRuntime, TaskPrioritizer
+from petals_amd.server.span_engine import SpanEngine, StepEntry
 from petals_amd.utils.misc import DUMMY, is_dummy
 
 logger = logging.getLogger(__name__)
@@ -80,6 +84,20 @@ class _SpanDecodeGraph:
         return self.graph.replay()
 
 
+@dataclasses.dataclass
+class _PagedStep:
+    """One session's step while it waits to be merged into a batch."""
+
+    hidden_states: Any  # [B, S, width] or a mesh receive handle
+    hypo_ids: Optional[torch.Tensor]
+    prompts: Optional[torch.Tensor]
+    sequences: List[Any]  # one PagedSequence per batch row
+    prefix_length: int
+    keep_on_device: bool
+    commit_cb: Any
+    reply_cb: Any
+
+
 def _dtype_str(dtype) -> str:
     from petals_amd.utils.serialization import _DTYPE_TO_STR
 
@@ -118,8 +136,10 @@ class TransformerConnectionHandler:
         mesh=None,
         default_compression: str = "none",
         tp_coord=None,
+        engine: Optional[SpanEngine] = None,
     ):
         self.backends = backends
+        self.engine = engine  # step function of paged blocks (None: per-session tensors)
         self.memory_cache = memory_cache
         self.runtime = runtime
         self.prioritizer = prioritizer or TaskPrioritizer()
@@ -162,6 +182,13 @@ class TransformerConnectionHandler:
         for uid in uids:
             if uid not in self.backends:
                 raise RpcError(f"uid {uid!r} is not served here")
+        if self.engine is not None:
+            try:
+                self.engine.check_chain(uids)
+            except ValueError as e:
+                raise RpcError(str(e)) from None
+            if meta.get("active_adapter"):
+                raise RpcError("these blocks have no adapters")
         return uids
 
     def _split_prompts(self, prompts: Optional[torch.Tensor], n: int, dtype, device) -> List[Optional[torch.Tensor]]:
@@ -198,12 +225,14 @@ class TransformerConnectionHandler:
         from petals_amd.utils.peft import using_adapter
 
         backend0 = self.backends[uids[0]]
-        device, dtype = backend0.device, backend0.dtype
+        device, dtype = backend0.device, backend0.stream_dtype
         hidden_states = hidden_states.to(device=device, dtype=dtype)
         if self.tp_coord is not None:
             p = prompts if (prompts is not None and not is_dummy(prompts)) else None
             self.tp_coord.forward(hidden_states, p)
         prompt_list = self._split_prompts(prompts, len(uids), dtype, device)
+        if self.engine is not None:
+            return self.engine.forward(uids, hidden_states, prompt_list).cpu()
         with using_adapter(active_adapter):
             for uid, prompt in zip(uids, prompt_list):
                 if prompt is not None:
@@ -252,13 +281,15 @@ class TransformerConnectionHandler:
         from petals_amd.utils.peft import using_adapter
 
         backend0 = self.backends[uids[0]]
-        device, dtype = backend0.device, backend0.dtype
+        device, dtype = backend0.device, backend0.stream_dtype
         inputs = inputs.to(device=device, dtype=dtype)
         grad_outputs = grad_outputs.to(device=device, dtype=dtype)
         if self.tp_coord is not None:
             p = prompts if (prompts is not None and not is_dummy(prompts)) else None
             self.tp_coord.backward(inputs, grad_outputs, p)
         prompt_list = self._split_prompts(prompts, len(uids), dtype, device)
+        if self.engine is not None:
+            return self._backward_paged(uids, inputs, grad_outputs, prompt_list)
         # re-run forward (plain no_grad, NOT inference_mode: these activations
         # feed autograd below) to recover intermediate inputs
         inter_inputs: List[torch.Tensor] = []
@@ -301,6 +332,41 @@ class TransformerConnectionHandler:
             grad_prompts_t = DUMMY
         return grad.cpu(), grad_prompts_t.cpu() if not is_dummy(grad_prompts_t) else DUMMY
 
+    def _backward_paged(self, uids, inputs, grad_outputs, prompt_list):
+        """Backward of paged blocks, in units of blocks that share a latent: a
+        unit is re-run with gradients as a whole, its prompts as leaves."""
+
+        def run(unit, hidden, prompts):
+            shared: Dict[int, torch.Tensor] = {}
+            for uid, prompt in zip(unit, prompts):
+                if prompt is not None:
+                    pre = prompt.shape[1]
+                    hidden = torch.cat([hidden[:, :pre] + prompt, hidden[:, pre:]], dim=1)
+                hidden = self.backends[uid].block(hidden, shared=shared)
+            return hidden
+
+        units, at = [], 0
+        for unit in self.engine.units(uids):
+            units.append((unit, prompt_list[at : at + len(unit)]))
+            at += len(unit)
+        unit_inputs = [inputs]
+        with torch.no_grad():
+            for unit, prompts in units[:-1]:
+                unit_inputs.append(run(unit, unit_inputs[-1], prompts))
+        grad, grad_prompts = grad_outputs, []
+        for (unit, prompts), hidden in zip(reversed(units), reversed(unit_inputs)):
+            with torch.enable_grad():
+                hidden = hidden.detach().clone().requires_grad_(True)
+                leaves = [None if p is None else p.detach().clone().requires_grad_(True) for p in prompts]
+                torch.autograd.backward([run(unit, hidden, leaves)], [grad])
+            grad = hidden.grad
+            grad_prompts.extend(None if p is None else p.grad for p in reversed(leaves))
+        grad_prompts.reverse()
+        ref = next((g for g in grad_prompts if g is not None), None)
+        if ref is None:
+            return grad.cpu(), DUMMY
+        return grad.cpu(), torch.stack([torch.zeros_like(ref) if g is None else g for g in grad_prompts]).cpu()
+
     async def _handle_backward(self, meta: Dict[str, Any], tensors: List[torch.Tensor]) -> List[torch.Tensor]:
         uids = self._parse_uids(meta)
         inputs, grad_outputs = tensors[0], tensors[1]
@@ -340,7 +406,7 @@ class TransformerConnectionHandler:
         """Runs IN the runtime thread: one inference step through the whole span
         (the single-process analog of reference _MergedInferenceStep)."""
         backend0 = self.backends[uids[0]]
-        device, dtype = backend0.device, backend0.dtype
+        device, dtype = backend0.device, backend0.stream_dtype
         if not torch.is_tensor(hidden_states):
             # MeshRecvHandle: the step was submitted BEFORE its input landed;
             # block here (the actual data dependency) instead of in the
@@ -442,6 +508,51 @@ class TransformerConnectionHandler:
             reply_cb(hidden_states)
         return hidden_states
 
+    def _merged_paged_step(self, uids: Tuple[ModuleUID, ...], items: List[_PagedStep]) -> List[Any]:
+        """Runs IN the runtime thread: the waiting steps of any number of
+        sessions as one ragged batch through the span engine. Returns each
+        session's output or the exception that kept it out."""
+        device, dtype = self.engine.device, self.backends[uids[0]].stream_dtype
+        results: List[Any] = [None] * len(items)
+        entries: List[StepEntry] = []
+        owners: List[int] = []
+        for i, item in enumerate(items):
+            try:
+                hidden = item.hidden_states
+                if not torch.is_tensor(hidden):  # mesh receive: wait for the data itself
+                    hidden = hidden.result(self.step_timeout)
+                hidden = hidden.to(device=device, dtype=dtype)
+                if hidden.shape[0] != len(item.sequences):
+                    raise RpcError(f"{hidden.shape[0]} rows for a session of batch size {len(item.sequences)}")
+                if item.hypo_ids is not None and not is_dummy(item.hypo_ids):
+                    self.engine.pool.reorder(item.sequences, item.hypo_ids.tolist())
+                prompts = self._split_prompts(item.prompts, len(uids), dtype, device)
+                has_prompts = any(p is not None for p in prompts)
+                for b, sequence in enumerate(item.sequences):
+                    own = [None if p is None else p[b] for p in prompts] if has_prompts else None
+                    entries.append(StepEntry(sequence, hidden[b], item.prefix_length, own))
+                    owners.append(i)
+            except Exception as e:  # noqa: BLE001 - this session's own failure
+                entries = [x for x, o in zip(entries, owners) if o != i]
+                owners = [o for o in owners if o != i]
+                results[i] = e
+        rows: List[List[torch.Tensor]] = [[] for _ in items]
+        for i, out in zip(owners, self.engine.step(uids, entries) if entries else []):
+            if isinstance(out, BaseException):
+                results[i] = out
+            rows[i].append(out)
+        for i, item in enumerate(items):
+            if results[i] is None:
+                out = torch.stack(rows[i])
+                results[i] = out if item.keep_on_device else out.cpu()
+                _commit_if_needed(item.commit_cb, results[i])
+        if device.type == "cuda" and any(item.reply_cb is not None for item in items):
+            torch.cuda.current_stream(device).synchronize()  # clients read on their own streams
+        for item, out in zip(items, results):
+            if item.reply_cb is not None and not isinstance(out, BaseException):
+                item.reply_cb(out)
+        return results
+
     async def rpc_inference(self, request: RpcMessage, stream: RpcStream) -> None:
         meta = request.meta
         uids = self._parse_uids(meta)
@@ -453,8 +564,10 @@ class TransformerConnectionHandler:
         session_id = meta.get("session_id") or f"anon-{id(stream)}"
         alloc_timeout = float(meta.get("alloc_timeout", self.memory_cache.alloc_timeout))
 
-        descriptors: List[TensorDescriptor] = []
-        for uid in uids:
+        descriptors: List[Any] = []
+        if self.engine is not None:
+            descriptors.append(PageDescriptor(self.engine.pool, batch_size, max_length))
+        for uid in uids if self.engine is None else ():
             descriptors.extend(self.backends[uid].get_inference_cache_descriptors(batch_size, max_length))
 
         session = _Session(session_id, uids, max_length)
@@ -463,6 +576,10 @@ class TransformerConnectionHandler:
         try:
             async with self.memory_cache.allocate_cache(*descriptors, timeout=alloc_timeout) as flat_handles:
                 handles = [tuple(flat_handles[2 * i : 2 * i + 2]) for i in range(len(uids))]
+                sequences = None
+                if self.engine is not None:
+                    with self.memory_cache.use_cache(flat_handles[0]) as (sequences,):
+                        pass
                 if self.tp_coord is not None:
                     session.tp_slot = next(self._tp_slots)
                     self.tp_coord.open_session(session.tp_slot, batch_size, max_length)
@@ -517,7 +634,7 @@ class TransformerConnectionHandler:
                     ack_task = None
                     if length_increment > 0:
                         out_shape = list(hidden_states.shape)  # blocks preserve shape
-                        out_dtype = self.backends[uids[0]].dtype
+                        out_dtype = self.backends[uids[0]].stream_dtype
                         if will_push:
                             mdst = self._mesh_dst(next_servers[0])
                             if mdst is not None:
@@ -585,7 +702,13 @@ class TransformerConnectionHandler:
                     if length_increment > 0:
                         priority = self.prioritizer.prioritize(hidden_states, type="inference")
                         try:
-                            output = await self.runtime.submit(
+                            output = await self.runtime.submit_merged(
+                                priority, ("step", tuple(uids)), functools.partial(self._merged_paged_step, tuple(uids)),
+                                _PagedStep(
+                                    hidden_states, hypo_ids, prompts, sequences, session.prefix_length,
+                                    keep_on_device, commit_cb, reply_cb,
+                                ),
+                            ) if self.engine is not None else await self.runtime.submit(
                                 priority,
                                 self._inference_step_chain,
                                 uids,

@@ -32,6 +32,7 @@ from petals_amd.server.from_pretrained import load_pretrained_block
 from petals_amd.server.handler import TransformerConnectionHandler
 from petals_amd.server.memory_cache import MemoryCache
 from petals_amd.server.scheduler import PriorityRuntime
+from petals_amd.server.span_engine import SpanEngine
 from petals_amd.server.throughput import get_server_throughput
 from petals_amd.utils.misc import get_size_in_bytes
 
@@ -109,6 +110,13 @@ class Server:
             self.block_indices = list(range(int(start), int(end)))
             num_blocks = len(self.block_indices)
         self.num_blocks = num_blocks or self._choose_num_blocks(attn_cache_tokens)
+        cuts = self.config.valid_cuts()
+        if self.block_indices and cuts is not None:
+            if not {self.block_indices[0], self.block_indices[-1] + 1} <= cuts:
+                raise ValueError(
+                    f"blocks {block_indices} cannot be served on their own: some block shares its cache across the "
+                    f"border; spans may start and end at {sorted(cuts)}"
+                )
 
         self.attn_cache_tokens = attn_cache_tokens
         self.max_batch_size = max_batch_size
@@ -119,6 +127,13 @@ class Server:
         self.mean_balance_check_period = mean_balance_check_period
         self.public_name = public_name
         self.adapters = tuple(adapters)
+        wanted = {
+            "adapters": bool(self.adapters), "quantization": quant_type != "none",
+            "tensor parallelism": tensor_parallel_ranks > 1,
+        }
+        refused = sorted(option for option in self.config.unsupported if wanted[option])
+        if refused:
+            raise ValueError(f"model_type {self.config.model_type!r} is served without {', '.join(refused)}")
         self._throughput_setting = throughput
         # LocalMesh for the co-located RCCL/xGMI activation hand-off tier
         self.mesh = mesh
@@ -173,12 +188,7 @@ class Server:
             dtype_bytes = 0.53125  # 4.25 bits/param (parity: block_utils.py:46)
         elif self.quant_type == "int8":
             dtype_bytes = 1.002  # 8 bits/param + per-column bf16 scales
-        h, inter = cfg.hidden_size, cfg.intermediate_size
-        kv = cfg.n_kv_heads * cfg.head_dim
-        attn = h * h + 2 * h * kv + h * h
-        n_experts = getattr(cfg, "num_local_experts", 1)
-        mlp = 3 * h * inter * n_experts
-        return int((attn + mlp) * dtype_bytes)
+        return int(cfg.block_param_count() * dtype_bytes)
 
     def _choose_num_blocks(self, attn_cache_tokens: int = 16384) -> int:
         """Fit blocks to device memory: block bytes + attn-cache + autograd
@@ -189,7 +199,8 @@ class Server:
             total = 16 << 30
         block_bytes = self._block_param_bytes()
         cache_bytes_per_block = (
-            2 * self.config.n_kv_heads * self.config.head_dim * attn_cache_tokens * get_size_in_bytes(self.torch_dtype)
+            max(self.config.cache_values_per_token(i) for i in range(self.config.num_blocks))
+            * attn_cache_tokens * get_size_in_bytes(self.torch_dtype)
         )
         autograd_reserve = 2 << 30
         usable = total * 0.92 - autograd_reserve
@@ -302,7 +313,9 @@ class Server:
             block_indices = self.block_indices
         else:
             infos, _ = await self._get_infos()
-            block_indices = block_selection.choose_best_blocks(self.num_blocks, infos)
+            block_indices = block_selection.choose_best_blocks(
+                self.num_blocks, infos, self.config.valid_cuts()
+            )
         logger.info("serving blocks %s..%s", block_indices[0], block_indices[-1])
 
         # --- throughput estimate (cheap on CPU; measured once per device/model)
@@ -324,13 +337,10 @@ class Server:
             # reference server/throughput.py:96-107)
             throughput *= 0.2
 
-        cache_bytes = int(
-            2
-            * self.config.n_kv_heads
-            * self.config.head_dim
+        cache_bytes = (
+            sum(self.config.cache_values_per_token(i) for i in block_indices)
             * self.attn_cache_tokens
             * get_size_in_bytes(self.torch_dtype)
-            * len(block_indices)
         )
         self.memory_cache = MemoryCache(cache_bytes, self.device, alloc_timeout=self.max_alloc_timeout)
 
@@ -380,7 +390,17 @@ class Server:
                 max_chunk_size_bytes=self.max_chunk_size_bytes,
             )
 
+        engine = None
+        blocks = {uid: b.block for uid, b in self.backends.items()}
+        if any(getattr(b, "paged", False) for b in blocks.values()):
+            pool = SpanEngine.pool_for(
+                list(blocks.values()), self.attn_cache_tokens, dtype=self.torch_dtype, device=self.device
+            )
+            self.memory_cache.max_size_bytes = pool.num_pages * pool.bytes_per_page
+            engine = SpanEngine(blocks, pool, max_length=self.inference_max_length)
+
         self.handler = TransformerConnectionHandler(
+            engine=engine,
             backends=self.backends,
             memory_cache=self.memory_cache,
             runtime=self.runtime,
@@ -440,7 +460,9 @@ class Server:
                 if self.block_indices is None and time.monotonic() > next_balance_check:
                     next_balance_check = time.monotonic() + random.random() * 2 * self.mean_balance_check_period
                     infos, _ = await self._get_infos()
-                    if block_selection.should_choose_other_blocks(self.p2p.peer_id, infos, self.balance_quality):
+                    if block_selection.should_choose_other_blocks(
+                        self.p2p.peer_id, infos, self.balance_quality, self.config.valid_cuts()
+                    ):
                         logger.info("swarm is imbalanced: restarting with a new span")
                         self._restart_requested = True
                         break
@@ -513,7 +535,7 @@ class Server:
             return
         first = next(iter(self.backends.values()), None)
         if first is not None and self.memory_cache is not None:
-            bytes_per_token = first.cache_bytes_per_token() * max(1, len(self.backends))
+            bytes_per_token = sum(b.cache_bytes_per_token() for b in self.backends.values())
             self.server_info.cache_tokens_left = int(self.memory_cache.bytes_left // max(1, bytes_per_token))
         uids = [
             make_uid(self.config.dht_prefix, i)

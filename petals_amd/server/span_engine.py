@@ -18,7 +18,7 @@ from typing import Any, Dict, List, Optional, Sequence, Tuple
 
 import torch
 
-from petals_amd.server.paged_cache import PagedBatch, PagedPool, PagedSequence, StaticDecodeBatch, pages_for
+from petals_amd.server.paged_cache import PAGE_SIZE, PagedBatch, PagedPool, PagedSequence, StaticDecodeBatch, pages_for
 
 MAX_STEP_TOKENS = 8192  # rows per pass; longer steps are cut into several
 
@@ -66,9 +66,10 @@ class SpanEngine:
             seen.add(block.layer_idx)
 
     @torch.inference_mode()
-    def step(self, uids: Sequence[Any], entries: Sequence[StepEntry]) -> List[Any]:
+    def step(self, uids: Sequence[Any], entries: Sequence[StepEntry], pool: Optional[PagedPool] = None) -> List[Any]:
         """Runs the chain `uids` on all entries; returns each entry's output rows
-        (or the exception that kept it out of the batch, e.g. a full cache)."""
+        (or the exception that kept it out of the batch, e.g. a full cache).
+        `pool`: where the entries' sequences live (default: the engine's own)."""
         uids = tuple(uids)
         assert all(e.hidden.shape[0] > 0 for e in entries)
         results: List[Any] = [None] * len(entries)
@@ -88,7 +89,7 @@ class SpanEngine:
                 budget -= n
                 batch.append((i, done, n))
             if batch:
-                x, at = self._run(uids, [(entries[i], done, n) for i, done, n in batch]), 0
+                x, at = self._run(uids, [(entries[i], done, n) for i, done, n in batch], pool or self.pool), 0
                 for i, done, n in batch:
                     entries[i].sequence.advance(n)
                     rows = x[at : at + n]
@@ -99,14 +100,14 @@ class SpanEngine:
             todo = later
         return results
 
-    def _run(self, uids, parts) -> torch.Tensor:
+    def _run(self, uids, parts, pool: PagedPool) -> torch.Tensor:
         hidden = [e.hidden[done : done + n].to(self.device, torch.float32) for e, done, n in parts]
         x = hidden[0] if len(hidden) == 1 else torch.cat(hidden)
         pages = [e.sequence.pages for e, _, _ in parts]
         starts = [e.start + done for e, done, _ in parts]
         lens = [n for _, _, n in parts]
         has_prompts = any(e.prompts is not None for e, _, _ in parts)
-        if not has_prompts and self._graphable(uids, lens):
+        if not has_prompts and pool is self.pool and self._graphable(uids, lens):
             key = (uids, len(lens))
             if key not in self._graphs:
                 self._graphs[key] = _DecodeGraph(self, uids, len(lens), x, pages, starts)
@@ -115,8 +116,45 @@ class SpanEngine:
         for b, uid in enumerate(uids):
             if has_prompts:
                 x = self._add_prompts(x, parts, b)
-            x = self.blocks[uid].forward_paged(x, batch, self.pool)
+            x = self.blocks[uid].forward_paged(x, batch, pool)
         return x
+
+    @torch.inference_mode()
+    def forward(
+        self, uids: Sequence[Any], hidden: torch.Tensor, prompts: Optional[Sequence[Optional[torch.Tensor]]] = None
+    ) -> torch.Tensor:
+        """Stateless pass over whole sequences [B, S, width] (a scratch pool holds
+        their state meanwhile). prompts[i]: [B, pre, width] or None for block i."""
+        self.check_chain(uids)
+        b, s, _ = hidden.shape
+        scratch = self.pool_for(
+            [self.blocks[u] for u in uids], b * pages_for(s) * PAGE_SIZE, dtype=self.pool.dtype, device=self.device
+        )
+        entries = [
+            StepEntry(
+                scratch.open(), hidden[i], 0,
+                None if prompts is None else [None if p is None else p[i] for p in prompts],
+            )
+            for i in range(b)
+        ]
+        out = self.step(uids, entries, scratch)
+        for r in out:
+            if isinstance(r, BaseException):
+                raise r
+        return torch.stack(out)
+
+    def units(self, uids: Sequence[Any]) -> List[List[Any]]:
+        """The chain in the smallest runs that share no state with each other."""
+        runs: List[List[Any]] = []
+        for uid in uids:
+            source = self.blocks[uid].latent_layer
+            keep = len(runs)
+            for i, run in enumerate(runs):
+                if any(self.blocks[u].layer_idx == source for u in run):
+                    keep = i
+                    break
+            runs[keep:] = [[u for run in runs[keep:] for u in run] + [uid]]
+        return runs
 
     @staticmethod
     def _add_prompts(x, parts, block: int) -> torch.Tensor:

@@ -103,6 +103,11 @@ def measure_compute_rps(
     block = build_empty_block(config, 0, device, dtype)
     init_random_block_(block, config, 0)
     block = block.eval()
+    if getattr(block, "paged", False):
+        return _measure_paged_rps(
+            config, block, device, dtype, n_infer_steps=n_infer_steps, n_forward_steps=n_forward_steps,
+            forward_tokens=forward_tokens,
+        )
 
     k_shape, v_shape = block.kv_cache_shape(1, 1024)
     k = torch.zeros(k_shape, device=device, dtype=dtype)
@@ -134,3 +139,30 @@ def measure_compute_rps(
     if device.type == "cuda":
         torch.cuda.empty_cache()
     return {"inference_rps": inference_rps, "forward_rps": forward_rps}
+
+
+def _measure_paged_rps(config, block, device, dtype, *, n_infer_steps, n_forward_steps, forward_tokens):
+    """The same two numbers for a paged block, through the step function that serves it."""
+    from petals_amd.server.span_engine import SpanEngine, StepEntry
+
+    if device.type == "cuda":
+        block.optimize_for_inference()
+    pool = SpanEngine.pool_for([block], 2048, dtype=dtype, device=device)
+    engine = SpanEngine({0: block}, pool, max_length=1024)
+    x = torch.randn(forward_tokens, config.hidden_size, device=device)
+
+    def timed(n_rows: int, steps: int) -> float:
+        sequence = pool.open()
+        engine.step([0], [StepEntry(sequence, x[:n_rows], 0)])  # warmup
+        if device.type == "cuda":
+            torch.cuda.synchronize(device)
+        t0 = time.perf_counter()
+        for i in range(steps):
+            start = i + 1 if n_rows == 1 else 0
+            engine.step([0], [StepEntry(sequence, x[:n_rows], start)])
+        if device.type == "cuda":
+            torch.cuda.synchronize(device)
+        sequence.close()
+        return steps * n_rows / (time.perf_counter() - t0)
+
+    return {"inference_rps": timed(1, n_infer_steps), "forward_rps": timed(forward_tokens, n_forward_steps)}

@@ -1,0 +1,348 @@
+"""Tulezen through the framework's entry points: servers, scheduler, client,
+generation, training, routing, and the trace command."""
+
+import asyncio
+import json
+import os
+import subprocess
+import sys
+import threading
+
+import pytest
+import torch
+
+import tulezen_oracle as oracle
+
+L = oracle.layer_dict
+LAYERS = [
+    L(window=12), L(heads=2, dim=8, vdim=16, kv_rank=48, window=40), L(kv_rank=48, window=7, kv_from=1, mlp=False),
+    L(heads=4, window=25, top=1), L(window=90, kv_from=3),
+]
+VOCAB, WIDTH = 101, 48
+
+
+@pytest.fixture(scope="module")
+def checkpoint(tmp_path_factory):
+    raw = oracle.config_dict(vocab=VOCAB, width=WIDTH, layers=LAYERS)
+    weights = oracle.random_model(raw, seed=11)
+    path = str(tmp_path_factory.mktemp("tulezen") / "model")
+    oracle.save_model(path, raw, weights)
+    return path, raw, weights
+
+
+def greedy(raw, weights, ids, n):
+    ids = list(ids)
+    for _ in range(n):
+        ids.append(int(oracle.run(raw, weights, ids)[-1].argmax()))
+    return ids
+
+
+def start_server(path, peers, blocks, device="cpu", dtype="float32", **kwargs):
+    from petals_amd.server.server import Server
+
+    return Server(
+        path, initial_peers=peers, host="127.0.0.1", device=device, torch_dtype=dtype, block_indices=blocks,
+        dht_prefix="test-tulezen", throughput=1.0, update_period=2.0, attn_cache_tokens=2048, **kwargs,
+    ).start()
+
+
+def make_client(path, peers, **kwargs):
+    from petals_amd.utils.auto_config import AutoDistributedModelForCausalLM
+
+    return AutoDistributedModelForCausalLM.from_pretrained(
+        path, initial_peers=peers, dht_prefix="test-tulezen", show_route=False, max_retries=2, min_backoff=0.2,
+        request_timeout=30.0, **kwargs,
+    )
+
+
+@pytest.fixture(scope="module")
+def swarm(checkpoint):
+    from petals_amd.dht.node import DHT
+
+    path, _, _ = checkpoint
+    boot = DHT(host="127.0.0.1")
+    servers = [start_server(path, [boot.listen_addr], b) for b in ("0:3", "3:5")]
+    yield boot, servers
+    for s in servers:
+        s.shutdown()
+    boot.shutdown()
+
+
+@pytest.fixture(scope="module")
+def client(swarm, checkpoint):
+    model = make_client(checkpoint[0], [swarm[0].listen_addr])
+    yield model
+    model.transformer.h.sequence_manager.shutdown()
+
+
+def test_forward_matches_oracle(client, checkpoint):
+    _, raw, weights = checkpoint
+    ids = torch.randint(0, VOCAB, (2, 50), generator=torch.Generator().manual_seed(0))
+    with torch.no_grad():
+        out = client(input_ids=ids).logits
+    for i in range(2):
+        want = oracle.run(raw, weights, ids[i].tolist())
+        assert (out[i].double() - want).abs().max() < 2e-3 * want.abs().max()
+
+
+def test_greedy_generation(client, checkpoint):
+    _, raw, weights = checkpoint
+    ids = torch.randint(0, VOCAB, (1, 30), generator=torch.Generator().manual_seed(1))
+    out = client.generate(ids, max_new_tokens=12, do_sample=False)
+    assert out[0].tolist() == greedy(raw, weights, ids[0].tolist(), 12)
+
+
+def test_batched_and_resumed_generation(client, checkpoint):
+    _, raw, weights = checkpoint
+    ids = torch.randint(0, VOCAB, (3, 9), generator=torch.Generator().manual_seed(2))
+    out = client.generate(ids, max_new_tokens=5, do_sample=False)
+    for i in range(3):
+        assert out[i].tolist() == greedy(raw, weights, ids[i].tolist(), 5)
+    with client.transformer.h.inference_session(max_length=40):
+        first = client.generate(ids[:1], max_new_tokens=4, do_sample=False)
+        again = client.generate(first, max_new_tokens=4, do_sample=False)
+    assert again[0].tolist() == greedy(raw, weights, ids[0].tolist(), 8)
+
+
+def test_beam_search_reorders_pages(client, checkpoint):
+    """A beam's reported tokens are the best-scoring path of a plain beam search."""
+    _, raw, weights = checkpoint
+    ids = [5, 17, 40, 3]
+    beams, n, k = [(0.0, ids)], 5, 3
+    for _ in range(n):
+        options = []
+        for score, seq in beams:
+            lp = torch.log_softmax(oracle.run(raw, weights, seq)[-1], -1)
+            options += [(score + float(lp[t]), seq + [t]) for t in lp.topk(k).indices.tolist()]
+        beams = sorted(options, reverse=True)[:k]
+    out = client.generate(torch.tensor([ids]), max_new_tokens=n, num_beams=k, do_sample=False)
+    assert out[0].tolist() == beams[0][1], beams
+
+
+def test_concurrent_sessions_share_steps(client, swarm, checkpoint):
+    """Sessions stepping at the same time are merged, and none notices."""
+    _, raw, weights = checkpoint
+    engine = swarm[1][0].handler.engine
+    sizes, run = [], engine._run
+
+    def counting(uids, parts, pool):
+        sizes.append(len(parts))
+        return run(uids, parts, pool)
+
+    engine._run = counting
+    results = {}
+
+    def worker(i):
+        ids = torch.randint(0, VOCAB, (1, 3 + 9 * i), generator=torch.Generator().manual_seed(i))
+        results[i] = (ids, client.generate(ids, max_new_tokens=10, do_sample=False))
+
+    try:
+        threads = [threading.Thread(target=worker, args=(i,)) for i in range(5)]
+        [t.start() for t in threads]
+        [t.join() for t in threads]
+    finally:
+        engine._run = run
+    for ids, out in results.values():
+        assert out[0].tolist() == greedy(raw, weights, ids[0].tolist(), 10)
+    assert len(results) == 5 and sum(sizes) >= 50
+    assert engine.pool.free_pages == engine.pool.num_pages
+
+
+def test_gradients_through_shared_latents(client, checkpoint):
+    _, raw, weights = checkpoint
+    x = torch.randn(2, 20, WIDTH, generator=torch.Generator().manual_seed(3))
+    ours = x.clone().requires_grad_(True)
+    (client.transformer.h(ours).pow(2).sum()).backward()
+    for i in range(2):
+        plain = x[i].double().requires_grad_(True)
+        residuals = []
+        oracle.run(raw, weights, [0] * 20, embeds=plain, residuals=residuals)
+        # clone in the oracle keeps the graph
+        residuals[-1].pow(2).sum().backward()
+        assert (ours.grad[i].double() - plain.grad).abs().max() < 2e-3 * plain.grad.abs().max()
+
+
+def test_deep_prompt_tuning_trains(swarm, checkpoint):
+    model = make_client(checkpoint[0], [swarm[0].listen_addr], tuning_mode="deep_ptune", pre_seq_len=3)
+    try:
+        ids = torch.randint(0, VOCAB, (2, 6), generator=torch.Generator().manual_seed(4))
+        model(input_ids=ids).logits.pow(2).mean().backward()
+        grad = model.transformer.intermediate_prompt_embeddings.weight.grad
+        assert grad is not None and torch.isfinite(grad).all() and grad.abs().sum() > 0
+        with torch.no_grad():
+            full = model(input_ids=ids).logits
+            with model.transformer.h.inference_session(max_length=16, batch_size=2):
+                step = model(input_ids=ids).logits
+        assert torch.allclose(full, step, atol=1e-4)
+    finally:
+        model.transformer.h.sequence_manager.shutdown()
+
+
+# ------------------------------------------------------- spans and routing
+
+
+def test_spans_cannot_split_a_shared_latent(checkpoint, swarm, client):
+    from petals_amd.p2p.transport import RpcError
+    from petals_amd.server.server import Server
+
+    path, _, _ = checkpoint
+    for blocks in ("0:2", "2:5", "3:4"):
+        with pytest.raises(ValueError, match="spans may start and end at"):
+            Server(path, block_indices=blocks, device="cpu")
+    handler = swarm[1][0].handler
+    with pytest.raises(RpcError, match="reads the cache"):
+        handler._parse_uids({"uids": ["test-tulezen.2"]})
+    for option in ({"quant_type": "nf4"}, {"adapters": ["x"]}, {"tensor_parallel_ranks": 2}):
+        with pytest.raises(ValueError, match="served without"):
+            Server(path, device="cpu", **option)
+
+
+def test_block_selection_respects_cuts():
+    from petals_amd.server.block_selection import choose_best_blocks, servable_length
+
+    cuts = frozenset({0, 1, 3, 5})
+    assert [servable_length(n, 5, cuts) for n in (1, 2, 3, 4, 5, 9)] == [1, 2, 3, 4, 5, 5]
+    assert servable_length(1, 4, frozenset({0, 4})) == 4  # nothing shorter exists
+    for n in range(1, 6):
+        span = choose_best_blocks(n, [None] * 5, cuts)
+        assert span[0] in cuts and span[-1] + 1 in cuts and len(span) <= n
+    assert choose_best_blocks(2, [None] * 5) == [0, 1]
+
+
+def test_routing_trims_servers_to_cuts():
+    from petals_amd.client.routing.sequence_info import RemoteSequenceInfo
+    from petals_amd.data_structures import RemoteModuleInfo, ServerInfo, ServerState
+
+    online = ServerInfo(state=ServerState.ONLINE, throughput=1.0)
+    hosts = {"a": range(0, 3), "b": range(2, 5), "c": range(0, 5), "d": range(2, 3)}
+    infos = [RemoteModuleInfo(f"m.{i}", {p: online for p, r in hosts.items() if i in r}) for i in range(5)]
+    seq = RemoteSequenceInfo.make_empty([f"m.{i}" for i in range(5)], frozenset({0, 1, 3, 5}))
+    seq.update_(infos)
+    assert sorted((s.peer_id, s.start, s.end) for s in seq.spans_by_priority) == [("a", 0, 3), ("b", 3, 5), ("c", 0, 5)]
+
+
+# -------------------------------------------------------------- scheduler
+
+
+def test_runtime_merges_what_waits_under_one_key():
+    from petals_amd.server.scheduler import PriorityRuntime
+
+    runtime = PriorityRuntime().start()
+    calls = []
+    gate = threading.Event()
+
+    def batch(items):
+        calls.append(list(items))
+        return [ValueError(x) if x == 3 else 10 * x for x in items]
+
+    async def main():
+        blocker = asyncio.ensure_future(runtime.submit(0.0, gate.wait))
+        await asyncio.sleep(0.05)
+        waiting = [asyncio.ensure_future(runtime.submit_merged(1.0, "k", batch, i)) for i in range(5)]
+        other = asyncio.ensure_future(runtime.submit_merged(1.0, "other", batch, 7))
+        await asyncio.sleep(0.05)
+        gate.set()
+        await blocker
+        return await asyncio.gather(*waiting, other, return_exceptions=True)
+
+    out = asyncio.new_event_loop().run_until_complete(main())
+    runtime.shutdown()
+    assert calls == [[0, 1, 2, 3, 4], [7]]
+    assert isinstance(out[3], ValueError) and [o for o in out if not isinstance(o, ValueError)] == [0, 10, 20, 40, 70]
+
+
+def test_sessions_wait_for_pages():
+    from petals_amd.server.memory_cache import AllocationFailed, MemoryCache
+    from petals_amd.server.paged_cache import PagedPool, PageDescriptor
+
+    async def main():
+        pool = PagedPool({0: 32}, 4, dtype=torch.float32, device="cpu")
+        cache = MemoryCache(pool.num_pages * pool.bytes_per_page, torch.device("cpu"))
+        async with cache.allocate_cache(PageDescriptor(pool, 2, 65)) as (handle,):
+            with cache.use_cache(handle) as (sequences,):
+                for s in sequences:
+                    s.prepare(0, 65)
+            assert pool.free_pages == 0
+            with pytest.raises(AllocationFailed):
+                async with cache.allocate_cache(PageDescriptor(pool, 1, 1), timeout=0.05):
+                    pass
+        assert pool.free_pages == 4 and cache.current_size_bytes == 0 and pool.live_sequences == 0
+
+    asyncio.new_event_loop().run_until_complete(main())
+
+
+# ------------------------------------------------------------ trace command
+
+DEVICES = ["cpu", pytest.param("cuda", marks=pytest.mark.gpu)]
+
+
+@pytest.mark.parametrize("device", DEVICES)
+def test_trace_run(checkpoint, tmp_path, device):
+    path, raw, weights = checkpoint
+    rng = torch.Generator().manual_seed(5)
+    ids = {k: torch.randint(0, VOCAB, (n,), generator=rng).tolist() for k, n in (("a", 130), ("b", 20), ("c", 70))}
+    steps = [
+        ([("a", 100), ("b", 1)], []), ([("b", 10), ("c", 2)], []), ([("a", 29), ("b", 9), ("c", 1)], ["b"]),
+        ([("c", 67), ("a", 1)], ["a", "c"]),
+    ]
+    at, lines, wanted = dict.fromkeys(ids, 0), [], []
+    for n, (entries, end) in enumerate(steps):
+        out, rows = [], []
+        for k, count in entries:
+            want = sorted({0, count - 1}) if (n, k) != (1, "c") else []
+            out.append({"id": k, "tokens": ids[k][at[k] : at[k] + count], "want": want})
+            rows += [(k, at[k] + w) for w in want]
+            at[k] += count
+        lines.append(json.dumps({"step": n, "entries": out, "end": end}))
+        wanted.append(rows)
+    runner = os.path.join(os.path.dirname(os.path.dirname(os.path.abspath(__file__))), "bin", "trace_run")
+    done = subprocess.run(
+        [sys.executable, runner, "--model", path, "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "320",
+         "--device", device],
+        input="\n".join(lines) + "\n", capture_output=True, text=True, timeout=110,
+    )
+    assert done.returncode == 0, done.stderr[-2000:]
+    assert [x for x in done.stdout.splitlines() if x.startswith("done")] == [f"done {i}" for i in range(len(steps))]
+    want = {k: oracle.run(raw, weights, ids[k]) for k in ids}
+    for n, rows in enumerate(wanted):
+        import numpy as np
+
+        got = torch.from_numpy(np.fromfile(tmp_path / f"{n}.f32", dtype="<f4")).view(len(rows), VOCAB).double()
+        for g, (k, pos) in zip(got, rows):
+            assert (g - want[k][pos]).abs().max() < 1e-3 * want[k][pos].abs().max()
+
+
+@pytest.mark.gpu
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_generation_on_gpu(tmp_path, dtype):
+    """Server and client on the GPU; concurrent greedy generations."""
+    from petals_amd.dht.node import DHT
+
+    raw = oracle.config_dict(vocab=VOCAB, width=WIDTH, layers=LAYERS)
+    weights = oracle.random_model(raw, seed=11, decided=True)
+    weights["head"] *= 4.0  # greedy choices that 16-bit rounding rarely turns
+    oracle.save_model(str(tmp_path), raw, weights)
+    boot = DHT(host="127.0.0.1")
+    server = start_server(str(tmp_path), [boot.listen_addr], "0:5", device="cuda", dtype=dtype)
+    model = make_client(str(tmp_path), [boot.listen_addr]).to(device="cuda", dtype=getattr(torch, dtype))
+    try:
+        results = {}
+
+        def worker(i):
+            ids = torch.randint(0, VOCAB, (1, 5 + 40 * i), generator=torch.Generator().manual_seed(i))
+            results[i] = model.generate(ids.cuda(), max_new_tokens=20, do_sample=False)[0].tolist()
+
+        threads = [threading.Thread(target=worker, args=(i,)) for i in range(4)]
+        [t.start() for t in threads]
+        [t.join(timeout=60) for t in threads]
+        assert len(results) == 4
+        for i, out in results.items():
+            logits = oracle.run(raw, weights, out[:-1])
+            start = 5 + 40 * i - 1
+            for pos in range(start, len(out) - 1):
+                best = logits[pos].max() - logits[pos][out[pos + 1]]
+                assert best <= (1e-3 if dtype == "float32" else 0.25) * logits[pos].std(), (i, pos, float(best))
+    finally:
+        model.transformer.h.sequence_manager.shutdown()
+        server.shutdown()
+        boot.shutdown()

@@ -2,9 +2,8 @@
 
 One function per mechanism, float64 throughout, whole sequences only: no cache,
 no pages, no batching, nothing imported from the framework. Weights come as a
-dict of tensors under their checkpoint names. The optional ``rope``-free latent
-attention, the windows and the expert selection are spelled out as loops or
-dense masks so that each can be read against its formula.
+dict of tensors under their checkpoint names. Windows and expert selection are
+spelled out as dense masks and loops, to be read against their formulas.
 
 ``faults`` plants a mistake on purpose (tests use it to show that their inputs
 would expose one): "window+1", "window-1", "no_share", "renorm_router",
@@ -130,8 +129,12 @@ def run(
     return zero_centered_norm(x, weights["final.norm"], eps, faults) @ weights["head"].T
 
 
-def random_model(config: dict, seed: int = 0, scale: float = 1.0) -> Dict[str, torch.Tensor]:
-    """bf16 checkpoint tensors of `config` (row scale ~ 1/sqrt(in), norms off their neutral value)."""
+def random_model(config: dict, seed: int = 0, scale: float = 1.0, decided: bool = False) -> Dict[str, torch.Tensor]:
+    """bf16 checkpoint tensors of `config` (row scale ~ 1/sqrt(in), norms off their neutral value).
+
+    decided: the routers read a few dimensions that no sublayer adds to (their
+    norm weights are -1), so that each token's experts are fixed by its embedding
+    and 16-bit rounding cannot turn a close call into another expert."""
     g = torch.Generator().manual_seed(seed)
 
     def mat(out, inp, gain=1.0):
@@ -141,6 +144,7 @@ def random_model(config: dict, seed: int = 0, scale: float = 1.0) -> Dict[str, t
         return (center + 0.3 * torch.randn(n, generator=g)).to(torch.bfloat16)
 
     d = config["width"]
+    fixed = max(2, d // 5)
     w = {"embed": torch.randn(config["vocab"], d, generator=g).to(torch.bfloat16),
          "head": mat(config["vocab"], d), "final.norm": vec(d, 0.0)}
     for i, layer in enumerate(config["layers"]):
@@ -159,10 +163,15 @@ def random_model(config: dict, seed: int = 0, scale: float = 1.0) -> Dict[str, t
             ff = layer["mlp"]["expert"]["ff"]
             n = layer["mlp"]["router"]["experts"]
             w[p + "mlp.router"] = mat(n, d, 2.0)
+            if decided:
+                w[p + "mlp.router"][:, fixed:] = 0
             for e in range(n):
                 w[p + f"mlp.e{e}.gate"] = mat(ff, d, 2.0)
                 w[p + f"mlp.e{e}.up"] = mat(ff, d, 2.0)
                 w[p + f"mlp.e{e}.down"] = mat(d, ff)
+        if decided:
+            for norm in ("norm1", "norm2")[: 1 if layer.get("mlp") is None else 2]:
+                w[p + norm][:fixed] = -1
     return w
 
 
@@ -171,7 +180,7 @@ def config_dict(vocab=97, width=40, eps=1e-6, layers=()) -> dict:
             "vocab": vocab, "width": width}
 
 
-def layer_dict(heads=3, dim=16, vdim=24, kv_rank=32, window=20, scale=0.21, kv_from=None, ff=40, limit=1.5,
+def layer_dict(heads=3, dim=16, vdim=24, kv_rank=32, window=20, scale=0.05, kv_from=None, ff=40, limit=1.5,
                experts=5, top=2, mlp=True) -> dict:
     mixer = {"heads": heads, "dim": dim, "vdim": vdim, "kv_rank": kv_rank, "scale": scale, "mask": {"size": window}}
     if kv_from is not None:
