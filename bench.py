@@ -253,7 +253,14 @@ def main():
                    help="serve (default): the REAL serving stack (DHT + Server + handler + client "
                         "sessions) with the RCCL mesh hand-off — what a user gets; pipeline: bare "
                         "rank-per-GPU RCCL pipeline (kernel-harness upper bound)")
+    p.add_argument("--compare", default=None, choices=["tulezen"],
+                   help="instead of the flagship run: layers of this family beside the closest other family's, "
+                        "one GPU, random weights (benchmarks/benchmark_tulezen.py)")
     args = p.parse_args()
+    if args.compare:
+        from benchmarks.benchmark_tulezen import main as compare
+
+        return compare(steps=args.steps, warmup=args.warmup)
 
     import torch.distributed as dist
 

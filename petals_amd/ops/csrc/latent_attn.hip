@@ -25,12 +25,20 @@ using bf16x8 = __attribute__((ext_vector_type(8))) short;
 using f32x4 = __attribute__((ext_vector_type(4))) float;
 
 #define PAGE 64   // tokens per page
-#define LKVT 32   // keys per staged tile
-#define LPAD 8    // LDS row padding (elements)
+#define LKVT 32   // keys per staged tile; tiles are aligned, so one lies in one page
+#define LPAD 16   // LDS row padding (elements): rows 8 banks apart
 
-// transposed tile addressing: XOR swizzle on the dim group (see prefill_attn.hip)
-#define LVT_BYTE(dim, key_byte) \
-  ((((unsigned)(dim)) * ((LKVT + LPAD) * 2) + (unsigned)(key_byte)) ^ ((((unsigned)(dim) >> 3) & 7u) << 4))
+using v4s = __attribute__((ext_vector_type(4))) short;
+
+// PV B-fragment: keys hi*8..hi*8+7 of one dim per lane, read from the row-major
+// tile by two transposing LDS loads. p: row hi*8 + (lane&15)/4, column
+// 4*(lane&3) of a 16-wide dim block; after the load lane i holds column i.
+__device__ __forceinline__ bf16x8 load_keys(const unsigned short* p, int row_elems) {
+  using lds_v4s = __attribute__((address_space(3))) v4s;
+  const v4s a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s*)p);
+  const v4s b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s*)(p + 4 * row_elems));
+  return bf16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+}
 
 struct PagedRows {
   const int* pos;     // [T] position of each row
@@ -58,9 +66,15 @@ template <> __device__ __forceinline__ void store_f32<unsigned short>(unsigned s
 
 // ------------------------------------------------------------ MFMA kernel
 
+// A workgroup is 4 waves = RG groups of 16 rows x DG slices of the latent's
+// dims: DG > 1 when there are few rows (decoding), so that all waves share the
+// staging and the weighted sum. Tiles are double-buffered in LDS and the next
+// one is loaded while the current one is used. The same staged tile is the keys
+// (row-major fragments) and the values (transposing LDS loads).
+//
 // RC = latent size in 32-wide MFMA k-chunks (columns past RP read as zero).
-// Grid: (token runs, groups of 16*NW rows, key splits); NW = blockDim.x / 64.
-template <int RC>
+// Grid: (token runs, groups of 16*RG rows, key splits).
+template <int RC, int DG>
 __global__ __launch_bounds__(256) void latent_attn_kernel(
     const unsigned short* __restrict__ q,      // [T, H, RP]
     const unsigned short* __restrict__ cache,  // [num_pages, PAGE, RP]
@@ -76,31 +90,33 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
     float scale_log2e,
     int n_splits) {
   constexpr int R = RC * 32;
-  const int nw = blockDim.x / WAVE;
+  constexpr int RG = 4 / DG;
+  constexpr int ROW = R + LPAD;                  // LDS row in elements
+  constexpr int LOADS = LKVT * (R / 8);          // 16-byte loads per tile
+  constexpr int NLD = (LOADS + 255) / 256;       // per thread
+  constexpr int DB = (R / 16 + DG - 1) / DG;     // 16-wide dim blocks per wave
   const int tok0 = tiles[2 * blockIdx.x];
   const int ntok = tiles[2 * blockIdx.x + 1];
   const int rows = ntok * heads;
-  const int g0 = blockIdx.y * 16 * nw;  // first row of this workgroup
+  const int g0 = blockIdx.y * 16 * RG;  // first row of this workgroup
   if (g0 >= rows) return;               // uniform over the workgroup
-  const int g1 = min(g0 + 16 * nw, rows);
+  const int g1 = min(g0 + 16 * RG, rows);
 
   const int tid = threadIdx.x;
   const int wave = tid / WAVE;
   const int lane = tid & (WAVE - 1);
   const int col = lane & 15;
   const int hi = lane >> 4;
-  const int r0 = g0 + wave * 16;  // first row of this wave
+  const int r0 = g0 + (wave / DG) * 16;  // first row of this wave
+  const int d0 = (wave % DG) * DB;       // first dim block of this wave
 
-  extern __shared__ unsigned char smem[];
-  unsigned short* k_lds = reinterpret_cast<unsigned short*>(smem);  // [LKVT][R + LPAD]
-  unsigned char* vt_raw = smem + LKVT * (R + LPAD) * 2;             // [R][LKVT + LPAD] swizzled
-  unsigned short* p_lds =
-      reinterpret_cast<unsigned short*>(vt_raw + R * (LKVT + LPAD) * 2) + wave * 16 * (LKVT + LPAD);
+  extern __shared__ unsigned short smem[];
+  unsigned short* p_lds = smem + 2 * LKVT * ROW + wave * 16 * (LKVT + 8);
 
   const int seq = b.owner[tok0];
   const int first_pos = b.pos[tok0 + g0 / heads];
   const int last_pos = b.pos[tok0 + (g1 - 1) / heads];
-  const int key_lo = window > 0 ? max(0, first_pos - window + 1) : 0;
+  const int key_lo = window > 0 ? max(0, first_pos - window + 1) / LKVT * LKVT : 0;
   const int key_hi = last_pos + 1;
   const int n_tiles = (key_hi - key_lo + LKVT - 1) / LKVT;
   const int per_split = (n_tiles + n_splits - 1) / n_splits;
@@ -121,11 +137,11 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
     }
   }
 
-  f32x4 acc_o[R / 16];
-  float m_row[4], l_row[4];
+  f32x4 acc_o[DB];
+  float m_row[4], l_row[4];  // l_row: this lane's share of the row's sum
   int row_pos[4], row_lo[4];
 #pragma unroll
-  for (int d = 0; d < R / 16; ++d) acc_o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
+  for (int d = 0; d < DB; ++d) acc_o[d] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     m_row[r] = NEG_SENTINEL;
@@ -135,27 +151,44 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
     row_lo[r] = window > 0 ? row_pos[r] - window + 1 : 0;
   }
   // keys that every row of this wave sees: [all_lo, all_hi]
-  const int wave_last = min(r0 + 15, rows - 1);
   const bool full_wave = r0 + 16 <= rows;
   const int all_hi = full_wave ? b.pos[tok0 + r0 / heads] : -1;
-  const int all_lo = full_wave && window > 0 ? b.pos[tok0 + wave_last / heads] - window + 1 : 0;
+  const int all_lo = full_wave && window > 0 ? b.pos[tok0 + (r0 + 15) / heads] - window + 1 : 0;
 
-  for (int j0 = j_begin; j0 < j_end; j0 += LKVT) {
-    __syncthreads();
-    for (int idx = tid; idx < LKVT * (R / 8); idx += blockDim.x) {
+  bf16x8 next[NLD];
+  // rows of tile j0 that lie in [0, j_end); zero elsewhere and past rp
+  auto fetch = [&](int j0) {
+    const long at = cache_row(b, seq, j0);
+#pragma unroll
+    for (int i = 0; i < NLD; ++i) {
+      const int idx = tid + i * 256;
       const int row = idx / (R / 8);
       const int c8 = (idx - row * (R / 8)) * 8;
-      bf16x8 v8 = {0, 0, 0, 0, 0, 0, 0, 0};
-      if (j0 + row < j_end && c8 < rp) {
-        const long at = cache_row(b, seq, j0 + row);
-        if (at >= 0) v8 = *reinterpret_cast<const bf16x8*>(cache + (size_t)at * rp + c8);
-      }
-      *reinterpret_cast<bf16x8*>(&k_lds[row * (R + LPAD) + c8]) = v8;
-#pragma unroll
-      for (int e = 0; e < 8; ++e)
-        *reinterpret_cast<unsigned short*>(&vt_raw[LVT_BYTE(c8 + e, row * 2)]) = (unsigned short)v8[e];
+      next[i] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+      if ((LOADS % 256 == 0 || idx < LOADS) && at >= 0 && j0 + row < j_end && c8 < rp)
+        next[i] = *reinterpret_cast<const bf16x8*>(cache + ((size_t)at + row) * rp + c8);
     }
-    __syncthreads();
+  };
+  auto stage = [&](unsigned short* buf) {
+#pragma unroll
+    for (int i = 0; i < NLD; ++i) {
+      const int idx = tid + i * 256;
+      const int row = idx / (R / 8);
+      const int c8 = (idx - row * (R / 8)) * 8;
+      if (LOADS % 256 == 0 || idx < LOADS) *reinterpret_cast<bf16x8*>(&buf[row * ROW + c8]) = next[i];
+    }
+  };
+
+  if (j_begin < j_end) {
+    fetch(j_begin);
+    stage(smem);
+  }
+  __syncthreads();
+  int which = 0;
+  for (int j0 = j_begin; j0 < j_end; j0 += LKVT, which ^= 1) {
+    const unsigned short* k_lds = smem + which * LKVT * ROW;
+    const bool more = j0 + LKVT < j_end;
+    if (more) fetch(j0 + LKVT);
 
     f32x4 s_acc[2];
 #pragma unroll
@@ -163,8 +196,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
       s_acc[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kc = 0; kc < RC; ++kc) {
-        const bf16x8 kt =
-            *reinterpret_cast<const bf16x8*>(&k_lds[(nb * 16 + col) * (R + LPAD) + kc * 32 + hi * 8]);
+        const bf16x8 kt = *reinterpret_cast<const bf16x8*>(&k_lds[(nb * 16 + col) * ROW + kc * 32 + hi * 8]);
         s_acc[nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q_frag[kc], kt, s_acc[nb], 0, 0, 0);
       }
     }
@@ -189,52 +221,59 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
       for (int off = 8; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, WAVE));
       const float m_new = fmaxf(m_row[r], mx);
       corr[r] = (m_row[r] <= NEG_THRESHOLD) ? 0.f : exp2f(m_row[r] - m_new);
-      float lsum = 0.f;
 #pragma unroll
-      for (int nb = 0; nb < 2; ++nb) {
-        p[nb][r] = (s[nb] <= NEG_THRESHOLD) ? 0.f : exp2f(s[nb] - m_new);
-        lsum += p[nb][r];
-      }
-#pragma unroll
-      for (int off = 8; off > 0; off >>= 1) lsum += __shfl_xor(lsum, off, WAVE);
-      l_row[r] = l_row[r] * corr[r] + lsum;
+      for (int nb = 0; nb < 2; ++nb) p[nb][r] = (s[nb] <= NEG_THRESHOLD) ? 0.f : exp2f(s[nb] - m_new);
+      l_row[r] = l_row[r] * corr[r] + (p[0][r] + p[1][r]);
       m_row[r] = m_new;
     }
+    // P to A-fragment layout through this wave's own LDS
 #pragma unroll
     for (int r = 0; r < 4; ++r)
 #pragma unroll
-      for (int nb = 0; nb < 2; ++nb)
-        p_lds[(hi * 4 + r) * (LKVT + LPAD) + nb * 16 + col] = f32_to_bf16(p[nb][r]);
-    __syncthreads();
+      for (int nb = 0; nb < 2; ++nb) p_lds[(hi * 4 + r) * (LKVT + 8) + nb * 16 + col] = f32_to_bf16(p[nb][r]);
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    const bf16x8 p_frag = *reinterpret_cast<const bf16x8*>(&p_lds[col * (LKVT + 8) + hi * 8]);
 
-    const bf16x8 p_frag = *reinterpret_cast<const bf16x8*>(&p_lds[col * (LKVT + LPAD) + hi * 8]);
+    const unsigned short* v_lds = k_lds + (hi * 8 + col / 4) * ROW + (col & 3) * 4;
 #pragma unroll
-    for (int d = 0; d < R / 16; ++d) {
+    for (int d = 0; d < DB; ++d) {
+      if (DG > 1 && d0 + d >= R / 16) break;  // uniform over the wave
 #pragma unroll
       for (int r = 0; r < 4; ++r) acc_o[d][r] *= corr[r];
-      const bf16x8 vfrag = *reinterpret_cast<const bf16x8*>(&vt_raw[LVT_BYTE(d * 16 + col, hi * 16)]);
-      acc_o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p_frag, vfrag, acc_o[d], 0, 0, 0);
+      acc_o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+          p_frag, load_keys(v_lds + (d0 + d) * 16, ROW), acc_o[d], 0, 0, 0);
     }
+    if (more) stage(smem + (which ^ 1) * LKVT * ROW);
+    __syncthreads();
   }
 
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
+    float l = l_row[r];
+#pragma unroll
+    for (int off = 8; off > 0; off >>= 1) l += __shfl_xor(l, off, WAVE);
     const int row = r0 + hi * 4 + r;
     if (row >= rows) continue;
     const size_t flat = (size_t)tok0 * heads + row;
     if (n_splits == 1) {
-      const float inv_l = l_row[r] > 0.f ? 1.0f / l_row[r] : 0.f;
+      const float inv_l = l > 0.f ? 1.0f / l : 0.f;
 #pragma unroll
-      for (int d = 0; d < R / 16; ++d)
-        if (d * 16 + col < rp) out[flat * rp + d * 16 + col] = f32_to_bf16(acc_o[d][r] * inv_l);
+      for (int d = 0; d < DB; ++d) {
+        const int c = (d0 + d) * 16 + col;
+        if (c < rp) out[flat * rp + c] = f32_to_bf16(acc_o[d][r] * inv_l);
+      }
     } else {
       const size_t at = (size_t)blockIdx.z * total_tokens * heads + flat;
 #pragma unroll
-      for (int d = 0; d < R / 16; ++d)
-        if (d * 16 + col < rp) part_o[at * rp + d * 16 + col] = acc_o[d][r];
-      if (col == 0) {
+      for (int d = 0; d < DB; ++d) {
+        const int c = (d0 + d) * 16 + col;
+        if (c < rp) part_o[at * rp + c] = acc_o[d][r];
+      }
+      if (col == 0 && wave % DG == 0) {
         part_ml[at * 2] = m_row[r];
-        part_ml[at * 2 + 1] = l_row[r];
+        part_ml[at * 2 + 1] = l;
       }
     }
   }
@@ -244,22 +283,31 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
 __global__ __launch_bounds__(128) void latent_attn_combine(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     unsigned short* __restrict__ out, int n_rows, int rp, int n_splits) {
+  __shared__ float share[WAVE];  // weight of each split in the row
   const int row = blockIdx.x;
-  float m = NEG_SENTINEL;
-  for (int s = 0; s < n_splits; ++s) m = fmaxf(m, part_ml[((size_t)s * n_rows + row) * 2]);
-  float l = 0.f;
-  for (int s = 0; s < n_splits; ++s) {
-    const float* ml = part_ml + ((size_t)s * n_rows + row) * 2;
-    if (ml[0] > NEG_THRESHOLD) l += ml[1] * exp2f(ml[0] - m);
-  }
-  const float inv_l = l > 0.f ? 1.f / l : 0.f;
-  for (int d = threadIdx.x; d < rp; d += blockDim.x) {
-    float o = 0.f;
-    for (int s = 0; s < n_splits; ++s) {
-      const float ms = part_ml[((size_t)s * n_rows + row) * 2];
-      if (ms > NEG_THRESHOLD) o += part_o[((size_t)s * n_rows + row) * rp + d] * exp2f(ms - m);
+  if (threadIdx.x < WAVE) {
+    const int s = threadIdx.x;
+    float m = NEG_SENTINEL, l = 0.f;
+    if (s < n_splits) {
+      m = part_ml[((size_t)s * n_rows + row) * 2];
+      l = part_ml[((size_t)s * n_rows + row) * 2 + 1];
     }
-    out[(size_t)row * rp + d] = f32_to_bf16(o * inv_l);
+    const float mx = wave_reduce_max(m);
+    const float w = m > NEG_THRESHOLD ? exp2f(m - mx) : 0.f;
+    const float sum = wave_reduce_sum(w * l);
+    share[s] = sum > 0.f ? w / sum : 0.f;
+  }
+  __syncthreads();
+  for (int d = threadIdx.x; d < rp; d += blockDim.x) {
+    const float* src = part_o + (size_t)row * rp + d;
+    const size_t step = (size_t)n_rows * rp;
+    float o[4] = {0.f, 0.f, 0.f, 0.f};
+    int s = 0;
+    for (; s + 4 <= n_splits; s += 4)
+#pragma unroll
+      for (int u = 0; u < 4; ++u) o[u] = fmaf(src[(s + u) * step], share[s + u], o[u]);
+    for (; s < n_splits; ++s) o[0] = fmaf(src[s * step], share[s], o[0]);
+    out[(size_t)row * rp + d] = f32_to_bf16((o[0] + o[1]) + (o[2] + o[3]));
   }
 }
 
@@ -367,22 +415,19 @@ static PagedRows paged_rows(const torch::Tensor& pos, const torch::Tensor& owner
 
 #define BF16P(t) reinterpret_cast<unsigned short*>((t).data_ptr())
 
-template <int RC>
-static void launch_mfma(dim3 grid, int nw, const torch::Tensor& q, const torch::Tensor& cache, torch::Tensor& out,
+template <int RC, int DG>
+static void launch_mfma(dim3 grid, const torch::Tensor& q, const torch::Tensor& cache, torch::Tensor& out,
                         torch::Tensor& part_o, torch::Tensor& part_ml, const torch::Tensor& tiles, PagedRows b,
                         int heads, int rp, int window, float scale, int n_splits) {
-  const size_t lds = LKVT * (RC * 32 + LPAD) * 2 + RC * 32 * (LKVT + LPAD) * 2 + (size_t)nw * 16 * (LKVT + LPAD) * 2;
+  constexpr size_t lds = (2 * LKVT * (RC * 32 + LPAD) + 4 * 16 * (LKVT + 8)) * 2;
   static bool allowed = false;
-  if (!allowed) {
-    const size_t most = LKVT * (RC * 32 + LPAD) * 2 + RC * 32 * (LKVT + LPAD) * 2 + 4 * 16 * (LKVT + LPAD) * 2;
-    if (most > 65536) {
-      hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<RC>),
-                                         hipFuncAttributeMaxDynamicSharedMemorySize, (int)most);
-      TORCH_CHECK(e == hipSuccess, "LDS request refused: ", hipGetErrorString(e));
-    }
+  if (lds > 65536 && !allowed) {
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<RC, DG>),
+                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    TORCH_CHECK(e == hipSuccess, "LDS request refused: ", hipGetErrorString(e));
     allowed = true;
   }
-  latent_attn_kernel<RC><<<grid, nw * WAVE, lds, at::cuda::getCurrentCUDAStream()>>>(
+  latent_attn_kernel<RC, DG><<<grid, 256, lds, at::cuda::getCurrentCUDAStream()>>>(
       BF16P(q), BF16P(cache), BF16P(out), part_o.numel() ? part_o.data_ptr<float>() : nullptr,
       part_ml.numel() ? part_ml.data_ptr<float>() : nullptr, tiles.data_ptr<int>(), b, (int)q.size(0), heads, rp,
       window, scale * 1.4426950408889634f, n_splits);
@@ -416,21 +461,29 @@ torch::Tensor latent_attention(
     HIP_CHECK_LAST();
     return out;
   }
+  TORCH_CHECK(splits <= 64, "at most 64 key splits");
   TORCH_CHECK(tiles.is_cuda() && tiles.dtype() == torch::kInt32 && tiles.is_contiguous() && tiles.dim() == 2);
   const int rows = (int)run_tokens * heads;
-  const int nw = std::min(4, (rows + 15) / 16);
-  dim3 grid(tiles.size(0), (rows + 16 * nw - 1) / (16 * nw), 1);
+  const int rg = rows <= 16 ? 1 : rows <= 32 ? 2 : 4;  // 16-row groups per workgroup
+  dim3 grid(tiles.size(0), (rows + 16 * rg - 1) / (16 * rg), 1);
   int n_splits = (int)splits;
   if (n_splits <= 0) {
-    // enough workgroups for the chip, at least two key tiles each
+    // enough workgroups for the chip
     const long wgs = (long)grid.x * grid.y;
-    n_splits = (int)std::max(1L, std::min({(long)((max_keys + 63) / 64), 512 / std::max(1L, wgs), 64L}));
+    n_splits = (int)std::max(1L, std::min({(long)((max_keys + LKVT - 1) / LKVT), 512 / std::max(1L, wgs), 64L}));
   }
   grid.z = n_splits;
   auto f32o = q.options().dtype(torch::kFloat32);
   auto part_o = torch::empty({n_splits > 1 ? (long)n_splits * t * heads * rp : 0}, f32o);
   auto part_ml = torch::empty({n_splits > 1 ? (long)n_splits * t * heads * 2 : 0}, f32o);
-#define LA(RC) launch_mfma<RC>(grid, nw, q, cache, out, part_o, part_ml, tiles, b, heads, rp, (int)window, (float)scale, n_splits)
+#define LA2(RC, DG) \
+  launch_mfma<RC, DG>(grid, q, cache, out, part_o, part_ml, tiles, b, heads, rp, (int)window, (float)scale, n_splits)
+#define LA(RC)                    \
+  do {                            \
+    if (rg == 1) LA2(RC, 4);      \
+    else if (rg == 2) LA2(RC, 2); \
+    else LA2(RC, 1);              \
+  } while (0)
   const int rc = rp / 32;
   if (rc <= 1) LA(1);
   else if (rc <= 2) LA(2);
@@ -441,6 +494,7 @@ torch::Tensor latent_attention(
   else if (rc <= 12) LA(12);
   else LA(16);
 #undef LA
+#undef LA2
   HIP_CHECK_LAST();
   if (n_splits > 1) {
     latent_attn_combine<<<t * heads, 128, 0, stream>>>(

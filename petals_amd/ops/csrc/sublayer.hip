@@ -25,6 +25,21 @@ __device__ __forceinline__ float ld(const unsigned short* p) { return bf16_to_f3
 __device__ __forceinline__ void st(float* p, float v) { *p = v; }
 __device__ __forceinline__ void st(unsigned short* p, float v) { *p = f32_to_bf16(v); }
 
+// 8 consecutive elements, 16-byte aligned
+__device__ __forceinline__ void ld8(const float* p, float* v) {
+#pragma unroll
+  for (int h = 0; h < 2; ++h) {
+    const f32x4 a = reinterpret_cast<const f32x4*>(p)[h];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[4 * h + e] = a[e];
+  }
+}
+__device__ __forceinline__ void ld8(const unsigned short* p, float* v) {
+  const bf16x8 a = *reinterpret_cast<const bf16x8*>(p);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = bf16_to_f32((unsigned short)a[e]);
+}
+
 // sum over the workgroup, the same value in every thread; red holds one float
 // per wave and is free again on return
 __device__ __forceinline__ float block_sum(float v, float* red) {
@@ -85,8 +100,15 @@ __global__ __launch_bounds__(1024) void sublayer_out_kernel(
   __syncthreads();
   const int wave = tid / WAVE, lane = tid & (WAVE - 1);
   for (int e = wave; e < experts; e += nt / WAVE) {
-    float z = 0.f;
-    for (int c = lane; c < d; c += WAVE) z = fmaf(row[c], ld(router + (size_t)e * dp + c), z);
+    float z = 0.f;  // row and router are zero between d and dp
+    const TW* re = router + (size_t)e * dp;
+#pragma unroll 4
+    for (int c = lane * 8; c < dp; c += WAVE * 8) {
+      float w[8];
+      ld8(re + c, w);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) z = fmaf(row[c + i], w[i], z);
+    }
     z = wave_reduce_sum(z);
     if (lane == 0) logit[e] = z;
   }
@@ -210,6 +232,36 @@ __global__ __launch_bounds__(256) void batched_linear_kernel(
         if (c < n_dim) st(out + (size_t)t * o_t + h * o_h + c, acc[m][n][r]);
       }
     }
+}
+
+// Few rows (t_dim <= 16): the 4 waves of a workgroup share 16 columns and split
+// k, so that even a single token spreads a head over many waves.
+template <typename TA, typename TO>
+__global__ __launch_bounds__(256) void batched_linear_few_kernel(
+    const TA* __restrict__ a, long a_t, long a_h, const unsigned short* __restrict__ w,
+    TO* __restrict__ out, long o_t, long o_h, int t_dim, int n_dim, int k_dim, bool a_wide, bool w_wide) {
+  __shared__ float part[4][16][17];
+  const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;
+  const int col = lane & 15, hi = lane >> 4;
+  const int n0 = blockIdx.x * 16;
+  const size_t h = blockIdx.y;
+  const bool a_ok = col < t_dim, w_ok = n0 + col < n_dim;
+  const TA* ap = a + (size_t)(a_ok ? col : 0) * a_t + h * a_h;
+  const unsigned short* wp = w + (h * n_dim + (w_ok ? n0 + col : 0)) * (size_t)k_dim;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k0 = wave * 32; k0 < k_dim; k0 += 128) {
+    const bf16x8 wf = w_ok ? frag8(wp, k0 + hi * 8, k_dim, w_wide) : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    const bf16x8 af = a_ok ? frag8(ap, k0 + hi * 8, k_dim, a_wide) : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af, wf, acc, 0, 0, 0);
+  }
+#pragma unroll
+  for (int r = 0; r < 4; ++r) part[wave][hi * 4 + r][col] = acc[r];
+  __syncthreads();
+  const int t = threadIdx.x >> 4, c = threadIdx.x & 15;
+  if (t < t_dim && n0 + c < n_dim)
+    st(out + (size_t)t * o_t + h * o_h + n0 + c,
+       (part[0][t][c] + part[1][t][c]) + (part[2][t][c] + part[3][t][c]));
 }
 
 __global__ __launch_bounds__(256) void batched_linear_f32_kernel(
@@ -343,6 +395,7 @@ std::vector<torch::Tensor> sublayer_out(
   if (router.has_value()) {
     rf = is_f32(*router);
     TORCH_CHECK(router->is_contiguous() && router->dim() == 2 && router->size(1) == dp);
+    TORCH_CHECK(dp % 8 == 0 && reinterpret_cast<uintptr_t>(router->data_ptr()) % 16 == 0);
     experts = router->size(0);
     TORCH_CHECK(top >= 1 && top <= experts);
     rp = router->data_ptr();
@@ -395,16 +448,19 @@ torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32) {
 #define BL(TA, TO, MT, NT, AP, OP)                                                                          \
   batched_linear_kernel<TA, TO, MT, NT><<<dim3((n + 64 * NT - 1) / (64 * NT), (t + 16 * MT - 1) / (16 * MT), h), \
                                           256, 0, stream>>>(AP, at_, ah, BF16P(w), OP, ot, oh, t, n, k, a_wide, w_wide)
-#define BLO(TA, MT, NT, AP)                                         \
-  do {                                                              \
-    if (out_f32) BL(TA, float, MT, NT, AP, out.data_ptr<float>());  \
-    else BL(TA, unsigned short, MT, NT, AP, BF16P(out));            \
+#define BF(TA, TO, AP, OP)                                                           \
+  batched_linear_few_kernel<TA, TO><<<dim3((n + 15) / 16, h), 256, 0, stream>>>(     \
+      AP, at_, ah, BF16P(w), OP, ot, oh, t, n, k, a_wide, w_wide)
+#define BLO(TA, AP)                                                       \
+  do {                                                                    \
+    if (t <= 16) {                                                        \
+      if (out_f32) BF(TA, float, AP, out.data_ptr<float>());              \
+      else BF(TA, unsigned short, AP, BF16P(out));                        \
+    } else if (out_f32) BL(TA, float, 4, 2, AP, out.data_ptr<float>());   \
+    else BL(TA, unsigned short, 4, 2, AP, BF16P(out));                    \
   } while (0)
-  if (af) {
-    if (t <= 16) BLO(float, 1, 1, a.data_ptr<float>()); else BLO(float, 4, 2, a.data_ptr<float>());
-  } else {
-    if (t <= 16) BLO(unsigned short, 1, 1, BF16P(a)); else BLO(unsigned short, 4, 2, BF16P(a));
-  }
+  if (af) BLO(float, a.data_ptr<float>()); else BLO(unsigned short, BF16P(a));
+#undef BF
 #undef BLO
 #undef BL
   HIP_CHECK_LAST();

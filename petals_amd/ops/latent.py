@@ -155,7 +155,9 @@ class LatentMoEFastPath:
     def _dense(self, x: torch.Tensor, w: torch.Tensor, few: bool) -> torch.Tensor:
         """x [T, in] (32-bit if few rows or float32, else the weight dtype) @ w [in, out]."""
         if few:
-            return self.hip.gemv_bf16(w, x, self._no_ws, None, _EPI_PLAIN_F32)
+            # 64 input rows a wave keeps the loads of a short gemv in flight
+            splits = max(1, min(w.shape[0] // 64, 1024 // (-(-w.shape[1] // 512))))
+            return self.hip.gemv_bf16(w, x, self._no_ws, None, _EPI_PLAIN_F32, splits)
         return x @ w
 
     def forward_paged(self, x: torch.Tensor, batch, cache: torch.Tensor) -> torch.Tensor:
