@@ -279,7 +279,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
   }
 }
 
-// one workgroup per (token, head) row
+// one workgroup per (token, head) row and 128 of its dims
 __global__ __launch_bounds__(128) void latent_attn_combine(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
     unsigned short* __restrict__ out, int n_rows, int rp, int n_splits) {
@@ -298,7 +298,8 @@ __global__ __launch_bounds__(128) void latent_attn_combine(
     share[s] = sum > 0.f ? w / sum : 0.f;
   }
   __syncthreads();
-  for (int d = threadIdx.x; d < rp; d += blockDim.x) {
+  const int d = blockIdx.y * blockDim.x + threadIdx.x;
+  if (d < rp) {
     const float* src = part_o + (size_t)row * rp + d;
     const size_t step = (size_t)n_rows * rp;
     float o[4] = {0.f, 0.f, 0.f, 0.f};
@@ -470,7 +471,7 @@ torch::Tensor latent_attention(
   if (n_splits <= 0) {
     // enough workgroups for the chip
     const long wgs = (long)grid.x * grid.y;
-    n_splits = (int)std::max(1L, std::min({(long)((max_keys + LKVT - 1) / LKVT), 512 / std::max(1L, wgs), 64L}));
+    n_splits = (int)std::max(1L, std::min({(long)((max_keys + LKVT - 1) / LKVT), 128 / std::max(1L, wgs), 64L}));
   }
   grid.z = n_splits;
   auto f32o = q.options().dtype(torch::kFloat32);
@@ -497,7 +498,7 @@ torch::Tensor latent_attention(
 #undef LA2
   HIP_CHECK_LAST();
   if (n_splits > 1) {
-    latent_attn_combine<<<t * heads, 128, 0, stream>>>(
+    latent_attn_combine<<<dim3(t * heads, (rp + 127) / 128), 128, 0, stream>>>(
         part_o.data_ptr<float>(), part_ml.data_ptr<float>(), BF16P(out), t * heads, rp, n_splits);
     HIP_CHECK_LAST();
   }

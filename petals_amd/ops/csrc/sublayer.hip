@@ -65,36 +65,53 @@ __global__ __launch_bounds__(1024) void sublayer_out_kernel(
     const float* __restrict__ norm_w, float eps,
     const float* __restrict__ x, float* __restrict__ xo, unsigned short* __restrict__ xb,
     const TW* __restrict__ router, int experts, int top, int* __restrict__ sel, float* __restrict__ sel_w,
-    int d, int dp) {
+    int d, int dp, bool y_wide) {
   extern __shared__ float sm[];
-  float* row = sm;          // [dp]
+  float* row = sm;          // [dp], dp % 8 == 0
   float* logit = row + dp;  // [experts]
   __shared__ float red[16];
   const int tid = threadIdx.x, nt = blockDim.x;
   const size_t t = blockIdx.x;
 
   float ss = 0.f;
-  for (int c = tid; c < d; c += nt) {
-    float v;
-    if (slot_w) {
-      v = 0.f;
-      for (int j = 0; j < k; ++j) v = fmaf(slot_w[t * k + j], ld(y + (t * k + j) * ys + c), v);
-    } else {
-      v = ld(y + t * ys + c);
+  for (int c = tid * 8; c < d; c += nt * 8) {
+    float v[8], u[8];
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] = 0.f;
+    for (int j = 0; j < k; ++j) {
+      const TY* src = y + (t * k + j) * ys + c;
+      const float w = slot_w ? slot_w[t * k + j] : 1.f;
+      if (y_wide) {
+        ld8(src, u);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) u[i] = c + i < d ? ld(src + i) : 0.f;
+      }
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[i] = fmaf(w, u[i], v[i]);
     }
-    row[c] = v;
-    ss = fmaf(v, v, ss);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      if (c + i >= d) v[i] = 0.f;
+      row[c + i] = v[i];
+      ss = fmaf(v[i], v[i], ss);
+    }
   }
   const float inv = 1.f / sqrtf(block_sum(ss, red) / d + eps);
-  for (int c = tid; c < dp; c += nt) {
-    float v = 0.f;
-    if (c < d) {
-      v = row[c] * inv * (1.f + norm_w[c]);
-      if (x) v += x[t * dp + c];
+  for (int c = tid * 4; c < dp; c += nt * 4) {
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (c + i < d) v[i] = row[c + i] * inv * (1.f + norm_w[c + i]);
+    if (x) v += *reinterpret_cast<const f32x4*>(x + t * dp + c);
+    *reinterpret_cast<f32x4*>(xo + t * dp + c) = v;
+    *reinterpret_cast<f32x4*>(row + c) = v;
+    if (xb) {
+      uint2 w;
+      w.x = f32_to_bf16(v[0]) | ((unsigned)f32_to_bf16(v[1]) << 16);
+      w.y = f32_to_bf16(v[2]) | ((unsigned)f32_to_bf16(v[3]) << 16);
+      *reinterpret_cast<uint2*>(xb + t * dp + c) = w;
     }
-    xo[t * dp + c] = v;
-    if (xb) xb[t * dp + c] = f32_to_bf16(v);
-    row[c] = v;
   }
   if (!router) return;
   __syncthreads();
@@ -171,20 +188,25 @@ __device__ __forceinline__ bf16x8 frag8(const float* p, int k, int k_dim, bool w
   return bf16x8{v[0], v[1], v[2], v[3], v[4], v[5], v[6], v[7]};
 }
 
-// A wave computes 16*MT rows x 16*NT columns of one head; 4 waves side by side
-// in n. Fragments come straight from global memory (the weights are read once
-// per 16*MT rows; k is short or the rows are few wherever this runs).
-template <typename TA, typename TO, int MT, int NT>
+// A wave computes 64 rows x 64 columns of one head; the waves of a workgroup
+// take consecutive tiles (columns first). Fragments come straight from global
+// memory; the weights are the MFMA's A operand, so that a lane ends up with 4
+// neighbouring columns of one row, and rows leave through LDS in 16-byte stores.
+template <typename TA, typename TO>
 __global__ __launch_bounds__(256) void batched_linear_kernel(
     const TA* __restrict__ a, long a_t, long a_h,   // strides of rows and heads
     const unsigned short* __restrict__ w,           // [H, N, K]
-    TO* __restrict__ out, long o_t, long o_h, int t_dim, int n_dim, int k_dim, bool a_wide, bool w_wide) {
+    TO* __restrict__ out, long o_t, long o_h, int t_dim, int n_dim, int k_dim, int n_tiles, bool a_wide,
+    bool w_wide, bool o_wide) {
+  constexpr int MT = 4, NT = 4;
+  __shared__ TO tile[4][16][16 * NT + 16 / sizeof(TO)];
   const int lane = threadIdx.x & (WAVE - 1), wave = threadIdx.x / WAVE;
   const int col = lane & 15, hi = lane >> 4;
-  const int n0 = (blockIdx.x * 4 + wave) * 16 * NT;
-  const int t0 = blockIdx.y * 16 * MT;
-  const size_t h = blockIdx.z;
-  if (n0 >= n_dim) return;
+  const int job = blockIdx.x * 4 + wave;
+  const int n0 = job % n_tiles * 16 * NT;
+  const int t0 = job / n_tiles * 16 * MT;
+  const size_t h = blockIdx.y;
+  if (t0 >= t_dim) return;  // no barrier below
   const TA* ap[MT];
   const unsigned short* wp[NT];
   bool a_ok[MT], w_ok[NT];
@@ -205,7 +227,7 @@ __global__ __launch_bounds__(256) void batched_linear_kernel(
   for (int m = 0; m < MT; ++m)
 #pragma unroll
     for (int n = 0; n < NT; ++n) acc[m][n] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
+#pragma unroll 2
   for (int k0 = 0; k0 < k_dim; k0 += 32) {
     bf16x8 af[MT], wf[NT];
 #pragma unroll
@@ -218,20 +240,35 @@ __global__ __launch_bounds__(256) void batched_linear_kernel(
     for (int m = 0; m < MT; ++m)
 #pragma unroll
       for (int n = 0; n < NT; ++n)
-        acc[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(af[m], wf[n], acc[m][n], 0, 0, 0);
+        acc[m][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[n], af[m], acc[m][n], 0, 0, 0);
   }
+  // acc[m][n][r]: row t0 + m*16 + col, column n0 + n*16 + hi*4 + r
+  constexpr int PER = 16 / sizeof(TO);  // elements of a 16-byte store
 #pragma unroll
-  for (int m = 0; m < MT; ++m)
+  for (int m = 0; m < MT; ++m) {
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const int t = t0 + m * 16 + hi * 4 + r;
-      if (t >= t_dim) continue;
+    for (int n = 0; n < NT; ++n)
 #pragma unroll
-      for (int n = 0; n < NT; ++n) {
-        const int c = n0 + n * 16 + col;
-        if (c < n_dim) st(out + (size_t)t * o_t + h * o_h + c, acc[m][n][r]);
+      for (int r = 0; r < 4; ++r) st(&tile[wave][col][n * 16 + hi * 4 + r], acc[m][n][r]);
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+#pragma unroll
+    for (int i = lane; i < 16 * 16 * NT / PER; i += WAVE) {
+      const int t = t0 + m * 16 + i / (16 * NT / PER), c = i % (16 * NT / PER) * PER;
+      if (t >= t_dim || n0 + c >= n_dim) continue;
+      const TO* src = &tile[wave][t - t0 - m * 16][c];
+      TO* dst = out + (size_t)t * o_t + h * o_h + n0 + c;
+      if (o_wide && n0 + c + PER <= n_dim) {
+        *reinterpret_cast<f32x4*>(dst) = *reinterpret_cast<const f32x4*>(src);
+      } else {
+        for (int e = 0; e < PER && n0 + c + e < n_dim; ++e) dst[e] = src[e];
       }
     }
+  }
 }
 
 // Few rows (t_dim <= 16): the 4 waves of a workgroup share 16 columns and split
@@ -380,7 +417,9 @@ std::vector<torch::Tensor> sublayer_out(
     t = slot_w->size(0);
     sw = slot_w->data_ptr<float>();
   }
-  TORCH_CHECK(y.size(0) == t * k && y.size(1) >= d && dp >= d, "sublayer rows do not fit");
+  TORCH_CHECK(y.size(0) == t * k && y.size(1) >= d && dp >= d && dp % 8 == 0, "sublayer rows do not fit");
+  // whole groups of 8 may be read: aligned rows that reach to the next multiple of 8
+  const bool y_wide = y.size(1) % 8 == 0 && reinterpret_cast<uintptr_t>(y.data_ptr()) % 16 == 0;
   auto f32o = y.options().dtype(torch::kFloat32);
   auto xo = torch::empty({t, (long)dp}, f32o);
   auto xb = torch::empty({want_bf16 ? t : 0, (long)dp}, y.options().dtype(torch::kBFloat16));
@@ -395,7 +434,7 @@ std::vector<torch::Tensor> sublayer_out(
   if (router.has_value()) {
     rf = is_f32(*router);
     TORCH_CHECK(router->is_contiguous() && router->dim() == 2 && router->size(1) == dp);
-    TORCH_CHECK(dp % 8 == 0 && reinterpret_cast<uintptr_t>(router->data_ptr()) % 16 == 0);
+    TORCH_CHECK(reinterpret_cast<uintptr_t>(router->data_ptr()) % 16 == 0);
     experts = router->size(0);
     TORCH_CHECK(top >= 1 && top <= experts);
     rp = router->data_ptr();
@@ -413,7 +452,7 @@ std::vector<torch::Tensor> sublayer_out(
 #define SO(TY, TW, YP)                                                                                     \
   sublayer_out_kernel<TY, TW><<<t, threads, lds, stream>>>(                                                \
       YP, (int)y.size(1), k, sw, norm_w.data_ptr<float>(), (float)eps, xp, xo.data_ptr<float>(), xbp,      \
-      reinterpret_cast<const TW*>(rp), experts, (int)top, selp, selwp, d, (int)dp)
+      reinterpret_cast<const TW*>(rp), experts, (int)top, selp, selwp, d, (int)dp, y_wide)
     if (yf && rf) SO(float, float, y.data_ptr<float>());
     else if (yf) SO(float, unsigned short, y.data_ptr<float>());
     else if (rf) SO(unsigned short, float, BF16P(y));
@@ -445,9 +484,12 @@ torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32) {
   const size_t ab = af ? 4 : 2;
   const bool a_wide = (reinterpret_cast<uintptr_t>(a.data_ptr()) % 16 == 0) && (at_ * ab) % 16 == 0 && (ah * ab) % 16 == 0;
   const bool w_wide = k % 8 == 0;
-#define BL(TA, TO, MT, NT, AP, OP)                                                                          \
-  batched_linear_kernel<TA, TO, MT, NT><<<dim3((n + 64 * NT - 1) / (64 * NT), (t + 16 * MT - 1) / (16 * MT), h), \
-                                          256, 0, stream>>>(AP, at_, ah, BF16P(w), OP, ot, oh, t, n, k, a_wide, w_wide)
+  const bool o_wide = (n * (out_f32 ? 4 : 2)) % 16 == 0;
+  const int n_tiles = (n + 63) / 64;
+  const long jobs = n_tiles * ((t + 63) / 64);
+#define BL(TA, TO, AP, OP)                                                               \
+  batched_linear_kernel<TA, TO><<<dim3((jobs + 3) / 4, h), 256, 0, stream>>>(            \
+      AP, at_, ah, BF16P(w), OP, ot, oh, t, n, k, n_tiles, a_wide, w_wide, o_wide)
 #define BF(TA, TO, AP, OP)                                                           \
   batched_linear_few_kernel<TA, TO><<<dim3((n + 15) / 16, h), 256, 0, stream>>>(     \
       AP, at_, ah, BF16P(w), OP, ot, oh, t, n, k, a_wide, w_wide)
@@ -456,8 +498,8 @@ torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32) {
     if (t <= 16) {                                                        \
       if (out_f32) BF(TA, float, AP, out.data_ptr<float>());              \
       else BF(TA, unsigned short, AP, BF16P(out));                        \
-    } else if (out_f32) BL(TA, float, 4, 2, AP, out.data_ptr<float>());   \
-    else BL(TA, unsigned short, 4, 2, AP, BF16P(out));                    \
+    } else if (out_f32) BL(TA, float, AP, out.data_ptr<float>());   \
+    else BL(TA, unsigned short, AP, BF16P(out));                    \
   } while (0)
   if (af) BLO(float, a.data_ptr<float>()); else BLO(unsigned short, BF16P(a));
 #undef BF
