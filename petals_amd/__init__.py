@@ -1,6 +1,6 @@
 """petals_amd — an MI355X-native swarm inference/fine-tuning engine for large LMs.
 
-Capabilities modeled on bigscience-workshop/petals (see SURVEY.md): transformer
+Capabilities modeled on bigscience-workshop/petals: transformer
 blocks sharded by layer across independent servers, a thin client holding only
 embeddings + LM head, DHT-based discovery, fault-tolerant autoregressive
 inference with server-side KV caches, and parameter-efficient fine-tuning

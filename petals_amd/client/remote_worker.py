@@ -12,7 +12,7 @@ Two execution modes:
   this removes two thread wake-ups per step (submit + result) — worth
   ~0.2-0.3 ms/token against a 13 ms step. Concurrent callers fall back to
   blocking on the lock (client sessions are sequential by nature).
-* THREAD (PETALS_AMD_WORKER_THREAD=1): the round-1 background-thread design.
+* THREAD (PETALS_AMD_WORKER_THREAD=1): the earlier background-thread design.
 """
 
 from __future__ import annotations

@@ -44,7 +44,7 @@ def build(verbose: bool = False, name: str = "core") -> str:
     build_dir = os.path.join(PKG_DIR, folder)
     os.makedirs(build_dir, exist_ok=True)
     # torch's hipify writes `<name>_hip.<ext>` next to each source and skips
-    # regeneration based on mtimes; a repo snapshot (gpurun) can scramble those
+    # regeneration based on mtimes; copying the tree can scramble those
     # and leave a stale artifact compiling instead of the real source. Purge
     # them so every build regenerates from the true sources.
     import glob

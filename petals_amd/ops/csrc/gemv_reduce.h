@@ -57,7 +57,7 @@ static __device__ __forceinline__ float gelu_tanh_f32(float x) {
 // cut each thread's serial chain 8x; a tiny LDS tree combines (deterministic
 // order preserved: fixed group partition, fixed add order).
 #define GEMV_REDUCE_GROUPS 16  // 16 split groups x 64 outputs (1024-thread
-// wgs): halves each thread's serial split chain vs the round-2 value of 8 —
+// wgs): halves each thread's serial split chain vs the earlier value of 8 —
 // +1.3 tok/s on every alternating A/B pair (profiles/qrr_groups_ab.log);
 // PETALS_REDUCE_GROUPS=8 selects the old width
 

@@ -71,7 +71,7 @@ __global__ __launch_bounds__(WAVES * 64) void attn_prefill_kernel(
   const int q0 = q0_wg + wave * QR;  // this wave's first q row
   // softmax runs in the log2 domain (exp2 instead of exp): q is pre-scaled by
   // scale*log2e at load, saving a VALU mul per score AND per exponential —
-  // the kernel was issue-bound on VALU at 17:1 VALU:MFMA (PMC, round 1)
+  // the kernel was issue-bound on VALU at 17:1 VALU:MFMA (PMC)
   const float slope = ALIBI ? alibi[qh] * 1.4426950408889634f : 0.f;  // wave-uniform
 
   // LDS: K tile row-major [KVT][HD+KPAD]; V tile transposed+swizzled

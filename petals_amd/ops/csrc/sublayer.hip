@@ -116,18 +116,29 @@ __global__ __launch_bounds__(1024) void sublayer_out_kernel(
   if (!router) return;
   __syncthreads();
   const int wave = tid / WAVE, lane = tid & (WAVE - 1);
-  for (int e = wave; e < experts; e += nt / WAVE) {
-    float z = 0.f;  // row and router are zero between d and dp
-    const TW* re = router + (size_t)e * dp;
+  // two experts per wave at a time; row and router are zero between d and dp
+  for (int e = wave * 2; e < experts; e += nt / WAVE * 2) {
+    const bool both = e + 1 < experts;
+    float z0 = 0.f, z1 = 0.f;
+    const TW* r0 = router + (size_t)e * dp;
+    const TW* r1 = both ? r0 + dp : r0;
 #pragma unroll 4
     for (int c = lane * 8; c < dp; c += WAVE * 8) {
-      float w[8];
-      ld8(re + c, w);
+      float w0[8], w1[8];
+      ld8(r0 + c, w0);
+      ld8(r1 + c, w1);
 #pragma unroll
-      for (int i = 0; i < 8; ++i) z = fmaf(row[c + i], w[i], z);
+      for (int i = 0; i < 8; ++i) {
+        z0 = fmaf(row[c + i], w0[i], z0);
+        z1 = fmaf(row[c + i], w1[i], z1);
+      }
     }
-    z = wave_reduce_sum(z);
-    if (lane == 0) logit[e] = z;
+    z0 = wave_reduce_sum(z0);
+    z1 = wave_reduce_sum(z1);
+    if (lane == 0) {
+      logit[e] = z0;
+      if (both) logit[e + 1] = z1;
+    }
   }
   __syncthreads();
   if (wave != 0) return;

@@ -48,7 +48,7 @@ def _get_ws(device: torch.device, key: str, numel: int) -> torch.Tensor:
             # NEVER free a replaced workspace: hipGraphs capture raw pointers,
             # so freeing it lets the allocator hand the memory to someone else
             # and a previously captured graph replays into foreign storage.
-            # (Root cause of the round-1 "bloom dual-graph hardware fault":
+            # (Root cause of the earlier "bloom dual-graph hardware fault":
             # the client LM-head graph for bloom's 250k vocab grew the shared
             # gemv workspace AFTER the span graph had captured the old one.)
             _retired_workspaces.append(ws)
@@ -172,8 +172,8 @@ class _FastWeight:
         """bf16 [in, out] view for prefill GEMMs. Quantized weights dequantize
         through a process-wide LRU (default 16 GiB of the 288 GB HBM,
         PETALS_AMD_DEQUANT_CACHE_MB) so chunked prefills and back-to-back
-        sessions stop paying the per-matmul dequant (~337 us/weight measured
-        round 1, PARITY.md)."""
+        sessions stop paying the per-matmul dequant (~337 us/weight
+        measured)."""
         if self.quant == "nf4":
             return _dequant_cached(self, lambda: self.hip.nf4_dequantize(self.packed, self.absmax))
         if self.quant == "int8":
@@ -669,7 +669,7 @@ def _bloom_qkv_perm(qh: int, hd: int) -> torch.Tensor:
 
 
 class BloomFastPath(_TPFastPathMixin):
-    # The round-1 "bloom dual-graph hardware fault" (a bloom span graph +
+    # The earlier "bloom dual-graph hardware fault" (a bloom span graph +
     # the client's LM-head graph faulting on replay while each was clean in
     # isolation) was ROOT-CAUSED to the shared gemv workspace: bloom's 250k
     # vocab made the head's workspace request GROW the shared buffer, freeing

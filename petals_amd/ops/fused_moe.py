@@ -11,7 +11,7 @@ once per token — the decode-time degenerate case of a grouped GEMM.
 (The reference runs Mixtral experts densely inside one server's HF block with
 host-side routing: reference models/mixtral/block.py:73-81.)
 
-int8 expert weights keep the round-1 host-routed per-expert GEMV path
+int8 expert weights keep the host-routed per-expert GEMV path
 (graph_safe = False).
 """
 

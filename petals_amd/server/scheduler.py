@@ -62,9 +62,8 @@ class PriorityRuntime:
         # keep-warm (opt-in, PETALS_AMD_KEEP_WARM=<seconds>): for a short
         # window after each task, keep the device queue non-empty while idle.
         # Per-token serving leaves ~10 ms host gaps in which this pool's host
-        # power management parks sclk, making ~every 3rd step run ~5x slower
-        # (PARITY.md "serving cadence"). 1-element ticks every 1 ms were NOT
-        # enough to hold clocks on the SR-IOV pool host; the knob stays for
+        # power management parks sclk, making ~every 3rd step run ~5x slower.
+        # 1-element ticks every 1 ms were NOT enough to hold clocks on the SR-IOV pool host; the knob stays for
         # bare-metal deployments where guest clocks are controllable.
         self._keep_warm_s = float(_os.environ.get("PETALS_AMD_KEEP_WARM", "0"))
         self._warm_until = 0.0

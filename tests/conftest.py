@@ -7,7 +7,7 @@ sys.path.insert(0, os.path.dirname(os.path.dirname(os.path.abspath(__file__))))
 
 
 def pytest_configure(config):
-    config.addinivalue_line("markers", "gpu: test requires an MI355X GPU (run via gpurun)")
+    config.addinivalue_line("markers", "gpu: test requires an MI355X GPU")
 
 
 @pytest.fixture(scope="session")

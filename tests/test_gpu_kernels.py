@@ -808,7 +808,7 @@ def test_block_fast_decode_with_adapter_matches_cpu(hip, preset, hidden):
 
 @requires_gpu
 def test_bloom_dual_graph_with_big_vocab_head(hip):
-    """Regression for the round-1 dual-graph fault: a bloom-layout span graph
+    """Regression for the dual-graph fault: a bloom-layout span graph
     must survive the client's LM-head graph growing the shared gemv workspace
     (bloom's 250k vocab). _get_ws retires replaced workspaces so captured raw
     pointers stay valid."""
