@@ -19,14 +19,11 @@ In float32 every product is a true 32-bit one.
 
 from __future__ import annotations
 
-from typing import Dict, Optional
-
 import torch
 
 from petals_amd.ops.fused_decode import _EPI_PLAIN_F32
 
 GATE_ALPHA = 1.702
-_EPI_RAW = -1
 _EPI_CLAMPED_SWIGLU_F32 = 5
 _MOE_TILE = 32  # rows of a moe_gemm tile
 _GEMV_ROWS = 8  # most rows of the dense GEMV
