@@ -65,6 +65,8 @@ def main(argv=None):
     parser.add_argument("--quant_type", type=str, default="none", choices=["none", "nf4", "int8"])
     parser.add_argument("--attn_cache_tokens", type=int, default=16384)
     parser.add_argument("--max_batch_size", type=int, default=8)
+    parser.add_argument("--max_sequences", type=int, default=None,
+                        help="sequences that may be live at once, for models with recurrent state (a slot each)")
     parser.add_argument("--max_chunk_size_bytes", type=int, default=256 * 1024 * 1024,
                         help="prefill chunking bound inside a span (attention score memory)")
     parser.add_argument("--max_alloc_timeout", type=float, default=600.0,
@@ -190,6 +192,7 @@ def main(argv=None):
         dht_prefix=args.dht_prefix,
         attn_cache_tokens=args.attn_cache_tokens,
         max_batch_size=args.max_batch_size,
+        max_sequences=args.max_sequences,
         inference_max_length=args.inference_max_length,
         throughput=args.throughput,
         update_period=args.update_period,

@@ -89,8 +89,17 @@ class _ServerSession:
 class InferenceSession:
     """Synchronous user-facing session over the full block range."""
 
-    def __init__(self, sequence_manager: RemoteSequenceManager, max_length: int, batch_size: int = 1):
+    def __init__(
+        self,
+        sequence_manager: RemoteSequenceManager,
+        max_length: int,
+        batch_size: int = 1,
+        rewindable: bool = True,
+    ):
+        """rewindable: whether servers can drop a session's last tokens; if not,
+        a rollback replays what is left from the start."""
         self._manager = sequence_manager
+        self._rewindable = rewindable
         self._max_length = max_length
         self._batch_size = batch_size
         self._position = 0
@@ -111,9 +120,10 @@ class InferenceSession:
         """Rollback for speculative decoding: next step sends
         start_from_position so servers rewind their KV caches."""
         assert new_position <= self._position, "position can only be rolled back"
+        keep = new_position if self._rewindable or new_position == self._position else 0
         self._position = new_position
         for s in self._sessions:
-            s.position = min(s.position, new_position)
+            s.position = min(s.position, keep)
             if s.history is not None and s.history.shape[1] > new_position:
                 s.history = s.history[:, :new_position] if new_position > 0 else None
 

@@ -20,6 +20,7 @@ class LMHead(nn.Module):
     def __init__(self, config):
         super().__init__()
         self.weight = nn.Parameter(torch.zeros(config.vocab_size, config.hidden_size), requires_grad=False)
+        self.scale = getattr(config, "logit_scale", 1.0)
         use_chunked = getattr(config, "use_chunked_forward", "auto")
         if use_chunked == "auto":
             # chunk on CPU fp32 to bound peak memory; never on GPU
@@ -28,6 +29,10 @@ class LMHead(nn.Module):
         self.chunked_forward_step = getattr(config, "chunked_forward_step", 16384)
 
     def forward(self, hidden_states: torch.Tensor) -> torch.Tensor:
+        logits = self._project(hidden_states)
+        return logits if self.scale == 1.0 else logits * self.scale
+
+    def _project(self, hidden_states: torch.Tensor) -> torch.Tensor:
         if (
             self.weight.dtype in (torch.float16, torch.bfloat16)
             and self.weight.device.type == "cpu"

@@ -69,7 +69,9 @@ class RemoteSequential(nn.Module):
 
     @contextmanager
     def inference_session(self, **kwargs) -> InferenceSession:
-        with InferenceSession(self.sequence_manager, **kwargs) as session, self.use_session(session):
+        with InferenceSession(
+            self.sequence_manager, rewindable=self.config.rewindable, **kwargs
+        ) as session, self.use_session(session):
             yield session
 
     def __getitem__(self, ix) -> "RemoteSequential":

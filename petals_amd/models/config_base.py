@@ -12,6 +12,7 @@ from __future__ import annotations
 
 import dataclasses
 import json
+import math
 import os
 from typing import Any, ClassVar, Dict, FrozenSet, Optional, Tuple, Type
 
@@ -59,6 +60,7 @@ class ModelConfig:
     tie_word_embeddings: bool = False
     torch_dtype: str = "bfloat16"
     name_or_path: str = ""
+    logit_scale: float = 1.0  # factor of the head's output
 
     model_type: ClassVar[str] = ""  # set by @register_config
     # server options that the family's blocks do not have
@@ -110,6 +112,17 @@ class ModelConfig:
         """dtype of the hidden states that travel between blocks served in `dtype`."""
         return dtype
 
+    @property
+    def stream_width(self) -> int:
+        """Values per token of the hidden states that travel between blocks."""
+        return self.hidden_size
+
+    @property
+    def rewindable(self) -> bool:
+        """Whether a session can drop its last tokens. State that is folded into
+        one matrix cannot: such a session is replayed from its start."""
+        return True
+
     def valid_cuts(self) -> Optional[FrozenSet[int]]:
         """Block indices at which the chain may be split between servers
         (None: anywhere). Families whose blocks read another block's cache
@@ -125,6 +138,14 @@ class ModelConfig:
     def cache_values_per_token(self, block_index: int = 0) -> int:
         """Elements that one token occupies in one block's attention cache."""
         return 2 * self.n_kv_heads * self.head_dim
+
+    def state_shapes(self, block_index: int = 0) -> Dict[str, Tuple[int, ...]]:
+        """Per-sequence 32-bit state of one block besides what each token leaves
+        in the cache: name -> shape."""
+        return {}
+
+    def state_values(self, block_index: int = 0) -> int:
+        return sum(math.prod(s) for s in self.state_shapes(block_index).values())
 
     # ------------------------------------------------------- HF conversion
 

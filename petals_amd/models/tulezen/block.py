@@ -40,7 +40,7 @@ class TulezenBlock(nn.Module):
         self.layer_idx = layer_idx
         spec = config.spec(layer_idx)
         self.attention, self.moe, self.eps = spec.attention, spec.moe, config.layer_norm_eps
-        self.latent_layer = layer_idx if spec.attention.kv_from is None else spec.attention.kv_from
+        self.source_layer = layer_idx if spec.attention.kv_from is None else spec.attention.kv_from
         d, a = config.hidden_size, spec.attention
 
         def param(*shape):
@@ -111,7 +111,7 @@ class TulezenBlock(nn.Module):
 
     def forward_paged(self, x: torch.Tensor, batch, pool) -> torch.Tensor:
         """x [T, D] 32-bit residual of the batch's rows; returns the new one."""
-        cache = pool.layer(self.latent_layer)
+        cache = pool.layer(self.source_layer)
         if self._fast is not None:
             return self._fast.forward_paged(x, batch, cache)
         if x.is_cuda:

@@ -190,12 +190,24 @@ def zero_centered_rms_norm(x, weight, eps: float):
     return reference.zero_centered_rms_norm(x, weight, eps)
 
 
+def rms_norm_f32(x, weight, eps: float):
+    """x / sqrt(mean(x^2) + eps) * weight over the last axis, 32-bit in and out."""
+    if x.is_cuda and not _grad_mode(x, weight):
+        from petals_amd.ops import hybrid
+
+        return hybrid.rms_norm_f32(x, weight, eps)
+    return reference.rms_norm(x.float(), weight.float(), eps)
+
+
 def linear_f32(x, weight):
     """x @ weight.T with a 32-bit result, the product in the weight's dtype."""
     if x.is_cuda:
-        from petals_amd.ops import latent
+        from petals_amd.ops import _hip
 
-        return latent.linear_f32(x, weight)
+        # in every library of the paged families: the one this process serves with
+        hip = _hip.first_loaded("latent", "hybrid")
+        rows = x.float().reshape(-1, 1, x.shape[-1]).contiguous()
+        return hip.batched_linear(rows, weight.contiguous().unsqueeze(0), True).view(*x.shape[:-1], weight.shape[0])
     return (x.to(weight.dtype) @ weight.t()).float()
 
 

@@ -8,6 +8,20 @@ import os
 from petals_amd.ops.build import EXTENSIONS, so_path
 
 
+_loaded = {}
+
+
+def first_loaded(*names: str):
+    """The first of these libraries that this process has loaded; if it has
+    loaded none, the first that is built."""
+    for name in names:
+        if name in _loaded:
+            return _loaded[name]
+    name = next((n for n in names if os.path.exists(so_path(n))), names[0])
+    _loaded[name] = load(name)
+    return _loaded[name]
+
+
 def load(name: str = "core"):
     import torch  # noqa: F401 — the extension links against loaded libtorch
 

@@ -29,17 +29,13 @@ _MOE_TILE = 32  # rows of a moe_gemm tile
 _GEMV_ROWS = 8  # most rows of the dense GEMV
 _MOE_GEMV_ROWS = 64  # most (token, slot) rows of the expert GEMV
 
-_hip = None
 
 
 def hip():
     """The compiled kernels; on a GPU there is nothing else to fall back to."""
-    global _hip
-    if _hip is None:
-        from petals_amd.ops import _hip as loader
+    from petals_amd.ops import _hip
 
-        _hip = loader.load("latent")
-    return _hip
+    return _hip.first_loaded("latent")
 
 
 def _up(n: int, to: int) -> int:
@@ -50,12 +46,6 @@ def zero_centered_rms_norm(x: torch.Tensor, weight: torch.Tensor, eps: float) ->
     rows = x.float().reshape(-1, x.shape[-1]).contiguous()
     out, _, _, _ = hip().sublayer_out(rows, None, weight.float().contiguous(), eps, None, rows.shape[1], False, None, 1)
     return out.view(x.shape)
-
-
-def linear_f32(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
-    """x @ weight.T with a 32-bit result; the product runs in the weight's dtype."""
-    rows = x.float().reshape(-1, 1, x.shape[-1]).contiguous()
-    return hip().batched_linear(rows, weight.contiguous().unsqueeze(0), True).view(*x.shape[:-1], weight.shape[0])
 
 
 class LatentMoEFastPath:

@@ -202,7 +202,7 @@ def paged_write(cache: torch.Tensor, batch, rows: torch.Tensor) -> None:
     for s, (lo, hi) in enumerate(batch.row_ranges()):
         pos = torch.arange(batch.starts[s], batch.starts[s] + hi - lo)
         pages = torch.as_tensor(batch.pages[s])[pos // page]
-        cache[pages, pos % page, : rows.shape[1]] = rows[lo:hi]
+        cache[pages, pos % page, : rows.shape[1]] = rows[lo:hi].to(cache.dtype)
 
 
 def latent_attention_paged(q, cache, batch, w_uk, w_uv, *, scale: float, window: int) -> torch.Tensor:
@@ -221,3 +221,59 @@ def latent_attention_paged(q, cache, batch, w_uk, w_uv, *, scale: float, window:
         mask = sliding_window_mask(n, len(pos), start - first, window)
         out[lo:hi] = masked_attention(q[lo:hi], k, v, mask, scale)
     return out
+
+
+# --------------------------------- gated delta rule, attention with a sink
+
+
+def short_conv(x: torch.Tensor, weight: torch.Tensor) -> torch.Tensor:
+    """Causal convolution per channel: x [B, taps - 1 + S, C] with the inputs before
+    the first output ahead, weight [C, taps] (last column: the current token)."""
+    taps = weight.shape[1]
+    s = x.shape[1] - taps + 1
+    return sum(x[:, j : j + s] * weight[:, j] for j in range(taps))
+
+
+def unit_vectors(x: torch.Tensor, eps: float = 1e-6) -> torch.Tensor:
+    return x * torch.rsqrt(x.pow(2).sum(-1, keepdim=True) + eps)
+
+
+def gated_delta_rule(q, k, v, g, beta, state=None):
+    """q, k, g [B, S, H, dim], v [B, S, H, vdim], beta [B, S, H]; 32-bit. Per token
+    S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q.
+    Returns (o [B, S, H, vdim], last state [B, H, dim, vdim])."""
+    b, s, h, dim = q.shape
+    if state is None:
+        state = torch.zeros(b, h, dim, v.shape[-1], device=q.device)
+    out = []
+    for t in range(s):
+        state = g[:, t, :, :, None] * state
+        u = beta[:, t, :, None] * (v[:, t] - torch.einsum("bhk,bhkv->bhv", k[:, t], state))
+        state = state + k[:, t, :, :, None] * u[:, :, None, :]
+        out.append(torch.einsum("bhk,bhkv->bhv", q[:, t], state))
+    return torch.stack(out, dim=1), state
+
+
+def distance_slopes(heads: int, device=None) -> torch.Tensor:
+    """2^(-8 (h + 1) / heads), for any number of heads."""
+    return torch.exp2(-8.0 * torch.arange(1, heads + 1, device=device).float() / heads)
+
+
+def query_temperature(pos: torch.Tensor, coef: float, every: int) -> torch.Tensor:
+    """1 + coef * ln(floor((p + 1) / every) + 1), 32-bit."""
+    return 1.0 + coef * torch.log1p(((pos + 1) // every).float())
+
+
+def biased_sink_attention(q, k, v, q_pos, k_pos, *, scale, window, sink, slopes, temperature) -> torch.Tensor:
+    """q [..., Sq, H, d], k/v [..., Sk, G, d]; a distance bias slope * (i - j) is taken
+    off the scores, and the softmax's denominator holds exp(sink) per head. 32-bit."""
+    group = q.shape[-2] // k.shape[-2]
+    k, v = (t.float().repeat_interleave(group, dim=-2).transpose(-3, -2) for t in (k, v))
+    q = (q.float() * temperature[:, None, None]).transpose(-3, -2)
+    gap = (q_pos[:, None] - k_pos[None, :]).float()
+    score = (q @ k.transpose(-1, -2)) * scale - slopes[:, None, None] * gap
+    seen = (gap >= 0) & (gap < window) if window > 0 else gap >= 0
+    score = score.masked_fill(~seen, float("-inf"))
+    sink = sink.float()[:, None, None].expand(*score.shape[:-1], 1)
+    p = torch.softmax(torch.cat([score, sink], dim=-1), dim=-1)[..., :-1]
+    return (p @ v).transpose(-3, -2)

@@ -200,9 +200,9 @@ class TransformerConnectionHandler:
     # ----------------------------------------------------------- rpc_info
 
     async def rpc_info(self, request: RpcMessage, stream: RpcStream) -> None:
-        first = next(iter(self.backends.values()), None)
         cache_bytes_left = self.memory_cache.bytes_left
-        bytes_per_token = first.cache_bytes_per_token() if first is not None else 1
+        # blocks may differ in what a token leaves in them: their average
+        bytes_per_token = sum(b.cache_bytes_per_token() for b in self.backends.values()) // max(1, len(self.backends))
         info = {
             "version": "petals_amd-0.1",
             "dht_client_mode": False,
@@ -341,6 +341,7 @@ class TransformerConnectionHandler:
             for uid, prompt in zip(unit, prompts):
                 if prompt is not None:
                     pre = prompt.shape[1]
+                    prompt = torch.nn.functional.pad(prompt, (0, hidden.shape[-1] - prompt.shape[-1]))
                     hidden = torch.cat([hidden[:, :pre] + prompt, hidden[:, pre:]], dim=1)
                 hidden = self.backends[uid].block(hidden, shared=shared)
             return hidden

@@ -54,6 +54,10 @@ class TensorDescriptor:
     def allocate(self, device: torch.device) -> torch.Tensor:
         return torch.zeros(self.shape, dtype=self.dtype, device=device)
 
+    def ready(self) -> bool:
+        """Whether there is more to wait for than bytes."""
+        return True
+
     def release(self, tensor: torch.Tensor) -> None:
         """Nothing to give back beyond the bytes."""
 
@@ -103,7 +107,8 @@ class MemoryCache:
             while True:
                 with self._lock:
                     is_turn = self._alloc_queue and self._alloc_queue[0] == ticket
-                    if is_turn and self._current_size + total_bytes <= self.max_size_bytes:
+                    fits = self._current_size + total_bytes <= self.max_size_bytes
+                    if is_turn and fits and all(d.ready() for d in descriptors):
                         handles = []
                         for d in descriptors:
                             handle = next(self._handle_counter)

@@ -7,7 +7,8 @@ portions of prompts beside single decoded tokens - run as one ragged batch:
 
   PagedPool      the pages of every cache-owning layer, a free list, reference
                  counts (beam hypotheses share full pages; a shared page is
-                 copied when it is about to be written)
+                 copied when it is about to be written); and, for recurrent
+                 layers, one state slot per sequence
   PagedSequence  one sequence's page list and length; grows page by page,
                  rolls back, closes
   PageDescriptor reserves a session's worst case from MemoryCache's byte budget
@@ -26,6 +27,7 @@ from petals_amd.server.memory_cache import AllocationFailed
 from petals_amd.utils.misc import get_size_in_bytes
 
 PAGE_SIZE = 64  # tokens
+DEFAULT_SLOTS = 64  # sequences of a pool with recurrent state, if nothing else is said
 
 
 def pages_for(tokens: int) -> int:
@@ -41,14 +43,29 @@ class PagedPool:
         dtype: torch.dtype,
         device: torch.device,
         max_sequences: Optional[int] = None,
+        states: Optional[Dict[int, Dict[str, Tuple[int, ...]]]] = None,
     ):
+        """states: recurrent layer -> {name: shape of one sequence's 32-bit state}.
+        A slot is not cleared when it is taken: the state of a sequence at
+        position 0 is zero whatever the slot holds."""
         self.num_pages, self.dtype, self.device = num_pages, dtype, torch.device(device)
+        self.recurrent = bool(states)
+        if self.recurrent and max_sequences is None:
+            max_sequences = DEFAULT_SLOTS
         self.max_sequences = max_sequences
         self._layers = {
             layer: torch.zeros(num_pages, PAGE_SIZE, width, dtype=dtype, device=device)
             for layer, width in layer_widths.items()
         }
         self.bytes_per_page = sum(layer_widths.values()) * PAGE_SIZE * get_size_in_bytes(dtype)
+        slots = max_sequences if self.recurrent else 0
+        self._states = {
+            layer: {name: torch.zeros(slots + 1, *shape, device=device) for name, shape in shapes.items()}
+            for layer, shapes in (states or {}).items()
+        }
+        self.bytes_per_sequence = sum(4 * t[0].numel() for s in self._states.values() for t in s.values())
+        self.scratch_slot = slots  # belongs to no sequence
+        self._free_slots = list(range(slots - 1, -1, -1))
         self._free = list(range(num_pages - 1, -1, -1))
         self._refs = [0] * num_pages
         self._lock = threading.Lock()
@@ -65,12 +82,27 @@ class PagedPool:
         except KeyError:
             raise ValueError(f"the cache of block {layer} is not in this server's span") from None
 
+    def state(self, layer: int) -> Dict[str, torch.Tensor]:
+        """name -> [slots + 1, ...] of one recurrent layer."""
+        try:
+            return self._states[layer]
+        except KeyError:
+            raise ValueError(f"the state of block {layer} is not in this server's span") from None
+
+    @property
+    def total_bytes(self) -> int:
+        return self.num_pages * self.bytes_per_page + self.scratch_slot * self.bytes_per_sequence
+
+    def can_open(self, n: int) -> bool:
+        return self.max_sequences is None or self.live_sequences + n <= self.max_sequences
+
     def open(self) -> "PagedSequence":
         with self._lock:
-            if self.max_sequences is not None and self.live_sequences >= self.max_sequences:
+            if not self.can_open(1):
                 raise AllocationFailed(f"all {self.max_sequences} sequence slots are in use")
             self.live_sequences += 1
-        return PagedSequence(self)
+            slot = self._free_slots.pop() if self.recurrent else 0
+        return PagedSequence(self, slot)
 
     # ------------------------------------------------------ page accounting
 
@@ -110,11 +142,17 @@ class PagedPool:
         for seq, (pages, length) in zip(sequences, new):
             self._release(seq.pages)
             seq.pages, seq.length = pages, length
+        if self.recurrent:
+            own = torch.tensor([s.slot for s in sequences], device=self.device)
+            source = own[torch.as_tensor(list(parents), device=self.device)]
+            for tensors in self._states.values():
+                for t in tensors.values():
+                    t[own] = t[source]
 
 
 class PagedSequence:
-    def __init__(self, pool: PagedPool):
-        self.pool = pool
+    def __init__(self, pool: PagedPool, slot: int = 0):
+        self.pool, self.slot = pool, slot
         self.pages: List[int] = []
         self.length = 0  # tokens whose state is valid
         self._open = True
@@ -126,6 +164,8 @@ class PagedSequence:
             raise RuntimeError("the sequence is closed")
         if start > self.length:
             raise ValueError(f"position {start} is ahead of the cache ({self.length} tokens)")
+        if self.pool.recurrent and start not in (0, self.length):
+            raise ValueError(f"the state behind {self.length} tokens cannot go back to {start}; replay from 0")
         pool = self.pool
         need = pages_for(start + n)
         if need > len(self.pages):
@@ -151,6 +191,8 @@ class PagedSequence:
             self.pages, self.length = [], 0
             with self.pool._lock:
                 self.pool.live_sequences -= 1
+                if self.pool.recurrent:
+                    self.pool._free_slots.append(self.slot)
 
 
 class PageDescriptor:
@@ -158,7 +200,10 @@ class PageDescriptor:
 
     def __init__(self, pool: PagedPool, batch_size: int, max_length: int):
         self.pool, self.batch_size = pool, batch_size
-        self.nbytes = batch_size * pages_for(max_length) * pool.bytes_per_page
+        self.nbytes = batch_size * (pages_for(max_length) * pool.bytes_per_page + pool.bytes_per_sequence)
+
+    def ready(self) -> bool:
+        return self.pool.can_open(self.batch_size)
 
     def allocate(self, device) -> List[PagedSequence]:
         return [self.pool.open() for _ in range(self.batch_size)]
@@ -170,14 +215,24 @@ class PageDescriptor:
 
 class PagedBatch:
     """Rows of one step, grouped by sequence: sequence s brings rows
-    [offsets[s], offsets[s+1]) at positions starts[s], starts[s]+1, ..."""
+    [offsets[s], offsets[s+1]) at positions starts[s], starts[s]+1, ... and its
+    recurrent state is in slot slots[s]."""
 
-    def __init__(self, pages: List[List[int]], starts: List[int], lens: List[int], device: torch.device):
+    def __init__(
+        self,
+        pages: List[List[int]],
+        starts: List[int],
+        lens: List[int],
+        device: torch.device,
+        slots: Optional[List[int]] = None,
+    ):
         self.pages, self.starts, self.lens = pages, starts, lens
+        self.slots = [0] * len(lens) if slots is None else slots
         self.tokens = sum(lens)
         self.device = torch.device(device)
         self.max_end = max(s + n for s, n in zip(starts, lens))
         self._tiles: Dict[int, torch.Tensor] = {}
+        self._chunks: Dict[int, torch.Tensor] = {}
         if self.device.type == "cuda":
             self._upload()
 
@@ -196,19 +251,21 @@ class PagedBatch:
         return torch.tensor(values, dtype=torch.int32, pin_memory=True)
 
     def _upload(self) -> None:
-        """One int32 copy to the device: pos [T], owner [T], tables [S, width]."""
+        """One int32 copy to the device: pos [T], owner [T], slot [S], tables [S, width]."""
         t, width = self.tokens, max(len(p) for p in self.pages)
         flat: List[int] = []
         for s, n in zip(self.starts, self.lens):
             flat.extend(range(s, s + n))
         for i, n in enumerate(self.lens):
             flat.extend([i] * n)
+        flat.extend(self.slots)
         for p in self.pages:
             flat.extend(p)
             flat.extend([0] * (width - len(p)))
         dev = self._host_ints(flat).to(self.device, non_blocking=True)
         self.pos, self.owner = dev[:t], dev[t : 2 * t]
-        self.tables = dev[2 * t :].view(len(self.pages), width)
+        self.slot = dev[2 * t : 2 * t + len(self.slots)]
+        self.tables = dev[2 * t + len(self.slots) :].view(len(self.pages), width)
 
     def run_tokens(self, heads: int) -> int:
         """Rows that share one attention tile: as many as give about 64
@@ -226,6 +283,15 @@ class PagedBatch:
             self._tiles[rows] = self._host_ints(flat).to(self.device, non_blocking=True).view(-1, 2)
         return self._tiles[rows]
 
+    def chunk_bounds(self, rows: int) -> torch.Tensor:
+        """[S + 1] int32: tiles(rows)[bounds[s] : bounds[s + 1]] are sequence s's."""
+        if rows not in self._chunks:
+            bounds = [0]
+            for n in self.lens:
+                bounds.append(bounds[-1] - (-n // rows))
+            self._chunks[rows] = self._host_ints(bounds).to(self.device, non_blocking=True)
+        return self._chunks[rows]
+
 
 class StaticDecodeBatch(PagedBatch):
     """One row for each of `size` sequences in device buffers that keep their
@@ -236,15 +302,20 @@ class StaticDecodeBatch(PagedBatch):
         self.device = torch.device(device)
         self.starts, self.pages = [0] * size, [[0]] * size
         self.max_end = width * PAGE_SIZE
-        self._tiles = {}
+        self._tiles, self._chunks = {}, {}
+        self.slots = [0] * size
+        self.slot = torch.zeros(size, dtype=torch.int32, device=device)
         self.pos = torch.zeros(size, dtype=torch.int32, device=device)
         self.owner = torch.arange(size, dtype=torch.int32, device=device)
         self.tables = torch.zeros(size, width, dtype=torch.int32, device=device)
         self._uploaded: List[Optional[List[int]]] = [None] * size
         self.tiles(1)
 
-    def load(self, pages: List[List[int]], starts: List[int]) -> None:
+    def load(self, pages: List[List[int]], starts: List[int], slots: List[int]) -> None:
         self.pos.copy_(self._host_ints(starts), non_blocking=True)
+        if slots != self.slots:
+            self.slot.copy_(self._host_ints(slots), non_blocking=True)
+            self.slots = list(slots)
         for i, p in enumerate(pages):
             if self._uploaded[i] != p:
                 self.tables[i, : len(p)].copy_(self._host_ints(p), non_blocking=True)

@@ -31,6 +31,7 @@ from petals_amd.server.backend import TransformerBackend
 from petals_amd.server.from_pretrained import load_pretrained_block
 from petals_amd.server.handler import TransformerConnectionHandler
 from petals_amd.server.memory_cache import MemoryCache
+from petals_amd.server.paged_cache import DEFAULT_SLOTS
 from petals_amd.server.scheduler import PriorityRuntime
 from petals_amd.server.span_engine import SpanEngine
 from petals_amd.server.throughput import get_server_throughput
@@ -58,6 +59,7 @@ class Server:
         dht_prefix: Optional[str] = None,
         attn_cache_tokens: int = 16384,
         max_batch_size: int = 8,
+        max_sequences: Optional[int] = None,
         inference_max_length: Optional[int] = None,
         throughput: str | float = "auto",
         update_period: float = 60.0,
@@ -109,7 +111,7 @@ class Server:
             start, end = block_indices.split(":")
             self.block_indices = list(range(int(start), int(end)))
             num_blocks = len(self.block_indices)
-        self.num_blocks = num_blocks or self._choose_num_blocks(attn_cache_tokens)
+        self.num_blocks = num_blocks or self._choose_num_blocks(attn_cache_tokens, max_sequences or DEFAULT_SLOTS)
         cuts = self.config.valid_cuts()
         if self.block_indices and cuts is not None:
             if not {self.block_indices[0], self.block_indices[-1] + 1} <= cuts:
@@ -120,6 +122,7 @@ class Server:
 
         self.attn_cache_tokens = attn_cache_tokens
         self.max_batch_size = max_batch_size
+        self.max_sequences = max_sequences or DEFAULT_SLOTS
         self.inference_max_length = inference_max_length or attn_cache_tokens
         self.update_period = update_period
         self.expiration = expiration or max(3 * update_period, 60.0)
@@ -190,7 +193,7 @@ class Server:
             dtype_bytes = 1.002  # 8 bits/param + per-column bf16 scales
         return int(cfg.block_param_count() * dtype_bytes)
 
-    def _choose_num_blocks(self, attn_cache_tokens: int = 16384) -> int:
+    def _choose_num_blocks(self, attn_cache_tokens: int = 16384, max_sequences: int = DEFAULT_SLOTS) -> int:
         """Fit blocks to device memory: block bytes + attn-cache + autograd
         reserve (parity: server.py:275-326)."""
         if self.device.type == "cuda":
@@ -201,6 +204,9 @@ class Server:
         cache_bytes_per_block = (
             max(self.config.cache_values_per_token(i) for i in range(self.config.num_blocks))
             * attn_cache_tokens * get_size_in_bytes(self.torch_dtype)
+        )
+        cache_bytes_per_block += (
+            max(self.config.state_values(i) for i in range(self.config.num_blocks)) * 4 * max_sequences
         )
         autograd_reserve = 2 << 30
         usable = total * 0.92 - autograd_reserve
@@ -394,9 +400,10 @@ class Server:
         blocks = {uid: b.block for uid, b in self.backends.items()}
         if any(getattr(b, "paged", False) for b in blocks.values()):
             pool = SpanEngine.pool_for(
-                list(blocks.values()), self.attn_cache_tokens, dtype=self.torch_dtype, device=self.device
+                list(blocks.values()), self.attn_cache_tokens, dtype=self.torch_dtype, device=self.device,
+                max_sequences=self.max_sequences if any(self.config.state_shapes(i) for i in block_indices) else None,
             )
-            self.memory_cache.max_size_bytes = pool.num_pages * pool.bytes_per_page
+            self.memory_cache.max_size_bytes = pool.total_bytes
             engine = SpanEngine(blocks, pool, max_length=self.inference_max_length)
 
         self.handler = TransformerConnectionHandler(

@@ -51,16 +51,19 @@ class SpanEngine:
     @staticmethod
     def pool_for(blocks: Sequence[torch.nn.Module], tokens: int, *, dtype, device, max_sequences=None) -> PagedPool:
         widths = {b.layer_idx: b.paged_cache_width() for b in blocks if b.paged_cache_width()}
-        return PagedPool(widths, max(1, pages_for(tokens)), dtype=dtype, device=device, max_sequences=max_sequences)
+        states = {b.layer_idx: b.state_shapes() for b in blocks if b.state_shapes()}
+        return PagedPool(
+            widths, max(1, pages_for(tokens)), dtype=dtype, device=device, max_sequences=max_sequences, states=states
+        )
 
     def check_chain(self, uids: Sequence[Any]) -> None:
-        """A chain must contain the owner of every latent it reads, in order."""
+        """A chain must contain the owner of every cache it reads, in order."""
         seen = set()
         for uid in uids:
             block = self.blocks[uid]
-            if block.latent_layer != block.layer_idx and block.latent_layer not in seen:
+            if block.source_layer != block.layer_idx and block.source_layer not in seen:
                 raise ValueError(
-                    f"block {block.layer_idx} reads the cache of block {block.latent_layer}: "
+                    f"block {block.layer_idx} reads the cache of block {block.source_layer}: "
                     "both must be in one server's part of the chain"
                 )
             seen.add(block.layer_idx)
@@ -102,17 +105,18 @@ class SpanEngine:
 
     def _run(self, uids, parts, pool: PagedPool) -> torch.Tensor:
         hidden = [e.hidden[done : done + n].to(self.device, torch.float32) for e, done, n in parts]
-        x = hidden[0] if len(hidden) == 1 else torch.cat(hidden)
+        x = torch.cat(hidden)  # a copy: blocks may update the stream in place
         pages = [e.sequence.pages for e, _, _ in parts]
         starts = [e.start + done for e, done, _ in parts]
         lens = [n for _, _, n in parts]
+        slots = [e.sequence.slot for e, _, _ in parts]
         has_prompts = any(e.prompts is not None for e, _, _ in parts)
         if not has_prompts and pool is self.pool and self._graphable(uids, lens):
             key = (uids, len(lens))
             if key not in self._graphs:
                 self._graphs[key] = _DecodeGraph(self, uids, len(lens), x, pages, starts)
-            return self._graphs[key].step(x, pages, starts)
-        batch = PagedBatch(pages, starts, lens, self.device)
+            return self._graphs[key].step(x, pages, starts, slots)
+        batch = PagedBatch(pages, starts, lens, self.device, slots)
         for b, uid in enumerate(uids):
             if has_prompts:
                 x = self._add_prompts(x, parts, b)
@@ -128,7 +132,8 @@ class SpanEngine:
         self.check_chain(uids)
         b, s, _ = hidden.shape
         scratch = self.pool_for(
-            [self.blocks[u] for u in uids], b * pages_for(s) * PAGE_SIZE, dtype=self.pool.dtype, device=self.device
+            [self.blocks[u] for u in uids], b * pages_for(s) * PAGE_SIZE, dtype=self.pool.dtype, device=self.device,
+            max_sequences=b,
         )
         entries = [
             StepEntry(
@@ -147,7 +152,7 @@ class SpanEngine:
         """The chain in the smallest runs that share no state with each other."""
         runs: List[List[Any]] = []
         for uid in uids:
-            source = self.blocks[uid].latent_layer
+            source = self.blocks[uid].source_layer
             keep = len(runs)
             for i, run in enumerate(runs):
                 if any(self.blocks[u].layer_idx == source for u in run):
@@ -163,7 +168,7 @@ class SpanEngine:
             p = e.prompts[block] if e.prompts is not None else None
             if p is not None and done < p.shape[0]:
                 stop = min(n, p.shape[0] - done)
-                x[at : at + stop] += p[done : done + stop].to(x.device, x.dtype)
+                x[at : at + stop, : p.shape[1]] += p[done : done + stop].to(x.device, x.dtype)
             at += n
         return x
 
@@ -188,8 +193,9 @@ class _DecodeGraph:
         self.width = width
         self.batch = StaticDecodeBatch(size, width, engine.device)
         self.x = torch.empty(size, x.shape[1], dtype=torch.float32, device=engine.device)
-        # the warm-up runs write the state of the step that is about to run
-        self._load(x, pages, starts)
+        # the warm-up runs write the cache of the step that is about to run, which
+        # writes it again, and no sequence's recurrent state
+        self._load(x, pages, starts, [engine.pool.scratch_slot] * size)
 
         def span_fn():
             h = self.x
@@ -199,13 +205,13 @@ class _DecodeGraph:
 
         self.graph = GraphedCallable(span_fn, [])
 
-    def _load(self, x, pages, starts) -> None:
+    def _load(self, x, pages, starts, slots) -> None:
         longest = max(len(p) for p in pages)
         if longest > self.width:
             raise ValueError(f"a sequence holds {longest} pages, the step graph was made for {self.width}")
         self.x.copy_(x)
-        self.batch.load(pages, starts)
+        self.batch.load(pages, starts, slots)
 
-    def step(self, x: torch.Tensor, pages, starts) -> torch.Tensor:
-        self._load(x, pages, starts)
+    def step(self, x: torch.Tensor, pages, starts, slots) -> torch.Tensor:
+        self._load(x, pages, starts, slots)
         return self.graph.replay().clone()

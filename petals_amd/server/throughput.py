@@ -149,7 +149,7 @@ def _measure_paged_rps(config, block, device, dtype, *, n_infer_steps, n_forward
         block.optimize_for_inference()
     pool = SpanEngine.pool_for([block], 2048, dtype=dtype, device=device)
     engine = SpanEngine({0: block}, pool, max_length=1024)
-    x = torch.randn(forward_tokens, config.hidden_size, device=device)
+    x = torch.randn(forward_tokens, config.stream_width, device=device)
 
     def timed(n_rows: int, steps: int) -> float:
         sequence = pool.open()
