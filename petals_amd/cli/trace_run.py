@@ -33,10 +33,12 @@ def main() -> int:
     args = p.parse_args()
 
     if args.device.startswith("cuda"):
+        from petals_amd.models.config_base import load_model_config
         from petals_amd.ops.build import build, so_path
 
-        if not os.path.exists(so_path("latent")):
-            build(name="latent")
+        library = load_model_config(args.model).kernel_library
+        if not os.path.exists(so_path(library)):
+            build(name=library)
 
     import torch
 

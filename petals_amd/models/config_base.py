@@ -63,6 +63,8 @@ class ModelConfig:
     logit_scale: float = 1.0  # factor of the head's output
 
     model_type: ClassVar[str] = ""  # set by @register_config
+    # library of HIP kernels (ops/build.py) that a process serving the family needs
+    kernel_library: ClassVar[str] = "core"
     # server options that the family's blocks do not have
     unsupported: ClassVar[FrozenSet[str]] = frozenset()
     # dht_prefix identifies the block namespace in the swarm: "{prefix}.{i}"

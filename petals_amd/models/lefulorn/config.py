@@ -100,6 +100,7 @@ class LefulornConfig(ModelConfig):
     layers: List[Dict[str, Any]] = dataclasses.field(default_factory=list)
     block_prefix: str = "l"
 
+    kernel_library: ClassVar[str] = "hybrid"
     unsupported: ClassVar[FrozenSet[str]] = frozenset({"adapters", "quantization", "tensor parallelism"})
 
     def __post_init__(self):

@@ -78,6 +78,7 @@ class TulezenConfig(ModelConfig):
     layers: List[Dict[str, Any]] = dataclasses.field(default_factory=list)
     block_prefix: str = "l"
 
+    kernel_library: ClassVar[str] = "latent"
     unsupported: ClassVar[FrozenSet[str]] = frozenset({"adapters", "quantization", "tensor parallelism"})
 
     def __post_init__(self):

@@ -1,11 +1,13 @@
 """Build the HIP extensions IN-TREE (the .so files must travel with the source
 tree to GPU boxes): `python -m petals_amd.ops.build [name ...]`.
 
-Cross-compiles for gfx950 (no GPU needed at build time). Two libraries:
+Cross-compiles for gfx950 (no GPU needed at build time). Three libraries:
 
   core    the kernels of the llama / bloom / falcon / mixtral families
   latent  latent attention, output norms and routed experts (tulezen); it is
           all that a process serving such a model needs
+  hybrid  windowed attention with a distance bias and a sink, gated delta rule,
+          input norms (lefulorn); likewise
 """
 
 from __future__ import annotations
@@ -27,6 +29,10 @@ EXTENSIONS = {
     "latent": (
         "_hip_latent.so", "petals_amd_hip_latent", os.path.join("_build", "latent"),
         ["latent_bindings.cpp", "latent_attn.hip", "sublayer.hip", "gemv.hip", "moe.hip"],
+    ),
+    "hybrid": (
+        "_hip_hybrid.so", "petals_amd_hip_hybrid", os.path.join("_build", "hybrid"),
+        ["hybrid_bindings.cpp", "paged_attn.hip", "delta.hip", "prenorm.hip", "sublayer.hip", "gemv.hip"],
     ),
 }
 

@@ -18,6 +18,7 @@ enum GemvEpilogue : int {
   EPI_GELU_F32 = 4,      // y_f32[b, out] = gelu_tanh(sum) (BLOOM/Falcon MLPs)
   EPI_CLAMPED_SWIGLU_F32 = 5,  // g = min(sum[:half], limit), u = clamp(sum[half:], +-limit):
                                // g * sigmoid(alpha g) * (u + 1), y_f32[b, half]
+  EPI_RELU2_F32 = 6,     // y_f32[b, out] = relu(sum)^2
 };
 
 // constants of EPI_CLAMPED_SWIGLU_F32
@@ -129,6 +130,9 @@ static __global__ __launch_bounds__(64 * G) void gemv_reduce_kernel_impl(
       reinterpret_cast<unsigned short*>(y)[row + o] = f32_to_bf16(sum);
     } else if (epilogue == EPI_GELU_F32) {
       reinterpret_cast<float*>(y)[row + o] = gelu_tanh_f32(sum);
+    } else if (epilogue == EPI_RELU2_F32) {
+      const float r = fmaxf(sum, 0.f);
+      reinterpret_cast<float*>(y)[row + o] = r * r;
     } else {  // EPI_RESIDUAL_BF16
       const float r = bf16_to_f32(residual[row + o]);
       const unsigned short packed = f32_to_bf16(r + sum);
@@ -159,7 +163,7 @@ static inline torch::Tensor launch_gemv_reduce(
   const bool pair = epilogue == EPI_SWIGLU_F32 || epilogue == EPI_CLAMPED_SWIGLU_F32;
   const int n_out = pair ? half : out_dim;
   torch::Tensor y;
-  if (epilogue == EPI_PLAIN_F32 || epilogue == EPI_GELU_F32)
+  if (epilogue == EPI_PLAIN_F32 || epilogue == EPI_GELU_F32 || epilogue == EPI_RELU2_F32)
     y = torch::empty({batch, out_dim}, f32_opts);
   else if (pair)
     y = torch::empty({batch, half}, f32_opts);

@@ -1,0 +1,153 @@
+// Sublayer kernels for blocks that norm each sublayer's INPUT and keep the
+// residual stream in 32-bit (CDNA4, gfx950).
+//
+//   residual_norm   x += y (+ bias), then RMS norm of x with a plain weight
+//   residual_sum    x += split-K partial sums (+ bias) of a decoding product
+//   bias_relu2      relu(y + bias)^2
+//
+// The stream's rows may be wider than the residual (what lies past it is left
+// alone); the norm is written in rows padded with zeros to a multiple of 8.
+
+#include "common.h"
+#include "paged.h"
+#include <torch/extension.h>
+#include <ATen/cuda/CUDAContext.h>
+
+// One workgroup per token. y null: x is only read; h null: nothing is normed.
+template <typename TY, typename TH>
+__global__ __launch_bounds__(1024) void residual_norm_kernel(
+    float* __restrict__ x, long x_stride, const TY* __restrict__ y, long y_stride, const float* __restrict__ bias,
+    const float* __restrict__ w, float eps, TH* __restrict__ h, int d, int dp) {
+  extern __shared__ float row[];  // [d]
+  __shared__ float red[16];
+  const int tid = threadIdx.x, nt = blockDim.x;
+  const size_t t = blockIdx.x;
+  float* xr = x + t * x_stride;
+  float ss = 0.f;
+  for (int c = tid; c < d; c += nt) {
+    float v = xr[c];
+    if (y) {
+      v += load_f32(y + t * y_stride + c) + (bias ? bias[c] : 0.f);
+      xr[c] = v;
+    }
+    row[c] = v;
+    ss = fmaf(v, v, ss);
+  }
+  if (!h) return;  // uniform
+  ss = wave_reduce_sum(ss);
+  if ((tid & (WAVE - 1)) == 0) red[tid / WAVE] = ss;
+  __syncthreads();
+  ss = 0.f;
+  for (int i = 0; i < nt / WAVE; ++i) ss += red[i];
+  const float inv = 1.f / sqrtf(ss / d + eps);
+  for (int c = tid; c < dp; c += nt) store_f32(h + t * dp + c, c < d ? row[c] * inv * w[c] : 0.f);
+}
+
+// 64 columns x 16 groups of splits per workgroup
+__global__ __launch_bounds__(1024) void residual_sum_kernel(
+    const float* __restrict__ partials,  // [n_splits, batch, n]
+    const float* __restrict__ bias, float* __restrict__ x, long x_stride, int n_splits, int batch, int n, int d) {
+  __shared__ float acc[16][64];
+  const int ol = threadIdx.x & 63, sg = threadIdx.x >> 6;
+  const int c = blockIdx.x * 64 + ol, b = blockIdx.y;
+  float v = 0.f;
+  if (c < d)
+    for (int s = sg; s < n_splits; s += 16) v += partials[((size_t)s * batch + b) * n + c];
+  acc[sg][ol] = v;
+  __syncthreads();
+  if (sg != 0 || c >= d) return;
+  float sum = bias ? bias[c] : 0.f;
+#pragma unroll
+  for (int k = 0; k < 16; ++k) sum += acc[k][ol];
+  x[(size_t)b * x_stride + c] += sum;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void bias_relu2_kernel(T* __restrict__ y, const float* __restrict__ bias, int n, long total) {
+  const long i = ((long)blockIdx.x * 256 + threadIdx.x) * 8;
+  if (i >= total) return;  // n % 8 == 0: a group of 8 never crosses a row
+  const int c = i % n;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) {
+    const float v = fmaxf(load_f32(y + i + e) + bias[c + e], 0.f);
+    store_f32(y + i + e, v * v);
+  }
+}
+
+// ------------------------------------------------------------------- host
+
+static bool wide(const torch::Tensor& t) {
+  TORCH_CHECK(t.is_cuda() && (t.dtype() == torch::kFloat32 || t.dtype() == torch::kBFloat16));
+  return t.dtype() == torch::kFloat32;
+}
+
+static const float* vec(const c10::optional<torch::Tensor>& t, int64_t n) {
+  if (!t.has_value()) return nullptr;
+  TORCH_CHECK(t->is_cuda() && t->dtype() == torch::kFloat32 && t->is_contiguous() && t->numel() >= n);
+  return t->data_ptr<float>();
+}
+
+// x [T, >= d] f32, updated in place if y is given; returns the norm [T, dp], or nothing if w is absent
+torch::Tensor residual_norm(torch::Tensor x, c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> bias,
+                            c10::optional<torch::Tensor> w, int64_t d, double eps, bool out_f32) {
+  TORCH_CHECK(x.is_cuda() && x.dtype() == torch::kFloat32 && x.dim() == 2 && x.stride(1) == 1 && x.size(1) >= d);
+  const long t = x.size(0), dp = w.has_value() ? (d + 7) / 8 * 8 : 0;
+  bool yf = true;
+  const void* yp = nullptr;
+  long ys = 0;
+  if (y.has_value()) {
+    yf = wide(*y);
+    TORCH_CHECK(y->dim() == 2 && y->stride(1) == 1 && y->size(0) == t && y->size(1) >= d);
+    yp = y->data_ptr();
+    ys = y->stride(0);
+  }
+  const float* bp = vec(bias, d);
+  const float* wp = vec(w, d);
+  auto h = torch::empty({wp ? t : 0, dp}, x.options().dtype(out_f32 ? torch::kFloat32 : torch::kBFloat16));
+  if (t == 0) return h;
+  const size_t lds = d * 4;
+  TORCH_CHECK(lds <= 65536 - 64, "width ", d, " is not supported");
+  const int threads = t < 512 ? 1024 : 256;
+  auto stream = at::cuda::getCurrentCUDAStream();
+#define RN(TY, TH)                                                                                          \
+  residual_norm_kernel<TY, TH><<<t, threads, lds, stream>>>(                                                \
+      x.data_ptr<float>(), x.stride(0), reinterpret_cast<const TY*>(yp), ys, bp, wp, (float)eps,            \
+      wp ? reinterpret_cast<TH*>(h.data_ptr()) : nullptr, (int)d, (int)dp)
+  if (yf && out_f32) RN(float, float);
+  else if (yf) RN(float, unsigned short);
+  else if (out_f32) RN(unsigned short, float);
+  else RN(unsigned short, unsigned short);
+#undef RN
+  HIP_CHECK_LAST();
+  return h;
+}
+
+// partials [splits, T, >= d] of gemv_bf16's raw mode
+void residual_sum(torch::Tensor partials, c10::optional<torch::Tensor> bias, torch::Tensor x, int64_t d) {
+  TORCH_CHECK(partials.is_cuda() && partials.dtype() == torch::kFloat32 && partials.dim() == 3 && partials.is_contiguous());
+  TORCH_CHECK(x.is_cuda() && x.dtype() == torch::kFloat32 && x.dim() == 2 && x.stride(1) == 1);
+  const int batch = partials.size(1), n = partials.size(2);
+  TORCH_CHECK(x.size(0) == batch && x.size(1) >= d && n >= d && batch <= 65535);
+  if (batch == 0) return;
+  residual_sum_kernel<<<dim3((d + 63) / 64, batch), 1024, 0, at::cuda::getCurrentCUDAStream()>>>(
+      partials.data_ptr<float>(), vec(bias, d), x.data_ptr<float>(), x.stride(0), (int)partials.size(0), batch, n, (int)d);
+  HIP_CHECK_LAST();
+}
+
+// in place
+torch::Tensor bias_relu2(torch::Tensor y, torch::Tensor bias) {
+  const bool f = wide(y);
+  TORCH_CHECK(y.dim() == 2 && y.is_contiguous() && y.size(1) % 8 == 0);
+  const float* bp = vec(bias, y.size(1));
+  const long total = y.numel();
+  if (total == 0) return y;
+  const long blocks = (total / 8 + 255) / 256;
+  auto stream = at::cuda::getCurrentCUDAStream();
+  if (f) {
+    bias_relu2_kernel<float><<<blocks, 256, 0, stream>>>(y.data_ptr<float>(), bp, (int)y.size(1), total);
+  } else {
+    bias_relu2_kernel<unsigned short><<<blocks, 256, 0, stream>>>(BF16P(y), bp, (int)y.size(1), total);
+  }
+  HIP_CHECK_LAST();
+  return y;
+}

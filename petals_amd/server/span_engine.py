@@ -51,7 +51,7 @@ class SpanEngine:
     @staticmethod
     def pool_for(blocks: Sequence[torch.nn.Module], tokens: int, *, dtype, device, max_sequences=None) -> PagedPool:
         widths = {b.layer_idx: b.paged_cache_width() for b in blocks if b.paged_cache_width()}
-        states = {b.layer_idx: b.state_shapes() for b in blocks if b.state_shapes()}
+        states = {b.layer_idx: b.state_shapes() for b in blocks if getattr(b, "state_shapes", dict)()}
         return PagedPool(
             widths, max(1, pages_for(tokens)), dtype=dtype, device=device, max_sequences=max_sequences, states=states
         )
