@@ -253,14 +253,15 @@ def main():
                    help="serve (default): the REAL serving stack (DHT + Server + handler + client "
                         "sessions) with the RCCL mesh hand-off — what a user gets; pipeline: bare "
                         "rank-per-GPU RCCL pipeline (kernel-harness upper bound)")
-    p.add_argument("--compare", default=None, choices=["tulezen"],
+    p.add_argument("--compare", default=None, choices=["tulezen", "lefulorn"],
                    help="instead of the flagship run: layers of this family beside the closest other family's, "
-                        "one GPU, random weights (benchmarks/benchmark_tulezen.py)")
+                        "one GPU, random weights (benchmarks/benchmark_<family>.py)")
     args = p.parse_args()
     if args.compare:
-        from benchmarks.benchmark_tulezen import main as compare
+        import importlib
 
-        return compare(steps=args.steps, warmup=args.warmup)
+        compare = importlib.import_module(f"benchmarks.benchmark_{args.compare}")
+        return compare.main(steps=args.steps, warmup=args.warmup)
 
     import torch.distributed as dist
 

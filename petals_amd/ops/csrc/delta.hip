@@ -47,7 +47,7 @@ template <typename TY>
 struct ConvInput {
   const TY* y;  // [T, stride]
   int stride;
-  const float* w;      // [channels, taps]
+  const float* w;      // [taps, channels]
   const float* state;  // [slots, taps, channels]
 };
 
@@ -62,9 +62,29 @@ __device__ __forceinline__ float conv_silu(
     float x = 0.f;
     if (ago <= back) x = load_f32(in.y + (size_t)(row - ago) * in.stride + col);
     else if (pos - ago >= 0) x = in.state[((size_t)slot * s.taps + (pos - ago) % s.taps) * s.channels() + ch];
-    acc = fmaf(in.w[ch * s.taps + j], x, acc);
+    acc = fmaf(in.w[j * s.channels() + ch], x, acc);
   }
   return acc / (1.f + expf(-acc));
+}
+
+// 8 neighbouring channels at once (aligned groups)
+template <typename TY>
+__device__ __forceinline__ void conv_silu8(
+    const ConvInput<TY>& in, const DeltaShape& s, int row, int back, int pos, int slot, int col, int ch, float* out) {
+  float acc[8], x[8], w[8];
+#pragma unroll
+  for (int e = 0; e < 8; ++e) acc[e] = 0.f;
+  for (int j = 0; j < s.taps; ++j) {
+    const int ago = s.taps - 1 - j;
+    if (ago <= back) load8(in.y + (size_t)(row - ago) * in.stride + col, x);
+    else if (pos - ago >= 0) load8(in.state + ((size_t)slot * s.taps + (pos - ago) % s.taps) * s.channels() + ch, x);
+    else continue;
+    load8(in.w + (size_t)j * s.channels() + ch, w);
+#pragma unroll
+    for (int e = 0; e < 8; ++e) acc[e] = fmaf(w[e], x[e], acc[e]);
+  }
+#pragma unroll
+  for (int e = 0; e < 8; ++e) out[e] = acc[e] / (1.f + expf(-acc[e]));
 }
 
 // log2 of the decay
@@ -81,8 +101,9 @@ __host__ __device__ __forceinline__ size_t unit_size(int dk, int dv) {
 
 // ---------------------------------------------------------------- per chunk
 
-// Grid: (chunks, heads), 256 threads: 16 per token.
-template <typename TY>
+// Grid: (chunks, heads), 256 threads: 16 per token. BY8: head sizes and columns
+// are multiples of 8.
+template <typename TY, bool BY8>
 __global__ __launch_bounds__(256) void delta_chunk_kernel(
     ConvInput<TY> in, const float* __restrict__ a,  // a: [T, H * dim]
     const float* __restrict__ a_exp, const float* __restrict__ dt_bias, const int* __restrict__ tiles,
@@ -113,7 +134,40 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(
   float* w_g = w_qk + CH * CH;            // [dk]      G_15
 
   float q2 = 0.f, k2 = 0.f;
-  for (int c = l16; c < s.dk; c += 16) {
+  if (BY8) {
+    for (int c = l16 * 8; c < s.dk; c += 128) {
+      float q[8], k[8], lg[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) q[e] = k[e] = lg[e] = 0.f;
+      if (valid && c < s.dim) {
+        const int cq = kvh * s.dim + c, ca = h * s.dim + c;
+        conv_silu8(in, s, row, back, p, slot, s.oq + cq, cq, q);
+        conv_silu8(in, s, row, back, p, slot, s.ok + cq, s.kv_heads * s.dim + cq, k);
+        float b[8];
+        load8(a + (size_t)row * s.heads * s.dim + ca, lg);
+        load8(dt_bias + ca, b);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) lg[e] = log_decay(lg[e], b[e], a_exp[h]);
+      }
+      store8(&sq[i * P + c], q);
+      store8(&sk[i * P + c], k);
+      store8(&sl[i * P + c], lg);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        q2 = fmaf(q[e], q[e], q2);
+        k2 = fmaf(k[e], k[e], k2);
+      }
+    }
+    for (int c = l16 * 8; c < s.dv; c += 128) {
+      float v[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = 0.f;
+      const int cv = h * s.vdim + c;
+      if (valid && c < s.vdim) conv_silu8(in, s, row, back, p, slot, s.ov + cv, 2 * s.kv_heads * s.dim + cv, v);
+      store8(w_v + i * s.dv + c, v);
+    }
+  }
+  for (int c = BY8 ? s.dk : l16; c < s.dk; c += 16) {
     float q = 0.f, k = 0.f, lg = 0.f;
     if (valid && c < s.dim) {
       const int cq = kvh * s.dim + c;
@@ -130,11 +184,12 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(
   }
   const float qn = 1.f / sqrtf(group16_reduce_sum(q2) + 1e-6f) / sqrtf((float)s.dim);
   const float kn = 1.f / sqrtf(group16_reduce_sum(k2) + 1e-6f);
+  __syncthreads();  // a row's channels were written by other lanes
   for (int c = l16; c < s.dk; c += 16) {
     sq[i * P + c] *= qn;
     sk[i * P + c] *= kn;
   }
-  for (int c = l16; c < s.dv; c += 16) {
+  for (int c = BY8 ? s.dv : l16; c < s.dv; c += 16) {
     float v = 0.f;
     if (valid && c < s.vdim) {
       const int cv = h * s.vdim + c;
@@ -206,14 +261,22 @@ __device__ __forceinline__ f32x4 mma16(const f32x4& a, const f32x4& b, f32x4 c) 
   return c;
 }
 
+// a barrier for data in LDS that leaves loads from memory in flight
+__device__ __forceinline__ void lds_barrier() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
 template <int TPW>
 struct ChunkOperands {
   f32x4 kt[TPW], qt[TPW], kh[TPW], g[TPW], t, qk;
   float v[4];
 };
 
-// Grid: (heads, 16-column slices of S, sequences). The 4 waves hold the 16-row
-// tiles of S in turn, TPW each.
+// Grid: (heads, 16-column slices of S, sequences): the slices of a head, which
+// share their operands, meet in one XCD's L2. The 4 waves hold the 16-row tiles
+// of S in turn, TPW each; operands are on their way 3 chunks ahead (1 if they are many).
 template <int TPW>
 __global__ __launch_bounds__(256) void delta_scan_kernel(
     const float* __restrict__ ws, const int* __restrict__ tiles, const int* __restrict__ bounds,
@@ -222,7 +285,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
     DeltaShape s) {
   __shared__ f32x4 part[2][4][2][WAVE];
   const int h = blockIdx.x, v0 = blockIdx.y * 16, seq = blockIdx.z;
-  const int wave = threadIdx.x / WAVE, lane = threadIdx.x & (WAVE - 1);
+  const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x / WAVE), lane = threadIdx.x & (WAVE - 1);
   const int col = lane & 15, hi = lane >> 4;
   const int c0 = bounds[seq], c1 = bounds[seq + 1];
   if (c0 >= c1) return;
@@ -247,25 +310,18 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
     const float* g = tt + 2 * CH * CH;
 #pragma unroll
     for (int t = 0; t < TPW; ++t) {
-      const int tile = wave + t * 4;
-      if (tile < n_tiles) {
-        o.kt[t] = *reinterpret_cast<const f32x4*>(unit + col * s.dk + tile * 16 + hi * 4);
-        o.qt[t] = *reinterpret_cast<const f32x4*>(unit + (CH + col) * s.dk + tile * 16 + hi * 4);
-        o.kh[t] = *reinterpret_cast<const f32x4*>(kh + (tile * 16 + col) * CH + hi * 4);
-        o.g[t] = *reinterpret_cast<const f32x4*>(g + tile * 16 + hi * 4);
-      } else {
-        o.kt[t] = o.qt[t] = o.kh[t] = o.g[t] = zero;
-      }
+      const int tile = min(wave + t * 4, n_tiles - 1);
+      o.kt[t] = *reinterpret_cast<const f32x4*>(unit + col * s.dk + tile * 16 + hi * 4);
+      o.qt[t] = *reinterpret_cast<const f32x4*>(unit + (CH + col) * s.dk + tile * 16 + hi * 4);
+      o.kh[t] = *reinterpret_cast<const f32x4*>(kh + (tile * 16 + col) * CH + hi * 4);
+      o.g[t] = *reinterpret_cast<const f32x4*>(g + tile * 16 + hi * 4);
     }
     o.t = *reinterpret_cast<const f32x4*>(tt + col * CH + hi * 4);
     o.qk = *reinterpret_cast<const f32x4*>(tt + CH * CH + col * CH + hi * 4);
 #pragma unroll
     for (int r = 0; r < 4; ++r) o.v[r] = v[(hi * 4 + r) * s.dv + v0 + col];
   };
-  ChunkOperands<TPW> now, next;
-  load(c0, now);
-  for (int c = c0; c < c1; ++c) {
-    if (c + 1 < c1) load(c + 1, next);
+  auto step = [&](int c, const ChunkOperands<TPW>& now) {
     f32x4 pk = zero, pq = zero;
 #pragma unroll
     for (int t = 0; t < TPW; ++t) {
@@ -275,7 +331,7 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
     const int buf = c & 1;
     part[buf][wave][0][lane] = pk;
     part[buf][wave][1][lane] = pq;
-    __syncthreads();
+    lds_barrier();
     pk = (part[buf][0][0][lane] + part[buf][1][0][lane]) + (part[buf][2][0][lane] + part[buf][3][0][lane]);
     f32x4 rest;
 #pragma unroll
@@ -285,7 +341,12 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
     for (int t = 0; t < TPW; ++t) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) acc[t][r] *= now.g[t][r];
-      acc[t] = mma16(now.kh[t], u, acc[t]);
+      // no branch around a product: the tile past the last one takes zeros
+      const bool live = wave + t * 4 < n_tiles;
+      f32x4 kh;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) kh[r] = live ? now.kh[t][r] : 0.f;
+      acc[t] = mma16(kh, u, acc[t]);
     }
     if (wave == 3) {  // the wave with the fewest tiles
       pq = (part[buf][0][1][lane] + part[buf][1][1][lane]) + (part[buf][2][1][lane] + part[buf][3][1][lane]);
@@ -296,7 +357,36 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(
         if (hi * 4 + r < n && v0 + col < s.vdim)
           out[((size_t)(row0 + hi * 4 + r) * s.heads + h) * s.vdim + v0 + col] = pq[r];
     }
-    now = next;
+  };
+  auto load_ahead = [&](int c, ChunkOperands<TPW>& o) { load(min(c, c1 - 1), o); };
+  ChunkOperands<TPW> o0, o1, o2, o3;  // written out: an indexed array would not stay in registers
+  load_ahead(c0, o0);
+  if constexpr (TPW <= 2) {
+    load_ahead(c0 + 1, o1);
+    load_ahead(c0 + 2, o2);
+    int c = c0;
+    for (; c + 4 <= c1; c += 4) {
+      load_ahead(c + 3, o3);
+      step(c, o0);
+      load_ahead(c + 4, o0);
+      step(c + 1, o1);
+      load_ahead(c + 5, o1);
+      step(c + 2, o2);
+      load_ahead(c + 6, o2);
+      step(c + 3, o3);
+    }
+    if (c < c1) step(c, o0);
+    if (c + 1 < c1) step(c + 1, o1);
+    if (c + 2 < c1) step(c + 2, o2);
+  } else {
+    int c = c0;
+    for (; c + 2 <= c1; c += 2) {
+      load_ahead(c + 1, o1);
+      step(c, o0);
+      load_ahead(c + 2, o0);
+      step(c + 1, o1);
+    }
+    if (c < c1) step(c, o0);
   }
 #pragma unroll
   for (int t = 0; t < TPW; ++t) {
@@ -323,21 +413,45 @@ __global__ __launch_bounds__(256) void delta_conv_tail(
     conv[((size_t)slot * s.taps + pos[row] % s.taps) * s.channels() + ch] = load_f32(y + (size_t)row * stride + col);
 }
 
-// out[t, h * vdim + c] = o / rms(o) * w * sigmoid(gate); a wave per (token, head)
+// out[t, h * vdim + c] = o / rms(o) * w * sigmoid(gate); 16 lanes per (token, head)
 template <typename TO>
 __global__ __launch_bounds__(256) void delta_norm_kernel(
     const float* __restrict__ o, const float* __restrict__ gate, const float* __restrict__ w, TO* __restrict__ out,
     int out_stride, int heads, int vdim, long total, float eps) {
-  const long th = (long)blockIdx.x * 4 + threadIdx.x / WAVE;
-  if (th >= total) return;
-  const int lane = threadIdx.x & (WAVE - 1);
+  const long th = (long)blockIdx.x * 16 + threadIdx.x / 16;
+  if (th >= total) return;  // all 16 lanes
+  const int lane = threadIdx.x & 15;
   const float* src = o + th * vdim;
   const float* gs = gate + th * vdim;
   TO* dst = out + th / heads * out_stride + th % heads * vdim;
   float ss = 0.f;
-  for (int c = lane; c < vdim; c += WAVE) ss = fmaf(src[c], src[c], ss);
-  const float inv = 1.f / sqrtf(wave_reduce_sum(ss) / vdim + eps);
-  for (int c = lane; c < vdim; c += WAVE) store_f32(dst + c, src[c] * inv * w[c] / (1.f + expf(-gs[c])));
+  if (vdim % 8 == 0 && vdim <= 256) {
+    float o8[2][8], g8[2][8];
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      const int c = lane * 8 + m * 128;
+      if (c < vdim) {
+        load8(src + c, o8[m]);
+        load8(gs + c, g8[m]);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) ss = fmaf(o8[m][e], o8[m][e], ss);
+      }
+    }
+    const float inv = 1.f / sqrtf(group16_reduce_sum(ss) / vdim + eps);
+#pragma unroll
+    for (int m = 0; m < 2; ++m) {
+      const int c = lane * 8 + m * 128;
+      if (c < vdim) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) o8[m][e] *= inv * w[c + e] / (1.f + expf(-g8[m][e]));
+        store8(dst + c, o8[m]);
+      }
+    }
+    return;
+  }
+  for (int c = lane; c < vdim; c += 16) ss = fmaf(src[c], src[c], ss);
+  const float inv = 1.f / sqrtf(group16_reduce_sum(ss) / vdim + eps);
+  for (int c = lane; c < vdim; c += 16) store_f32(dst + c, src[c] * inv * w[c] / (1.f + expf(-gs[c])));
 }
 
 // ----------------------------------------------------------------- decoding
@@ -351,9 +465,13 @@ struct LowRank {
 template <typename TY, typename TW>
 __device__ __forceinline__ float quad_dot(const TY* x, const TW* w, int rank, int part) {
   float s = 0.f;
-  for (int r = part * 8; r < rank; r += 32)
+  for (int r = part * 8; r < rank; r += 32) {
+    float a[8], b[8];
+    load8(w + r, a);
+    load8(x + r, b);
 #pragma unroll
-    for (int e = 0; e < 8; ++e) s = fmaf(load_f32(w + r + e), load_f32(x + r + e), s);
+    for (int e = 0; e < 8; ++e) s = fmaf(a[e], b[e], s);
+  }
   s += __shfl_xor(s, 1, WAVE);
   s += __shfl_xor(s, 2, WAVE);
   return s;
@@ -517,8 +635,8 @@ static DeltaShape delta_shape(const torch::Tensor& y, int64_t heads, int64_t kv_
   const long width = y.size(1);
   TORCH_CHECK(cols[0] >= 0 && cols[0] + kv_heads * dim <= width && cols[1] >= 0 && cols[1] + kv_heads * dim <= width &&
               cols[2] >= 0 && cols[2] + heads * vdim <= width && cols[3] >= 0 && cols[3] + heads <= width);
-  TORCH_CHECK(conv_w.dim() == 2 && conv_w.size(0) == s.channels());
-  s.taps = conv_w.size(1);
+  TORCH_CHECK(conv_w.dim() == 2 && conv_w.size(1) == s.channels());
+  s.taps = conv_w.size(0);
   check_f32(conv_w, (long)s.channels() * s.taps, "convolution weights");
   TORCH_CHECK(delta.dim() == 4 && conv.dim() == 3);
   s.slots = delta.size(0);
@@ -557,21 +675,26 @@ torch::Tensor delta_prefill(
   const int *bp = bounds.data_ptr<int>(), *pp = pos.data_ptr<int>(), *op = owner.data_ptr<int>(), *sp = slot.data_ptr<int>();
   const int stride = y.size(1);
   const dim3 tail_grid(seqs, (s.channels() + 255) / 256);
-#define DC(TY, YP)                                                                                                    \
+#define DC(TY, BY8, YP)                                                                                               \
   do {                                                                                                                \
     if (lds > 65536) {                                                                                                \
-      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_chunk_kernel<TY>),                \
+      const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&delta_chunk_kernel<TY, BY8>),           \
                                                hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);                 \
       TORCH_CHECK(e == hipSuccess, "LDS request refused: ", hipGetErrorString(e));                                    \
     }                                                                                                                 \
     const ConvInput<TY> in{YP, stride, conv_w.data_ptr<float>(), conv.data_ptr<float>()};                             \
-    delta_chunk_kernel<TY><<<dim3(chunks, heads), 256, lds, stream>>>(in, a.data_ptr<float>(), a_exp.data_ptr<float>(), \
+    delta_chunk_kernel<TY, BY8><<<dim3(chunks, heads), 256, lds, stream>>>(in, a.data_ptr<float>(), a_exp.data_ptr<float>(), \
         dt_bias.data_ptr<float>(), tp, bp, pp, op, sp, s, ws.data_ptr<float>());                                      \
     HIP_CHECK_LAST();                                                                                                 \
     delta_conv_tail<TY><<<tail_grid, 256, 0, stream>>>(YP, stride, tp, bp, pp, sp, conv.data_ptr<float>(), s);        \
   } while (0)
-  if (yf) DC(float, y.data_ptr<float>());
-  else DC(unsigned short, BF16P(y));
+  bool by8 = dim % 8 == 0 && vdim % 8 == 0 && stride % 8 == 0;
+  for (int i = 0; i < 3; ++i) by8 = by8 && cols[i] % 8 == 0;
+  for (const auto& p : {y, a, conv_w, dt_bias, conv}) by8 = by8 && reinterpret_cast<uintptr_t>(p.data_ptr()) % 16 == 0;
+  if (yf && by8) DC(float, true, y.data_ptr<float>());
+  else if (yf) DC(float, false, y.data_ptr<float>());
+  else if (by8) DC(unsigned short, true, BF16P(y));
+  else DC(unsigned short, false, BF16P(y));
 #undef DC
   HIP_CHECK_LAST();
   const dim3 grid(heads, s.dv / 16, seqs);
@@ -595,14 +718,14 @@ torch::Tensor delta_norm(torch::Tensor o, torch::Tensor gate, torch::Tensor w, i
   check_f32(o, t * heads * vdim, "delta output");
   check_f32(gate, t * heads * vdim, "delta gate");
   check_f32(w, vdim, "delta norm");
-  TORCH_CHECK(width >= heads * vdim);
+  TORCH_CHECK(width >= heads * vdim && (vdim % 8 || width % 8 == 0));
   const auto opt = o.options().dtype(f32 ? torch::kFloat32 : torch::kBFloat16);
   auto out = width == heads * vdim ? torch::empty({t, width}, opt) : torch::zeros({t, width}, opt);
   if (t == 0) return out;
   const long total = t * heads;
   auto stream = at::cuda::getCurrentCUDAStream();
 #define DN(TO, OP)                                                                                              \
-  delta_norm_kernel<TO><<<(total + 3) / 4, 256, 0, stream>>>(o.data_ptr<float>(), gate.data_ptr<float>(),       \
+  delta_norm_kernel<TO><<<(total + 15) / 16, 256, 0, stream>>>(o.data_ptr<float>(), gate.data_ptr<float>(),       \
       w.data_ptr<float>(), OP, (int)width, (int)heads, (int)vdim, total, (float)eps)
   if (f32) DN(float, out.data_ptr<float>());
   else DN(unsigned short, BF16P(out));
@@ -632,6 +755,7 @@ torch::Tensor delta_decode(
     int64_t vdim, std::vector<int64_t> cols, int64_t width, double eps) {
   const DeltaShape s = delta_shape(y, heads, kv_heads, dim, vdim, cols, conv_w, delta, conv);
   const long t = y.size(0);
+  const int stride = y.size(1);
   check_f32(a_exp, heads, "decay rates");
   check_f32(dt_bias, heads * dim, "decay bias");
   check_f32(norm_w, vdim, "delta norm");
@@ -644,6 +768,7 @@ torch::Tensor delta_decode(
                 w.dtype() == (wf ? torch::kFloat32 : torch::kBFloat16), "low-rank projections");
   TORCH_CHECK(a2.size(0) == heads * dim && g2.size(0) == heads * vdim && (yf || !wf));
   const LowRank lr{(int)a1_col, (int)g1_col, (int)a2.size(1), (int)g2.size(1)};
+  TORCH_CHECK(a1_col % 8 == 0 && g1_col % 8 == 0 && stride % 8 == 0, "low-rank columns are read in groups of 8");
   TORCH_CHECK(a1_col >= 0 && a1_col + lr.a_rank <= y.size(1) && g1_col >= 0 && g1_col + lr.g_rank <= y.size(1));
   const int nr = decode_rows(s);
   TORCH_CHECK(delta_decodes(dim, vdim), "head sizes ", dim, " and ", vdim, " are not supported");
@@ -652,7 +777,6 @@ torch::Tensor delta_decode(
   if (t == 0) return out;
   auto stream = at::cuda::getCurrentCUDAStream();
   const size_t lds = (size_t)(3 * s.dk + 2 * s.dv + 2048) * 4;
-  const int stride = y.size(1);
 #define DD(TY, TW, N, YP, OP, A2, G2)                                                                              \
   delta_decode_kernel<TY, TW, N><<<dim3(t, heads), 512, lds, stream>>>(                                            \
       ConvInput<TY>{YP, stride, conv_w.data_ptr<float>(), conv.data_ptr<float>()}, conv.data_ptr<float>(), A2, G2, \

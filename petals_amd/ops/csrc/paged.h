@@ -34,6 +34,32 @@ template <typename T> __device__ __forceinline__ void store_f32(T* p, float v);
 template <> __device__ __forceinline__ void store_f32<float>(float* p, float v) { *p = v; }
 template <> __device__ __forceinline__ void store_f32<unsigned short>(unsigned short* p, float v) { *p = f32_to_bf16(v); }
 
+// 8 consecutive elements, 16-byte aligned
+static __device__ __forceinline__ void load8(const float* p, float* v) {
+#pragma unroll
+  for (int h = 0; h < 2; ++h) {
+    const f32x4 a = reinterpret_cast<const f32x4*>(p)[h];
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[4 * h + e] = a[e];
+  }
+}
+static __device__ __forceinline__ void load8(const unsigned short* p, float* v) {
+  const bf16x8 a = *reinterpret_cast<const bf16x8*>(p);
+#pragma unroll
+  for (int e = 0; e < 8; ++e) v[e] = bf16_to_f32((unsigned short)a[e]);
+}
+static __device__ __forceinline__ void store8(float* p, const float* v) {
+#pragma unroll
+  for (int h = 0; h < 2; ++h)
+    reinterpret_cast<f32x4*>(p)[h] = f32x4{v[4 * h], v[4 * h + 1], v[4 * h + 2], v[4 * h + 3]};
+}
+static __device__ __forceinline__ void store8(unsigned short* p, const float* v) {
+  bf16x8 a;
+#pragma unroll
+  for (int e = 0; e < 8; ++e) a[e] = (short)f32_to_bf16(v[e]);
+  *reinterpret_cast<bf16x8*>(p) = a;
+}
+
 using v4s = __attribute__((ext_vector_type(4))) short;
 
 // PV B-fragment: keys hi*8..hi*8+7 of one dim per lane, read from the row-major

@@ -98,8 +98,9 @@ __device__ __forceinline__ void softmax_tile(
 
 // ------------------------------------------------------------ MFMA kernel
 
-// RC: 32-wide chunks of the key size, VB: 16-wide blocks of the value size (at
-// least as many as there are; what lies past dk and dv is skipped).
+// RC: 32-wide chunks of the key size, VB: 16-wide blocks of the value size, at
+// least as many as there are: tiles are filled up with zeros, so that no branch
+// stands between products.
 // Grid: (token runs, kv heads x groups of 64 rows, key splits).
 template <int RC, int VB>
 __global__ __launch_bounds__(256) void paged_attn_kernel(
@@ -111,7 +112,9 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
     const int* __restrict__ tiles,             // [n, 2] first token, token count
     PagedRows b, AttnShape a, int total_tokens, int n_splits) {
   constexpr int KROW = RC * 32 + TPAD, VROW = VB * 16 + TPAD;
-  constexpr int NLD = RC * 4 * KVT / 256 + VB * 2 * KVT / 256;  // 16-byte loads per thread, at most
+  constexpr int K8 = RC * 4, V8 = VB * 2;                    // 16-byte groups of a row
+  constexpr int K_LOADS = KVT * K8, LOADS = KVT * (K8 + V8);
+  constexpr int NLD = (LOADS + 255) / 256;                   // per thread
   const int tok0 = tiles[2 * blockIdx.x];
   const int ntok = tiles[2 * blockIdx.x + 1];
   const int group = a.heads / a.kv_heads;
@@ -124,7 +127,6 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid & (WAVE - 1);
   const int col = lane & 15, hi = lane >> 4;
   const int r0 = g0 + wave * 16;
-  const int kc_n = a.dk / 32, vb_n = a.dv / 16;
 
   extern __shared__ unsigned short smem[];
   unsigned short* p_lds = smem + 2 * KVT * (KROW + VROW) + wave * 16 * (KVT + 8);
@@ -145,8 +147,8 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
     const size_t at = ((size_t)(tok0 + row / group) * a.heads + kvh * group + row % group) * a.dk;
 #pragma unroll
     for (int kc = 0; kc < RC; ++kc)
-      q_frag[kc] = row < rows && kc < kc_n ? *reinterpret_cast<const bf16x8*>(q + at + kc * 32 + hi * 8)
-                                           : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+      q_frag[kc] = row < rows && kc * 32 < a.dk ? *reinterpret_cast<const bf16x8*>(q + at + kc * 32 + hi * 8)
+                                                : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
   }
 
   f32x4 acc_o[VB];
@@ -170,8 +172,6 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
   const int all_lo = full_wave && a.window > 0 ? wave_last - a.window + 1 : 0;
   const int any_hi = wave_last, any_lo = a.window > 0 ? wave_first - a.window + 1 : 0;
 
-  const int k8 = a.dk / 8, v8 = a.dv / 8;
-  const int k_loads = KVT * k8, loads = k_loads + KVT * v8;
   const int width = a.kv_heads * (a.dk + a.dv);
   bf16x8 next[NLD];
   // rows of tile j0 that lie in [0, j_end); zero elsewhere
@@ -181,12 +181,12 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
     for (int i = 0; i < NLD; ++i) {
       const int idx = tid + i * 256;
       next[i] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
-      if (idx < loads) {
-        const bool is_v = idx >= k_loads;
-        const int at8 = is_v ? idx - k_loads : idx, per = is_v ? v8 : k8;
-        const int row = at8 / per, c8 = (at8 - row * per) * 8;
+      if (LOADS % 256 == 0 || idx < LOADS) {
+        const bool is_v = idx >= K_LOADS;
+        const int row = is_v ? (idx - K_LOADS) / V8 : idx / K8;
+        const int c8 = (is_v ? (idx - K_LOADS) % V8 : idx % K8) * 8;
         const int c = is_v ? a.kv_heads * a.dk + kvh * a.dv + c8 : kvh * a.dk + c8;
-        if (at >= 0 && j0 + row < j_end)
+        if (at >= 0 && j0 + row < j_end && c8 < (is_v ? a.dv : a.dk))
           next[i] = *reinterpret_cast<const bf16x8*>(cache + ((size_t)at + row) * width + c);
       }
     }
@@ -195,10 +195,10 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
 #pragma unroll
     for (int i = 0; i < NLD; ++i) {
       const int idx = tid + i * 256;
-      if (idx < loads) {
-        const bool is_v = idx >= k_loads;
-        const int at8 = is_v ? idx - k_loads : idx, per = is_v ? v8 : k8;
-        const int row = at8 / per, c8 = (at8 - row * per) * 8;
+      if (LOADS % 256 == 0 || idx < LOADS) {
+        const bool is_v = idx >= K_LOADS;
+        const int row = is_v ? (idx - K_LOADS) / V8 : idx / K8;
+        const int c8 = (is_v ? (idx - K_LOADS) % V8 : idx % K8) * 8;
         unsigned short* dst = is_v ? buf + KVT * KROW + row * VROW + c8 : buf + row * KROW + c8;
         *reinterpret_cast<bf16x8*>(dst) = next[i];
       }
@@ -223,7 +223,6 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
         s_acc[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int kc = 0; kc < RC; ++kc) {
-          if (kc >= kc_n) break;
           const bf16x8 kt = *reinterpret_cast<const bf16x8*>(&k_lds[(nb * 16 + col) * KROW + kc * 32 + hi * 8]);
           s_acc[nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q_frag[kc], kt, s_acc[nb], 0, 0, 0);
         }
@@ -241,7 +240,6 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
       const unsigned short* v_lds = k_lds + KVT * KROW + (hi * 8 + col / 4) * VROW + (col & 3) * 4;
 #pragma unroll
       for (int d = 0; d < VB; ++d) {
-        if (d >= vb_n) break;
 #pragma unroll
         for (int r = 0; r < 4; ++r) acc_o[d][r] *= corr[r];
         acc_o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p_frag, load_keys(v_lds + d * 16, VROW), acc_o[d], 0, 0, 0);
@@ -270,12 +268,12 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
       const float inv_l = l > 0.f ? scale / l : 0.f;
 #pragma unroll
       for (int d = 0; d < VB; ++d)
-        if (d < vb_n) write_gated(g, a, tok, head, d * 16 + col, acc_o[d][r] * inv_l);
+        if (d * 16 < a.dv) write_gated(g, a, tok, head, d * 16 + col, acc_o[d][r] * inv_l);
     } else {
       const size_t at = ((size_t)blockIdx.z * total_tokens + tok) * a.heads + head;
 #pragma unroll
       for (int d = 0; d < VB; ++d)
-        if (d < vb_n) part_o[at * a.dv + d * 16 + col] = acc_o[d][r];
+        if (d * 16 < a.dv) part_o[at * a.dv + d * 16 + col] = acc_o[d][r];
       if (col == 0) {
         part_ml[at * 2] = w.m[r];
         part_ml[at * 2 + 1] = l;
@@ -293,12 +291,12 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
     const unsigned short* __restrict__ q, const unsigned short* __restrict__ cache, GatedOut g,
     float* __restrict__ part_o, float* __restrict__ part_ml, PagedRows b, AttnShape a, int total_tokens, int n_splits) {
   constexpr int VROW = VB * 16 + TPAD;
-  constexpr int NLD = VB * 2 * KVT / WAVE;  // 16-byte value loads per lane, at most
+  constexpr int V8 = VB * 2;                // 16-byte groups of a row
+  constexpr int NLD = V8 * KVT / WAVE;      // value loads per lane
   const int tok = blockIdx.x, kvh = blockIdx.y;
   const int group = a.heads / a.kv_heads;
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid & (WAVE - 1);
   const int col = lane & 15, hi = lane >> 4;
-  const int kc_n = a.dk / 32, vb_n = a.dv / 16;
   extern __shared__ unsigned short smem[];
   unsigned short* v_tile = smem + wave * (KVT * VROW + 16 * (KVT + 8));
   unsigned short* p_lds = v_tile + KVT * VROW;
@@ -314,8 +312,8 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
   const size_t q_at = ((size_t)tok * a.heads + kvh * group + col) * a.dk;
 #pragma unroll
   for (int kc = 0; kc < RC; ++kc)
-    q_frag[kc] = col < group && kc < kc_n ? *reinterpret_cast<const bf16x8*>(q + q_at + kc * 32 + hi * 8)
-                                          : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+    q_frag[kc] = col < group && kc * 32 < a.dk ? *reinterpret_cast<const bf16x8*>(q + q_at + kc * 32 + hi * 8)
+                                               : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
   f32x4 acc_o[VB];
   SoftmaxRows w;
 #pragma unroll
@@ -329,7 +327,7 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
     w.lo[r] = a.window > 0 ? pos - a.window + 1 : 0;
     w.slope[r] = row < group && a.slopes ? a.slopes[kvh * group + row] * LOG2E : 0.f;
   }
-  const int v8 = a.dv / 8, width = a.kv_heads * (a.dk + a.dv);
+  const int width = a.kv_heads * (a.dk + a.dv);
   const float scale_l2 = a.scale * LOG2E;
   for (int j0 = j_begin + wave * KVT; j0 < j_end; j0 += 4 * KVT) {
     const long at = cache_row(b, seq, j0);
@@ -340,15 +338,15 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
       for (int kc = 0; kc < RC; ++kc) {
         const int row = nb * 16 + col;
         kt[nb][kc] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
-        if (kc < kc_n && at >= 0 && j0 + row < j_end)
+        if (kc * 32 < a.dk && at >= 0 && j0 + row < j_end)
           kt[nb][kc] = *reinterpret_cast<const bf16x8*>(
               cache + ((size_t)at + row) * width + kvh * a.dk + kc * 32 + hi * 8);
       }
 #pragma unroll
     for (int i = 0; i < NLD; ++i) {
-      const int idx = lane + i * WAVE, row = idx / v8, c8 = (idx - row * v8) * 8;
+      const int idx = lane + i * WAVE, row = idx / V8, c8 = idx % V8 * 8;
       vals[i] = bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
-      if (row < KVT && at >= 0 && j0 + row < j_end)
+      if (at >= 0 && j0 + row < j_end && c8 < a.dv)
         vals[i] = *reinterpret_cast<const bf16x8*>(
             cache + ((size_t)at + row) * width + a.kv_heads * a.dk + kvh * a.dv + c8);
     }
@@ -358,15 +356,15 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
       s_acc[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int kc = 0; kc < RC; ++kc)
-        if (kc < kc_n) s_acc[nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q_frag[kc], kt[nb][kc], s_acc[nb], 0, 0, 0);
+        s_acc[nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q_frag[kc], kt[nb][kc], s_acc[nb], 0, 0, 0);
     }
     float corr[4], p[2][4];
     softmax_tile(w, s_acc, j0, col, j_end, false, scale_l2, corr, p);
     wave_lds_fence();  // the last tile's reads are done
 #pragma unroll
     for (int i = 0; i < NLD; ++i) {
-      const int idx = lane + i * WAVE, row = idx / v8, c8 = (idx - row * v8) * 8;
-      if (row < KVT) *reinterpret_cast<bf16x8*>(&v_tile[row * VROW + c8]) = vals[i];
+      const int idx = lane + i * WAVE, row = idx / V8, c8 = idx % V8 * 8;
+      *reinterpret_cast<bf16x8*>(&v_tile[row * VROW + c8]) = vals[i];
     }
 #pragma unroll
     for (int r = 0; r < 4; ++r)
@@ -377,7 +375,6 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
     const unsigned short* v_lds = v_tile + (hi * 8 + col / 4) * VROW + (col & 3) * 4;
 #pragma unroll
     for (int d = 0; d < VB; ++d) {
-      if (d >= vb_n) break;
 #pragma unroll
       for (int r = 0; r < 4; ++r) acc_o[d][r] *= corr[r];
       acc_o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p_frag, load_keys(v_lds + d * 16, VROW), acc_o[d], 0, 0, 0);
@@ -400,7 +397,7 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
     }
 #pragma unroll
     for (int d = 0; d < VB; ++d)
-      if (d < vb_n) os[(wave * group + row) * a.dv + d * 16 + col] = acc_o[d][r];
+      if (d * 16 < a.dv) os[(wave * group + row) * a.dv + d * 16 + col] = acc_o[d][r];
   }
   __syncthreads();
   for (int i = tid; i < group * a.dv; i += 256) {
@@ -535,6 +532,7 @@ struct MixValues {
   float* first;         // a row's first-layer values: first[t * stride + kvh * vdim + c], or null
   long stride;
   int vdim;             // unpadded
+  bool aligned;         // groups of 8 of `first` may be moved at once
 };
 
 // y [T, >= H*dk + G*(dk+dv)]: queries, keys, values. 8 columns per thread; a
@@ -548,9 +546,11 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
   if (c0 >= nq + nk + nv) return;
   const size_t t = blockIdx.y;
   const int pos = b.pos[t];
-  float v[8];
+  float v[8], w[8];
+  load8(y + t * y_stride + c0, v);
+  load8(bias + c0, w);
 #pragma unroll
-  for (int e = 0; e < 8; ++e) v[e] = load_f32(y + t * y_stride + c0 + e) + bias[c0 + e];
+  for (int e = 0; e < 8; ++e) v[e] += w[e];
   TC* dst;
   if (c0 < nq) {
     if (temp_coef != 0.f) {
@@ -566,18 +566,27 @@ __global__ __launch_bounds__(256) void attn_prepare_kernel(
       const int kvh = c / a.dv, d0 = c - kvh * a.dv;
       float* own = mix.first + t * mix.stride + kvh * mix.vdim + d0;
       const float lam = mix.lambda ? *mix.lambda : 0.f;
+      if (mix.aligned && d0 + 8 <= mix.vdim) {
+        if (mix.lambda) {
+          load8(own, w);
 #pragma unroll
-      for (int e = 0; e < 8; ++e)
-        if (d0 + e < mix.vdim) {
-          if (mix.lambda) v[e] = (1.f - lam) * v[e] + lam * own[e];
-          else own[e] = v[e];
+          for (int e = 0; e < 8; ++e) v[e] = (1.f - lam) * v[e] + lam * w[e];
+        } else {
+          store8(own, v);
         }
+      } else {
+#pragma unroll
+        for (int e = 0; e < 8; ++e)
+          if (d0 + e < mix.vdim) {
+            if (mix.lambda) v[e] = (1.f - lam) * v[e] + lam * own[e];
+            else own[e] = v[e];
+          }
+      }
     }
     if (row < 0) return;
     dst = cache + (size_t)row * (nk + nv) + (c0 - nq);
   }
-#pragma unroll
-  for (int e = 0; e < 8; ++e) store_f32(dst + e, v[e]);
+  store8(dst, v);
 }
 
 // ------------------------------------------------------------------- host
@@ -690,11 +699,13 @@ torch::Tensor paged_attention(
 #define PA(RC, VB) launch_attn<RC, VB>(decode, grid, q, cache, g, po, pml, tiles.data_ptr<int>(), b, a, n_splits)
 #define PAV(RC)            \
   do {                     \
-    if (dv <= 64) PA(RC, 4); \
+    if (dv <= 32) PA(RC, 2); \
+    else if (dv <= 64) PA(RC, 4); \
     else if (dv <= 128) PA(RC, 8); \
     else PA(RC, 16);       \
   } while (0)
-  if (dk <= 64) PAV(2);
+  if (dk <= 32) PAV(1);
+  else if (dk <= 64) PAV(2);
   else if (dk <= 128) PAV(4);
   else PAV(8);
 #undef PAV
@@ -722,14 +733,16 @@ torch::Tensor attn_prepare(
   const PagedRows b = paged_rows(pos, owner, tables, cache, t);
   const AttnShape a = attn_shape(heads, kv_heads, dk, dv, cache);
   const long cols = heads * dk + kv_heads * (dk + dv);
-  TORCH_CHECK(y.size(1) >= cols, "projection too narrow");
+  TORCH_CHECK(y.size(1) >= cols && y.size(1) % 8 == 0, "projection too narrow");
+  for (const auto& p : {y, bias, cache}) TORCH_CHECK(reinterpret_cast<uintptr_t>(p.data_ptr()) % 16 == 0);
   TORCH_CHECK(bias.is_cuda() && bias.dtype() == torch::kFloat32 && bias.is_contiguous() && bias.numel() >= cols);
-  MixValues mix{nullptr, nullptr, 0, (int)vdim};
+  MixValues mix{nullptr, nullptr, 0, (int)vdim, false};
   if (first.has_value()) {
     TORCH_CHECK(first->is_cuda() && first->dtype() == torch::kFloat32 && first->dim() == 2 && first->stride(1) == 1);
     TORCH_CHECK(first->size(0) == t && first->size(1) >= kv_heads * vdim && vdim <= dv);
     mix.first = first->data_ptr<float>();
     mix.stride = first->stride(0);
+    mix.aligned = vdim % 8 == 0 && mix.stride % 4 == 0 && reinterpret_cast<uintptr_t>(mix.first) % 16 == 0;
     if (lambda.has_value()) {
       TORCH_CHECK(lambda->is_cuda() && lambda->dtype() == torch::kFloat32 && lambda->numel() == 1);
       mix.lambda = lambda->data_ptr<float>();

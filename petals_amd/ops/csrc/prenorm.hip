@@ -13,18 +13,44 @@
 #include <torch/extension.h>
 #include <ATen/cuda/CUDAContext.h>
 
+__device__ __forceinline__ f32x4 load4(const float* p) { return *reinterpret_cast<const f32x4*>(p); }
+__device__ __forceinline__ f32x4 load4(const unsigned short* p) {
+  const v4s a = *reinterpret_cast<const v4s*>(p);
+  return f32x4{bf16_to_f32(a[0]), bf16_to_f32(a[1]), bf16_to_f32(a[2]), bf16_to_f32(a[3])};
+}
+__device__ __forceinline__ void store4(float* p, f32x4 v) { *reinterpret_cast<f32x4*>(p) = v; }
+__device__ __forceinline__ void store4(unsigned short* p, f32x4 v) {
+  *reinterpret_cast<v4s*>(p) = v4s{(short)f32_to_bf16(v[0]), (short)f32_to_bf16(v[1]), (short)f32_to_bf16(v[2]),
+                                   (short)f32_to_bf16(v[3])};
+}
+
 // One workgroup per token. y null: x is only read; h null: nothing is normed.
 template <typename TY, typename TH>
 __global__ __launch_bounds__(1024) void residual_norm_kernel(
     float* __restrict__ x, long x_stride, const TY* __restrict__ y, long y_stride, const float* __restrict__ bias,
-    const float* __restrict__ w, float eps, TH* __restrict__ h, int d, int dp) {
+    const float* __restrict__ w, float eps, TH* __restrict__ h, int d, int dp, bool by4) {
   extern __shared__ float row[];  // [d]
   __shared__ float red[16];
   const int tid = threadIdx.x, nt = blockDim.x;
   const size_t t = blockIdx.x;
   float* xr = x + t * x_stride;
   float ss = 0.f;
-  for (int c = tid; c < d; c += nt) {
+  if (by4) {
+    for (int c = tid * 4; c < d; c += nt * 4) {
+      f32x4 v = load4(xr + c);
+      if (y) {
+        const f32x4 u = load4(y + t * y_stride + c);
+        const f32x4 b = bias ? load4(bias + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] += u[e] + b[e];
+        store4(xr + c, v);
+      }
+      store4(row + c, v);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) ss = fmaf(v[e], v[e], ss);
+    }
+  }
+  for (int c = by4 ? d : tid; c < d; c += nt) {
     float v = xr[c];
     if (y) {
       v += load_f32(y + t * y_stride + c) + (bias ? bias[c] : 0.f);
@@ -40,7 +66,16 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
   ss = 0.f;
   for (int i = 0; i < nt / WAVE; ++i) ss += red[i];
   const float inv = 1.f / sqrtf(ss / d + eps);
-  for (int c = tid; c < dp; c += nt) store_f32(h + t * dp + c, c < d ? row[c] * inv * w[c] : 0.f);
+  if (by4) {
+    for (int c = tid * 4; c < d; c += nt * 4) {
+      f32x4 v = load4(row + c);
+      const f32x4 g = load4(w + c);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] *= inv * g[e];
+      store4(h + t * dp + c, v);
+    }
+  }
+  for (int c = by4 ? d + tid : tid; c < dp; c += nt) store_f32(h + t * dp + c, c < d ? row[c] * inv * w[c] : 0.f);
 }
 
 // 64 columns x 16 groups of splits per workgroup
@@ -108,11 +143,14 @@ torch::Tensor residual_norm(torch::Tensor x, c10::optional<torch::Tensor> y, c10
   const size_t lds = d * 4;
   TORCH_CHECK(lds <= 65536 - 64, "width ", d, " is not supported");
   const int threads = t < 512 ? 1024 : 256;
+  auto aligned = [](const void* p, int bytes) { return reinterpret_cast<uintptr_t>(p) % bytes == 0; };
+  const bool by4 = d % 4 == 0 && x.stride(0) % 4 == 0 && ys % 4 == 0 && aligned(x.data_ptr(), 16) &&
+                   aligned(yp, yf ? 16 : 8) && aligned(bp, 16) && aligned(wp, 16);
   auto stream = at::cuda::getCurrentCUDAStream();
 #define RN(TY, TH)                                                                                          \
   residual_norm_kernel<TY, TH><<<t, threads, lds, stream>>>(                                                \
       x.data_ptr<float>(), x.stride(0), reinterpret_cast<const TY*>(yp), ys, bp, wp, (float)eps,            \
-      wp ? reinterpret_cast<TH*>(h.data_ptr()) : nullptr, (int)d, (int)dp)
+      wp ? reinterpret_cast<TH*>(h.data_ptr()) : nullptr, (int)d, (int)dp, by4)
   if (yf && out_f32) RN(float, float);
   else if (yf) RN(float, unsigned short);
   else if (out_f32) RN(unsigned short, float);

@@ -155,9 +155,11 @@ class HybridFastPath:
         self.w_g2 = self._zeros(m.heads * m.vdim, _up(g_rank, 8))
         self._place(block, "a2", self.w_a2[:, :a_rank])
         self._place(block, "g2", self.w_g2[:, :g_rank])
-        self.conv_w = torch.cat([getattr(block, f"{n}_conv").detach().float() for n in ("q", "k", "v")]).contiguous()
+        # [taps, channels]
+        conv_w = torch.cat([getattr(block, f"{n}_conv").detach().float() for n in ("q", "k", "v")])
+        self.conv_w = conv_w.t().contiguous()
         rows = [getattr(block, f"{n}_conv").shape[0] for n in ("q", "k", "v")]
-        self._views.update(zip(("q_conv", "k_conv", "v_conv"), self.conv_w.split(rows)))
+        self._views.update(zip(("q_conv", "k_conv", "v_conv"), self.conv_w.t().split(rows)))
         self.a_exp = self._f32(block, "A_log").exp()
         self.dt_bias, self.o_norm = self._f32(block, "dt_bias"), self._f32(block, "o_norm")
         self.wide = _up(m.heads * m.vdim, 8)

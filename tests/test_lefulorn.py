@@ -671,9 +671,11 @@ def test_delta_kernels(heads, kv, dim, vdim, taps, dtype):
     torch.manual_seed(0)
     hip, dt = hybrid.hip(), getattr(torch, dtype)
     sizes = [kv * dim, kv * dim, heads * vdim, heads]
-    cols = [0, kv * dim + 3, 2 * kv * dim + 3, 2 * kv * dim + heads * vdim + 3]
+    gap = 8 if dim % 8 == 0 else 3  # aligned columns and others
+    cols = [0, kv * dim + gap, 2 * kv * dim + gap, 2 * kv * dim + heads * vdim + gap]
     rank, g_rank = 8, 16
-    at_a, at_g = cols[3] + heads, cols[3] + heads + rank
+    at_a = -(-(cols[3] + heads) // 8) * 8
+    at_g = at_a + rank
     width = at_g + g_rank
     lens = [37, 1, 16, 50]
     total, tail = [x + 5 for x in lens], 5
@@ -703,7 +705,7 @@ def test_delta_kernels(heads, kv, dim, vdim, taps, dtype):
         delta[s, :, dim:] = 0
         delta[s, :, :, vdim:] = 0
     conv = torch.full((7, taps, conv_w.shape[0]), 9.0, device="cuda")
-    cu = [t.cuda() for t in (conv_w, a_log.exp(), dt_bias, norm_w, a2, g2)]
+    cu = [t.cuda() for t in (conv_w.t().contiguous(), a_log.exp(), dt_bias, norm_w, a2, g2)]
     tol = 2e-4 if dtype == "float32" else 3e-2
 
     def batch_of(starts, counts):
@@ -722,7 +724,7 @@ def test_delta_kernels(heads, kv, dim, vdim, taps, dtype):
         gate = (y[:, at_g : at_g + g_rank].float() @ cu[5].float().T).contiguous()
         o = hip.delta_prefill(y, a, cu[0], cu[1], cu[2], b.tiles(16), b.chunk_bounds(16), b.pos, b.owner, b.slot, delta,
                               conv, heads, kv, dim, vdim, cols)
-        out = hip.delta_norm(o, gate, cu[3], heads, heads * vdim + 3, True, eps)
+        out = hip.delta_norm(o, gate, cu[3], heads, heads * vdim + 8, True, eps)
         assert (out[:, heads * vdim :] == 0).all()
         for i, (lo, hi) in zip(live, b.row_ranges()):
             assert rel(out[lo:hi, : heads * vdim], wants[i][starts[i] : starts[i] + hi - lo]) < tol
