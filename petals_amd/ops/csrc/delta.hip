@@ -89,8 +89,13 @@ __device__ __forceinline__ void conv_silu8(
 
 // log2 of the decay
 __device__ __forceinline__ float log_decay(float a, float dt_bias, float a_exp) {
-  const float x = a + dt_bias;
-  const float softplus = x > 20.f ? x : log1pf(expf(x));
+  // softplus(x) = max(x, 0) + log1p(u), u = exp(-|x|); log1p(u) = log(w) u / (w - 1)
+  // with w = 1 + u as it is rounded
+  const float x = a + dt_bias, u = expf(-fabsf(x));
+  float w = 1.f + u;
+  asm volatile("" : "+v"(w));  // or fast math would take w - 1 for u
+  const float d = w - 1.f;
+  const float softplus = fmaxf(x, 0.f) + (d > 0.f ? logf(w) * (u / d) : u);
   return -a_exp * softplus * LOG2E;
 }
 
@@ -461,29 +466,28 @@ struct LowRank {
   int a_rank, g_rank;  // multiples of 8, zero-padded
 };
 
-// sum_r w[r] x[r] by 4 neighbouring lanes, the same value in each
+// sum_r w[r] x[r] by 2 neighbouring lanes, the same value in both
 template <typename TY, typename TW>
-__device__ __forceinline__ float quad_dot(const TY* x, const TW* w, int rank, int part) {
+__device__ __forceinline__ float pair_dot(const TY* x, const TW* w, int rank, int part) {
   float s = 0.f;
-  for (int r = part * 8; r < rank; r += 32) {
+#pragma unroll 8
+  for (int r = part * 8; r < rank; r += 16) {
     float a[8], b[8];
     load8(w + r, a);
     load8(x + r, b);
 #pragma unroll
     for (int e = 0; e < 8; ++e) s = fmaf(a[e], b[e], s);
   }
-  s += __shfl_xor(s, 1, WAVE);
-  s += __shfl_xor(s, 2, WAVE);
-  return s;
+  return s + __shfl_xor(s, 1, WAVE);
 }
 
-// Grid: (tokens, heads), one token per sequence. 512 threads hold S, 4 columns
+// Grid: (tokens, heads); row t is sequence t's only one. 512 threads hold S, 4 columns
 // and NR rows each.
 template <typename TY, typename TW, int NR>
 __global__ __launch_bounds__(512) void delta_decode_kernel(
     ConvInput<TY> in, float* __restrict__ conv_out, const TW* __restrict__ a2, const TW* __restrict__ g2, LowRank lr,
     const float* __restrict__ a_exp, const float* __restrict__ dt_bias, const float* __restrict__ norm_w,
-    const int* __restrict__ pos, const int* __restrict__ owner, const int* __restrict__ slot_of,
+    const int* __restrict__ pos, const int* __restrict__ slot_of,
     float* __restrict__ state, TY* __restrict__ out, int out_stride, DeltaShape s, float eps) {
   extern __shared__ float sm[];
   float* sq = sm;            // [dk]
@@ -495,7 +499,7 @@ __global__ __launch_bounds__(512) void delta_decode_kernel(
   __shared__ float scal[3];
   const int tid = threadIdx.x, lane = tid & (WAVE - 1);
   const int row = blockIdx.x, h = blockIdx.y, group = s.heads / s.kv_heads, kvh = h / group;
-  const int p = pos[row], slot = min(max(slot_of[owner[row]], 0), s.slots - 1);
+  const int p = pos[row], slot = min(max(slot_of[row], 0), s.slots - 1);
   const TY* yr = in.y + (size_t)row * in.stride;
 
   // S is on its way while the vectors are made
@@ -510,6 +514,8 @@ __global__ __launch_bounds__(512) void delta_decode_kernel(
                                            : f32x4{0.f, 0.f, 0.f, 0.f};
   }
 
+  const int ring_row = p % s.taps;
+#pragma unroll 1
   for (int i = tid; i < 2 * s.dk + s.dv; i += 512) {
     const int part = i < s.dk ? 0 : i < 2 * s.dk ? 1 : 2;
     const int c = i - part * s.dk;
@@ -518,28 +524,39 @@ __global__ __launch_bounds__(512) void delta_decode_kernel(
       const int at = part < 2 ? kvh * s.dim + c : h * s.vdim + c;
       const int col = (part == 0 ? s.oq : part == 1 ? s.ok : s.ov) + at;
       const int ch = part * s.kv_heads * s.dim + at;
-      x = conv_silu(in, s, row, 0, p, slot, col, ch);
-      // row p % taps is read by no other workgroup
-      if (part == 2 || h % group == 0)
-        conv_out[((size_t)slot * s.taps + p % s.taps) * s.channels() + ch] = load_f32(yr + col);
+      const float own = load_f32(yr + col);
+      x = own * in.w[(s.taps - 1) * s.channels() + ch];
+      const float* w = in.w + (s.taps - 1) * s.channels() + ch;
+      const float* ring = in.state + (size_t)slot * s.taps * s.channels() + ch;
+      for (int a0 = 1; a0 < s.taps; a0 += 4) {  // 4 loads on their way at once
+        float v[4], wt[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const int ago = a0 + e < s.taps ? a0 + e : 0;
+          v[e] = ring[(ring_row >= ago ? ring_row - ago : ring_row - ago + s.taps) * s.channels()];
+          wt[e] = w[-ago * s.channels()];
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) x = a0 + e < s.taps && a0 + e <= p ? fmaf(wt[e], v[e], x) : x;
+      }
+      x /= 1.f + expf(-x);
+      // this row is read by no other workgroup, and not used above
+      if (part == 2 || h == kvh * group)
+        conv_out[((size_t)slot * s.taps + ring_row) * s.channels() + ch] = own;
     }
     (part == 0 ? sq : part == 1 ? sk : sv)[c] = x;
   }
-  for (int i = tid; i < (s.dk + s.dv) * 4; i += 512) {
-    const int c = i >> 2, part = i & 3;
-    if (c < s.dk) {
-      float g = 0.f;
-      if (c < s.dim) {
-        const int ca = h * s.dim + c;
-        g = exp2f(log_decay(quad_dot(yr + lr.a1, a2 + (size_t)ca * lr.a_rank, lr.a_rank, part), dt_bias[ca], a_exp[h]));
-      }
-      if (part == 0) sg[c] = g;
-    } else {
-      float g = 0.f;
-      if (c - s.dk < s.vdim)
-        g = 1.f / (1.f + expf(-quad_dot(yr + lr.g1, g2 + (size_t)(h * s.vdim + c - s.dk) * lr.g_rank, lr.g_rank, part)));
-      if (part == 0) gate[c - s.dk] = g;
-    }
+#pragma unroll 1
+  for (int i = tid; i < (s.dk + s.dv) * 2; i += 512) {
+    const int part = i & 1;
+    const bool decays = i < s.dk * 2;
+    const int c = (i >> 1) - (decays ? 0 : s.dk), n = decays ? s.dim : s.vdim, at = h * n + min(c, n - 1);
+    const int rank = decays ? lr.a_rank : lr.g_rank;
+    const float z = pair_dot(yr + (decays ? lr.a1 : lr.g1), (decays ? a2 : g2) + (size_t)at * rank, rank, part);
+    float g = 0.f;
+    if (decays) g = exp2f(log_decay(z, dt_bias[at], a_exp[h]));
+    else g = 1.f / (1.f + expf(-z));
+    if (part == 0) (decays ? sg : gate)[c] = c < n ? g : 0.f;
   }
   __syncthreads();
   if (tid < 2 * WAVE) {
@@ -750,8 +767,8 @@ bool delta_decodes(int64_t dim, int64_t vdim) {
 // One row per sequence; returns [T, width] in y's dtype, normed and gated.
 torch::Tensor delta_decode(
     torch::Tensor y, torch::Tensor conv_w, torch::Tensor a2, torch::Tensor g2, int64_t a1_col, int64_t g1_col,
-    torch::Tensor a_exp, torch::Tensor dt_bias, torch::Tensor norm_w, torch::Tensor pos, torch::Tensor owner,
-    torch::Tensor slot, torch::Tensor delta, torch::Tensor conv, int64_t heads, int64_t kv_heads, int64_t dim,
+    torch::Tensor a_exp, torch::Tensor dt_bias, torch::Tensor norm_w, torch::Tensor pos, torch::Tensor slot,
+    torch::Tensor delta, torch::Tensor conv, int64_t heads, int64_t kv_heads, int64_t dim,
     int64_t vdim, std::vector<int64_t> cols, int64_t width, double eps) {
   const DeltaShape s = delta_shape(y, heads, kv_heads, dim, vdim, cols, conv_w, delta, conv);
   const long t = y.size(0);
@@ -760,7 +777,7 @@ torch::Tensor delta_decode(
   check_f32(dt_bias, heads * dim, "decay bias");
   check_f32(norm_w, vdim, "delta norm");
   check_i32(pos, t, "positions");
-  check_i32(owner, t, "owners");
+  TORCH_CHECK(slot.numel() == t, "one row per sequence");
   check_i32(slot, t, "slots");
   const bool yf = y.dtype() == torch::kFloat32, wf = a2.dtype() == torch::kFloat32;
   for (const auto& w : {a2, g2})
@@ -781,7 +798,7 @@ torch::Tensor delta_decode(
   delta_decode_kernel<TY, TW, N><<<dim3(t, heads), 512, lds, stream>>>(                                            \
       ConvInput<TY>{YP, stride, conv_w.data_ptr<float>(), conv.data_ptr<float>()}, conv.data_ptr<float>(), A2, G2, \
       lr, a_exp.data_ptr<float>(), dt_bias.data_ptr<float>(), norm_w.data_ptr<float>(), pos.data_ptr<int>(),       \
-      owner.data_ptr<int>(), slot.data_ptr<int>(), delta.data_ptr<float>(), OP, (int)width, s, (float)eps)
+      slot.data_ptr<int>(), delta.data_ptr<float>(), OP, (int)width, s, (float)eps)
 #define DDN(TY, TW, YP, OP, A2, G2)                      \
   do {                                                   \
     if (nr == 4) DD(TY, TW, 4, YP, OP, A2, G2);          \

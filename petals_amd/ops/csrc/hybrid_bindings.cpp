@@ -32,8 +32,8 @@ torch::Tensor delta_norm(
 bool delta_decodes(int64_t dim, int64_t vdim);
 torch::Tensor delta_decode(
     torch::Tensor y, torch::Tensor conv_w, torch::Tensor a2, torch::Tensor g2, int64_t a1_col, int64_t g1_col,
-    torch::Tensor a_exp, torch::Tensor dt_bias, torch::Tensor norm_w, torch::Tensor pos, torch::Tensor owner,
-    torch::Tensor slot, torch::Tensor delta, torch::Tensor conv, int64_t heads, int64_t kv_heads, int64_t dim,
+    torch::Tensor a_exp, torch::Tensor dt_bias, torch::Tensor norm_w, torch::Tensor pos, torch::Tensor slot,
+    torch::Tensor delta, torch::Tensor conv, int64_t heads, int64_t kv_heads, int64_t dim,
     int64_t vdim, std::vector<int64_t> cols, int64_t width, double eps);
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {

@@ -228,7 +228,7 @@ class HybridFastPath:
         if batch.decode_only and self.captures:
             return h.delta_decode(
                 y, self.conv_w, self.w_a2, self.w_g2, self.at_a1, self.at_g1, self.a_exp, self.dt_bias, self.o_norm,
-                batch.pos, batch.owner, batch.slot, delta, conv, *sizes, self.wide, self.eps,
+                batch.pos, batch.slot, delta, conv, *sizes, self.wide, self.eps,
             )
         a, gate = (
             self._outer(y[:, at : at + w.shape[1]], w) for at, w in ((self.at_a1, self.w_a2), (self.at_g1, self.w_g2))

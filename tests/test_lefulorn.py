@@ -734,7 +734,7 @@ def test_delta_kernels(heads, kv, dim, vdim, taps, dtype):
     for step in range(tail):
         b = batch_of(starts, [1] * 4)
         y = torch.stack([t[s] for t, s in zip(ys, starts)]).cuda()
-        out = hip.delta_decode(y, cu[0], cu[4], cu[5], at_a, at_g, cu[1], cu[2], cu[3], b.pos, b.owner, b.slot, delta, conv,
+        out = hip.delta_decode(y, cu[0], cu[4], cu[5], at_a, at_g, cu[1], cu[2], cu[3], b.pos, b.slot, delta, conv,
                                heads, kv, dim, vdim, cols, heads * vdim, eps)
         for i in range(4):
             assert rel(out[i], wants[i][starts[i]]) < tol
