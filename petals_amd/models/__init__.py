@@ -37,6 +37,7 @@ def _ensure_families():
         import petals_amd.models.mixtral  # noqa: F401
         import petals_amd.models.tulezen  # noqa: F401
         import petals_amd.models.lefulorn  # noqa: F401
+        import petals_amd.models.soselix  # noqa: F401
 
         _loaded = True
 

@@ -264,16 +264,65 @@ def query_temperature(pos: torch.Tensor, coef: float, every: int) -> torch.Tenso
     return 1.0 + coef * torch.log1p(((pos + 1) // every).float())
 
 
-def biased_sink_attention(q, k, v, q_pos, k_pos, *, scale, window, sink, slopes, temperature) -> torch.Tensor:
+def biased_sink_attention(
+    q, k, v, q_pos, k_pos, *, scale, window, sink, slopes=None, temperature=None
+) -> torch.Tensor:
     """q [..., Sq, H, d], k/v [..., Sk, G, d]; a distance bias slope * (i - j) is taken
     off the scores, and the softmax's denominator holds exp(sink) per head. 32-bit."""
     group = q.shape[-2] // k.shape[-2]
     k, v = (t.float().repeat_interleave(group, dim=-2).transpose(-3, -2) for t in (k, v))
-    q = (q.float() * temperature[:, None, None]).transpose(-3, -2)
+    q = (q.float() if temperature is None else q.float() * temperature[:, None, None]).transpose(-3, -2)
     gap = (q_pos[:, None] - k_pos[None, :]).float()
-    score = (q @ k.transpose(-1, -2)) * scale - slopes[:, None, None] * gap
+    score = (q @ k.transpose(-1, -2).contiguous()) * scale
+    if slopes is not None:
+        score = score - slopes[:, None, None] * gap
     seen = (gap >= 0) & (gap < window) if window > 0 else gap >= 0
     score = score.masked_fill(~seen, float("-inf"))
     sink = sink.float()[:, None, None].expand(*score.shape[:-1], 1)
     p = torch.softmax(torch.cat([score, sink], dim=-1), dim=-1)[..., :-1]
     return (p @ v).transpose(-3, -2)
+
+
+# ------------------- rotated halves, gated linear attention, group norm, xIELU
+
+
+def rotate_halves(x: torch.Tensor, pos: torch.Tensor, dims: int, base: float) -> torch.Tensor:
+    """x [..., n] at positions pos (broadcast over x's leading axes): the pair
+    (i, i + dims/2) of the first `dims` values turns by pos * base^(-2i/dims)."""
+    if dims == 0:
+        return x
+    i = torch.arange(dims // 2, device=x.device, dtype=torch.float64)
+    angle = pos[..., None].double() * base ** (-2.0 * i / dims)
+    cos, sin = angle.cos().float(), angle.sin().float()
+    u, v, rest = x.split([dims // 2, dims // 2, x.shape[-1] - dims], dim=-1)
+    return torch.cat([u * cos - v * sin, v * cos + u * sin, rest], dim=-1)
+
+
+def forget_gate(z: torch.Tensor, lower: torch.Tensor):
+    """f = lower + (1 - lower) sigmoid(z); returns (1 - f, f), the first without cancellation."""
+    return (1.0 - lower) * torch.sigmoid(-z), lower + (1.0 - lower) * torch.sigmoid(z)
+
+
+def gated_linear_attention(q, k, v, g, state=None):
+    """q, k [B, S, H, dim], v [B, S, H, vdim], g [B, S, H, dim or 1]; 32-bit. Per token
+    S <- g S + k v^T;  o = S^T q. Returns (o [B, S, H, vdim], last state [B, H, dim, vdim])."""
+    if state is None:
+        state = torch.zeros(q.shape[0], q.shape[2], q.shape[3], v.shape[3], device=q.device)
+    out = []
+    for t in range(q.shape[1]):
+        state = g[:, t, :, :, None] * state + k[:, t, :, :, None] * v[:, t, :, None, :]
+        out.append(torch.einsum("bhk,bhkv->bhv", q[:, t], state))
+    return torch.stack(out, dim=1), state
+
+
+def group_rms_norm(x: torch.Tensor, weight: torch.Tensor, groups: int, eps: float) -> torch.Tensor:
+    """RMS norm of each of `groups` equal parts of the last axis, one weight per value."""
+    parts = x.unflatten(-1, (groups, -1))
+    return (parts * torch.rsqrt(parts.pow(2).mean(-1, keepdim=True) + eps)).flatten(-2) * weight
+
+
+def xielu(z: torch.Tensor, p: torch.Tensor, q: torch.Tensor) -> torch.Tensor:
+    """z > 0: softplus(p) z^2 + z/2;  z <= 0: (1/2 + softplus(q)) (exp(z) - 1 - z) + z/2."""
+    low = z.clamp(max=0.0)
+    negative = (0.5 + F.softplus(q)) * (torch.expm1(low) - low)
+    return torch.where(z > 0, F.softplus(p) * z * z, negative) + 0.5 * z
