@@ -205,7 +205,7 @@ def linear_f32(x, weight):
         from petals_amd.ops import _hip
 
         # in every library of the paged families: the one this process serves with
-        hip = _hip.first_loaded("latent", "hybrid")
+        hip = _hip.first_loaded("latent", "hybrid", "recurrent")
         rows = x.float().reshape(-1, 1, x.shape[-1]).contiguous()
         return hip.batched_linear(rows, weight.contiguous().unsqueeze(0), True).view(*x.shape[:-1], weight.shape[0])
     return (x.to(weight.dtype) @ weight.t()).float()

@@ -1,13 +1,15 @@
 """Build the HIP extensions IN-TREE (the .so files must travel with the source
 tree to GPU boxes): `python -m petals_amd.ops.build [name ...]`.
 
-Cross-compiles for gfx950 (no GPU needed at build time). Three libraries:
+Cross-compiles for gfx950 (no GPU needed at build time). Four libraries:
 
   core    the kernels of the llama / bloom / falcon / mixtral families
   latent  latent attention, output norms and routed experts (tulezen); it is
           all that a process serving such a model needs
   hybrid  windowed attention with a distance bias and a sink, gated delta rule,
           input norms (lefulorn); likewise
+  recurrent  gated linear attention, latent attention with a rotated key part,
+          input norms (soselix); likewise
 """
 
 from __future__ import annotations
@@ -33,6 +35,11 @@ EXTENSIONS = {
     "hybrid": (
         "_hip_hybrid.so", "petals_amd_hip_hybrid", os.path.join("_build", "hybrid"),
         ["hybrid_bindings.cpp", "paged_attn.hip", "delta.hip", "prenorm.hip", "sublayer.hip", "gemv.hip"],
+    ),
+    "recurrent": (
+        "_hip_recurrent.so", "petals_amd_hip_recurrent", os.path.join("_build", "recurrent"),
+        ["recurrent_bindings.cpp", "linear_attn.hip", "latent_attn.hip", "rotary_latent.hip", "prenorm.hip",
+         "sublayer.hip", "gemv.hip"],
     ),
 }
 

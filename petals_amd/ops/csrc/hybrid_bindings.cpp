@@ -7,11 +7,11 @@ torch::Tensor gemv_bf16(
     torch::Tensor wt, torch::Tensor x, torch::Tensor workspace,
     c10::optional<torch::Tensor> residual, int64_t epilogue, int64_t splits_override,
     c10::optional<torch::Tensor> bias);
-torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32);
+torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32, c10::optional<torch::Tensor> out);
 torch::Tensor residual_norm(
     torch::Tensor x, c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> bias,
-    c10::optional<torch::Tensor> w, int64_t d, double eps, bool out_f32);
-void residual_sum(torch::Tensor partials, c10::optional<torch::Tensor> bias, torch::Tensor x, int64_t d);
+    c10::optional<torch::Tensor> w, int64_t d, double eps, bool out_f32, double mult);
+void residual_sum(torch::Tensor partials, c10::optional<torch::Tensor> bias, torch::Tensor x, int64_t d, double mult);
 torch::Tensor bias_relu2(torch::Tensor y, torch::Tensor bias);
 torch::Tensor paged_attention(
     torch::Tensor q, torch::Tensor cache, torch::Tensor pos, torch::Tensor owner, torch::Tensor tables,
@@ -40,9 +40,13 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("gemv_bf16", &gemv_bf16, "split-K bf16 gemv with fused epilogue",
         py::arg("wt"), py::arg("x"), py::arg("workspace"), py::arg("residual"), py::arg("epilogue"),
         py::arg("splits") = 0, py::arg("bias") = py::none());
-  m.def("batched_linear", &batched_linear, "out[t,h,n] = sum_k a[t,h,k] w[h,n,k]");
-  m.def("residual_norm", &residual_norm, "x += y + bias; RMS norm of x");
-  m.def("residual_sum", &residual_sum, "x += split-K partial sums + bias");
+  m.def("batched_linear", &batched_linear, "out[t,h,n] = sum_k a[t,h,k] w[h,n,k]",
+        py::arg("a"), py::arg("w"), py::arg("out_f32"), py::arg("out") = py::none());
+  m.def("residual_norm", &residual_norm, "x += mult (y + bias); RMS norm of x",
+        py::arg("x"), py::arg("y"), py::arg("bias"), py::arg("w"), py::arg("d"), py::arg("eps"), py::arg("out_f32"),
+        py::arg("mult") = 1.0);
+  m.def("residual_sum", &residual_sum, "x += mult (split-K partial sums + bias)",
+        py::arg("partials"), py::arg("bias"), py::arg("x"), py::arg("d"), py::arg("mult") = 1.0);
   m.def("bias_relu2", &bias_relu2, "relu(y + bias)^2 in place");
   m.def("paged_attention", &paged_attention, "windowed attention with distance bias, sink and gate over paged keys and values",
         py::arg("q"), py::arg("cache"), py::arg("pos"), py::arg("owner"), py::arg("tables"), py::arg("tiles"),

@@ -8,8 +8,12 @@
 // rows of an mfma_f32_16x16x32_bf16 tile, so a staged latent tile serves every
 // head and every token of the run.
 //
+// A cached row may be longer than what is summed: its first VP values are keys
+// and values, the rest (a rotated part that all heads share) are keys only.
+//
 //   latent_attn_kernel     MFMA flash kernel, prompts and decoding, ragged
-//                          batches, sliding window, optional key split
+//                          batches, sliding window, optional key split; a sink in
+//                          the softmax and a factor per head on the result
 //   latent_attn_combine    merges key splits
 //   latent_attn_simple     any latent size, 32-bit or bf16 storage
 //   latent_write           RMS-normalises new latents into their pages
@@ -23,7 +27,26 @@
 #include <ATen/cuda/CUDAContext.h>
 
 #define LKVT 32   // keys per staged tile; tiles are aligned, so one lies in one page
-#define LPAD 16   // LDS row padding (elements): rows 8 banks apart
+#define LOG2E 1.4426950408889634f
+
+// LDS row padding (elements): 16, or 8 where two workgroups would not fit in a CU otherwise
+constexpr int lds_pad(int rc) { return rc > 16 ? 8 : 16; }
+
+// what is done to a row's weighted sum at the end
+struct LatentEnd {
+  const float* sink;    // [H] score of one more entry of the softmax, without a value; or null
+  const float* factor;  // [T, H] or null
+};
+
+// factor of sum_j exp2(s_j - m) v_j, given l = sum_j exp2(s_j - m)
+__device__ __forceinline__ float end_factor(const LatentEnd& e, size_t flat, int heads, float m, float l) {
+  float f = l > 0.f ? 1.f / l : 0.f;
+  if (e.sink) {
+    const float s = e.sink[flat % heads] * LOG2E, mx = fmaxf(m, s), w = exp2f(m - mx);
+    f = w / fmaf(l, w, exp2f(s - mx));
+  }
+  return e.factor ? f * e.factor[flat] : f;
+}
 
 // ------------------------------------------------------------ MFMA kernel
 
@@ -33,29 +56,31 @@
 // one is loaded while the current one is used. The same staged tile is the keys
 // (row-major fragments) and the values (transposing LDS loads).
 //
-// RC = latent size in 32-wide MFMA k-chunks (columns past RP read as zero).
-// Grid: (token runs, groups of 16*RG rows, key splits).
-template <int RC, int DG>
+// RC = row size in 32-wide MFMA k-chunks (columns past RP read as zero), VC = those
+// of them that are values. Grid: (token runs, groups of 16*RG rows, key splits).
+template <int RC, int VC, int DG>
 __global__ __launch_bounds__(256) void latent_attn_kernel(
     const unsigned short* __restrict__ q,      // [T, H, RP]
     const unsigned short* __restrict__ cache,  // [num_pages, PAGE, RP]
-    unsigned short* __restrict__ out,          // [T, H, RP] (n_splits == 1)
-    float* __restrict__ part_o,                // [n_splits, T*H, RP]
+    unsigned short* __restrict__ out,          // [T, H, VP] (n_splits == 1)
+    float* __restrict__ part_o,                // [n_splits, T*H, VP]
     float* __restrict__ part_ml,               // [n_splits, T*H, 2]
     const int* __restrict__ tiles,             // [n, 2] first token, token count
     PagedRows b,
     int total_tokens,
     int heads,
     int rp,
+    int vp,
     int window,
     float scale_log2e,
-    int n_splits) {
+    int n_splits,
+    LatentEnd end) {
   constexpr int R = RC * 32;
   constexpr int RG = 4 / DG;
-  constexpr int ROW = R + LPAD;                  // LDS row in elements
+  constexpr int ROW = R + lds_pad(RC);           // LDS row in elements
   constexpr int LOADS = LKVT * (R / 8);          // 16-byte loads per tile
   constexpr int NLD = (LOADS + 255) / 256;       // per thread
-  constexpr int DB = (R / 16 + DG - 1) / DG;     // 16-wide dim blocks per wave
+  constexpr int DB = (VC * 2 + DG - 1) / DG;     // 16-wide dim blocks per wave
   const int tok0 = tiles[2 * blockIdx.x];
   const int ntok = tiles[2 * blockIdx.x + 1];
   const int rows = ntok * heads;
@@ -200,7 +225,7 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
     const unsigned short* v_lds = k_lds + (hi * 8 + col / 4) * ROW + (col & 3) * 4;
 #pragma unroll
     for (int d = 0; d < DB; ++d) {
-      if (DG > 1 && d0 + d >= R / 16) break;  // uniform over the wave
+      if (VC * 2 % DG != 0 && d0 + d >= VC * 2) break;  // uniform over the wave
 #pragma unroll
       for (int r = 0; r < 4; ++r) acc_o[d][r] *= corr[r];
       acc_o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
@@ -219,18 +244,18 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
     if (row >= rows) continue;
     const size_t flat = (size_t)tok0 * heads + row;
     if (n_splits == 1) {
-      const float inv_l = l > 0.f ? 1.0f / l : 0.f;
+      const float f = end_factor(end, flat, heads, m_row[r], l);
 #pragma unroll
       for (int d = 0; d < DB; ++d) {
         const int c = (d0 + d) * 16 + col;
-        if (c < rp) out[flat * rp + c] = f32_to_bf16(acc_o[d][r] * inv_l);
+        if (c < vp) out[flat * vp + c] = f32_to_bf16(acc_o[d][r] * f);
       }
     } else {
       const size_t at = (size_t)blockIdx.z * total_tokens * heads + flat;
 #pragma unroll
       for (int d = 0; d < DB; ++d) {
         const int c = (d0 + d) * 16 + col;
-        if (c < rp) part_o[at * rp + c] = acc_o[d][r];
+        if (c < vp) part_o[at * vp + c] = acc_o[d][r];
       }
       if (col == 0 && wave % DG == 0) {
         part_ml[at * 2] = m_row[r];
@@ -243,7 +268,8 @@ __global__ __launch_bounds__(256) void latent_attn_kernel(
 // one workgroup per (token, head) row and 128 of its dims
 __global__ __launch_bounds__(128) void latent_attn_combine(
     const float* __restrict__ part_o, const float* __restrict__ part_ml,
-    unsigned short* __restrict__ out, int n_rows, int rp, int n_splits) {
+    unsigned short* __restrict__ out, int n_rows, int heads, int vp, int n_splits,
+    LatentEnd end) {
   __shared__ float share[WAVE];  // weight of each split in the row
   const int row = blockIdx.x;
   if (threadIdx.x < WAVE) {
@@ -255,21 +281,20 @@ __global__ __launch_bounds__(128) void latent_attn_combine(
     }
     const float mx = wave_reduce_max(m);
     const float w = m > NEG_THRESHOLD ? exp2f(m - mx) : 0.f;
-    const float sum = wave_reduce_sum(w * l);
-    share[s] = sum > 0.f ? w / sum : 0.f;
+    share[s] = w * end_factor(end, row, heads, mx, wave_reduce_sum(w * l));
   }
   __syncthreads();
   const int d = blockIdx.y * blockDim.x + threadIdx.x;
-  if (d < rp) {
-    const float* src = part_o + (size_t)row * rp + d;
-    const size_t step = (size_t)n_rows * rp;
+  if (d < vp) {
+    const float* src = part_o + (size_t)row * vp + d;
+    const size_t step = (size_t)n_rows * vp;
     float o[4] = {0.f, 0.f, 0.f, 0.f};
     int s = 0;
     for (; s + 4 <= n_splits; s += 4)
 #pragma unroll
       for (int u = 0; u < 4; ++u) o[u] = fmaf(src[(s + u) * step], share[s + u], o[u]);
     for (; s < n_splits; ++s) o[0] = fmaf(src[s * step], share[s], o[0]);
-    out[(size_t)row * rp + d] = f32_to_bf16((o[0] + o[1]) + (o[2] + o[3]));
+    out[(size_t)row * vp + d] = f32_to_bf16((o[0] + o[1]) + (o[2] + o[3]));
   }
 }
 
@@ -281,12 +306,12 @@ template <typename T>
 __global__ __launch_bounds__(256) void latent_attn_simple(
     const T* __restrict__ q,      // [T, H, RP]
     const T* __restrict__ cache,  // [num_pages, PAGE, RP]
-    T* __restrict__ out,          // [T, H, RP]
-    PagedRows b, int heads, int rp, int window, float scale) {
+    T* __restrict__ out,          // [T, H, VP]
+    PagedRows b, int heads, int rp, int vp, int window, float scale, LatentEnd end) {
   extern __shared__ float sm[];
   float* qs = sm;           // [rp]
-  float* acc = qs + rp;     // [rp]
-  float* p = acc + rp;      // [256]
+  float* acc = qs + rp;     // [vp, rounded up to even]
+  float* p = acc + (vp + 1) / 2 * 2;  // [256]
   long* at = reinterpret_cast<long*>(p + 256);  // [256]
   __shared__ float red[4];
   const int tid = threadIdx.x;
@@ -294,10 +319,8 @@ __global__ __launch_bounds__(256) void latent_attn_simple(
   const int seq = b.owner[tok];
   const int pos = b.pos[tok];
   const int lo = window > 0 ? max(0, pos - window + 1) : 0;
-  for (int d = tid; d < rp; d += 256) {
-    qs[d] = load_f32(q + (size_t)blockIdx.x * rp + d);
-    acc[d] = 0.f;
-  }
+  for (int d = tid; d < rp; d += 256) qs[d] = load_f32(q + (size_t)blockIdx.x * rp + d);
+  for (int d = tid; d < vp; d += 256) acc[d] = 0.f;
   float m = NEG_SENTINEL, l = 0.f;
   for (int j0 = lo; j0 <= pos; j0 += 256) {
     __syncthreads();
@@ -325,15 +348,15 @@ __global__ __launch_bounds__(256) void latent_attn_simple(
     l = l * corr + ((red[0] + red[1]) + (red[2] + red[3]));
     m = m_new;
     const int n = min(256, pos - j0 + 1);
-    for (int d = tid; d < rp; d += 256) {
+    for (int d = tid; d < vp; d += 256) {
       float o = acc[d] * corr;
       for (int j = 0; j < n; ++j)
         if (at[j] >= 0) o = fmaf(p[j], load_f32(cache + (size_t)at[j] * rp + d), o);
       acc[d] = o;
     }
   }
-  const float inv_l = l > 0.f ? 1.f / l : 0.f;
-  for (int d = tid; d < rp; d += 256) store_f32(out + (size_t)blockIdx.x * rp + d, acc[d] * inv_l);
+  const float f = end_factor(end, blockIdx.x, heads, m * LOG2E, l);
+  for (int d = tid; d < vp; d += 256) store_f32(out + (size_t)blockIdx.x * vp + d, acc[d] * f);
 }
 
 // ---------------------------------------------------------- latent writing
@@ -364,22 +387,22 @@ __global__ __launch_bounds__(256) void latent_write_kernel(
 
 // ------------------------------------------------------------------- host
 
-template <int RC, int DG>
+template <int RC, int VC, int DG>
 static void launch_mfma(dim3 grid, const torch::Tensor& q, const torch::Tensor& cache, torch::Tensor& out,
                         torch::Tensor& part_o, torch::Tensor& part_ml, const torch::Tensor& tiles, PagedRows b,
-                        int heads, int rp, int window, float scale, int n_splits) {
-  constexpr size_t lds = (2 * LKVT * (RC * 32 + LPAD) + 4 * 16 * (LKVT + 8)) * 2;
+                        int heads, int rp, int vp, int window, float scale, int n_splits, LatentEnd end) {
+  constexpr size_t lds = (2 * LKVT * (RC * 32 + lds_pad(RC)) + 4 * 16 * (LKVT + 8)) * 2;
   static bool allowed = false;
   if (lds > 65536 && !allowed) {
-    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<RC, DG>),
+    hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(&latent_attn_kernel<RC, VC, DG>),
                                        hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     TORCH_CHECK(e == hipSuccess, "LDS request refused: ", hipGetErrorString(e));
     allowed = true;
   }
-  latent_attn_kernel<RC, DG><<<grid, 256, lds, at::cuda::getCurrentCUDAStream()>>>(
+  latent_attn_kernel<RC, VC, DG><<<grid, 256, lds, at::cuda::getCurrentCUDAStream()>>>(
       BF16P(q), BF16P(cache), BF16P(out), part_o.numel() ? part_o.data_ptr<float>() : nullptr,
-      part_ml.numel() ? part_ml.data_ptr<float>() : nullptr, tiles.data_ptr<int>(), b, (int)q.size(0), heads, rp,
-      window, scale * 1.4426950408889634f, n_splits);
+      part_ml.numel() ? part_ml.data_ptr<float>() : nullptr, tiles.data_ptr<int>(), b, (int)q.size(0), heads, rp, vp,
+      window, scale * LOG2E, n_splits, end);
 }
 
 torch::Tensor latent_attention(
@@ -389,24 +412,38 @@ torch::Tensor latent_attention(
     torch::Tensor tiles,   // [n, 2] int32 runs of at most run_tokens tokens
     int64_t run_tokens,
     int64_t max_keys,      // most keys that any row sees
-    int64_t window, double scale, int64_t splits) {
+    int64_t window, double scale,
+    int64_t values,        // size of the result: the first values of a row, 0 for all of them
+    c10::optional<torch::Tensor> sink,    // [H] f32
+    c10::optional<torch::Tensor> factor,  // [T, H] f32
+    int64_t splits) {
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() && q.dtype() == cache.dtype());
-  const int t = q.size(0), heads = q.size(1), rp = q.size(2);
-  TORCH_CHECK(cache.size(2) == rp && rp % 32 == 0, "latent width mismatch");
+  const int t = q.size(0), heads = q.size(1), rp = q.size(2), vp = values > 0 ? (int)values : rp;
+  TORCH_CHECK(cache.size(2) == rp && rp % 32 == 0 && vp <= rp, "latent width mismatch");
   const PagedRows b = paged_rows(pos, owner, tables, cache, t);
-  auto out = torch::empty_like(q);
+  LatentEnd end{nullptr, nullptr};
+  auto f32_values = [](const c10::optional<torch::Tensor>& x, long n) -> const float* {
+    if (!x.has_value()) return nullptr;
+    TORCH_CHECK(x->is_cuda() && x->dtype() == torch::kFloat32 && x->is_contiguous() && x->numel() == n);
+    return x->data_ptr<float>();
+  };
+  end.sink = f32_values(sink, heads);
+  end.factor = f32_values(factor, (long)t * heads);
+  auto out = torch::empty({t, heads, vp}, q.options());
+  if (t == 0) return out;
   auto stream = at::cuda::getCurrentCUDAStream();
   const bool f32 = q.dtype() == torch::kFloat32;
   TORCH_CHECK(f32 || q.dtype() == torch::kBFloat16);
-  if (f32 || rp > 512) {
-    const size_t lds = (2 * (size_t)rp + 256) * 4 + 256 * 8;
+  if (f32 || rp > 18 * 32 || vp > 16 * 32) {
+    const size_t lds = ((size_t)rp + (vp + 1) / 2 * 2 + 256) * 4 + 256 * 8;
     TORCH_CHECK(lds <= 65536, "latent size ", rp, " is not supported");
     if (f32)
       latent_attn_simple<float><<<t * heads, 256, lds, stream>>>(
-          q.data_ptr<float>(), cache.data_ptr<float>(), out.data_ptr<float>(), b, heads, rp, (int)window, (float)scale);
+          q.data_ptr<float>(), cache.data_ptr<float>(), out.data_ptr<float>(), b, heads, rp, vp, (int)window,
+          (float)scale, end);
     else
       latent_attn_simple<unsigned short><<<t * heads, 256, lds, stream>>>(
-          BF16P(q), BF16P(cache), BF16P(out), b, heads, rp, (int)window, (float)scale);
+          BF16P(q), BF16P(cache), BF16P(out), b, heads, rp, vp, (int)window, (float)scale, end);
     HIP_CHECK_LAST();
     return out;
   }
@@ -423,31 +460,38 @@ torch::Tensor latent_attention(
   }
   grid.z = n_splits;
   auto f32o = q.options().dtype(torch::kFloat32);
-  auto part_o = torch::empty({n_splits > 1 ? (long)n_splits * t * heads * rp : 0}, f32o);
+  auto part_o = torch::empty({n_splits > 1 ? (long)n_splits * t * heads * vp : 0}, f32o);
   auto part_ml = torch::empty({n_splits > 1 ? (long)n_splits * t * heads * 2 : 0}, f32o);
-#define LA2(RC, DG) \
-  launch_mfma<RC, DG>(grid, q, cache, out, part_o, part_ml, tiles, b, heads, rp, (int)window, (float)scale, n_splits)
-#define LA(RC)                    \
-  do {                            \
-    if (rg == 1) LA2(RC, 4);      \
-    else if (rg == 2) LA2(RC, 2); \
-    else LA2(RC, 1);              \
+#define LA2(RC, VC, DG)                                                                                              \
+  launch_mfma<RC, VC, DG>(grid, q, cache, out, part_o, part_ml, tiles, b, heads, rp, vp, (int)window, (float)scale, \
+                          n_splits, end)
+#define LA(RC, VC)                    \
+  do {                                \
+    if (rg == 1) LA2(RC, VC, 4);      \
+    else if (rg == 2) LA2(RC, VC, 2); \
+    else LA2(RC, VC, 1);              \
   } while (0)
-  const int rc = rp / 32;
-  if (rc <= 1) LA(1);
-  else if (rc <= 2) LA(2);
-  else if (rc <= 3) LA(3);
-  else if (rc <= 4) LA(4);
-  else if (rc <= 6) LA(6);
-  else if (rc <= 8) LA(8);
-  else if (rc <= 12) LA(12);
-  else LA(16);
+  const int rc = rp / 32, vc = (vp + 31) / 32;
+  if (rc <= 1) LA(1, 1);
+  else if (rc <= 2 && vc <= 1) LA(2, 1);
+  else if (rc <= 2) LA(2, 2);
+  else if (rc <= 3 && vc <= 2) LA(3, 2);
+  else if (rc <= 3) LA(3, 3);
+  else if (rc <= 4) LA(4, 4);
+  else if (rc <= 5 && vc <= 4) LA(5, 4);
+  else if (rc <= 6) LA(6, 6);
+  else if (rc <= 8) LA(8, 8);
+  else if (rc <= 10 && vc <= 8) LA(10, 8);
+  else if (rc <= 12) LA(12, 12);
+  else if (rc <= 14 && vc <= 12) LA(14, 12);
+  else if (rc <= 16) LA(16, 16);
+  else LA(18, 16);
 #undef LA
 #undef LA2
   HIP_CHECK_LAST();
   if (n_splits > 1) {
-    latent_attn_combine<<<dim3(t * heads, (rp + 127) / 128), 128, 0, stream>>>(
-        part_o.data_ptr<float>(), part_ml.data_ptr<float>(), BF16P(out), t * heads, rp, n_splits);
+    latent_attn_combine<<<dim3(t * heads, (vp + 127) / 128), 128, 0, stream>>>(
+        part_o.data_ptr<float>(), part_ml.data_ptr<float>(), BF16P(out), t * heads, heads, vp, n_splits, end);
     HIP_CHECK_LAST();
   }
   return out;

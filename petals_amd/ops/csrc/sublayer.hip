@@ -475,16 +475,20 @@ std::vector<torch::Tensor> sublayer_out(
 }
 
 // a: [T, H, K] view (any row and head stride, unit k stride); w: [H, N, K]
-torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32) {
+// into: where the result goes, a view [t, h, n] with unit stride in n (default: a new tensor)
+torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32, c10::optional<torch::Tensor> into) {
   const bool af = is_f32(a), wf = is_f32(w);
   TORCH_CHECK(a.dim() == 3 && w.dim() == 3 && w.is_contiguous() && a.stride(2) == 1);
   const long t = a.size(0), h = a.size(1), k = a.size(2), n = w.size(1);
   TORCH_CHECK(w.size(0) == h && w.size(2) == k, "batched_linear shapes");
   TORCH_CHECK(!wf || (af && out_f32), "32-bit weights need 32-bit rows");
-  auto out = torch::empty({t, h, n}, a.options().dtype(out_f32 ? torch::kFloat32 : torch::kBFloat16));
+  auto out = into.has_value() ? *into
+                              : torch::empty({t, h, n}, a.options().dtype(out_f32 ? torch::kFloat32 : torch::kBFloat16));
+  TORCH_CHECK(out.is_cuda() && out.dtype() == (out_f32 ? torch::kFloat32 : torch::kBFloat16) && out.dim() == 3 &&
+              out.size(0) == t && out.size(1) == h && out.size(2) == n && out.stride(2) == 1, "batched_linear result");
   if (t == 0) return out;
   auto stream = at::cuda::getCurrentCUDAStream();
-  const long at_ = a.stride(0), ah = a.stride(1), ot = h * n, oh = n;
+  const long at_ = a.stride(0), ah = a.stride(1), ot = out.stride(0), oh = out.stride(1);
   if (wf) {
     TORCH_CHECK(t <= 65535 && h <= 65535);
     batched_linear_f32_kernel<<<dim3((n + 3) / 4, t, h), 256, 0, stream>>>(
@@ -495,7 +499,8 @@ torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32) {
   const size_t ab = af ? 4 : 2;
   const bool a_wide = (reinterpret_cast<uintptr_t>(a.data_ptr()) % 16 == 0) && (at_ * ab) % 16 == 0 && (ah * ab) % 16 == 0;
   const bool w_wide = k % 8 == 0;
-  const bool o_wide = (n * (out_f32 ? 4 : 2)) % 16 == 0;
+  const long ob = out_f32 ? 4 : 2;
+  const bool o_wide = ot * ob % 16 == 0 && oh * ob % 16 == 0 && reinterpret_cast<uintptr_t>(out.data_ptr()) % 16 == 0;
   const int n_tiles = (n + 63) / 64;
   const long jobs = n_tiles * ((t + 63) / 64);
 #define BL(TA, TO, AP, OP)                                                               \

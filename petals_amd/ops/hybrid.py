@@ -6,16 +6,8 @@ of their own (ops/build.py "hybrid").
 
 Everything that reads the normed input is one product: queries, keys, values and
 gate of attention; queries, keys, values, beta and the inner low-rank projections
-of the delta rule. Weights are padded once, at load, to the tile sizes of the
-kernels with zeros that contribute nothing; any size works, and none is assumed.
-
-A batch takes one of two routes, whatever mix of requests it holds:
-  few rows   split-K GEMVs with 32-bit activations; no library product and no host
-             synchronisation, so the engine captures single-token batches in a
-             hipGraph
-  many rows  hipBLASLt products
-In float32 every product is a true 32-bit one. The delta rule has a kernel for
-batches of single tokens and a chunked one for all others.
+of the delta rule. The delta rule has a kernel for batches of single tokens and a
+chunked one for all others. Packing and routes: ops/packed.py.
 """
 
 from __future__ import annotations
@@ -24,12 +16,10 @@ import torch
 
 from petals_amd.models.lefulorn.config import KEY_PAD, VALUE_PAD
 from petals_amd.ops import reference
-from petals_amd.ops.fused_decode import _EPI_PLAIN_F32
+from petals_amd.ops.packed import CHUNK, PackedBlock, rms_norm_rows
+from petals_amd.ops.packed import round_up as _up
 
 _EPI_RELU2_F32 = 6
-_EPI_RAW = -1  # the split-K partial sums
-_GEMV_ROWS = 8  # most rows of the GEMV
-_CHUNK = 16  # tokens of a chunk of the delta rule
 
 
 def hip():
@@ -39,30 +29,17 @@ def hip():
     return _hip.first_loaded("hybrid")
 
 
-def _up(n: int, to: int) -> int:
-    return -(-n // to) * to
-
-
 def rms_norm_f32(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
-    d = x.shape[-1]
-    rows = x.float().reshape(-1, d).contiguous()
-    return hip().residual_norm(rows, None, None, weight.float().contiguous(), d, eps, True)[:, :d].reshape(x.shape)
+    from petals_amd.ops import _hip
+
+    # in every library of pre-norm blocks: the one this process serves with
+    return rms_norm_rows(_hip.first_loaded("hybrid", "recurrent"), x, weight, eps)
 
 
-class HybridFastPath:
-    quant = "none"
-
+class HybridFastPath(PackedBlock):
     def __init__(self, block):
-        self.hip = hip()
-        self.spec, self.mlp, self.eps, self.mix = block.mixer, block.mlp, block.eps, block.mix
-        dtype, dev = block.q.dtype, block.q.device
-        if dtype not in (torch.bfloat16, torch.float32):
-            raise ValueError(f"these blocks are served in bfloat16 or float32, not {dtype}")
-        self.dtype, self.f32, self.device = dtype, dtype == torch.float32, dev
-        self.d = block.config.hidden_size
-        self.dp = _up(self.d, 8)
-        self.carried = block.config.carried_values
-        self._views = {}  # checkpoint-shaped views of packed weights
+        super().__init__(block, hip())
+        self.mix, self.carried = block.mix, block.config.carried_values
         self.norm1 = self._f32(block, "norm1")
         if block.delta:
             self._pack_delta(block)
@@ -70,57 +47,9 @@ class HybridFastPath:
             self._pack_attention(block)
         if self.mlp is not None:
             self.norm2 = self._f32(block, "norm2")
-            ffp = _up(self.mlp.ff, 8)
-            self.w_up, self.w_down = self._zeros(self.dp, ffp), self._zeros(ffp, self.dp)
-            self._place(block, "up", self.w_up[: self.d, : self.mlp.ff].t())
-            self._place(block, "down", self.w_down[: self.mlp.ff, : self.d].t())
-            self.b_up = torch.zeros(ffp, device=dev)
-            self._place(block, "up_bias", self.b_up[: self.mlp.ff])
-            self.b_down = self._f32(block, "down_bias")
+        self._finish(block)
+        if self.mlp is not None:
             self.b_up_gemv = self.b_up.to(torch.bfloat16)
-        self.max_gemv_rows = _GEMV_ROWS
-        # batches that the engine may capture: only kernels of this library run
-        self.max_graph_rows = 0 if self.f32 or not self.captures else self.max_gemv_rows
-        self.graph_safe = self.max_graph_rows > 0
-        self._no_ws = torch.empty(0, dtype=torch.float32, device=dev)
-        empty = torch.empty(0, dtype=dtype, device=dev)
-        for p in block.parameters():
-            p.data = empty
-
-    # ---------------------------------------------------------------- weights
-
-    def _zeros(self, *shape):
-        return torch.zeros(*shape, dtype=self.dtype, device=self.device)
-
-    def _f32(self, block, name):
-        t = getattr(block, name).detach().float().contiguous()
-        self._views[name] = t
-        return t
-
-    def _place(self, block, name, view):
-        """Copy a parameter into its place in a packed weight."""
-        view.copy_(getattr(block, name).detach().view(view.shape))
-        self._views[name] = view
-
-    def weight(self, name: str) -> torch.Tensor:
-        """A checkpoint-shaped weight (stateless forward, backward)."""
-        view = self._views[name]
-        if view.dim() == 3:  # padded heads
-            view = view.reshape(-1, view.shape[-1]) if name != "o" else view.reshape(view.shape[0], -1)
-        return view
-
-    def _columns(self, block, parts):
-        """w_in [dp, n]: the named weights [out, d] side by side; parts: (name, heads,
-        size, padded size). Returns each part's first column."""
-        starts, n = [], 0
-        for _, heads, _, padded in parts:
-            starts.append(n)
-            n += _up(heads * padded, 8)
-        self.w_in = self._zeros(self.dp, n)
-        for at, (name, heads, size, padded) in zip(starts, parts):
-            heads_view = self.w_in[: self.d, at : at + heads * padded].unflatten(1, (heads, padded))[:, :, :size]
-            self._place(block, name, heads_view.permute(1, 2, 0))
-        return starts
 
     def _pack_attention(self, block):
         a = self.spec
@@ -169,23 +98,6 @@ class HybridFastPath:
 
     # ---------------------------------------------------------------- forward
 
-    def _splits(self, w: torch.Tensor) -> int:
-        # 64 input rows a wave keeps the loads of a short gemv in flight
-        return max(1, min(w.shape[0] // 64, 1024 // (-(-w.shape[1] // 512))))
-
-    def _dense(self, x, w, few: bool, epilogue: int = _EPI_PLAIN_F32, bias=None):
-        """x [T, in] (32-bit if few rows or float32, else the weight dtype) @ w [in, out]."""
-        if few:
-            return self.hip.gemv_bf16(w, x, self._no_ws, None, epilogue, self._splits(w), bias)
-        return x @ w
-
-    def _add(self, x, y, w, few: bool, bias=None):
-        """x += y @ w (+ bias), for the last product before x is read again."""
-        if few:
-            self.hip.residual_sum(self._dense(y, w, True, _EPI_RAW), bias, x, self.d)
-        else:
-            self.hip.residual_norm(x, y @ w, bias, None, self.d, self.eps, True)
-
     def forward_paged(self, x: torch.Tensor, batch, cache=None, state=None) -> torch.Tensor:
         """x [T, stream width] 32-bit, updated in place."""
         h = self.hip
@@ -196,12 +108,10 @@ class HybridFastPath:
         if self.mlp is None:
             self._add(x, y, self.w_o, few)
             return x
+        n = self._add_and_norm(x, y, self.w_o, few, self.norm2)
         if few:
-            self._add(x, y, self.w_o, few)
-            n = h.residual_norm(x, None, None, self.norm2, self.d, self.eps, wide)
             act = self._dense(n, self.w_up, few, _EPI_RELU2_F32, self.b_up_gemv)
         else:
-            n = h.residual_norm(x, y @ self.w_o, None, self.norm2, self.d, self.eps, wide)
             act = h.bias_relu2(n @ self.w_up, self.b_up)
         self._add(x, act, self.w_down, few, self.b_down)
         return x
@@ -234,7 +144,7 @@ class HybridFastPath:
             self._outer(y[:, at : at + w.shape[1]], w) for at, w in ((self.at_a1, self.w_a2), (self.at_g1, self.w_g2))
         )
         o = h.delta_prefill(
-            y, a, self.conv_w, self.a_exp, self.dt_bias, batch.tiles(_CHUNK), batch.chunk_bounds(_CHUNK), batch.pos,
+            y, a, self.conv_w, self.a_exp, self.dt_bias, batch.tiles(CHUNK), batch.chunk_bounds(CHUNK), batch.pos,
             batch.owner, batch.slot, delta, conv, *sizes,
         )
         return h.delta_norm(o, gate, self.o_norm, m.heads, self.wide, wide, self.eps)
