@@ -113,7 +113,8 @@ def _parse_layer(index: int, entry: Dict[str, Any]) -> LayerSpec:
         mixer = Hgrn2Spec(**_sizes(index, m, heads="heads", dim="dim", vdim="vdim"))
     elif kind == "mamba2":
         mixer = Mamba2Spec(**_sizes(
-            index, m, heads="heads", vdim="vdim", state="state", groups="groups", taps="conv", norm_groups="norm_groups"
+            index, {"groups": 1, "norm_groups": 1, **m}, heads="heads", vdim="vdim", state="state", groups="groups",
+            taps="conv", norm_groups="norm_groups",
         ))
         if mixer.heads % mixer.groups or mixer.inner % mixer.norm_groups:
             raise ValueError(

@@ -8,9 +8,25 @@ single captured graph replays for every token of a session.
 
 from __future__ import annotations
 
+import contextlib
+import gc
 from typing import Callable, Sequence
 
 import torch
+
+
+@contextlib.contextmanager
+def no_garbage_collection():
+    """While a graph is captured nothing may be collected: the destructor of an
+    older graph in a reference cycle synchronizes the device, which a capture does
+    not allow, and an error in a destructor ends the process."""
+    enabled = gc.isenabled()
+    gc.disable()
+    try:
+        yield
+    finally:
+        if enabled:
+            gc.enable()
 
 
 class GraphedCallable:
@@ -29,7 +45,7 @@ class GraphedCallable:
         torch.cuda.current_stream().wait_stream(stream)
 
         self.graph = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(self.graph):
+        with no_garbage_collection(), torch.cuda.graph(self.graph):
             out = fn(*self.static_inputs)
         self.static_outputs = out if isinstance(out, (tuple, list)) else (out,)
         self._single = not isinstance(out, (tuple, list))

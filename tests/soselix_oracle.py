@@ -47,18 +47,16 @@ def softplus(x):
 def rotate(x, positions, dims, base, faults=NONE):
     """x [S, ..., n]: pairs (i, i + dims/2) of the first `dims` turned by position * base^(-2i/dims)."""
     half = dims // 2
-    out = x.clone()
     if "no_rotation" in faults:
-        return out
+        return x
+    out = list(x.unbind(-1))
     for i in range(half):
-        j = i + half
-        if "rotate_neighbours" in faults:
-            i, j = 2 * i, 2 * i + 1
-        angle = positions.to(F64) * base ** (-2.0 * (i if j == i + half else i // 2) / dims)
+        angle = positions.to(F64) * base ** (-2.0 * i / dims)
         angle = angle.view(-1, *[1] * (x.dim() - 2))
-        out[..., i] = x[..., i] * torch.cos(angle) - x[..., j] * torch.sin(angle)
-        out[..., j] = x[..., j] * torch.cos(angle) + x[..., i] * torch.sin(angle)
-    return out
+        i, j = (2 * i, 2 * i + 1) if "rotate_neighbours" in faults else (i, i + half)
+        out[i] = x[..., i] * torch.cos(angle) - x[..., j] * torch.sin(angle)
+        out[j] = x[..., j] * torch.cos(angle) + x[..., i] * torch.sin(angle)
+    return torch.stack(out, dim=-1)
 
 
 def latent_rows(h, w, m, eps, faults=NONE):
@@ -90,15 +88,14 @@ def latent_attention(h, w, m, eps, rows, faults=NONE):
     seen = gap >= 0
     if "forgets_far" in faults:
         seen = seen & (gap < 64)
-    out = torch.zeros(s, heads, vdim, dtype=h.dtype)
+    out = []
     gate = torch.sigmoid(h @ w["g"].T)
     for n in range(heads):
         score = (q_plain[:, n] @ k[:, n].T + q_turned[:, n] @ shared.T) * m["scale"]
         score = score.masked_fill(~seen, -math.inf)
-        out[:, n] = sink_softmax(score, w["sink"][n], faults) @ v[:, n]
-        if "no_gate" not in faults:
-            out[:, n] = out[:, n] * gate[:, n : n + 1]
-    return out.reshape(s, heads * vdim) @ w["o"].T
+        o = sink_softmax(score, w["sink"][n], faults) @ v[:, n]
+        out.append(o if "no_gate" in faults else o * gate[:, n : n + 1])
+    return torch.cat(out, dim=1) @ w["o"].T
 
 
 # -------------------------------------------------------------------- hgrn2

@@ -78,3 +78,38 @@ def test_constants_and_misc():
     picked = sample_up_to(range(10), 3)
     assert len(picked) == 3 and set(picked) <= set(range(10))
     assert sample_up_to([1, 2], 5) == [1, 2]
+
+
+def test_nothing_is_collected_while_a_graph_is_captured(monkeypatch):
+    import contextlib
+    import gc
+
+    from petals_amd.utils import graphs
+
+    class Fake:
+        wait_stream = replay = lambda self, *_: None
+
+    capturing = []
+
+    @contextlib.contextmanager
+    def capture(_graph):
+        capturing.append(True)
+        yield
+        capturing.pop()
+
+    for name, value in (("Stream", Fake), ("CUDAGraph", Fake), ("current_stream", Fake), ("graph", capture),
+                        ("stream", lambda _s: contextlib.nullcontext())):
+        monkeypatch.setattr(graphs.torch.cuda, name, value)
+    seen = []
+    graphs.GraphedCallable(lambda: seen.append((bool(capturing), gc.isenabled())), [])
+    assert seen == [(False, True), (False, True), (True, False)] and gc.isenabled()
+
+    def fails():
+        if capturing:
+            raise RuntimeError("no capture")
+
+    try:
+        graphs.GraphedCallable(fails, [])
+    except RuntimeError:
+        pass
+    assert gc.isenabled()
