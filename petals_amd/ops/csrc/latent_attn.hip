@@ -412,11 +412,10 @@ torch::Tensor latent_attention(
     torch::Tensor tiles,   // [n, 2] int32 runs of at most run_tokens tokens
     int64_t run_tokens,
     int64_t max_keys,      // most keys that any row sees
-    int64_t window, double scale,
+    int64_t window, double scale, int64_t splits,
     int64_t values,        // size of the result: the first values of a row, 0 for all of them
-    c10::optional<torch::Tensor> sink,    // [H] f32
-    c10::optional<torch::Tensor> factor,  // [T, H] f32
-    int64_t splits) {
+    c10::optional<torch::Tensor> sink,      // [H] f32
+    c10::optional<torch::Tensor> factor) {  // [T, H] f32
   TORCH_CHECK(q.is_cuda() && q.dim() == 3 && q.is_contiguous() && q.dtype() == cache.dtype());
   const int t = q.size(0), heads = q.size(1), rp = q.size(2), vp = values > 0 ? (int)values : rp;
   TORCH_CHECK(cache.size(2) == rp && rp % 32 == 0 && vp <= rp, "latent width mismatch");

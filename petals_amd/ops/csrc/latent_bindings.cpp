@@ -15,8 +15,8 @@ torch::Tensor moe_gemm(
     torch::Tensor tile_expert, int64_t k_per_tok, int64_t n_rows);
 torch::Tensor latent_attention(
     torch::Tensor q, torch::Tensor cache, torch::Tensor pos, torch::Tensor owner, torch::Tensor tables,
-    torch::Tensor tiles, int64_t run_tokens, int64_t max_keys, int64_t window, double scale, int64_t values,
-    c10::optional<torch::Tensor> sink, c10::optional<torch::Tensor> factor, int64_t splits);
+    torch::Tensor tiles, int64_t run_tokens, int64_t max_keys, int64_t window, double scale, int64_t splits,
+    int64_t values, c10::optional<torch::Tensor> sink, c10::optional<torch::Tensor> factor);
 void latent_write(
     torch::Tensor y, int64_t offset, torch::Tensor w, torch::Tensor cache,
     torch::Tensor pos, torch::Tensor owner, torch::Tensor tables, double eps);
@@ -39,8 +39,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("moe_gemm", &moe_gemm, "grouped MFMA GEMM over expert-sorted pairs");
   m.def("latent_attention", &latent_attention, "sliding-window latent attention over a paged cache",
         py::arg("q"), py::arg("cache"), py::arg("pos"), py::arg("owner"), py::arg("tables"), py::arg("tiles"),
-        py::arg("run_tokens"), py::arg("max_keys"), py::arg("window"), py::arg("scale"), py::arg("values") = 0,
-        py::arg("sink") = py::none(), py::arg("factor") = py::none(), py::arg("splits") = 0);
+        py::arg("run_tokens"), py::arg("max_keys"), py::arg("window"), py::arg("scale"), py::arg("splits") = 0,
+        py::arg("values") = 0, py::arg("sink") = py::none(), py::arg("factor") = py::none());
   m.def("latent_write", &latent_write, "RMS-normalise latents into their cache pages");
   m.def("sublayer_out", &sublayer_out, "output norm + 32-bit residual (+ router)");
   m.def("batched_linear", &batched_linear, "out[t,h,n] = sum_k a[t,h,k] w[h,n,k]",

@@ -15,8 +15,8 @@ void residual_sum(torch::Tensor partials, c10::optional<torch::Tensor> bias, tor
 torch::Tensor bias_xielu(torch::Tensor y, torch::Tensor bias, double pos, double neg);
 torch::Tensor latent_attention(
     torch::Tensor q, torch::Tensor cache, torch::Tensor pos, torch::Tensor owner, torch::Tensor tables,
-    torch::Tensor tiles, int64_t run_tokens, int64_t max_keys, int64_t window, double scale, int64_t values,
-    c10::optional<torch::Tensor> sink, c10::optional<torch::Tensor> factor, int64_t splits);
+    torch::Tensor tiles, int64_t run_tokens, int64_t max_keys, int64_t window, double scale, int64_t splits,
+    int64_t values, c10::optional<torch::Tensor> sink, c10::optional<torch::Tensor> factor);
 std::vector<torch::Tensor> latent_rows(
     torch::Tensor y, int64_t at_q, torch::Tensor w_q, int64_t q_pad, bool q_f32, int64_t at_kv,
     c10::optional<torch::Tensor> w_kv, int64_t kv_pad, int64_t rot, torch::Tensor quarters, torch::Tensor cache,
@@ -60,8 +60,8 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("bias_xielu", &bias_xielu, "xIELU of y + bias, in place or of split-K partial sums");
   m.def("latent_attention", &latent_attention, "latent attention over a paged cache",
         py::arg("q"), py::arg("cache"), py::arg("pos"), py::arg("owner"), py::arg("tables"), py::arg("tiles"),
-        py::arg("run_tokens"), py::arg("max_keys"), py::arg("window"), py::arg("scale"), py::arg("values") = 0,
-        py::arg("sink") = py::none(), py::arg("factor") = py::none(), py::arg("splits") = 0);
+        py::arg("run_tokens"), py::arg("max_keys"), py::arg("window"), py::arg("scale"), py::arg("splits") = 0,
+        py::arg("values") = 0, py::arg("sink") = py::none(), py::arg("factor") = py::none());
   m.def("latent_rows", &latent_rows, "norms of the latents, rotated key part and gates; writes the cache");
   m.def("rotate_queries", &rotate_queries, "rotated part of the queries");
   m.def("forget_prefill", &forget_prefill, "linear attention with a forget gate over chunks of 16 tokens");

@@ -160,7 +160,7 @@ class RecurrentFastPath(PackedBlock):
         h.rotate_queries(qs, self.at_turned, m.rot_pad, self.quarters, batch.pos, q, m.latent_pad)
         run = batch.run_tokens(m.heads)
         lat = h.latent_attention(
-            q, cache, batch.pos, batch.owner, batch.tables, batch.tiles(run), run, batch.max_end, 0, m.scale,
+            q, cache, batch.pos, batch.owner, batch.tables, batch.tiles(run), run, batch.max_end, 0, m.scale, 0,
             m.latent_pad, self.sink, gate,
         )
         return h.batched_linear(lat, self.w_uv, wide).view(t, m.heads * self.vdim_p)

@@ -65,10 +65,11 @@ SHAPES = {
 
 
 class Model:
-    """A random model served by a SpanEngine, and its oracle."""
+    """A random model served by a SpanEngine, and its oracle. (A norm over few values that
+    happen to be small amplifies bf16 rounding without bound if eps is tiny.)"""
 
     def __init__(self, tmp_path, layers, path=("cpu", "float32"), *, width=40, vocab=97, tokens=1024, seed=0, edit=None,
-                 eps=1e-6, sequences=None, mult=0.6):
+                 eps=1e-2, sequences=None, mult=0.6):
         self.device, self.dtype = path
         self.raw = oracle.config_dict(vocab=vocab, width=width, layers=layers, eps=eps, mult=mult)
         self.weights = oracle.random_model(self.raw, seed)
@@ -594,7 +595,7 @@ def test_latent_attention_kernel(heads, rank, rot, dtype):
             for splits in (0, 1, 2, 5):
                 got = recurrent.hip().latent_attention(
                     q, cache, batch.pos, batch.owner, batch.tables, batch.tiles(run), run, batch.max_end, 0, scale,
-                    rank, sink_, factor_, splits,
+                    splits, rank, sink_, factor_,
                 )
                 assert got.shape == (batch.tokens, heads, rank)
                 assert (got.double().cpu() - want).abs().max() < (2e-5 if dtype == "float32" else 3e-2)
@@ -796,7 +797,7 @@ def test_group_norm_kernel(t, groups, size, shared):
         for f32 in (True, False):
             got = recurrent.hip().group_norm(o, gate, w, groups, groups * size, f32, 1e-2)
             assert got.dtype == (torch.float32 if f32 else torch.bfloat16)
-            assert (got.double() - want).abs().max() < (1e-4 if f32 else 0.05)
+            assert (got.double() - want).abs().max() < (1e-4 if f32 else 1e-2) * want.abs().max()
 
 
 @pytest.mark.gpu
