@@ -52,11 +52,10 @@ def bloom_config(s):
     )
 
 
-def lefulorn_runs(s, device, batch, kind):
-    """(prefill callable, decode callable)"""
+def engine_runs(config, device, batch):
+    """(prefill callable, decode callable) of a paged family's layers"""
     from petals_amd.server.span_engine import SpanEngine, StepEntry
 
-    config = lefulorn_config(s, kind)
     blocks = build(config, device)
     length = CONTEXT + 64 * 8
     pool = SpanEngine.pool_for(blocks, (batch + 1) * length, dtype=torch.bfloat16, device=device, max_sequences=batch + 1)
@@ -110,7 +109,7 @@ def main(steps: int = 20, warmup: int = 5, sizes=None, families=FAMILIES, batche
         for batch in batches:
             row = {"size": name, "layers": LAYERS, "batch": batch, "prefill_tokens": PREFILL, "context": CONTEXT}
             for f in families:  # in turn, on the same box
-                runs = bloom_runs(s, device, batch) if f == "bloom" else lefulorn_runs(s, device, batch, f)
+                runs = bloom_runs(s, device, batch) if f == "bloom" else engine_runs(lefulorn_config(s, f), device, batch)
                 prefill, decode = runs
                 if batch == 1:
                     row[f"{f}_prefill_tok_s"] = round(PREFILL / timed(prefill, max(3, steps // 4), 2))

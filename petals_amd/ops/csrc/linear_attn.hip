@@ -208,25 +208,58 @@ __device__ __forceinline__ void load_n(const float* p, float (&v)[1]) { v[0] = *
 __device__ __forceinline__ void load_n(const unsigned short* p, float (&v)[1]) { v[0] = bf16_to_f32(*p); }
 template <typename T> __device__ __forceinline__ void load_n(const T* p, float (&v)[8]) { load8(p, v); }
 
-// 16 rows x 16 groups of V columns per workgroup. V = 8 needs aligned groups.
-template <typename TY, int V>
+#define CONV_ROWS 4  // rows of a thread
+
+// 4 groups of CONV_ROWS rows x 64 groups of V columns per workgroup. V = 8 needs
+// aligned groups; TAPS: the number of taps, 0 for any.
+template <typename TY, int V, int TAPS>
 __global__ __launch_bounds__(256) void ssm_conv_kernel(
     const TY* __restrict__ y, int stride, ConvWeights cw, const float* __restrict__ state, ChunkRows b, SsmShape s,
     int rows, float* __restrict__ mixed) {
-  const int row = blockIdx.x * 16 + threadIdx.x / 16, c = (blockIdx.y * 16 + (threadIdx.x & 15)) * V;
-  if (row >= rows || c >= s.mixed()) return;
-  const int ch = ssm_channel(s, c);
-  float acc[V], x[V], w[V];
+  const int row0 = (blockIdx.x * 4 + threadIdx.x / 64) * CONV_ROWS, c = (blockIdx.y * 64 + (threadIdx.x & 63)) * V;
+  if (row0 >= rows || c >= s.mixed()) return;
+  const int ch = ssm_channel(s, c), n = min(CONV_ROWS, rows - row0);
+  float* dst = mixed + (size_t)row0 * s.mixed() + c;
+  const TY* src = y + (size_t)row0 * stride + s.o_conv + ch;
+  const int first_seq = b.owner[row0];
+  float acc[V], x[V], w[V], bias[V];
+  if (ch < 0) {
+    for (int r = 0; r < n; ++r)
 #pragma unroll
-  for (int e = 0; e < V; ++e) acc[e] = 0.f;
-  if (ch >= 0) {
-    const int seq = b.owner[row], p = b.pos[row];
+      for (int e = 0; e < V; ++e) dst[(size_t)r * s.mixed() + e] = 0.f;
+    return;
+  }
+  load_n(cw.bias + ch, bias);
+  if constexpr (TAPS > 0) {
+    // all inputs are rows of this step
+    if (n == CONV_ROWS && b.owner[row0 + n - 1] == first_seq && row0 - b.tiles[2 * b.bounds[first_seq]] >= TAPS - 1) {
+      float in[CONV_ROWS + TAPS - 1][V], taps[TAPS][V];
+#pragma unroll
+      for (int r = 0; r < CONV_ROWS + TAPS - 1; ++r) load_n(src + (long)(r - TAPS + 1) * stride, in[r]);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) load_n(cw.w + (size_t)j * s.channels() + ch, taps[j]);
+#pragma unroll
+      for (int r = 0; r < CONV_ROWS; ++r) {
+#pragma unroll
+        for (int e = 0; e < V; ++e) {
+          float sum = bias[e];
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j) sum = fmaf(taps[j][e], in[r + j][e], sum);
+          dst[(size_t)r * s.mixed() + e] = silu_f32(sum);
+        }
+      }
+      return;
+    }
+  }
+  for (int r = 0; r < n; ++r) {
+    const int row = row0 + r, seq = b.owner[row], p = b.pos[row];
     const int back = row - b.tiles[2 * b.bounds[seq]];
     const int slot = min(max(b.slot[seq], 0), s.slots - 1);
-    load_n(cw.bias + ch, acc);
+#pragma unroll
+    for (int e = 0; e < V; ++e) acc[e] = bias[e];
     for (int j = 0; j < s.taps; ++j) {
       const int ago = s.taps - 1 - j;
-      if (ago <= back) load_n(y + (size_t)(row - ago) * stride + s.o_conv + ch, x);
+      if (ago <= back) load_n(src + (long)(r - ago) * stride, x);
       else if (p - ago >= 0) load_n(state + ((size_t)slot * s.taps + (p - ago) % s.taps) * s.channels() + ch, x);
       else continue;
       load_n(cw.w + (size_t)j * s.channels() + ch, w);
@@ -234,11 +267,8 @@ __global__ __launch_bounds__(256) void ssm_conv_kernel(
       for (int e = 0; e < V; ++e) acc[e] = fmaf(w[e], x[e], acc[e]);
     }
 #pragma unroll
-    for (int e = 0; e < V; ++e) acc[e] = silu_f32(acc[e]);
+    for (int e = 0; e < V; ++e) dst[(size_t)r * s.mixed() + e] = silu_f32(acc[e]);
   }
-  float* dst = mixed + (size_t)row * s.mixed() + c;
-#pragma unroll
-  for (int e = 0; e < V; ++e) dst[e] = acc[e];
 }
 
 // floats of one (chunk, head): QK [16][16], G [16], G_15/G dt [16]
@@ -322,7 +352,7 @@ struct ScanInput {
   const float* mixed;  // convolved rows
   int mixed_stride, at_k, at_q, per_group;
   const float* skip;   // [H] D
-};
+};  // mixed_stride is v_stride
 
 template <int TPW, int NS, bool SSM>
 struct ScanOperands {
@@ -348,7 +378,9 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
   const int c0 = b.bounds[seq], c1 = b.bounds[seq + 1];
   if (c0 >= c1) return;
   const int slot = min(max(b.slot[seq], 0), s.slots - 1);
-  const bool fresh = b.pos[b.tiles[2 * c0]] == 0;
+  // a sequence's rows are consecutive and all its chunks but the last are full
+  const int seq_row0 = b.tiles[2 * c0], rows = b.tiles[2 * c1 - 2] + b.tiles[2 * c1 - 1] - seq_row0;
+  const bool fresh = b.pos[seq_row0] == 0;
   const int n_tiles = s.dk / 16;
   float* st = state + ((size_t)slot * s.heads + h) * s.dk * s.dv + v0 + col;
   f32x4 acc[NS][TPW];
@@ -362,91 +394,136 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
         acc[u][t][r] = !fresh && tile < n_tiles ? st[(size_t)(tile * 16 + hi * 4 + r) * s.dv + u * 16] : 0.f;
     }
   const float skip = SSM ? in.skip[h] : 0.f;
+  // Addresses are a base that moves with the chunk plus offsets that do not. Rows past
+  // the end of the last chunk read its last one.
+  const int tail = rows - (c1 - 1 - c0) * CH - 1;
+  unsigned row_v[4], tail_v[4], col_v[NS], at_row[TPW], at_col[TPW];
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    row_v[r] = (hi * 4 + r) * in.v_stride;
+    tail_v[r] = min(hi * 4 + r, tail) * in.v_stride;
+  }
+#pragma unroll
+  for (int u = 0; u < NS; ++u) col_v[u] = min(u * 16 + col, s.vdim - 1 - v0);
+#pragma unroll
+  for (int t = 0; t < TPW; ++t) {
+    const int tile = min(wave + t * 4, n_tiles - 1);
+    at_row[t] = tile * 16 + hi * 4;
+    at_col[t] = tile * 16 + col;
+  }
+  const unsigned row_q = col * in.mixed_stride, tail_q = min(col, tail) * in.mixed_stride;
   auto load = [&](int c, ScanOperands<TPW, NS, SSM>& o) {
-    const int row0 = b.tiles[2 * c], last = b.tiles[2 * c + 1] - 1;
+    const size_t row0 = seq_row0 + (size_t)(c - c0) * CH;
+    const bool last = c == c1 - 1;  // uniform
     if constexpr (SSM) {
       const float* unit = in.ws + ((size_t)c * s.heads + h) * SSM_UNIT;
-      const float* mixed = in.mixed + (size_t)row0 * in.mixed_stride + h / in.per_group * s.dk;
-      o.qk = unit[col * CH + hi * 4 + wave];
-      o.qg = unit[CH * CH + col];
+      const float* key = in.mixed + row0 * in.mixed_stride + in.at_k + h / in.per_group * s.dk;
+      const float* query = key + (in.at_q - in.at_k);
+      o.qk = unit[(unsigned)(col * CH + hi * 4 + wave)];
+      o.qg = unit[(unsigned)(CH * CH + col)];
       o.g15 = unit[CH * CH + 15];
-      o.g[0] = *reinterpret_cast<const f32x4*>(unit + CH * CH + CH + hi * 4);
+      o.g[0] = *reinterpret_cast<const f32x4*>(unit + (unsigned)(CH * CH + CH + hi * 4));
+      const unsigned rq = last ? tail_q : row_q;
 #pragma unroll
       for (int t = 0; t < TPW; ++t) {
-        const int tile = min(wave + t * 4, n_tiles - 1);
-        o.q[t] = *reinterpret_cast<const f32x4*>(mixed + (size_t)min(col, last) * in.mixed_stride + in.at_q + tile * 16 + hi * 4);
+        o.q[t] = *reinterpret_cast<const f32x4*>(query + (rq + at_row[t]));
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          o.k[t][r] = mixed[(size_t)min(hi * 4 + r, last) * in.mixed_stride + in.at_k + tile * 16 + col];
+        for (int r = 0; r < 4; ++r) o.k[t][r] = key[(last ? tail_v[r] : row_v[r]) + at_col[t]];
       }
     } else {
       const float* unit = in.ws + ((size_t)c * s.heads + h) * forget_unit(s.dk);
       const float* kh = unit + CH * s.dk;
       const float* qk = kh + CH * s.dk;
       const float* g = qk + CH * CH;
-      o.qk = qk[col * CH + hi * 4 + wave];
+      o.qk = qk[(unsigned)(col * CH + hi * 4 + wave)];
 #pragma unroll
       for (int t = 0; t < TPW; ++t) {
-        const int tile = min(wave + t * 4, n_tiles - 1);
-        o.q[t] = *reinterpret_cast<const f32x4*>(unit + col * s.dk + tile * 16 + hi * 4);
-        o.k[t] = *reinterpret_cast<const f32x4*>(kh + (tile * 16 + col) * CH + hi * 4);
-        o.g[t] = *reinterpret_cast<const f32x4*>(g + tile * 16 + hi * 4);
+        o.q[t] = *reinterpret_cast<const f32x4*>(unit + (unsigned)(col * s.dk + at_row[t]));
+        o.k[t] = *reinterpret_cast<const f32x4*>(kh + (at_col[t] * CH + hi * 4));
+        o.g[t] = *reinterpret_cast<const f32x4*>(g + at_row[t]);
       }
     }
+    const TV* v = in.v + row0 * in.v_stride + in.o_v + h * s.vdim + v0;
+#pragma unroll
+    for (int u = 0; u < NS; ++u)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o.v[u][r] = load_f32(v + ((last ? tail_v[r] : row_v[r]) + col_v[u]));
+  };
+  float mine[NS] = {};  // this wave's row of each group of 4 rows of the last chunk's values
+  // What the waves have left in LDS for chunk c. `between` runs when it is read, ahead
+  // of the branch around the store.
+  auto finish = [&](int c, auto&& between) {
+    lds_barrier();
+    float o[NS];
 #pragma unroll
     for (int u = 0; u < NS; ++u) {
-      const int vc = v0 + u * 16 + col;
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        o.v[u][r] = load_f32(in.v + (size_t)(row0 + min(hi * 4 + r, last)) * in.v_stride + in.o_v + h * s.vdim + min(vc, s.vdim - 1));
+      const float(*share)[WAVE] = part[c & 1][u][wave];
+      o[u] = (share[0][lane] + share[1][lane]) + (share[2][lane] + share[3][lane]);
+      if (SSM) o[u] = fmaf(skip, mine[u], o[u]);
     }
+    between();
+    const int row = (c - c0) * CH + hi * 4 + wave;
+    float* dst = out + ((seq_row0 + (long)(c - c0) * CH) * s.heads + h) * s.vdim + v0;
+#pragma unroll
+    for (int u = 0; u < NS; ++u)
+      if (row >= 0 && row < rows && v0 + u * 16 + col < s.vdim)
+        dst[(unsigned)((hi * 4 + wave) * s.heads * s.vdim + u * 16 + col)] = o[u];
   };
+  // The products of chunk c, then the result of the one before: the waves do not wait
+  // for each other's share of a chunk right after it.
   auto step = [&](int c, const ScanOperands<TPW, NS, SSM>& now) {
-    const int buf = c & 1;
-    f32x4 v[NS], p[NS];
-    float mine[NS];  // this wave's row of each group of 4
+    f32x4 v[NS], q[TPW], k[TPW], p[NS][TPW], old[NS][TPW];
+    float next[NS];
+#pragma unroll
+    for (int t = 0; t < TPW; ++t) {
+      const bool live = wave + t * 4 < n_tiles;
+      q[t] = now.q[t];
+      k[t] = now.k[t];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        if (SSM) {
+          q[t][r] *= now.qg;
+          k[t][r] *= now.g[0][r];
+        }
+        // no branch around a product: the tile past the last one takes zeros
+        k[t][r] = live ? k[t][r] : 0.f;
+      }
+    }
 #pragma unroll
     for (int u = 0; u < NS; ++u) {
 #pragma unroll
       for (int r = 0; r < 4; ++r) v[u][r] = v0 + u * 16 + col < s.vdim ? now.v[u][r] : 0.f;
-      mine[u] = wave == 0 ? v[u][0] : wave == 1 ? v[u][1] : wave == 2 ? v[u][2] : v[u][3];
-      p[u] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.qk, mine[u], f32x4{0.f, 0.f, 0.f, 0.f}, 0, 0, 0);
-    }
+      const float low = wave & 1 ? v[u][1] : v[u][0], high = wave & 1 ? v[u][3] : v[u][2];
+      next[u] = wave & 2 ? high : low;
 #pragma unroll
-    for (int t = 0; t < TPW; ++t) {
-      const bool live = wave + t * 4 < n_tiles;
-      f32x4 q = now.q[t], k = now.k[t];
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        if (SSM) {
-          q[r] *= now.qg;
-          k[r] *= now.g[0][r];
-        }
-        // no branch around a product: the tile past the last one takes zeros
-        k[r] = live ? k[r] : 0.f;
-      }
-#pragma unroll
-      for (int u = 0; u < NS; ++u) {
-        p[u] = mma16(q, acc[u][t], p[u]);
+      for (int t = 0; t < TPW; ++t) {
+        p[u][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+        old[u][t] = acc[u][t];
 #pragma unroll
         for (int r = 0; r < 4; ++r) acc[u][t][r] *= SSM ? now.g15 : now.g[SSM ? 0 : t][r];
-        acc[u][t] = mma16(k, v[u], acc[u][t]);
       }
+      p[u][0] = __builtin_amdgcn_mfma_f32_16x16x4f32(now.qk, next[u], p[u][0], 0, 0, 0);
     }
+    // independent chains side by side
 #pragma unroll
-    for (int u = 0; u < NS; ++u)
+    for (int r = 0; r < 4; ++r)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) part[buf][u][r][wave][lane] = p[u][r];
-    lds_barrier();
-    const int row0 = b.tiles[2 * c], n = b.tiles[2 * c + 1], row = hi * 4 + wave;
+      for (int t = 0; t < TPW; ++t)
 #pragma unroll
-    for (int u = 0; u < NS; ++u) {
-      const float(*share)[WAVE] = part[buf][u][wave];
-      float o = (share[0][lane] + share[1][lane]) + (share[2][lane] + share[3][lane]);
-      if (SSM) o = fmaf(skip, mine[u], o);
-      const int vc = v0 + u * 16 + col;
-      if (row < n && vc < s.vdim) out[((size_t)(row0 + row) * s.heads + h) * s.vdim + vc] = o;
-    }
+        for (int u = 0; u < NS; ++u) {
+          p[u][t] = __builtin_amdgcn_mfma_f32_16x16x4f32(q[t][r], old[u][t][r], p[u][t], 0, 0, 0);
+          acc[u][t] = __builtin_amdgcn_mfma_f32_16x16x4f32(k[t][r], v[u][r], acc[u][t], 0, 0, 0);
+        }
+    finish(c - 1, [&] {  // nothing is stored for the chunk before the first
+#pragma unroll
+      for (int u = 0; u < NS; ++u) {
+        mine[u] = next[u];
+#pragma unroll
+        for (int t = 1; t < TPW; ++t) p[u][0] += p[u][t];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) part[c & 1][u][r][wave][lane] = p[u][0][r];
+      }
+    });
   };
   auto load_ahead = [&](int c, ScanOperands<TPW, NS, SSM>& o) { load(min(c, c1 - 1), o); };
   ScanOperands<TPW, NS, SSM> o0, o1, o2, o3;  // written out: an indexed array would not stay in registers
@@ -478,6 +555,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(
     }
     if (c < c1) step(c, o0);
   }
+  finish(c1 - 1, [] {});
 #pragma unroll
   for (int u = 0; u < NS; ++u)
 #pragma unroll
@@ -855,14 +933,15 @@ torch::Tensor ssm_prefill(
   const size_t lds = (size_t)2 * CH * (s.dk + 4) * 4;
   const ConvWeights cw{conv_w.data_ptr<float>(), conv_b.data_ptr<float>()};
   const dim3 chunk_grid(chunks, groups, (per + 15) / 16);
+#define SC(TY, YP, V, TAPS)                                                                                         \
+  ssm_conv_kernel<TY, V, TAPS><<<dim3((t + 4 * CONV_ROWS - 1) / (4 * CONV_ROWS), (s.mixed() + 64 * V - 1) / (64 * V)), \
+                                 256, 0, stream>>>(YP, stride, cw, conv.data_ptr<float>(), b, s, (int)t,            \
+                                                   mixed.data_ptr<float>())
 #define SP(TY, YP)                                                                                                  \
   do {                                                                                                              \
-    if (by8)                                                                                                        \
-      ssm_conv_kernel<TY, 8><<<dim3((t + 15) / 16, (s.mixed() + 127) / 128), 256, 0, stream>>>(                     \
-          YP, stride, cw, conv.data_ptr<float>(), b, s, (int)t, mixed.data_ptr<float>());                           \
-    else                                                                                                            \
-      ssm_conv_kernel<TY, 1><<<dim3((t + 15) / 16, (s.mixed() + 15) / 16), 256, 0, stream>>>(                       \
-          YP, stride, cw, conv.data_ptr<float>(), b, s, (int)t, mixed.data_ptr<float>());                           \
+    if (by8 && s.taps == 4) SC(TY, YP, 8, 4);                                                                       \
+    else if (by8) SC(TY, YP, 8, 0);                                                                                 \
+    else SC(TY, YP, 1, 0);                                                                                          \
     HIP_CHECK_LAST();                                                                                               \
     ssm_conv_tail<TY><<<dim3(seqs, (s.channels() + 255) / 256), 256, 0, stream>>>(YP, stride, b,                    \
                                                                                   conv.data_ptr<float>(), s);       \
@@ -876,6 +955,7 @@ torch::Tensor ssm_prefill(
   if (y.dtype() == torch::kFloat32) SP(float, y.data_ptr<float>());
   else SP(unsigned short, BF16P(y));
 #undef SP
+#undef SC
   launch_scan<float, true>(
       ScanInput<float>{ws.data_ptr<float>(), mixed.data_ptr<float>(), s.mixed(), 0, mixed.data_ptr<float>(), s.mixed(),
                        s.at_k(), s.at_q(), per, skip.data_ptr<float>()},

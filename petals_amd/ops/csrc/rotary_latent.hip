@@ -58,23 +58,23 @@ struct LatentColumns {
   int gate, heads;
 };
 
-// One workgroup per token.
-template <typename TY, typename TC, typename TQ>
-__global__ __launch_bounds__(256) void latent_rows_kernel(
+// One workgroup of NT threads per token.
+template <typename TY, typename TC, typename TQ, int NT>
+__global__ __launch_bounds__(NT) void latent_rows_kernel(
     const TY* __restrict__ y, int stride, LatentColumns n, const float* __restrict__ w_q, const float* __restrict__ w_kv,
     Rotation rot, TC* __restrict__ cache, int width, PagedRows b, TQ* __restrict__ cq, float* __restrict__ factor,
     float eps) {
-  __shared__ float red[2][4];
+  __shared__ float red[2][NT / WAVE];
   const int tid = threadIdx.x;
   const size_t t = blockIdx.x;
   const TY* row = y + t * stride;
   float q2 = 0.f, c2 = 0.f;
-  for (int d = tid; d < n.q_rank; d += 256) {
+  for (int d = tid; d < n.q_rank; d += NT) {
     const float v = load_f32(row + n.q + d);
     q2 = fmaf(v, v, q2);
   }
   if (n.kv >= 0)
-    for (int d = tid; d < n.kv_rank; d += 256) {
+    for (int d = tid; d < n.kv_rank; d += NT) {
       const float v = load_f32(row + n.kv + d);
       c2 = fmaf(v, v, c2);
     }
@@ -85,19 +85,25 @@ __global__ __launch_bounds__(256) void latent_rows_kernel(
     red[1][tid / WAVE] = c2;
   }
   __syncthreads();
-  const float iq = 1.f / sqrtf(((red[0][0] + red[0][1]) + (red[0][2] + red[0][3])) / n.q_rank + eps);
-  for (int d = tid; d < n.q_pad; d += 256)
+  q2 = c2 = 0.f;
+#pragma unroll
+  for (int i = 0; i < NT / WAVE; ++i) {
+    q2 += red[0][i];
+    c2 += red[1][i];
+  }
+  const float iq = 1.f / sqrtf(q2 / n.q_rank + eps);
+  for (int d = tid; d < n.q_pad; d += NT)
     store_f32(cq + t * n.q_pad + d, d < n.q_rank ? load_f32(row + n.q + d) * iq * w_q[d] : 0.f);
-  for (int h = tid; h < n.heads; h += 256) factor[t * n.heads + h] = 1.f / (1.f + expf(-load_f32(row + n.gate + h)));
+  for (int h = tid; h < n.heads; h += NT) factor[t * n.heads + h] = 1.f / (1.f + expf(-load_f32(row + n.gate + h)));
   if (n.kv < 0) return;
   const int pos = b.pos[t];
   const long at = cache_row(b, b.owner[t], pos);
   if (at < 0) return;
-  const float ic = 1.f / sqrtf(((red[1][0] + red[1][1]) + (red[1][2] + red[1][3])) / n.kv_rank + eps);
+  const float ic = 1.f / sqrtf(c2 / n.kv_rank + eps);
   TC* dst = cache + (size_t)at * width;
-  for (int d = tid; d < n.kv_pad; d += 256)
+  for (int d = tid; d < n.kv_pad; d += NT)
     store_f32(dst + d, d < n.kv_rank ? load_f32(row + n.kv + d) * ic * w_kv[d] : 0.f);
-  for (int d = tid; d < width - n.kv_pad; d += 256)
+  for (int d = tid; d < width - n.kv_pad; d += NT)
     store_f32(dst + n.kv_pad + d, d < n.rot ? rotated(row + n.kv + n.kv_rank, d, pos, rot) : 0.f);
 }
 
@@ -154,11 +160,16 @@ std::vector<torch::Tensor> latent_rows(
   auto factor = torch::empty({t, heads}, y.options().dtype(torch::kFloat32));
   if (t == 0) return {cq, factor};
   auto stream = at::cuda::getCurrentCUDAStream();
-#define LR(TY, TC, TQ)                                                                                       \
-  latent_rows_kernel<TY, TC, TQ><<<t, 256, 0, stream>>>(                                                     \
+#define LRN(TY, TC, TQ, NT)                                                                                  \
+  latent_rows_kernel<TY, TC, TQ, NT><<<t, NT, 0, stream>>>(                                                  \
       reinterpret_cast<const TY*>(y.data_ptr()), (int)width, n, w_q.data_ptr<float>(), wkv, r,               \
       reinterpret_cast<TC*>(cache.data_ptr()), (int)cache.size(2), b, reinterpret_cast<TQ*>(cq.data_ptr()),  \
       factor.data_ptr<float>(), (float)eps)
+#define LR(TY, TC, TQ)                    \
+  do {                                    \
+    if (t < 512) LRN(TY, TC, TQ, 1024);   \
+    else LRN(TY, TC, TQ, 256);            \
+  } while (0)
 #define LRQ(TY, TC)                       \
   do {                                    \
     if (q_f32) LR(TY, TC, float);         \
@@ -170,6 +181,7 @@ std::vector<torch::Tensor> latent_rows(
   else LRQ(unsigned short, unsigned short);
 #undef LRQ
 #undef LR
+#undef LRN
   HIP_CHECK_LAST();
   return {cq, factor};
 }
