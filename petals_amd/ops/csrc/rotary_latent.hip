@@ -107,16 +107,35 @@ __global__ __launch_bounds__(NT) void latent_rows_kernel(
     store_f32(dst + n.kv_pad + d, d < n.rot ? rotated(row + n.kv + n.kv_rank, d, pos, rot) : 0.f);
 }
 
-// Grid: (values of a token / 256, tokens)
+// One workgroup per token; a thread turns one pair of every (256 / columns)th head,
+// where a row's columns are its pairs and, behind them, the values that pass.
 template <typename TY, typename TQ>
 __global__ __launch_bounds__(256) void rotate_queries_kernel(
     const TY* __restrict__ y, int stride, int first, int heads, int rot_pad, Rotation rot, const int* __restrict__ pos,
     TQ* __restrict__ q, int width, int offset) {
-  const int i = blockIdx.x * 256 + threadIdx.x;
-  if (i >= heads * rot_pad) return;
-  const int h = i / rot_pad, d = i - h * rot_pad;
-  const size_t t = blockIdx.y;
-  store_f32(q + (t * heads + h) * width + offset + d, rotated(y + t * stride + first + h * rot_pad, d, pos[t], rot));
+  const size_t t = blockIdx.x;
+  const int half = rot.turned / 2, columns = rot_pad - half, p = pos[t];
+  const int per = max(1, 256 / columns), h0 = threadIdx.x / columns;
+  if (columns <= 256 && h0 >= per) return;
+  const TY* src = y + t * stride + first;
+  TQ* dst = q + t * heads * width + offset;
+  for (int i = columns <= 256 ? threadIdx.x - h0 * columns : threadIdx.x; i < columns; i += 256) {
+    const bool pair = i < half;
+    float s = 0.f, c = 1.f;
+    if (pair) sin_cos(p * rot.quarters[i], s, c);
+#pragma unroll 4
+    for (int h = columns <= 256 ? h0 : 0; h < heads; h += per) {
+      const TY* x = src + h * rot_pad;
+      TQ* o = dst + (size_t)h * width;
+      if (pair) {
+        const float u = load_f32(x + i), v = load_f32(x + i + half);
+        store_f32(o + i, u * c - v * s);
+        store_f32(o + i + half, fmaf(v, c, u * s));
+      } else {
+        store_f32(o + i + half, load_f32(x + i + half));
+      }
+    }
+  }
 }
 
 // ------------------------------------------------------------------- host
@@ -196,12 +215,11 @@ void rotate_queries(torch::Tensor y, int64_t first, int64_t rot_pad, torch::Tens
   TORCH_CHECK(first >= 0 && first + heads * rot_pad <= y.size(1) && offset >= 0 && offset + rot_pad <= q.size(2));
   TORCH_CHECK(pos.is_cuda() && pos.dtype() == torch::kInt32 && pos.is_contiguous() && pos.numel() == t);
   const Rotation r = rotation(quarters);
-  TORCH_CHECK(r.turned <= rot_pad && t <= 65535, "rotation of ", r.turned, " of ", rot_pad, " values, ", t, " rows");
+  TORCH_CHECK(r.turned <= rot_pad, "rotation of ", r.turned, " of ", rot_pad, " values");
   if (t == 0 || rot_pad == 0) return;
   auto stream = at::cuda::getCurrentCUDAStream();
-  const dim3 grid((heads * rot_pad + 255) / 256, t);
 #define RQ(TY, TQ)                                                                                                \
-  rotate_queries_kernel<TY, TQ><<<grid, 256, 0, stream>>>(                                                        \
+  rotate_queries_kernel<TY, TQ><<<t, 256, 0, stream>>>(                                                           \
       reinterpret_cast<const TY*>(y.data_ptr()), (int)y.size(1), (int)first, (int)heads, (int)rot_pad, r,         \
       pos.data_ptr<int>(), reinterpret_cast<TQ*>(q.data_ptr()), (int)q.size(2), (int)offset)
   if (yf && qf) RQ(float, float);
