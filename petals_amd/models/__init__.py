@@ -38,6 +38,7 @@ def _ensure_families():
         import petals_amd.models.tulezen  # noqa: F401
         import petals_amd.models.lefulorn  # noqa: F401
         import petals_amd.models.soselix  # noqa: F401
+        import petals_amd.models.zudarax  # noqa: F401
 
         _loaded = True
 

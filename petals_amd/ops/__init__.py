@@ -190,13 +190,14 @@ def zero_centered_rms_norm(x, weight, eps: float):
     return reference.zero_centered_rms_norm(x, weight, eps)
 
 
-def rms_norm_f32(x, weight, eps: float):
-    """x / sqrt(mean(x^2) + eps) * weight over the last axis, 32-bit in and out."""
+def rms_norm_f32(x, weight, eps: float, groups: int = 1):
+    """x / sqrt(mean(x^2) + eps) * weight over each of `groups` equal parts of the last
+    axis, 32-bit in and out."""
     if x.is_cuda and not _grad_mode(x, weight):
-        from petals_amd.ops import hybrid
+        from petals_amd.ops import packed
 
-        return hybrid.rms_norm_f32(x, weight, eps)
-    return reference.rms_norm(x.float(), weight.float(), eps)
+        return packed.rms_norm_f32(x, weight, eps, groups)
+    return reference.group_rms_norm(x.float(), weight.float(), groups, eps)
 
 
 def linear_f32(x, weight):
@@ -205,7 +206,7 @@ def linear_f32(x, weight):
         from petals_amd.ops import _hip
 
         # in every library of the paged families: the one this process serves with
-        hip = _hip.first_loaded("latent", "hybrid", "recurrent")
+        hip = _hip.first_loaded("latent", "hybrid", "recurrent", "scores")
         rows = x.float().reshape(-1, 1, x.shape[-1]).contiguous()
         return hip.batched_linear(rows, weight.contiguous().unsqueeze(0), True).view(*x.shape[:-1], weight.shape[0])
     return (x.to(weight.dtype) @ weight.t()).float()

@@ -16,7 +16,7 @@ import torch
 
 from petals_amd.models.lefulorn.config import KEY_PAD, VALUE_PAD
 from petals_amd.ops import reference
-from petals_amd.ops.packed import CHUNK, PackedBlock, rms_norm_rows
+from petals_amd.ops.packed import CHUNK, PackedBlock
 from petals_amd.ops.packed import round_up as _up
 
 _EPI_RELU2_F32 = 6
@@ -27,13 +27,6 @@ def hip():
     from petals_amd.ops import _hip
 
     return _hip.first_loaded("hybrid")
-
-
-def rms_norm_f32(x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
-    from petals_amd.ops import _hip
-
-    # in every library of pre-norm blocks: the one this process serves with
-    return rms_norm_rows(_hip.first_loaded("hybrid", "recurrent"), x, weight, eps)
 
 
 class HybridFastPath(PackedBlock):

@@ -1,5 +1,5 @@
 """What the fast paths of pre-norm blocks with a dense feed-forward have in common
-(ops/hybrid.py, ops/recurrent.py): weights packed once at load, and the two routes
+(ops/hybrid.py, ops/recurrent.py, ops/scores.py): weights packed once at load, and the two routes
 of a batch, whatever mix of requests it holds:
 
   few rows   split-K GEMVs with 32-bit activations; no library product and no host
@@ -27,10 +27,14 @@ def round_up(n: int, to: int) -> int:
     return -(-n // to) * to
 
 
-def rms_norm_rows(hip, x: torch.Tensor, weight: torch.Tensor, eps: float) -> torch.Tensor:
+def rms_norm_f32(x: torch.Tensor, weight: torch.Tensor, eps: float, groups: int = 1) -> torch.Tensor:
+    from petals_amd.ops import _hip
+
+    # in every library of pre-norm blocks: the one this process serves with
+    hip = _hip.first_loaded("hybrid", "recurrent", "scores")
     d = x.shape[-1]
     rows = x.float().reshape(-1, d).contiguous()
-    return hip.residual_norm(rows, None, None, weight.float().contiguous(), d, eps, True)[:, :d].reshape(x.shape)
+    return hip.residual_norm(rows, None, None, weight.float().contiguous(), d, eps, True, 1.0, groups)[:, :d].reshape(x.shape)
 
 
 class PackedBlock:

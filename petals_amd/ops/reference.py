@@ -286,16 +286,38 @@ def biased_sink_attention(
 # ------------------- rotated halves, gated linear attention, group norm, xIELU
 
 
+def rotary_frequencies(dims: int, base: float, yarn=None, device=None):
+    """(radians per position of each of dims/2 pairs, 64-bit; factor of cos and sin).
+    yarn: an object with factor, original, fast and slow, or None."""
+    i = torch.arange(dims // 2, device=device, dtype=torch.float64)
+    freqs = base ** (-2.0 * i / max(dims, 1))
+    if yarn is None or dims == 0:
+        return freqs, 1.0
+
+    def pair(turns):  # (2 x) the pair that turns this often over the original positions
+        return dims * math.log(yarn.original / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+    lo, hi = max(math.floor(pair(yarn.fast)), 0), min(math.ceil(pair(yarn.slow)), dims - 1)
+    ramp = ((i - lo) / max(hi - lo, 0.001)).clamp(0.0, 1.0)
+    return freqs / yarn.factor * ramp + freqs * (1.0 - ramp), 0.1 * math.log(yarn.factor) + 1.0
+
+
+def rotate_pairs(x: torch.Tensor, pos: torch.Tensor, freqs: torch.Tensor, factor: float = 1.0) -> torch.Tensor:
+    """x [..., n] at positions pos (broadcast over x's leading axes): pair (i, i + len(freqs))
+    turns by pos * freqs[i] and grows by `factor`; the values behind the pairs pass."""
+    half = len(freqs)
+    if half == 0:
+        return x
+    angle = pos[..., None].double() * freqs
+    cos, sin = (angle.cos() * factor).float(), (angle.sin() * factor).float()
+    u, v, rest = x.split([half, half, x.shape[-1] - 2 * half], dim=-1)
+    return torch.cat([u * cos - v * sin, v * cos + u * sin, rest], dim=-1)
+
+
 def rotate_halves(x: torch.Tensor, pos: torch.Tensor, dims: int, base: float) -> torch.Tensor:
     """x [..., n] at positions pos (broadcast over x's leading axes): the pair
     (i, i + dims/2) of the first `dims` values turns by pos * base^(-2i/dims)."""
-    if dims == 0:
-        return x
-    i = torch.arange(dims // 2, device=x.device, dtype=torch.float64)
-    angle = pos[..., None].double() * base ** (-2.0 * i / dims)
-    cos, sin = angle.cos().float(), angle.sin().float()
-    u, v, rest = x.split([dims // 2, dims // 2, x.shape[-1] - dims], dim=-1)
-    return torch.cat([u * cos - v * sin, v * cos + u * sin, rest], dim=-1)
+    return rotate_pairs(x, pos, rotary_frequencies(dims, base, device=x.device)[0])
 
 
 def forget_gate(z: torch.Tensor, lower: torch.Tensor):
@@ -326,3 +348,43 @@ def xielu(z: torch.Tensor, p: torch.Tensor, q: torch.Tensor) -> torch.Tensor:
     low = z.clamp(max=0.0)
     negative = (0.5 + F.softplus(q)) * (torch.expm1(low) - low)
     return torch.where(z > 0, F.softplus(p) * z * z, negative) + 0.5 * z
+
+
+# ---------------- capped, differential and sigmoid attention, PolyNorm
+
+
+def visible(q_pos: torch.Tensor, k_pos: torch.Tensor, chunk: int = 0) -> torch.Tensor:
+    """[Sq, Sk]: keys at or before the query, in its own run of `chunk` positions (0: all of them)."""
+    seen = k_pos[None, :] <= q_pos[:, None]
+    if chunk > 0:
+        seen = seen & (k_pos[None, :] // chunk == q_pos[:, None] // chunk)
+    return seen
+
+
+def scored_attention(q, k, v, seen, *, scale, softcap=0.0, sigmoid_bias=None) -> torch.Tensor:
+    """q [..., Sq, H, d], k/v [..., Sk, G, d]; 32-bit. Scores are capped by a tanh if `softcap` is
+    given; weights are a softmax, or sigmoids of scores plus a bias per head."""
+    group = q.shape[-2] // k.shape[-2]
+    q = q.float().transpose(-3, -2)
+    k, v = (t.float().repeat_interleave(group, dim=-2).transpose(-3, -2) for t in (k, v))
+    score = (q @ k.transpose(-1, -2).contiguous()) * scale
+    if softcap > 0:
+        score = softcap * torch.tanh(score / softcap)
+    if sigmoid_bias is not None:
+        p = torch.sigmoid(score + sigmoid_bias.float()[:, None, None]).masked_fill(~seen, 0.0)
+    else:
+        p = torch.softmax(score.masked_fill(~seen, float("-inf")), dim=-1)
+    return (p @ v).transpose(-3, -2)
+
+
+def differential_share(lq1, lk1, lq2, lk2, diff: float) -> torch.Tensor:
+    """exp(lq1 . lk1) - exp(lq2 . lk2) + diff: how much of the second map is taken off the first."""
+    first, second = ((a.float() * b.float()).sum().exp() for a, b in ((lq1, lk1), (lq2, lk2)))
+    return first - second + diff
+
+
+def poly_norm(z: torch.Tensor, act: torch.Tensor, eps: float) -> torch.Tensor:
+    """a N(z) + b N(z^2) + c N(z^3) + e, act = (a, b, c, e); N divides a row by its root mean square."""
+    one = z.new_ones(())
+    a, b, c, e = act
+    return a * rms_norm(z, one, eps) + b * rms_norm(z * z, one, eps) + c * rms_norm(z * z * z, one, eps) + e

@@ -21,7 +21,7 @@ def _ensure_registered():
     import petals_amd.models as m
 
     m._ensure_families()
-    for family in ("llama", "bloom", "falcon", "mixtral", "tulezen", "lefulorn", "soselix"):
+    for family in ("llama", "bloom", "falcon", "mixtral", "tulezen", "lefulorn", "soselix", "zudarax"):
         if family not in _REGISTRY:
             mod = getattr(__import__(f"petals_amd.models.{family}", fromlist=["_register_models"]), "_register_models")
             mod()
