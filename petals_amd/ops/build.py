@@ -1,7 +1,7 @@
 """Build the HIP extensions IN-TREE (the .so files must travel with the source
 tree to GPU boxes): `python -m petals_amd.ops.build [name ...]`.
 
-Cross-compiles for gfx950 (no GPU needed at build time). Four libraries:
+Cross-compiles for gfx950 (no GPU needed at build time). Five libraries:
 
   core    the kernels of the llama / bloom / falcon / mixtral families
   latent  latent attention, output norms and routed experts (tulezen); it is
@@ -10,6 +10,8 @@ Cross-compiles for gfx950 (no GPU needed at build time). Four libraries:
           input norms (lefulorn); likewise
   recurrent  gated linear attention, latent attention with a rotated key part,
           input norms (soselix); likewise
+  scores  attention with capped scores, two maps or sigmoid weights, short
+          convolutions ahead of it, PolyNorm (zudarax); likewise
 """
 
 from __future__ import annotations
@@ -39,6 +41,11 @@ EXTENSIONS = {
     "recurrent": (
         "_hip_recurrent.so", "petals_amd_hip_recurrent", os.path.join("_build", "recurrent"),
         ["recurrent_bindings.cpp", "linear_attn.hip", "latent_attn.hip", "rotary_latent.hip", "prenorm.hip",
+         "sublayer.hip", "gemv.hip"],
+    ),
+    "scores": (
+        "_hip_scores.so", "petals_amd_hip_scores", os.path.join("_build", "scores"),
+        ["scores_bindings.cpp", "paired_attn.hip", "capped_attn.hip", "sigmoid_attn.hip", "prepare_rows.hip", "prenorm.hip",
          "sublayer.hip", "gemv.hip"],
     ),
 }

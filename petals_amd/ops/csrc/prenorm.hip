@@ -1,7 +1,8 @@
 // Sublayer kernels for blocks that norm each sublayer's INPUT and keep the
 // residual stream in 32-bit (CDNA4, gfx950).
 //
-//   residual_norm   x += mult (y + bias), then RMS norm of x with a plain weight
+//   residual_norm   x += mult (y + bias), then RMS norm of x with a plain weight, of the
+//                   whole row or of equal parts of it
 //   residual_sum    x += mult (split-K partial sums + bias) of a decoding product
 //   bias_relu2      relu(y + bias)^2
 //   bias_xielu      xIELU of y + bias, y a matrix (in place) or split-K partial sums
@@ -29,8 +30,8 @@ __device__ __forceinline__ void store4(unsigned short* p, f32x4 v) {
 template <typename TY, typename TH>
 __global__ __launch_bounds__(1024) void residual_norm_kernel(
     float* __restrict__ x, long x_stride, const TY* __restrict__ y, long y_stride, const float* __restrict__ bias,
-    const float* __restrict__ w, float eps, TH* __restrict__ h, int d, int dp, bool by4, float mult) {
-  extern __shared__ float row[];  // [d]
+    const float* __restrict__ w, float eps, TH* __restrict__ h, int d, int dp, bool by4, float mult, int groups) {
+  extern __shared__ float row[];  // [d], then of each group
   __shared__ float red[16];
   const int tid = threadIdx.x, nt = blockDim.x;
   const size_t t = blockIdx.x;
@@ -61,6 +62,40 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
     ss = fmaf(v, v, ss);
   }
   if (!h) return;  // uniform
+  if (groups > 1) {  // the waves share the groups
+    const int part = d / groups, waves = nt / WAVE, per = max(1, waves / groups), lane = tid & (WAVE - 1);
+    float* inv_of = row + (d + 3) / 4 * 4;  // [groups]
+    float* sums = inv_of + groups;          // [groups * per]
+    __syncthreads();
+    for (int i = tid / WAVE; i < groups * per; i += waves) {
+      const float* src = row + i / per * part;
+      float s2 = 0.f;
+      for (int c = i % per * WAVE + lane; c < part; c += per * WAVE) s2 = fmaf(src[c], src[c], s2);
+      s2 = wave_reduce_sum(s2);
+      if (lane == 0) sums[i] = s2;
+    }
+    __syncthreads();
+    for (int g = tid; g < groups; g += nt) {
+      float s2 = 0.f;
+      for (int i = 0; i < per; ++i) s2 += sums[g * per + i];
+      inv_of[g] = 1.f / sqrtf(s2 / part + eps);
+    }
+    __syncthreads();
+    const bool quads = by4 && part % 4 == 0;
+    if (quads) {
+      for (int c = tid * 4; c < d; c += nt * 4) {
+        f32x4 v = load4(row + c);
+        const f32x4 g = load4(w + c);
+        const float inv = inv_of[c / part];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] *= inv * g[e];
+        store4(h + t * dp + c, v);
+      }
+    }
+    for (int c = quads ? d + tid : tid; c < dp; c += nt)
+      store_f32(h + t * dp + c, c < d ? row[c] * inv_of[c / part] * w[c] : 0.f);
+    return;
+  }
   ss = wave_reduce_sum(ss);
   if ((tid & (WAVE - 1)) == 0) red[tid / WAVE] = ss;
   __syncthreads();
@@ -180,10 +215,13 @@ static const float* vec(const c10::optional<torch::Tensor>& t, int64_t n) {
   return t->data_ptr<float>();
 }
 
-// x [T, >= d] f32, updated in place if y is given; returns the norm [T, dp], or nothing if w is absent
+// x [T, >= d] f32, updated in place if y is given; returns the norm [T, dp] of `groups` equal parts, or
+// nothing if w is absent
 torch::Tensor residual_norm(torch::Tensor x, c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> bias,
-                            c10::optional<torch::Tensor> w, int64_t d, double eps, bool out_f32, double mult) {
+                            c10::optional<torch::Tensor> w, int64_t d, double eps, bool out_f32, double mult,
+                            int64_t groups) {
   TORCH_CHECK(x.is_cuda() && x.dtype() == torch::kFloat32 && x.dim() == 2 && x.stride(1) == 1 && x.size(1) >= d);
+  TORCH_CHECK(groups >= 1 && d % groups == 0, d, " values in ", groups, " groups");
   const long t = x.size(0), dp = w.has_value() ? (d + 7) / 8 * 8 : 0;
   bool yf = true;
   const void* yp = nullptr;
@@ -198,8 +236,8 @@ torch::Tensor residual_norm(torch::Tensor x, c10::optional<torch::Tensor> y, c10
   const float* wp = vec(w, d);
   auto h = torch::empty({wp ? t : 0, dp}, x.options().dtype(out_f32 ? torch::kFloat32 : torch::kBFloat16));
   if (t == 0) return h;
-  const size_t lds = d * 4;
-  TORCH_CHECK(lds <= 65536 - 64, "width ", d, " is not supported");
+  const size_t lds = d * 4 + (groups > 1 ? (2 * groups + 16 + 4) * 4 : 0);
+  TORCH_CHECK(lds <= 65536 - 64, "width ", d, " in ", groups, " groups is not supported");
   const int threads = t < 512 ? 1024 : 256;
   auto aligned = [](const void* p, int bytes) { return reinterpret_cast<uintptr_t>(p) % bytes == 0; };
   const bool by4 = d % 4 == 0 && x.stride(0) % 4 == 0 && ys % 4 == 0 && aligned(x.data_ptr(), 16) &&
@@ -208,7 +246,7 @@ torch::Tensor residual_norm(torch::Tensor x, c10::optional<torch::Tensor> y, c10
 #define RN(TY, TH)                                                                                          \
   residual_norm_kernel<TY, TH><<<t, threads, lds, stream>>>(                                                \
       x.data_ptr<float>(), x.stride(0), reinterpret_cast<const TY*>(yp), ys, bp, wp, (float)eps,            \
-      wp ? reinterpret_cast<TH*>(h.data_ptr()) : nullptr, (int)d, (int)dp, by4, (float)mult)
+      wp ? reinterpret_cast<TH*>(h.data_ptr()) : nullptr, (int)d, (int)dp, by4, (float)mult, (int)groups)
   if (yf && out_f32) RN(float, float);
   else if (yf) RN(float, unsigned short);
   else if (out_f32) RN(unsigned short, float);

@@ -10,7 +10,7 @@ torch::Tensor gemv_bf16(
 torch::Tensor batched_linear(torch::Tensor a, torch::Tensor w, bool out_f32, c10::optional<torch::Tensor> out);
 torch::Tensor residual_norm(
     torch::Tensor x, c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> bias,
-    c10::optional<torch::Tensor> w, int64_t d, double eps, bool out_f32, double mult);
+    c10::optional<torch::Tensor> w, int64_t d, double eps, bool out_f32, double mult, int64_t groups);
 void residual_sum(torch::Tensor partials, c10::optional<torch::Tensor> bias, torch::Tensor x, int64_t d, double mult);
 torch::Tensor bias_xielu(torch::Tensor y, torch::Tensor bias, double pos, double neg);
 torch::Tensor latent_attention(
@@ -54,7 +54,7 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("a"), py::arg("w"), py::arg("out_f32"), py::arg("out") = py::none());
   m.def("residual_norm", &residual_norm, "x += mult (y + bias); RMS norm of x",
         py::arg("x"), py::arg("y"), py::arg("bias"), py::arg("w"), py::arg("d"), py::arg("eps"), py::arg("out_f32"),
-        py::arg("mult") = 1.0);
+        py::arg("mult") = 1.0, py::arg("groups") = 1);
   m.def("residual_sum", &residual_sum, "x += mult (split-K partial sums + bias)",
         py::arg("partials"), py::arg("bias"), py::arg("x"), py::arg("d"), py::arg("mult") = 1.0);
   m.def("bias_xielu", &bias_xielu, "xIELU of y + bias, in place or of split-K partial sums");

@@ -63,6 +63,10 @@ class PackedBlock:
             self.b_up = torch.zeros(ffp, device=self.device)
             self._place(block, "up_bias", self.b_up[: self.mlp.ff])
             self.b_down = self._f32(block, "down_bias")
+        self._release(block)
+
+    def _release(self, block) -> None:
+        """Frees the block's own weights; all are packed."""
         self.max_gemv_rows = _GEMV_ROWS
         # batches that the engine may capture: only kernels of this library run
         self.max_graph_rows = 0 if self.f32 or not self.captures else self.max_gemv_rows
