@@ -253,7 +253,7 @@ def main():
                    help="serve (default): the REAL serving stack (DHT + Server + handler + client "
                         "sessions) with the RCCL mesh hand-off — what a user gets; pipeline: bare "
                         "rank-per-GPU RCCL pipeline (kernel-harness upper bound)")
-    p.add_argument("--compare", default=None, choices=["tulezen", "lefulorn", "soselix"],
+    p.add_argument("--compare", default=None, choices=["tulezen", "lefulorn", "soselix", "zudarax"],
                    help="instead of the flagship run: layers of this family beside the closest other family's, "
                         "one GPU, random weights (benchmarks/benchmark_<family>.py)")
     args = p.parse_args()

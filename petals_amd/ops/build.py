@@ -71,6 +71,11 @@ def build(verbose: bool = False, name: str = "core") -> str:
 
     for stale in glob.glob(os.path.join(SRC_DIR, "*_hip.*")):
         os.unlink(stale)
+    # headers are not among the dependencies that torch writes for hipcc
+    newest = max(os.path.getmtime(h) for h in glob.glob(os.path.join(SRC_DIR, "*.h")))
+    for obj in glob.glob(os.path.join(build_dir, "*.o")):
+        if os.path.getmtime(obj) < newest:
+            os.unlink(obj)
     load(
         name=ext_name,
         sources=[os.path.join(SRC_DIR, s) for s in files],

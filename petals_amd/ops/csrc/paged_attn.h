@@ -13,7 +13,7 @@
 // A token's cache row is [G heads of MAPS x DK keys | G heads of DV values], DK a
 // multiple of 32 and DV of 16 (padded with zeros when weights are packed).
 //
-//   paged_attn_kernel   MFMA flash kernel for prompts and portions: 4 waves of 16
+//   paged_attn_kernel   MFMA flash kernel for prompts and portions: 4 waves of 16 or 32
 //                       (token, head) rows share double-buffered key/value tiles
 //   paged_attn_decode   few rows per kv head: every wave takes tiles of its own,
 //                       keys straight from memory, merged through LDS at the end
@@ -29,7 +29,7 @@
 #include <c10/hip/HIPStream.h>
 #include <algorithm>
 
-#define KVT 32   // keys per tile; tiles are aligned, so one lies in one page
+#define KVT 32   // keys per tile of a decoding wave; tiles are aligned, so one lies in one page
 #define TPAD 16  // LDS row padding (elements)
 #define LOG2E 1.4426950408889634f
 
@@ -61,19 +61,48 @@ struct GatedOut {
   long gate_stride;
   bool per_head;     // one gate per head
   bool f32;          // both in 32-bit, else bf16
+  bool by4;          // groups of 4 of the result are aligned
 };
+
+__device__ __forceinline__ float gate_of(const GatedOut& g, size_t at) {
+  const float z = g.f32 ? reinterpret_cast<const float*>(g.gate)[at]
+                        : bf16_to_f32(reinterpret_cast<const unsigned short*>(g.gate)[at]);
+  return 1.f / (1.f + expf(-z));
+}
 
 __device__ __forceinline__ void write_gated(const GatedOut& g, const AttnShape& a, size_t tok, int head, int c, float v) {
   const int col = head * a.dv + c;
-  if (g.gate) {
-    const size_t at = tok * g.gate_stride + (g.per_head ? head : col);
-    const float z = g.f32 ? reinterpret_cast<const float*>(g.gate)[at]
-                          : bf16_to_f32(reinterpret_cast<const unsigned short*>(g.gate)[at]);
-    v /= 1.f + expf(-z);
-  }
+  if (g.gate) v *= gate_of(g, tok * g.gate_stride + (g.per_head ? head : col));
   const size_t to = tok * g.out_stride + col;
   if (g.f32) reinterpret_cast<float*>(g.out)[to] = v;
   else reinterpret_cast<unsigned short*>(g.out)[to] = f32_to_bf16(v);
+}
+
+// 4 neighbouring values, c a multiple of 4
+__device__ __forceinline__ void write_gated4(const GatedOut& g, const AttnShape& a, size_t tok, int head, int c, f32x4 v) {
+  const int col = head * a.dv + c;
+  if (g.gate) {
+    const size_t at = tok * g.gate_stride + (g.per_head ? head : col);
+    if (g.per_head) {
+      v *= gate_of(g, at);
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[e] *= gate_of(g, at + e);
+    }
+  }
+  const size_t to = tok * g.out_stride + col;
+  if (!g.by4) {
+#pragma unroll
+    for (int e = 0; e < 4; ++e) {
+      if (g.f32) reinterpret_cast<float*>(g.out)[to + e] = v[e];
+      else reinterpret_cast<unsigned short*>(g.out)[to + e] = f32_to_bf16(v[e]);
+    }
+  } else if (g.f32) {
+    *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(g.out) + to) = v;
+  } else {
+    *reinterpret_cast<v4s*>(reinterpret_cast<unsigned short*>(g.out) + to) =
+        v4s{(short)f32_to_bf16(v[0]), (short)f32_to_bf16(v[1]), (short)f32_to_bf16(v[2]), (short)f32_to_bf16(v[3])};
+  }
 }
 
 __device__ __forceinline__ void wave_lds_fence() {
@@ -82,92 +111,169 @@ __device__ __forceinline__ void wave_lds_fence() {
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
+// A tile's scores are computed as K Q^T and its result as V^T P^T: a lane then holds
+// keys (or value dimensions) of ONE query row, the row of its column lane&15, so that a
+// softmax's maximum and sum take two exchanges between lanes, and the weights are the
+// next product's operand as they are. In the C layout, register r of block nb is key
+// nb*16 + hi*4 + r; as operand of a product over 32 keys, registers 0-3 of two blocks
+// are its 8 elements, so the values are read in the same order (load_values).
+
 // factors of a raw score, in log2 units
 struct ScoreScale {
-  float in;   // SOFTMAX, SIGMOID: scale; CAPPED: 2 scale / cap
-  float cap;  // CAPPED
+  float in;      // SOFTMAX, SIGMOID: scale; CAPPED: 2 scale / cap
+  float cap;     // CAPPED
+  bool bounded;  // weights need no maximum: the cap keeps them and their sums in range
 };
 
 template <int KIND>
 __device__ __forceinline__ ScoreScale score_scale(const AttnShape& a) {
-  if (KIND == CAPPED) return ScoreScale{2.f * a.scale / a.cap * LOG2E, a.cap * LOG2E};
-  return ScoreScale{a.scale * LOG2E, 0.f};
+  if (KIND == CAPPED) return ScoreScale{2.f * a.scale / a.cap * LOG2E, a.cap * LOG2E, a.cap * LOG2E <= 80.f};
+  return ScoreScale{a.scale * LOG2E, 0.f, KIND == SIGMOID};
 }
 
-// Scores of a 16-row x 32-key tile (C layout: key col of block nb, rows hi*4+r)
-// -> weights. A softmax updates the running maximum and this lane's share of the
-// sum; sigmoid weights need neither.
-struct WeightRows {
-  float m[4], l[4], lin[4];  // lin in log2 units: SOFTMAX: slope per distance; SIGMOID: bias
-};
-struct SeenRows {
-  int pos[4], lo[4];  // the row sees keys in [lo, pos]
+__device__ __forceinline__ float first_maximum(const ScoreScale& k) { return k.bounded ? 0.f : NEG_SENTINEL; }
+
+// the keys that a lane's query row sees: [lo, pos], none if pos < 0
+struct SeenRow {
+  int pos, lo;
 };
 
-template <int KIND>
-__device__ __forceinline__ void weigh_tile(
-    WeightRows& w, const SeenRows& n, const f32x4* s_acc, int j0, int col, int j_end, bool interior, ScoreScale k,
-    float corr[4], float p[2][4]) {
-#pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    float s[2];
-#pragma unroll
-    for (int nb = 0; nb < 2; ++nb) {
-      if (KIND == SOFTMAX) {
-        s[nb] = s_acc[nb][r] * k.in - w.lin[r] * (float)(n.pos[r] - (j0 + nb * 16 + col));
-      } else if (KIND == CAPPED) {  // tanh(x) = 1 - 2 / (exp(2x) + 1)
-        s[nb] = fmaf(-2.f * k.cap, __builtin_amdgcn_rcpf(exp2f(fminf(s_acc[nb][r] * k.in, 80.f)) + 1.f), k.cap);
-      } else {
-        s[nb] = fmaf(s_acc[nb][r], k.in, w.lin[r]);
-      }
-    }
-    if (KIND == SIGMOID) {
-#pragma unroll
-      for (int nb = 0; nb < 2; ++nb) p[nb][r] = __builtin_amdgcn_rcpf(1.f + exp2f(fminf(-s[nb], 100.f)));
-      if (!interior) {
-#pragma unroll
-        for (int nb = 0; nb < 2; ++nb) {
-          const int key = j0 + nb * 16 + col;
-          if (key >= j_end || key > n.pos[r] || key < n.lo[r]) p[nb][r] = 0.f;
-        }
-      }
-      continue;
-    }
-    // masking and the running max stay in separate loops (see prefill_attn.hip)
-    if (!interior) {
-#pragma unroll
-      for (int nb = 0; nb < 2; ++nb) {
-        const int key = j0 + nb * 16 + col;
-        if (key >= j_end || key > n.pos[r] || key < n.lo[r]) s[nb] = NEG_SENTINEL;
-      }
-    }
-    float mx = fmaxf(s[0], s[1]);
-#pragma unroll
-    for (int off = 8; off > 0; off >>= 1) mx = fmaxf(mx, __shfl_xor(mx, off, WAVE));
-    const float m_new = fmaxf(w.m[r], mx);
-    corr[r] = (w.m[r] <= NEG_THRESHOLD) ? 0.f : exp2f(w.m[r] - m_new);
-#pragma unroll
-    for (int nb = 0; nb < 2; ++nb) p[nb][r] = (s[nb] <= NEG_THRESHOLD) ? 0.f : exp2f(s[nb] - m_new);
-    w.l[r] = w.l[r] * corr[r] + (p[0][r] + p[1][r]);
-    w.m[r] = m_new;
-  }
-}
-
-// row of a weight in `lin`: head's slope or bias
+// in log2 units: SOFTMAX: slope per distance; SIGMOID: bias
 template <int KIND>
 __device__ __forceinline__ float linear_term(const AttnShape& a, int head) {
   if (KIND == SOFTMAX) return a.slopes ? a.slopes[head] * LOG2E : 0.f;
   return KIND == SIGMOID && a.bias ? a.bias[head] * LOG2E : 0.f;
 }
 
+// maximum and sum over the lanes of a query row
+__device__ __forceinline__ float row_max(float x) {
+  x = fmaxf(x, __shfl_xor(x, 16, WAVE));
+  return fmaxf(x, __shfl_xor(x, 32, WAVE));
+}
+__device__ __forceinline__ float row_sum(float x) {
+  x += __shfl_xor(x, 16, WAVE);
+  return x + __shfl_xor(x, 32, WAVE);
+}
+
+// Scores of a lane's row and NB blocks of 16 keys from j0 -> weights, in place.
+// m: the row's maximum so far; l: this lane's share of the sum. Returns whether m grew
+// in some row of the wave; what has been summed is then to be scaled by corr.
+template <int KIND, int NB>
+__device__ __forceinline__ bool weigh_tile(
+    f32x4* s, float& m, float& l, float lin, SeenRow n, int j0, int hi, int j_end, bool interior, ScoreScale k,
+    float& corr) {
+  const int first = j0 + hi * 4;  // key of register 0 in block 0
+  if (KIND == SIGMOID) {
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        s[nb][r] = __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(fminf(fmaf(s[nb][r], -k.in, -lin), 100.f)));
+    if (!interior) {
+#pragma unroll
+      for (int nb = 0; nb < NB; ++nb)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int key = first + nb * 16 + r;
+          if (key >= j_end || key > n.pos || key < n.lo) s[nb][r] = 0.f;
+        }
+    }
+    return false;
+  }
+  const float base = KIND == SOFTMAX ? lin * (float)(n.pos - first) : 0.f;
+#pragma unroll
+  for (int nb = 0; nb < NB; ++nb)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      if (KIND == SOFTMAX) {
+        s[nb][r] = fmaf(s[nb][r], k.in, fmaf(lin, (float)(nb * 16 + r), -base));
+      } else {  // tanh(x) = 1 - 2 / (exp(2x) + 1)
+        const float e = __builtin_amdgcn_exp2f(fminf(s[nb][r] * k.in, 80.f));
+        s[nb][r] = fmaf(-2.f * k.cap, __builtin_amdgcn_rcpf(e + 1.f), k.cap);
+      }
+    }
+  // masking and the maximum stay in separate loops (see prefill_attn.hip)
+  if (!interior) {
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = first + nb * 16 + r;
+        if (key >= j_end || key > n.pos || key < n.lo) s[nb][r] = NEG_SENTINEL;
+      }
+  }
+  bool grew = false;
+  corr = 1.f;
+  if (KIND != CAPPED || !k.bounded) {
+    float mx = m;
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[nb][r]);
+    const float m_new = row_max(mx);
+    grew = __any(m_new > m);
+    if (grew) {
+      corr = m <= NEG_THRESHOLD ? 0.f : exp2f(m - m_new);
+      l *= corr;
+      m = m_new;
+    }
+  }
+  const float top = m <= NEG_THRESHOLD ? 0.f : m;  // nothing seen yet: weights of 0
+  float sum = 0.f;
+#pragma unroll
+  for (int nb = 0; nb < NB; ++nb)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      s[nb][r] = __builtin_amdgcn_exp2f(s[nb][r] - top);
+      sum += s[nb][r];
+    }
+  l += sum;
+  return grew;
+}
+
+// weights of 32 keys as an operand
+__device__ __forceinline__ bf16x8 weight_operand(const f32x4& a, const f32x4& b) {
+  using f32x8 = __attribute__((ext_vector_type(8))) float;
+  using nbf16x8 = __attribute__((ext_vector_type(8))) __bf16;
+  const f32x8 v = {a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+  return __builtin_bit_cast(bf16x8, __builtin_convertvector(v, nbf16x8));
+}
+
+// Values of one dimension per lane (column lane&15 of a block) in the order of
+// weight_operand, by two transposing LDS loads. p: row hi*4 + (lane&15)/4, column
+// 4*(lane&3) of the block, in the tile's rows of these 32 keys.
+__device__ __forceinline__ bf16x8 load_values(const unsigned short* p, int row_elems) {
+  using lds_v4s = __attribute__((address_space(3))) v4s;
+  const v4s a = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s*)p);
+  const v4s b = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4s*)(p + 16 * row_elems));
+  return bf16x8{a[0], a[1], a[2], a[3], b[0], b[1], b[2], b[3]};
+}
+
 // ------------------------------------------------------------ MFMA kernel
+
+// The token run (x) and the heads (y) of a workgroup. Workgroups are dealt to the 8
+// chiplets in turn: each chiplet takes heads of its own, whose keys and values then stay
+// in its cache. Late rows see most and come first; every second 32 are turned round, so
+// that a compute unit (there are 32 on a chiplet) that gets two gets a long and a short one.
+__device__ __forceinline__ int2 spread_tiles(int nx, int ny) {
+  unsigned at = blockIdx.y * nx + blockIdx.x;
+  if (ny % 8 == 0) {
+    const unsigned per = ny / 8;
+    unsigned i = at / 8;
+    if (i / 32 * 32 + 32 <= nx * per && (i & 32)) i = i / 32 * 32 + 31 - i % 32;
+    return int2{(int)(nx - 1 - i / per), (int)((at & 7) * per + i % per)};
+  }
+  if (nx * ny % 8 == 0) at = (at & 7) * (nx * ny / 8) + at / 8;
+  return int2{(int)(nx - 1 - at % nx), (int)(at / nx)};
+}
 
 // RC: 32-wide chunks of the key size, VB: 16-wide blocks of the value size, at
 // least as many as there are: tiles are filled up with zeros, so that no branch
-// stands between products. A wave holds all maps of its rows.
-// Grid: (token runs, kv heads x groups of 64 rows, key splits).
-template <int KIND, int MAPS, int RC, int VB>
-__global__ __launch_bounds__(256) void paged_attn_kernel(
+// stands between products. A wave holds all maps of its QB blocks of 16 rows; a tile
+// has KT keys and lies in one page.
+// Grid: (token runs, kv heads x groups of 64 QB rows, key splits).
+template <int KIND, int MAPS, int RC, int VB, int QB, int KT>
+__global__ __launch_bounds__(256, QB) void paged_attn_kernel(
     const unsigned short* __restrict__ q,      // [T, H, MAPS, dk]
     const unsigned short* __restrict__ cache,  // [pages, PAGE, G * (MAPS * dk + dv)]
     GatedOut g,                                // n_splits == 1
@@ -175,81 +281,69 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
     float* __restrict__ part_ml,               // [n_splits, T*H, MAPS, 2]
     const int* __restrict__ tiles,             // [n, 2] first token, token count
     PagedRows b, AttnShape a, int total_tokens, int n_splits) {
+  constexpr int ROWS = 64 * QB, NB = KT / 16;
   constexpr int KROW = MAPS * RC * 32 + TPAD, VROW = VB * 16 + TPAD;
   constexpr int K8 = MAPS * RC * 4, V8 = VB * 2;             // 16-byte groups of a row
-  constexpr int K_LOADS = KVT * K8, LOADS = KVT * (K8 + V8);
+  constexpr int K_LOADS = KT * K8, LOADS = KT * (K8 + V8);
   constexpr int NLD = (LOADS + 255) / 256;                   // per thread
-  // Workgroups are dealt to the 8 chiplets in turn: each chiplet takes heads of its own,
-  // whose keys and values then stay in its cache, and late rows, which see most, first.
-  int bx = blockIdx.x, by = blockIdx.y;
-  if ((gridDim.x * gridDim.y & 7) == 0) {
-    const unsigned at = by * gridDim.x + bx, mine = (at & 7) * (gridDim.x * gridDim.y / 8) + at / 8;
-    by = mine / gridDim.x;
-    bx = mine - by * gridDim.x;
-  }
-  bx = gridDim.x - 1 - bx;
+  const int2 own = spread_tiles(gridDim.x, gridDim.y);
+  const int bx = own.x, by = own.y;
   const int tok0 = tiles[2 * bx];
   const int ntok = tiles[2 * bx + 1];
   const int group = a.heads / a.kv_heads;
   const int rows = ntok * group;
   const int kvh = by % a.kv_heads;
-  const int g0 = by / a.kv_heads * 64;
+  const int g0 = by / a.kv_heads * ROWS;
   if (g0 >= rows) return;  // uniform over the workgroup
-  const int g1 = min(g0 + 64, rows);
+  const int g1 = min(g0 + ROWS, rows);
 
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid & (WAVE - 1);
   const int col = lane & 15, hi = lane >> 4;
-  const int r0 = g0 + wave * 16;
+  const int r0 = g0 + wave * 16 * QB;
 
   extern __shared__ unsigned short smem[];
-  unsigned short* p_lds = smem + 2 * KVT * (KROW + VROW) + wave * MAPS * 16 * (KVT + 8);
 
   const int seq = b.owner[tok0];
   const int first_pos = b.pos[tok0 + g0 / group];
   const int last_pos = b.pos[tok0 + (g1 - 1) / group];
-  const int key_lo = max(0, first_key(a, first_pos)) / KVT * KVT;
+  const int key_lo = max(0, first_key(a, first_pos)) / KT * KT;
   const int key_hi = last_pos + 1;
-  const int n_tiles = (key_hi - key_lo + KVT - 1) / KVT;
+  const int n_tiles = (key_hi - key_lo + KT - 1) / KT;
   const int per_split = (n_tiles + n_splits - 1) / n_splits;
-  const int j_begin = key_lo + blockIdx.z * per_split * KVT;
-  const int j_end = min(key_hi, j_begin + per_split * KVT);
+  const int j_begin = key_lo + blockIdx.z * per_split * KT;
+  const int j_end = min(key_hi, j_begin + per_split * KT);
 
-  bf16x8 q_frag[MAPS][RC];
-  {
-    const int row = r0 + col;
-    const size_t at = ((size_t)(tok0 + row / group) * a.heads + kvh * group + row % group) * MAPS * a.dk;
+  const ScoreScale scale = score_scale<KIND>(a);
+  bf16x8 q_frag[QB][MAPS][RC];
+  f32x4 acc_o[QB][MAPS][VB];
+  float m[QB][MAPS], l[QB][MAPS], lin[QB];
+  SeenRow seen[QB];
 #pragma unroll
-    for (int u = 0; u < MAPS; ++u)
-#pragma unroll
-      for (int kc = 0; kc < RC; ++kc)
-        q_frag[u][kc] = row < rows && kc * 32 < a.dk
-                            ? *reinterpret_cast<const bf16x8*>(q + at + u * a.dk + kc * 32 + hi * 8)
-                            : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
-  }
-
-  f32x4 acc_o[MAPS][VB];
-  WeightRows w[MAPS];
-  SeenRows seen;
-#pragma unroll
-  for (int u = 0; u < MAPS; ++u)
-#pragma unroll
-    for (int d = 0; d < VB; ++d) acc_o[u][d] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const int row = r0 + hi * 4 + r;
-    seen.pos[r] = row < rows ? b.pos[tok0 + row / group] : -1;  // -1: sees nothing
-    seen.lo[r] = row < rows ? first_key(a, seen.pos[r]) : 0;
+  for (int i = 0; i < QB; ++i) {
+    const int row = r0 + i * 16 + col;
+    const bool live = row < rows;
+    const int head = live ? kvh * group + row % group : 0;
+    const size_t at = ((size_t)(tok0 + (live ? row / group : 0)) * a.heads + head) * MAPS * a.dk;
+    seen[i].pos = live ? b.pos[tok0 + row / group] : -1;  // -1: sees nothing
+    seen[i].lo = live ? first_key(a, seen[i].pos) : 0;
+    lin[i] = live ? linear_term<KIND>(a, head) : 0.f;
 #pragma unroll
     for (int u = 0; u < MAPS; ++u) {
-      w[u].m[r] = NEG_SENTINEL;
-      w[u].l[r] = 0.f;
-      w[u].lin[r] = row < rows ? linear_term<KIND>(a, kvh * group + row % group) : 0.f;
+      m[i][u] = first_maximum(scale);
+      l[i][u] = 0.f;
+#pragma unroll
+      for (int kc = 0; kc < RC; ++kc)
+        q_frag[i][u][kc] = live && kc * 32 < a.dk
+                               ? *reinterpret_cast<const bf16x8*>(q + at + u * a.dk + kc * 32 + hi * 8)
+                               : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
+#pragma unroll
+      for (int d = 0; d < VB; ++d) acc_o[i][u][d] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
   }
   // keys that every row of this wave sees: [all_lo, all_hi]; those that some row sees: [any_lo, any_hi]
-  const bool full_wave = r0 + 16 <= rows;
+  const bool full_wave = r0 + 16 * QB <= rows;
   const int wave_first = r0 < rows ? b.pos[tok0 + r0 / group] : -1;
-  const int wave_last = r0 < rows ? b.pos[tok0 + (min(r0 + 16, rows) - 1) / group] : -1;
+  const int wave_last = r0 < rows ? b.pos[tok0 + (min(r0 + 16 * QB, rows) - 1) / group] : -1;
   const int all_hi = full_wave ? wave_first : -1;
   const int all_lo = full_wave ? first_key(a, wave_last) : 0;
   const int any_hi = wave_last, any_lo = r0 < rows ? first_key(a, wave_first) : 0;
@@ -282,80 +376,78 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
         const bool is_v = idx >= K_LOADS;
         const int row = is_v ? (idx - K_LOADS) / V8 : idx / K8;
         const int c8 = (is_v ? (idx - K_LOADS) % V8 : idx % K8) * 8;
-        unsigned short* dst = is_v ? buf + KVT * KROW + row * VROW + c8 : buf + row * KROW + c8;
+        unsigned short* dst = is_v ? buf + KT * KROW + row * VROW + c8 : buf + row * KROW + c8;
         *reinterpret_cast<bf16x8*>(dst) = next[i];
       }
     }
   };
 
-  const ScoreScale scale = score_scale<KIND>(a);
   if (j_begin < j_end) {
     fetch(j_begin);
     stage(smem);
   }
   __syncthreads();
   int which = 0;
-  for (int j0 = j_begin; j0 < j_end; j0 += KVT, which ^= 1) {
-    const unsigned short* k_lds = smem + which * KVT * (KROW + VROW);
-    const bool more = j0 + KVT < j_end;
-    if (more) fetch(j0 + KVT);
-    if (j0 <= any_hi && j0 + KVT > any_lo) {  // uniform over the wave
-      const bool interior = j0 >= all_lo && j0 + KVT - 1 <= all_hi && j0 + KVT <= j_end;
-      float corr[MAPS][4];
+  for (int j0 = j_begin; j0 < j_end; j0 += KT, which ^= 1) {
+    const unsigned short* k_lds = smem + which * KT * (KROW + VROW);
+    const bool more = j0 + KT < j_end;
+    if (more) fetch(j0 + KT);
+    if (j0 <= any_hi && j0 + KT > any_lo) {  // uniform over the wave
+      const bool interior = j0 >= all_lo && j0 + KT - 1 <= all_hi && j0 + KT <= j_end;
+      bf16x8 p_frag[QB][MAPS][NB / 2];
 #pragma unroll
       for (int u = 0; u < MAPS; ++u) {
-        f32x4 s_acc[2];
+        f32x4 s[QB][NB];
 #pragma unroll
-        for (int nb = 0; nb < 2; ++nb) {
-          s_acc[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int nb = 0; nb < NB; ++nb) {
+#pragma unroll
+          for (int i = 0; i < QB; ++i) s[i][nb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int kc = 0; kc < RC; ++kc) {
             const bf16x8 kt =
                 *reinterpret_cast<const bf16x8*>(&k_lds[(nb * 16 + col) * KROW + (u * RC + kc) * 32 + hi * 8]);
-            s_acc[nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q_frag[u][kc], kt, s_acc[nb], 0, 0, 0);
+#pragma unroll
+            for (int i = 0; i < QB; ++i)
+              s[i][nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt, q_frag[i][u][kc], s[i][nb], 0, 0, 0);
           }
         }
-        float p[2][4];
-        weigh_tile<KIND>(w[u], seen, s_acc, j0, col, j_end, interior, scale, corr[u], p);
-        // P to A-fragment layout through this wave's own LDS
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
+        for (int i = 0; i < QB; ++i) {
+          float corr;
+          if (weigh_tile<KIND, NB>(s[i], m[i][u], l[i][u], lin[i], seen[i], j0, hi, j_end, interior, scale, corr)) {
 #pragma unroll
-          for (int nb = 0; nb < 2; ++nb)
-            p_lds[(u * 16 + hi * 4 + r) * (KVT + 8) + nb * 16 + col] = f32_to_bf16(p[nb][r]);
-      }
-      wave_lds_fence();
-      bf16x8 p_frag[MAPS];
-#pragma unroll
-      for (int u = 0; u < MAPS; ++u)
-        p_frag[u] = *reinterpret_cast<const bf16x8*>(&p_lds[(u * 16 + col) * (KVT + 8) + hi * 8]);
-      const unsigned short* v_lds = k_lds + KVT * KROW + (hi * 8 + col / 4) * VROW + (col & 3) * 4;
-#pragma unroll
-      for (int d = 0; d < VB; ++d) {
-        const bf16x8 vt = load_keys(v_lds + d * 16, VROW);
-#pragma unroll
-        for (int u = 0; u < MAPS; ++u) {
-          if (KIND != SIGMOID) {
-#pragma unroll
-            for (int r = 0; r < 4; ++r) acc_o[u][d][r] *= corr[u][r];
+            for (int d = 0; d < VB; ++d) acc_o[i][u][d] *= corr;
           }
-          acc_o[u][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p_frag[u], vt, acc_o[u][d], 0, 0, 0);
+#pragma unroll
+          for (int ks = 0; ks < NB / 2; ++ks) p_frag[i][u][ks] = weight_operand(s[i][2 * ks], s[i][2 * ks + 1]);
         }
       }
+      const unsigned short* v_lds = k_lds + KT * KROW + (hi * 4 + col / 4) * VROW + (col & 3) * 4;
+#pragma unroll
+      for (int d = 0; d < VB; ++d)
+#pragma unroll
+        for (int ks = 0; ks < NB / 2; ++ks) {
+          const bf16x8 vt = load_values(v_lds + ks * 32 * VROW + d * 16, VROW);
+#pragma unroll
+          for (int i = 0; i < QB; ++i)
+#pragma unroll
+            for (int u = 0; u < MAPS; ++u)
+              acc_o[i][u][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, p_frag[i][u][ks], acc_o[i][u][d], 0, 0, 0);
+        }
     }
-    if (more) stage(smem + (which ^ 1) * KVT * (KROW + VROW));
+    if (more) stage(smem + (which ^ 1) * KT * (KROW + VROW));
     __syncthreads();
   }
 
 #pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    float l[MAPS];
-#pragma unroll
-    for (int u = 0; u < MAPS; ++u) l[u] = KIND == SIGMOID ? 1.f : group16_reduce_sum(w[u].l[r]);
-    const int row = r0 + hi * 4 + r;
+  for (int i = 0; i < QB; ++i) {
+    const int row = r0 + i * 16 + col;
     const bool live = row < rows;
     const size_t tok = tok0 + (live ? row / group : 0);
     const int head = kvh * group + (live ? row % group : 0);
+    float inv[MAPS];
+#pragma unroll
+    for (int u = 0; u < MAPS; ++u) inv[u] = KIND == SIGMOID ? 1.f : row_sum(l[i][u]);
     if (n_splits > 1) {
       if (!live) continue;
       const size_t at = (((size_t)blockIdx.z * total_tokens + tok) * a.heads + head) * MAPS;
@@ -363,39 +455,42 @@ __global__ __launch_bounds__(256) void paged_attn_kernel(
       for (int u = 0; u < MAPS; ++u) {
 #pragma unroll
         for (int d = 0; d < VB; ++d)
-          if (d * 16 < a.dv) part_o[(at + u) * a.dv + d * 16 + col] = acc_o[u][d][r];
-        if (KIND != SIGMOID && col == 0) {
-          part_ml[(at + u) * 2] = w[u].m[r];
-          part_ml[(at + u) * 2 + 1] = l[u];
+          if (d * 16 < a.dv) *reinterpret_cast<f32x4*>(part_o + (at + u) * a.dv + d * 16 + hi * 4) = acc_o[i][u][d];
+        if (KIND != SIGMOID && hi == 0) {
+          part_ml[(at + u) * 2] = m[i][u];
+          part_ml[(at + u) * 2 + 1] = inv[u];
         }
       }
       continue;
     }
-    float inv[MAPS];
+    if (KIND != SIGMOID) {
 #pragma unroll
-    for (int u = 0; u < MAPS; ++u) {
-      float up = 1.f;
-      if (KIND != SIGMOID && a.sink) {
-        const float z = a.sink[head] * LOG2E, m = fmaxf(w[u].m[r], z);
-        up = exp2f(w[u].m[r] - m);
-        l[u] = l[u] * up + exp2f(z - m);
+      for (int u = 0; u < MAPS; ++u) {
+        float up = 1.f, sum = inv[u];
+        if (a.sink) {
+          const float z = a.sink[head] * LOG2E, top = fmaxf(m[i][u], z);
+          up = exp2f(m[i][u] - top);
+          sum = sum * up + exp2f(z - top);
+        }
+        inv[u] = sum > 0.f ? up / sum : 0.f;
       }
-      inv[u] = l[u] > 0.f ? up / l[u] : 0.f;
     }
     if (MAPS == 2) {
       float ss = 0.f;
 #pragma unroll
-      for (int d = 0; d < VB; ++d) {
-        const float o = acc_o[0][d][r] * inv[0] - a.share * (acc_o[MAPS - 1][d][r] * inv[MAPS - 1]);
-        acc_o[0][d][r] = o;
-        ss = fmaf(o, o, ss);  // padding is zero
-      }
-      inv[0] = a.factor / sqrtf(group16_reduce_sum(ss) / a.vdim + a.eps);
+      for (int d = 0; d < VB; ++d)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const float o = acc_o[i][0][d][r] * inv[0] - a.share * (acc_o[i][MAPS - 1][d][r] * inv[MAPS - 1]);
+          acc_o[i][0][d][r] = o;
+          ss = fmaf(o, o, ss);  // padding is zero
+        }
+      inv[0] = a.factor / sqrtf(row_sum(ss) / a.vdim + a.eps);
     }
     if (!live) continue;
 #pragma unroll
     for (int d = 0; d < VB; ++d)
-      if (d * 16 < a.dv) write_gated(g, a, tok, head, d * 16 + col, acc_o[0][d][r] * inv[0]);
+      if (d * 16 < a.dv) write_gated4(g, a, tok, head, d * 16 + hi * 4, acc_o[i][0][d] * inv[0]);
   }
 }
 
@@ -416,8 +511,7 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
   const int tid = threadIdx.x, wave = tid / WAVE, lane = tid & (WAVE - 1);
   const int col = lane & 15, hi = lane >> 4;
   extern __shared__ unsigned short smem[];
-  unsigned short* v_tile = smem + wave * (KVT * VROW + MAPS * 16 * (KVT + 8));
-  unsigned short* p_lds = v_tile + KVT * VROW;
+  unsigned short* v_tile = smem + wave * KVT * VROW;
 
   const int seq = b.owner[tok], pos = b.pos[tok];
   const int lo = first_key(a, pos), key_lo = max(0, lo) / KVT * KVT;
@@ -426,36 +520,27 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
   const int j_begin = key_lo + blockIdx.z * per_split * KVT;
   const int j_end = min(pos + 1, j_begin + per_split * KVT);
 
+  const ScoreScale scale = score_scale<KIND>(a);
+  const bool live = col < group;
+  const SeenRow seen{live ? pos : -1, lo};
+  const float lin = live ? linear_term<KIND>(a, kvh * group + col) : 0.f;
   bf16x8 q_frag[MAPS][RC];
+  f32x4 acc_o[MAPS][VB];
+  float m[MAPS], l[MAPS];
   const size_t q_at = ((size_t)tok * a.heads + kvh * group + col) * MAPS * a.dk;
 #pragma unroll
-  for (int u = 0; u < MAPS; ++u)
+  for (int u = 0; u < MAPS; ++u) {
+    m[u] = first_maximum(scale);
+    l[u] = 0.f;
 #pragma unroll
     for (int kc = 0; kc < RC; ++kc)
-      q_frag[u][kc] = col < group && kc * 32 < a.dk
+      q_frag[u][kc] = live && kc * 32 < a.dk
                           ? *reinterpret_cast<const bf16x8*>(q + q_at + u * a.dk + kc * 32 + hi * 8)
                           : bf16x8{0, 0, 0, 0, 0, 0, 0, 0};
-  f32x4 acc_o[MAPS][VB];
-  WeightRows w[MAPS];
-  SeenRows seen;
-#pragma unroll
-  for (int u = 0; u < MAPS; ++u)
 #pragma unroll
     for (int d = 0; d < VB; ++d) acc_o[u][d] = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-  for (int r = 0; r < 4; ++r) {
-    const int row = hi * 4 + r;
-    seen.pos[r] = row < group ? pos : -1;
-    seen.lo[r] = lo;
-#pragma unroll
-    for (int u = 0; u < MAPS; ++u) {
-      w[u].m[r] = NEG_SENTINEL;
-      w[u].l[r] = 0.f;
-      w[u].lin[r] = row < group ? linear_term<KIND>(a, kvh * group + row) : 0.f;
-    }
   }
   const int width = a.kv_heads * (MAPS * a.dk + a.dv);
-  const ScoreScale scale = score_scale<KIND>(a);
   for (int j0 = j_begin + wave * KVT; j0 < j_end; j0 += 4 * KVT) {
     const long at = cache_row(b, seq, j0);
     bf16x8 vals[NLD], kt[MAPS][2][RC];
@@ -479,18 +564,23 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
         vals[i] = *reinterpret_cast<const bf16x8*>(
             cache + ((size_t)at + row) * width + a.kv_heads * MAPS * a.dk + kvh * a.dv + c8);
     }
-    float corr[MAPS][4], p[MAPS][2][4];
+    bf16x8 p_frag[MAPS];
 #pragma unroll
     for (int u = 0; u < MAPS; ++u) {
-      f32x4 s_acc[2];
+      f32x4 s[2];
 #pragma unroll
       for (int nb = 0; nb < 2; ++nb) {
-        s_acc[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
+        s[nb] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int kc = 0; kc < RC; ++kc)
-          s_acc[nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(q_frag[u][kc], kt[u][nb][kc], s_acc[nb], 0, 0, 0);
+          s[nb] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kt[u][nb][kc], q_frag[u][kc], s[nb], 0, 0, 0);
       }
-      weigh_tile<KIND>(w[u], seen, s_acc, j0, col, j_end, false, scale, corr[u], p[u]);
+      float corr;
+      if (weigh_tile<KIND, 2>(s, m[u], l[u], lin, seen, j0, hi, j_end, false, scale, corr)) {
+#pragma unroll
+        for (int d = 0; d < VB; ++d) acc_o[u][d] *= corr;
+      }
+      p_frag[u] = weight_operand(s[0], s[1]);
     }
     wave_lds_fence();  // the last tile's reads are done
 #pragma unroll
@@ -498,30 +588,14 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
       const int idx = lane + i * WAVE, row = idx / V8, c8 = idx % V8 * 8;
       *reinterpret_cast<bf16x8*>(&v_tile[row * VROW + c8]) = vals[i];
     }
-#pragma unroll
-    for (int u = 0; u < MAPS; ++u)
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-#pragma unroll
-        for (int nb = 0; nb < 2; ++nb)
-          p_lds[(u * 16 + hi * 4 + r) * (KVT + 8) + nb * 16 + col] = f32_to_bf16(p[u][nb][r]);
     wave_lds_fence();
-    bf16x8 p_frag[MAPS];
-#pragma unroll
-    for (int u = 0; u < MAPS; ++u)
-      p_frag[u] = *reinterpret_cast<const bf16x8*>(&p_lds[(u * 16 + col) * (KVT + 8) + hi * 8]);
-    const unsigned short* v_lds = v_tile + (hi * 8 + col / 4) * VROW + (col & 3) * 4;
+    const unsigned short* v_lds = v_tile + (hi * 4 + col / 4) * VROW + (col & 3) * 4;
 #pragma unroll
     for (int d = 0; d < VB; ++d) {
-      const bf16x8 vt = load_keys(v_lds + d * 16, VROW);
+      const bf16x8 vt = load_values(v_lds + d * 16, VROW);
 #pragma unroll
-      for (int u = 0; u < MAPS; ++u) {
-        if (KIND != SIGMOID) {
-#pragma unroll
-          for (int r = 0; r < 4; ++r) acc_o[u][d][r] *= corr[u][r];
-        }
-        acc_o[u][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(p_frag[u], vt, acc_o[u][d], 0, 0, 0);
-      }
+      for (int u = 0; u < MAPS; ++u)
+        acc_o[u][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vt, p_frag[u], acc_o[u][d], 0, 0, 0);
     }
   }
   // merge the waves: [MAPS][4][16] maxima and sums, then [MAPS][4][group][dv] weighted sums
@@ -529,58 +603,56 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
   float* ml = reinterpret_cast<float*>(smem);   // [MAPS][4][16][2]
   float* os = ml + MAPS * 4 * 16 * 2;           // [MAPS][4][group][dv]
 #pragma unroll
-  for (int u = 0; u < MAPS; ++u)
-#pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float l = KIND == SIGMOID ? 1.f : group16_reduce_sum(w[u].l[r]);
-      const int row = hi * 4 + r;
-      if (row >= group) continue;
-      if (col == 0) {
-        ml[((u * 4 + wave) * 16 + row) * 2] = w[u].m[r];
-        ml[((u * 4 + wave) * 16 + row) * 2 + 1] = l;
-      }
-#pragma unroll
-      for (int d = 0; d < VB; ++d)
-        if (d * 16 < a.dv) os[((u * 4 + wave) * group + row) * a.dv + d * 16 + col] = acc_o[u][d][r];
+  for (int u = 0; u < MAPS; ++u) {
+    const float sum = KIND == SIGMOID ? 1.f : row_sum(l[u]);
+    if (!live) continue;
+    if (hi == 0) {
+      ml[((u * 4 + wave) * 16 + col) * 2] = m[u];
+      ml[((u * 4 + wave) * 16 + col) * 2 + 1] = sum;
     }
+#pragma unroll
+    for (int d = 0; d < VB; ++d)
+      if (d * 16 < a.dv)
+        *reinterpret_cast<f32x4*>(os + ((u * 4 + wave) * group + col) * a.dv + d * 16 + hi * 4) = acc_o[u][d];
+  }
   __syncthreads();
   for (int i = tid; i < MAPS * group * a.dv; i += 256) {
     const int u = MAPS == 1 ? 0 : i / (group * a.dv), in = i - u * group * a.dv;
     const int row = in / a.dv, c = in - row * a.dv, head = kvh * group + row;
     const float* mlu = ml + u * 4 * 16 * 2;
     const float* osu = os + u * 4 * group * a.dv;
-    float l = 0.f, o = 0.f, m = 0.f;
+    float sum = 0.f, o = 0.f, top = 0.f;
     if (KIND == SIGMOID) {
 #pragma unroll
       for (int v = 0; v < 4; ++v) o += osu[(v * group + row) * a.dv + c];
     } else {
-      m = NEG_SENTINEL;
+      top = NEG_SENTINEL;
 #pragma unroll
-      for (int v = 0; v < 4; ++v) m = fmaxf(m, mlu[(v * 16 + row) * 2]);
+      for (int v = 0; v < 4; ++v) top = fmaxf(top, mlu[(v * 16 + row) * 2]);
     }
-    const float top = m;
+    const float own = top;
     if (KIND != SIGMOID) {
-      if (MAPS == 1 && n_splits == 1 && a.sink) m = fmaxf(m, a.sink[head] * LOG2E);
+      if (MAPS == 1 && n_splits == 1 && a.sink) top = fmaxf(top, a.sink[head] * LOG2E);
 #pragma unroll
       for (int v = 0; v < 4; ++v) {
-        const float mu = mlu[(v * 16 + row) * 2];
-        const float e = mu > NEG_THRESHOLD ? exp2f(mu - m) : 0.f;
-        l = fmaf(e, mlu[(v * 16 + row) * 2 + 1], l);
+        const float mv = mlu[(v * 16 + row) * 2];
+        const float e = mv > NEG_THRESHOLD ? exp2f(mv - top) : 0.f;
+        sum = fmaf(e, mlu[(v * 16 + row) * 2 + 1], sum);
         o = fmaf(e, osu[(v * group + row) * a.dv + c], o);
       }
     }
     if (MAPS == 1 && n_splits == 1) {
       if (KIND != SIGMOID) {
-        if (a.sink) l += exp2f(a.sink[head] * LOG2E - m);
-        o = l > 0.f ? o / l : 0.f;
+        if (a.sink) sum += exp2f(a.sink[head] * LOG2E - top);
+        o = sum > 0.f ? o / sum : 0.f;
       }
       write_gated(g, a, tok, head, c, o);
     } else {
       const size_t at = (((size_t)blockIdx.z * total_tokens + tok) * a.heads + head) * MAPS + u;
       part_o[at * a.dv + c] = o;
       if (KIND != SIGMOID && c == 0) {
-        part_ml[at * 2] = top;
-        part_ml[at * 2 + 1] = l;
+        part_ml[at * 2] = own;
+        part_ml[at * 2 + 1] = sum;
       }
     }
   }
@@ -766,7 +838,8 @@ static GatedOut gated_out(const torch::Tensor& out, const c10::optional<torch::T
                           const AttnShape& a) {
   const bool f32 = f32_or_bf16(out);
   TORCH_CHECK(out.dim() == 2 && out.stride(1) == 1 && out.size(0) == t && out.size(1) >= (long)a.heads * a.dv);
-  GatedOut g{out.data_ptr(), out.stride(0), nullptr, 0, false, f32};
+  const bool by4 = out.stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(out.data_ptr()) % 16 == 0;
+  GatedOut g{out.data_ptr(), out.stride(0), nullptr, 0, false, f32, by4};
   if (gate.has_value()) {
     TORCH_CHECK(gate->is_cuda() && gate->dim() == 2 && gate->stride(1) == 1 && gate->dtype() == out.dtype());
     g.per_head = gate->size(1) == a.heads;
@@ -786,24 +859,39 @@ static void allow_lds(K kernel, size_t lds) {
   TORCH_CHECK(e == hipSuccess, "LDS request refused: ", hipGetErrorString(e));
 }
 
+template <int KIND, int MAPS, int RC, int VB, int QB>
+static void launch_tiles(dim3 grid, const torch::Tensor& q, const torch::Tensor& cache, GatedOut g, float* po,
+                         float* pml, const int* tiles, PagedRows b, AttnShape a, int n_splits) {
+  constexpr int KT = MAPS * RC * 32 + VB * 16 <= 256 ? 64 : 32;
+  static_assert(PAGE % KT == 0, "a tile lies in one page");
+  const size_t lds = 2 * KT * (MAPS * RC * 32 + VB * 16 + 2 * TPAD) * 2;
+  allow_lds(&paged_attn_kernel<KIND, MAPS, RC, VB, QB, KT>, lds);
+  paged_attn_kernel<KIND, MAPS, RC, VB, QB, KT><<<grid, 256, lds, c10::hip::getCurrentHIPStream().stream()>>>(
+      BF16P(q), BF16P(cache), g, po, pml, tiles, b, a, (int)q.size(0), n_splits);
+}
+
+// blocks of 16 rows that a wave takes of `rows` rows of a token run: two share the reading of a tile
+template <int MAPS>
+static int row_blocks(int rows, int dk, int dv) {
+  return MAPS == 1 && rows >= 128 && dk <= 128 && dv <= 128 ? 2 : 1;
+}
+
 template <int KIND, int MAPS, int RC, int VB>
-static void launch_attn(bool decode, dim3 grid, const torch::Tensor& q, const torch::Tensor& cache, GatedOut g,
-                        float* po, float* pml, const int* tiles, PagedRows b, AttnShape a, int n_splits) {
-  auto stream = c10::hip::getCurrentHIPStream().stream();
-  const int t = q.size(0);
+static void launch_attn(bool decode, int blocks, dim3 grid, const torch::Tensor& q, const torch::Tensor& cache,
+                        GatedOut g, float* po, float* pml, const int* tiles, PagedRows b, AttnShape a, int n_splits) {
   if (decode) {
-    const size_t tile = 4 * (KVT * (VB * 16 + TPAD) + MAPS * 16 * (KVT + 8)) * 2;
+    const size_t tile = 4 * KVT * (VB * 16 + TPAD) * 2;
     const size_t merge = MAPS * (4 * 16 * 2 + 4 * (size_t)(a.heads / a.kv_heads) * a.dv) * 4;
     const size_t lds = std::max(tile, merge);
     allow_lds(&paged_attn_decode<KIND, MAPS, RC, VB>, lds);
-    paged_attn_decode<KIND, MAPS, RC, VB>
-        <<<grid, 256, lds, stream>>>(BF16P(q), BF16P(cache), g, po, pml, b, a, t, n_splits);
-  } else {
-    const size_t lds = (2 * KVT * (MAPS * RC * 32 + VB * 16 + 2 * TPAD) + 4 * MAPS * 16 * (KVT + 8)) * 2;
-    allow_lds(&paged_attn_kernel<KIND, MAPS, RC, VB>, lds);
-    paged_attn_kernel<KIND, MAPS, RC, VB>
-        <<<grid, 256, lds, stream>>>(BF16P(q), BF16P(cache), g, po, pml, tiles, b, a, t, n_splits);
+    paged_attn_decode<KIND, MAPS, RC, VB><<<grid, 256, lds, c10::hip::getCurrentHIPStream().stream()>>>(
+        BF16P(q), BF16P(cache), g, po, pml, b, a, (int)q.size(0), n_splits);
+    return;
   }
+  if constexpr (MAPS == 1 && RC <= 4 && VB <= 8) {
+    if (blocks == 2) return launch_tiles<KIND, MAPS, RC, VB, 2>(grid, q, cache, g, po, pml, tiles, b, a, n_splits);
+  }
+  launch_tiles<KIND, MAPS, RC, VB, 1>(grid, q, cache, g, po, pml, tiles, b, a, n_splits);
 }
 
 // q [T, H, dk] or [T, H, 2, dk] in the cache's dtype; tiles [n, 2] int32 runs of at most
@@ -834,7 +922,8 @@ static void run_attention(const torch::Tensor& q, const torch::Tensor& cache, co
   TORCH_CHECK(tiles.is_cuda() && tiles.dtype() == torch::kInt32 && tiles.is_contiguous() && tiles.dim() == 2);
   const int group = a.heads / a.kv_heads;
   const bool decode = run_tokens == 1 && group <= 16 && tiles.size(0) == t;
-  const int row_groups = ((int)run_tokens * group + 63) / 64;
+  const int blocks = decode ? 1 : row_blocks<MAPS>((int)run_tokens * group, a.dk, a.dv);
+  const int row_groups = ((int)run_tokens * group + 64 * blocks - 1) / (64 * blocks);
   dim3 grid(tiles.size(0), a.kv_heads * (decode ? 1 : row_groups), 1);
   int n_splits = (int)splits;
   if (n_splits <= 0) {
@@ -852,7 +941,7 @@ static void run_attention(const torch::Tensor& q, const torch::Tensor& cache, co
   float* po = parts ? part_o.data_ptr<float>() : nullptr;
   float* pml = parts ? part_ml.data_ptr<float>() : nullptr;
 #define PA(RC, VB) \
-  launch_attn<KIND, MAPS, RC, VB>(decode, grid, q, cache, g, po, pml, tiles.data_ptr<int>(), b, a, n_splits)
+  launch_attn<KIND, MAPS, RC, VB>(decode, blocks, grid, q, cache, g, po, pml, tiles.data_ptr<int>(), b, a, n_splits)
 #define PAV(RC)              \
   do {                       \
     if (a.dv <= 32) PA(RC, 2); \

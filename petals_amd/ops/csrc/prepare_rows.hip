@@ -279,6 +279,197 @@ __global__ __launch_bounds__(NT) void prepare_rows_kernel(
   }
 }
 
+// one workgroup per row
+template <typename T, int NT>
+__global__ __launch_bounds__(NT) void poly_kernel(
+    const T* __restrict__ y, int stride, float eps, PolyPart poly, T* __restrict__ act, long act_stride) {
+  const size_t t = blockIdx.x;
+  poly_row<T, NT>(y + t * stride + poly.at, poly, eps, act + t * act_stride);
+}
+
+// ------------------------------------------------------------ prompts' rows
+
+#define TILE_ROWS 4
+
+// columns c .. c+7 of TILE_ROWS rows from t behind the convolution, whose inputs all are rows of this step
+template <int TAPS>
+__device__ __forceinline__ void convolved_rows(
+    const unsigned short* __restrict__ y, int stride, const RowShape& s, const RowWeights& w, size_t t, int c,
+    float (&v)[TILE_ROWS][8]) {
+  constexpr int AHEAD = TAPS > 0 ? TAPS - 1 : 0;
+  Packed8<unsigned short> in[TILE_ROWS + AHEAD];
+#pragma unroll
+  for (int r = 0; r < TILE_ROWS + AHEAD; ++r) in[r].load(y + (t + r - AHEAD) * stride + c);
+  float bias[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  if (w.bias) load8(w.bias + c, bias);
+  if (TAPS == 0) {
+#pragma unroll
+    for (int r = 0; r < TILE_ROWS; ++r)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[r][e] = in[r][e] + bias[e];
+    return;
+  }
+#pragma unroll
+  for (int r = 0; r < TILE_ROWS; ++r)
+#pragma unroll
+    for (int e = 0; e < 8; ++e) v[r][e] = 0.f;
+#pragma unroll
+  for (int j = 0; j < TAPS; ++j) {
+    float f[8];
+    load8(w.conv + (size_t)j * s.columns() + c, f);
+#pragma unroll
+    for (int r = 0; r < TILE_ROWS; ++r)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[r][e] = fmaf(f[e], in[r + j][e] + bias[e], v[r][e]);
+  }
+}
+
+// As prepare_rows_kernel, for TILE_ROWS rows at once: weights and a row's inputs are read
+// once for all of them, and nothing but sums and angles leaves the registers. A thread has
+// two groups of 8 columns that are rotated with each other (or pass). Needs half % 8 == 0
+// and a part of at most 16 NT columns. Grid: (tiles, queries / keys / values).
+template <int TAPS, int NT>
+__global__ __launch_bounds__(NT) void prepare_tile_kernel(
+    const unsigned short* __restrict__ y, int stride, RowShape s, RowWeights w, ConvState st, Rotation rot,
+    float turn_factor, PagedRows b, unsigned short* __restrict__ q, unsigned short* __restrict__ cache, float eps,
+    int rows) {
+  constexpr int R = TILE_ROWS;
+  extern __shared__ __attribute__((aligned(16))) float table[];  // [R][2][half]
+  __shared__ float red[R][NT / WAVE];
+  const int tid = threadIdx.x, part = blockIdx.y, waves = blockDim.x / WAVE;
+  const int tile = (blockIdx.x & 7) * (gridDim.x >> 3) + (blockIdx.x >> 3);
+  const int t0 = tile * R, live = min(R, rows - t0);
+  if (live <= 0) return;
+  int p[R], seq[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    p[r] = b.pos[t0 + min(r, live - 1)];
+    seq[r] = b.owner[t0 + min(r, live - 1)];
+  }
+  const bool straight = live == R && seq[0] == seq[R - 1] &&
+                        (TAPS == 0 || (t0 >= TAPS - 1 && b.owner[max(t0 - TAPS + 1, 0)] == seq[0]));
+  auto columns = [&](int c, float (&v)[R][8]) {
+    if (straight) {
+      convolved_rows<TAPS>(y, stride, s, w, t0, c, v);
+      return;
+    }
+    float bias[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+    if (w.bias) load8(w.bias + c, bias);
+#pragma unroll
+    for (int r = 0; r < R; ++r) {  // rows at a sequence's edge
+      const int t = t0 + min(r, live - 1);
+      const float* ring = nullptr;
+      if (TAPS > 0) ring = st.inputs + (size_t)min(max(st.slot[seq[r]], 0), s.slots - 1) * TAPS * s.columns() + c;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[r][e] = 0.f;
+#pragma unroll 1
+      for (int ago = 0; ago < max(TAPS, 1) && ago <= p[r]; ++ago) {
+        float x[8], f[8];
+        if (ago <= t && b.owner[t - ago] == seq[r]) {
+          load8(y + (size_t)(t - ago) * stride + c, x);
+#pragma unroll
+          for (int e = 0; e < 8; ++e) x[e] += bias[e];
+        } else {
+          load8(ring + (size_t)((p[r] - ago) % max(TAPS, 1)) * s.columns(), x);
+        }
+        if (TAPS > 0) load8(w.conv + (size_t)(TAPS - 1 - ago) * s.columns() + c, f);
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[r][e] = TAPS > 0 ? fmaf(f[e], x[e], v[r][e]) : x[e];
+      }
+    }
+  };
+  const int width = s.nk + s.nv;
+  float v[2][R][8];
+  if (part == 2) {
+    for (int c = tid * 8; c < s.nv; c += blockDim.x * 8) {
+      columns(s.nq + s.nk + c, v[0]);
+#pragma unroll
+      for (int r = 0; r < R; ++r)
+        if (r < live) {
+          const long at = cache_row(b, seq[r], p[r]);
+          if (at >= 0) store8(cache + (size_t)at * width + s.nk + c, v[0][r]);
+        }
+    }
+    return;
+  }
+  const int n = part == 0 ? s.nq : s.nk, first = part == 0 ? 0 : s.nq, half = rot.turned / 2;
+  const bool busy = tid < n / 16;
+  const int head = tid / (s.dk / 16), unit = tid - head * (s.dk / 16);
+  const bool turns = unit < half / 8;
+  const int d0 = turns ? unit * 8 : 2 * half + (unit - half / 8) * 16;
+  const int c0 = head * s.dk + d0, c1 = c0 + (turns ? half : 8);
+  float ss[R];
+#pragma unroll
+  for (int r = 0; r < R; ++r) ss[r] = 0.f;
+  if (busy) {
+    columns(first + c0, v[0]);
+    columns(first + c1, v[1]);
+    if (w.norm) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i) {
+        float g[8];
+        load8(w.norm + first + (i ? c1 : c0), g);
+#pragma unroll
+        for (int r = 0; r < R; ++r)
+#pragma unroll
+          for (int e = 0; e < 8; ++e) {
+            ss[r] = fmaf(v[i][r][e], v[i][r][e], ss[r]);
+            v[i][r][e] *= g[e];
+          }
+      }
+    }
+  }
+  for (int i = tid; i < R * half; i += blockDim.x) {
+    const int r = i / half, d = i - r * half;
+    float si, co;
+    sin_cos((straight ? p[0] + r : b.pos[t0 + min(r, live - 1)]) * rot.quarters[d], si, co);
+    table[r * 2 * half + d] = co * turn_factor;
+    table[r * 2 * half + half + d] = si * turn_factor;
+  }
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    ss[r] = wave_reduce_sum(ss[r]);
+    if ((tid & (WAVE - 1)) == 0) red[r][tid / WAVE] = ss[r];
+  }
+  __syncthreads();
+  if (!busy) return;
+#pragma unroll
+  for (int r = 0; r < R; ++r) {
+    if (r >= live) break;
+    float inv = 1.f;
+    if (w.norm) {
+      float sum = 0.f;
+      for (int i = 0; i < waves; ++i) sum += red[r][i];
+      inv = 1.f / sqrtf(sum / (part == 0 ? s.q_size : s.k_size) + eps);
+    }
+    if (turns) {
+      float co[8], si[8];
+      load8(table + r * 2 * half + d0, co);
+      load8(table + r * 2 * half + half + d0, si);
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float x = v[0][r][e], z = v[1][r][e];
+        v[0][r][e] = x * co[e] - z * si[e];
+        v[1][r][e] = fmaf(z, co[e], x * si[e]);
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[i][r][e] *= inv;
+    unsigned short* dst;
+    if (part == 0) {
+      dst = q + (size_t)(t0 + r) * n;
+    } else {
+      const long at = cache_row(b, seq[r], p[r]);
+      if (at < 0) continue;
+      dst = cache + (size_t)at * width;
+    }
+    store8(dst + c0, v[0][r]);
+    store8(dst + c1, v[1][r]);
+  }
+}
+
 // Grid: (sequences, groups of 2048 columns)
 template <typename TY>
 __global__ __launch_bounds__(256) void conv_tail_kernel(
@@ -314,6 +505,21 @@ static const float* opt(const c10::optional<torch::Tensor>& t, int64_t n) {
   TORCH_CHECK(t->is_cuda() && t->dtype() == torch::kFloat32 && t->is_contiguous() && t->numel() == n);
   TORCH_CHECK(reinterpret_cast<uintptr_t>(t->data_ptr()) % 16 == 0);
   return t->data_ptr<float>();
+}
+
+static void conv_tail(const torch::Tensor& y, const RowShape& s, const RowWeights& w, const ConvState& st, bool single,
+                      const torch::Tensor& pos, const c10::optional<torch::Tensor>& tiles,
+                      const c10::optional<torch::Tensor>& bounds) {
+  if (s.taps <= 1 || single) return;
+  const dim3 grid(bounds->numel() - 1, (s.columns() / 8 + 255) / 256);
+  auto stream = at::cuda::getCurrentCUDAStream();
+#define CT(TY)                                                                                                        \
+  conv_tail_kernel<TY><<<grid, 256, 0, stream>>>(reinterpret_cast<const TY*>(y.data_ptr()), (int)y.size(1), s, w.bias, st, \
+                                                 pos.data_ptr<int>(), tiles->data_ptr<int>(), bounds->data_ptr<int>())
+  if (y.dtype() == torch::kFloat32) CT(float);
+  else CT(unsigned short);
+#undef CT
+  HIP_CHECK_LAST();
 }
 
 // y [T, ys]: columns of `heads` query vectors of dk values, kv_heads key vectors, `values` value
@@ -379,6 +585,38 @@ torch::Tensor prepare_rows(
   const size_t lds = ((size_t)std::max(s.nq, s.nk) + r.turned) * 4;
   TORCH_CHECK(lds <= 160 * 1024 - 1024, "query projections of ", s.nq, " values are not supported");
   auto stream = at::cuda::getCurrentCUDAStream();
+  const int half = r.turned / 2, most = std::max(s.nq, s.nk);
+  if (!yf && t >= 512 && half % 8 == 0 && most <= 16 * 512 && s.taps <= 4 && s.taps != 1) {  // a prompt's rows
+    const dim3 tiles_grid(((t + TILE_ROWS - 1) / TILE_ROWS + 7) / 8 * 8, 3);
+    const size_t table = (size_t)TILE_ROWS * 2 * half * 4;
+    TORCH_CHECK(table <= 32768, "rotation of ", r.turned, " values is not supported");
+    const int threads = std::max(64, (most / 16 + 63) / 64 * 64);
+#define PTN(TAPS, NT)                                                                                                   \
+  prepare_tile_kernel<TAPS, NT><<<tiles_grid, threads, table, stream>>>(BF16P(y), (int)y.size(1), s, w, st, r,          \
+                                                                        (float)turn_factor, b, BF16P(q), BF16P(cache),  \
+                                                                        (float)eps, (int)t)
+#define PT(TAPS)                        \
+  do {                                  \
+    if (threads <= 256) PTN(TAPS, 256); \
+    else PTN(TAPS, 512);                \
+  } while (0)
+    switch (s.taps) {
+      case 0: PT(0); break;
+      case 2: PT(2); break;
+      case 3: PT(3); break;
+      default: PT(4);
+    }
+#undef PT
+#undef PTN
+    HIP_CHECK_LAST();
+    if (!poly.empty()) {
+      const auto poly_rows = &poly_kernel<unsigned short, 256>;
+      poly_rows<<<dim3(t), 256, 0, stream>>>(BF16P(y), (int)y.size(1), (float)eps, pp, BF16P(*act), act_stride);
+      HIP_CHECK_LAST();
+    }
+    conv_tail(y, s, w, st, single, pos, tiles, bounds);
+    return q;
+  }
   const bool spread = t >= 64;
   const dim3 grid(spread ? (t + 7) / 8 * 8 : t, poly.empty() ? 3 : 4);
 #define PRN(TY, TC, NT)                                                                                                \
@@ -404,15 +642,6 @@ torch::Tensor prepare_rows(
 #undef PR
 #undef PRN
   HIP_CHECK_LAST();
-  if (s.taps > 1 && !single) {
-    const dim3 tail(tables.size(0), (columns / 8 + 255) / 256);
-#define CT(TY)                                                                                                        \
-  conv_tail_kernel<TY><<<tail, 256, 0, stream>>>(reinterpret_cast<const TY*>(y.data_ptr()), (int)y.size(1), s, w.bias, st, \
-                                                 pos.data_ptr<int>(), tiles->data_ptr<int>(), bounds->data_ptr<int>())
-    if (yf) CT(float);
-    else CT(unsigned short);
-#undef CT
-    HIP_CHECK_LAST();
-  }
+  conv_tail(y, s, w, st, single, pos, tiles, bounds);
   return q;
 }

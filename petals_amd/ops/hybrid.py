@@ -16,7 +16,7 @@ import torch
 
 from petals_amd.models.lefulorn.config import KEY_PAD, VALUE_PAD
 from petals_amd.ops import reference
-from petals_amd.ops.packed import CHUNK, PackedBlock
+from petals_amd.ops.packed import CHUNK, PackedBlock, attention_run
 from petals_amd.ops.packed import round_up as _up
 
 _EPI_RELU2_F32 = 6
@@ -116,8 +116,7 @@ class HybridFastPath(PackedBlock):
             y, self.b_in, cache, batch.pos, batch.owner, batch.tables, a.heads, a.kv_heads, self.dk, self.dv,
             a.temp_coef, a.temp_every, first, self.lam, a.vdim,
         )
-        group = a.heads // a.kv_heads
-        run = batch.run_tokens(group)
+        run = attention_run(batch, a.heads, a.kv_heads)
         max_keys = min(batch.max_end, a.window) if a.window > 0 else batch.max_end
         return h.paged_attention(
             q, cache, batch.pos, batch.owner, batch.tables, batch.tiles(run), run, max_keys, a.kv_heads, self.dv,

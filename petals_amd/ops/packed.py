@@ -37,6 +37,11 @@ def rms_norm_f32(x: torch.Tensor, weight: torch.Tensor, eps: float, groups: int 
     return hip.residual_norm(rows, None, None, weight.float().contiguous(), d, eps, True, 1.0, groups)[:, :d].reshape(x.shape)
 
 
+def attention_run(batch, heads: int, kv_heads: int) -> int:
+    """Rows of a paged attention tile: twice as many where that still fills the chip."""
+    return batch.run_tokens(heads // kv_heads, 128 if batch.tokens * heads >= 1 << 16 else 64)
+
+
 class PackedBlock:
     quant = "none"
     captures = True  # whether the mixer's decoding kernels take its sizes

@@ -19,7 +19,7 @@ import math
 import torch
 
 from petals_amd.ops import reference
-from petals_amd.ops.packed import _EPI_RAW, CHUNK, PackedBlock
+from petals_amd.ops.packed import _EPI_RAW, CHUNK, PackedBlock, attention_run
 from petals_amd.ops.packed import round_up as _up
 
 
@@ -116,7 +116,7 @@ class ScoresFastPath(PackedBlock):
     def _attend(self, q, cache, batch, y, out):
         """The heads' results into the first columns of `out`."""
         m, h, t = self.spec, self.hip, q.shape[0]
-        run = batch.run_tokens(m.heads // m.kv_heads)
+        run = attention_run(batch, m.heads, m.kv_heads)
         max_keys = min(batch.max_end, m.chunk) if m.chunk else batch.max_end
         rows = (
             cache, batch.pos, batch.owner, batch.tables, batch.tiles(run), run, max_keys, m.kv_heads, self.dv, m.chunk,

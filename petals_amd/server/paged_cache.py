@@ -267,10 +267,10 @@ class PagedBatch:
         self.slot = dev[2 * t : 2 * t + len(self.slots)]
         self.tables = dev[2 * t + len(self.slots) :].view(len(self.pages), width)
 
-    def run_tokens(self, heads: int) -> int:
-        """Rows that share one attention tile: as many as give about 64
+    def run_tokens(self, heads: int, rows: int = 64) -> int:
+        """Rows that share one attention tile: as many as give about `rows`
         (row, head) pairs."""
-        return 1 if self.decode_only else max(1, 64 // heads)
+        return 1 if self.decode_only else max(1, rows // heads)
 
     def tiles(self, rows: int) -> torch.Tensor:
         """[n, 2] int32 (first row, row count): the batch's rows in runs of at
