@@ -1,8 +1,8 @@
 // Sublayer kernels for blocks that norm each sublayer's INPUT and keep the
 // residual stream in 32-bit (CDNA4, gfx950).
 //
-//   residual_norm   x += mult (y + bias), then RMS norm of x with a plain weight, of the
-//                   whole row or of equal parts of it
+//   residual_norm   x += mult (y + bias), y one matrix or several to be summed, then RMS
+//                   norm of x with a plain weight, of the whole row or of equal parts of it
 //   residual_sum    x += mult (split-K partial sums + bias) of a decoding product
 //   bias_relu2      relu(y + bias)^2
 //   bias_xielu      xIELU of y + bias, y a matrix (in place) or split-K partial sums
@@ -26,11 +26,13 @@ __device__ __forceinline__ void store4(unsigned short* p, f32x4 v) {
                                    (short)f32_to_bf16(v[3])};
 }
 
-// One workgroup per token. y null: x is only read; h null: nothing is normed.
+// One workgroup per token. y null: x is only read; h null: nothing is normed. y: `parts`
+// matrices, part_stride apart.
 template <typename TY, typename TH>
 __global__ __launch_bounds__(1024) void residual_norm_kernel(
     float* __restrict__ x, long x_stride, const TY* __restrict__ y, long y_stride, const float* __restrict__ bias,
-    const float* __restrict__ w, float eps, TH* __restrict__ h, int d, int dp, bool by4, float mult, int groups) {
+    const float* __restrict__ w, float eps, TH* __restrict__ h, int d, int dp, bool by4, float mult, int groups,
+    int parts, long part_stride) {
   extern __shared__ float row[];  // [d], then of each group
   __shared__ float red[16];
   const int tid = threadIdx.x, nt = blockDim.x;
@@ -41,8 +43,13 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
     for (int c = tid * 4; c < d; c += nt * 4) {
       f32x4 v = load4(xr + c);
       if (y) {
-        const f32x4 u = load4(y + t * y_stride + c);
+        f32x4 u = load4(y + t * y_stride + c);
         const f32x4 b = bias ? load4(bias + c) : f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int i = 1; i < parts; ++i) {
+          const f32x4 more = load4(y + i * part_stride + t * y_stride + c);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) u[e] += more[e];
+        }
 #pragma unroll
         for (int e = 0; e < 4; ++e) v[e] = fmaf(mult, u[e] + b[e], v[e]);
         store4(xr + c, v);
@@ -55,7 +62,9 @@ __global__ __launch_bounds__(1024) void residual_norm_kernel(
   for (int c = by4 ? d : tid; c < d; c += nt) {
     float v = xr[c];
     if (y) {
-      v = fmaf(mult, load_f32(y + t * y_stride + c) + (bias ? bias[c] : 0.f), v);
+      float u = load_f32(y + t * y_stride + c);
+      for (int i = 1; i < parts; ++i) u += load_f32(y + i * part_stride + t * y_stride + c);
+      v = fmaf(mult, u + (bias ? bias[c] : 0.f), v);
       xr[c] = v;
     }
     row[c] = v;
@@ -215,7 +224,7 @@ static const float* vec(const c10::optional<torch::Tensor>& t, int64_t n) {
   return t->data_ptr<float>();
 }
 
-// x [T, >= d] f32, updated in place if y is given; returns the norm [T, dp] of `groups` equal parts, or
+// x [T, >= d] f32, updated in place if y [T, >= d] or [parts, T, >= d] is given; returns the norm [T, dp] of `groups` equal parts, or
 // nothing if w is absent
 torch::Tensor residual_norm(torch::Tensor x, c10::optional<torch::Tensor> y, c10::optional<torch::Tensor> bias,
                             c10::optional<torch::Tensor> w, int64_t d, double eps, bool out_f32, double mult,
@@ -225,12 +234,18 @@ torch::Tensor residual_norm(torch::Tensor x, c10::optional<torch::Tensor> y, c10
   const long t = x.size(0), dp = w.has_value() ? (d + 7) / 8 * 8 : 0;
   bool yf = true;
   const void* yp = nullptr;
-  long ys = 0;
+  long ys = 0, part_stride = 0;
+  int parts = 1;
   if (y.has_value()) {
     yf = wide(*y);
-    TORCH_CHECK(y->dim() == 2 && y->stride(1) == 1 && y->size(0) == t && y->size(1) >= d);
+    TORCH_CHECK((y->dim() == 2 || y->dim() == 3) && y->stride(-1) == 1 && y->size(-2) == t && y->size(-1) >= d);
     yp = y->data_ptr();
-    ys = y->stride(0);
+    ys = y->stride(-2);
+    if (y->dim() == 3) {
+      parts = y->size(0);
+      part_stride = y->stride(0);
+      TORCH_CHECK(parts >= 1);
+    }
   }
   const float* bp = vec(bias, d);
   const float* wp = vec(w, d);
@@ -240,13 +255,13 @@ torch::Tensor residual_norm(torch::Tensor x, c10::optional<torch::Tensor> y, c10
   TORCH_CHECK(lds <= 65536 - 64, "width ", d, " in ", groups, " groups is not supported");
   const int threads = t < 512 ? 1024 : 256;
   auto aligned = [](const void* p, int bytes) { return reinterpret_cast<uintptr_t>(p) % bytes == 0; };
-  const bool by4 = d % 4 == 0 && x.stride(0) % 4 == 0 && ys % 4 == 0 && aligned(x.data_ptr(), 16) &&
+  const bool by4 = d % 4 == 0 && x.stride(0) % 4 == 0 && ys % 4 == 0 && part_stride % 4 == 0 && aligned(x.data_ptr(), 16) &&
                    aligned(yp, yf ? 16 : 8) && aligned(bp, 16) && aligned(wp, 16);
   auto stream = at::cuda::getCurrentCUDAStream();
 #define RN(TY, TH)                                                                                          \
   residual_norm_kernel<TY, TH><<<t, threads, lds, stream>>>(                                                \
       x.data_ptr<float>(), x.stride(0), reinterpret_cast<const TY*>(yp), ys, bp, wp, (float)eps,            \
-      wp ? reinterpret_cast<TH*>(h.data_ptr()) : nullptr, (int)d, (int)dp, by4, (float)mult, (int)groups)
+      wp ? reinterpret_cast<TH*>(h.data_ptr()) : nullptr, (int)d, (int)dp, by4, (float)mult, (int)groups, parts, part_stride)
   if (yf && out_f32) RN(float, float);
   else if (yf) RN(float, unsigned short);
   else if (out_f32) RN(unsigned short, float);

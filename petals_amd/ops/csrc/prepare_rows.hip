@@ -529,8 +529,8 @@ static void conv_tail(const torch::Tensor& y, const RowShape& s, const RowWeight
 //   quarters [pairs] f64: quarter turns per position; turn_factor: of what is turned
 //   conv [slots, taps, columns] f32 and slot: absent if there is nothing to remember; single: one row per sequence,
 //   else tiles, bounds: the sequences' rows
-//   poly: (a, b, c, e) and columns [poly_at, poly_at + ff) of y go through PolyNorm to act [T, >= ff padded to 8];
-//   empty: none
+//   poly: (a, b, c, e) and columns [poly_at, poly_at + ff) of y go through PolyNorm to act [T, padded], a multiple
+//   of 8; y has as many columns, zero behind the first ff; empty: none
 torch::Tensor prepare_rows(
     torch::Tensor y, torch::Tensor cache, torch::Tensor pos, torch::Tensor owner, torch::Tensor tables, int64_t heads,
     int64_t kv_heads, int64_t dk, int64_t dim, int64_t values, c10::optional<torch::Tensor> bias,
@@ -573,10 +573,10 @@ torch::Tensor prepare_rows(
   PolyPart pp{0, 0, 0, 0.f, 0.f, 0.f, 0.f};
   long act_stride = 0;
   if (!poly.empty()) {
-    TORCH_CHECK(poly.size() == 4 && ff >= 1 && poly_at % 8 == 0 && act.has_value() && act->dtype() == y.dtype());
-    pp = PolyPart{(int)poly_at, (int)ff, (int)((ff + 7) / 8 * 8), (float)poly[0], (float)poly[1], (float)poly[2], (float)poly[3]};
-    TORCH_CHECK(poly_at >= 0 && poly_at + pp.padded <= y.size(1));
-    TORCH_CHECK(act->is_cuda() && act->dim() == 2 && act->stride(1) == 1 && act->size(0) == t && act->size(1) >= pp.padded);
+    TORCH_CHECK(poly.size() == 4 && ff >= 1 && poly_at % 8 == 0 && act.has_value() && act->dtype() == y.dtype() && act->dim() == 2);
+    pp = PolyPart{(int)poly_at, (int)ff, (int)act->size(1), (float)poly[0], (float)poly[1], (float)poly[2], (float)poly[3]};
+    TORCH_CHECK(poly_at >= 0 && pp.padded >= ff && pp.padded % 8 == 0 && poly_at + pp.padded <= y.size(1));
+    TORCH_CHECK(act->is_cuda() && act->dim() == 2 && act->stride(1) == 1 && act->size(0) == t);
     TORCH_CHECK(act->stride(0) % 8 == 0 && reinterpret_cast<uintptr_t>(act->data_ptr()) % 16 == 0);
     act_stride = act->stride(0);
   }

@@ -128,16 +128,27 @@ class PackedBlock:
             return self.hip.gemv_bf16(w, x, self._no_ws, None, epilogue, self._splits(w), bias)
         return x @ w
 
+    def _parts(self, x, w):
+        """x [T, in] @ w [in, out], as [parts, T, out] to be summed where whole tiles of the
+        result (256 x 256) would leave compute units idle: the parts share the inputs."""
+        tiles = -(-x.shape[0] // 256) * -(-w.shape[1] // 256)
+        parts = 1 if self.f32 else 8
+        while parts > 1 and (parts * tiles > 256 or w.shape[0] % (8 * parts) or w.shape[0] < 512 * parts):
+            parts //= 2
+        if parts == 1:
+            return x @ w
+        return torch.bmm(x.view(x.shape[0], parts, -1).transpose(0, 1), w.view(parts, -1, w.shape[1]))
+
     def _add(self, x, y, w, few: bool, bias=None):
         """x += mult (y @ w + bias), for the last product before x is read again."""
         if few:
             self.hip.residual_sum(self._dense(y, w, True, _EPI_RAW), bias, x, self.d, self.mult)
         else:
-            self.hip.residual_norm(x, y @ w, bias, None, self.d, self.eps, True, self.mult)
+            self.hip.residual_norm(x, self._parts(y, w), bias, None, self.d, self.eps, True, self.mult)
 
     def _add_and_norm(self, x, y, w, few: bool, norm):
         """x += mult (y @ w); the norm of the new x, the input of a dense product."""
         if few:
             self._add(x, y, w, True)
             return self.hip.residual_norm(x, None, None, norm, self.d, self.eps, True)
-        return self.hip.residual_norm(x, y @ w, None, norm, self.d, self.eps, self.f32, self.mult)
+        return self.hip.residual_norm(x, self._parts(y, w), None, norm, self.d, self.eps, self.f32, self.mult)

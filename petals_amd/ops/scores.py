@@ -19,7 +19,7 @@ import math
 import torch
 
 from petals_amd.ops import reference
-from petals_amd.ops.packed import _EPI_RAW, CHUNK, PackedBlock, attention_run
+from petals_amd.ops.packed import CHUNK, PackedBlock, attention_run
 from petals_amd.ops.packed import round_up as _up
 
 
@@ -39,12 +39,14 @@ class ScoresFastPath(PackedBlock):
         self.dk, self.dv = m.dim_pad, m.vdim_pad
         heads = {"q": (m.heads * m.maps, m.dim, self.dk), "k": (m.kv_heads * m.maps, m.dim, self.dk),
                  "v": (m.kv_heads, m.vdim, self.dv)}
+        self.wide = m.heads * self.dv
         ff = 0 if self.mlp is None else self.mlp.ff
+        ffp = _up(self.wide + ff, 64) - self.wide if ff else 0  # a sum of products that is cut in equal parts
         parts = [(name, *sizes) for name, sizes in heads.items()]
         if m.head_gate:
             parts.append(("g", m.heads, 1, 1))
         if ff:
-            parts.append(("up", 1, ff, ff))
+            parts.append(("up", 1, ff, ffp))
         starts = dict(zip([p[0] for p in parts], self._columns(block, parts)))
         self.at_gate, self.at_up = starts.get("g"), starts.get("up", 0)
         self.bias = self._vector(block, "bias", heads) if m.bias else None
@@ -59,7 +61,6 @@ class ScoresFastPath(PackedBlock):
                 self._views[f"{name}_conv"] = view.reshape(n * size, m.taps)
                 at += n * padded
         # the attended values' rows, then the feed-forward's
-        self.wide, ffp = m.heads * self.dv, _up(ff, 8)
         self.w_out = self._zeros(self.wide + ffp, self.dp)
         o = self.w_out[: self.wide].view(m.heads, self.dv, self.dp)[:, : m.vdim, :d].permute(2, 0, 1)
         self._place(block, "o", o)
@@ -107,10 +108,7 @@ class ScoresFastPath(PackedBlock):
             self.mlp.ff if self.poly else 0, out[:, self.wide :] if self.poly else None, self.eps,
         )
         self._attend(q, cache, batch, y, out)
-        if few:
-            h.residual_sum(self._dense(out, self.w_out, True, _EPI_RAW), None, x, self.d, 1.0)
-        else:
-            h.residual_norm(x, out @ self.w_out, None, None, self.d, self.eps, True)
+        self._add(x, out, self.w_out, few)
         return x
 
     def _attend(self, q, cache, batch, y, out):

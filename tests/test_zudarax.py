@@ -271,10 +271,8 @@ def test_prompt_matches_oracle(tmp_path, shape, path):
 
 
 @pytest.mark.parametrize("path", PATHS)
-@pytest.mark.parametrize("width,vocab,eps,groups", [(8, 11, 1e-6, 1), (131, 40, 1e-3, 131), (132, 60, 1e-4, 11), (256, 300, 0.3, 4)])
+@pytest.mark.parametrize("width,vocab,eps,groups", [(8, 11, 1e-6, 1), (131, 40, 0.5, 131), (132, 60, 1e-4, 11), (256, 300, 0.3, 4)])
 def test_other_widths_and_constants(tmp_path, width, vocab, eps, groups, path):
-    if groups == width and path[1] == "bfloat16":
-        pytest.skip("each value normed by itself keeps only its sign; its rounding is without bound around 0")
     m = Model(tmp_path, SHAPES["mixed"], path, width=width, vocab=vocab, eps=eps, seed=3, groups=groups)
     ids = ids_of(90, vocab)
     want = m.expected(ids)
@@ -572,8 +570,9 @@ def test_long_steps_are_cut(tmp_path, path):
 
 @pytest.mark.parametrize("path", PATHS)
 def test_many_rows_in_a_step(tmp_path, path):
-    """More rows than the kernels' small layouts take, in several sequences."""
-    m = Model(tmp_path, [C(ff=40), P(), S(conv=3)], path, tokens=1600)
+    """More rows than the kernels' small layouts take, in several sequences, and sums long
+    enough to be cut in parts."""
+    m = Model(tmp_path, [C(ff=2100), P(ff=1000), S(conv=3)], path, tokens=1600)
     ids = [ids_of(n, seed=n) for n in (601, 3, 210)]
     seqs = [m.engine.pool.open() for _ in ids]
     ys = m.engine.step(m.uids, [StepEntry(s, m.embed(t), 0) for s, t in zip(seqs, ids)])
