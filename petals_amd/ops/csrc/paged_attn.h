@@ -658,13 +658,14 @@ __global__ __launch_bounds__(256) void paged_attn_decode(
   }
 }
 
-// one workgroup per (token, head) row
+#define COMBINE_THREADS(MAPS) ((MAPS) == 1 ? 128 : 512)
+
+// one workgroup per (token, head) row; two maps (dv <= 256): half of the threads for each
 template <int KIND, int MAPS>
-__global__ __launch_bounds__(128) void paged_attn_combine(
+__global__ __launch_bounds__(COMBINE_THREADS(MAPS)) void paged_attn_combine(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, GatedOut g, AttnShape a, int n_rows,
     int n_splits) {
   __shared__ float share[MAPS][WAVE];  // weight of each split in the row
-  __shared__ float red[2];
   const int row = blockIdx.x, head = row % a.heads, tid = threadIdx.x;
   if (KIND == SIGMOID) {
     if (tid < WAVE) share[0][tid] = 1.f;
@@ -699,23 +700,20 @@ __global__ __launch_bounds__(128) void paged_attn_combine(
     for (int d = tid; d < a.dv; d += 128) write_gated(g, a, row / a.heads, head, d, summed(0, d));
     return;
   }
-  float o[2] = {0.f, 0.f};  // dv <= 256
-  float ss = 0.f;
-#pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int d = tid + i * 128;
-    if (d < a.dv) o[i] = summed(0, d) - a.share * summed(MAPS - 1, d);
-    ss = fmaf(o[i], o[i], ss);
-  }
-  ss = wave_reduce_sum(ss);
-  if ((tid & (WAVE - 1)) == 0) red[tid / WAVE] = ss;
+  __shared__ float second[256], red[4];
+  const int d = tid & 255;
+  float o = d < a.dv ? summed(tid / 256, d) : 0.f;
+  if (tid >= 256) second[d] = o;
   __syncthreads();
-  const float inv = a.factor / sqrtf((red[0] + red[1]) / a.vdim + a.eps);
-#pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int d = tid + i * 128;
-    if (d < a.dv) write_gated(g, a, row / a.heads, head, d, o[i] * inv);
+  if (tid < 256) {
+    o -= a.share * second[d];
+    const float ss = wave_reduce_sum(o * o);
+    if ((tid & (WAVE - 1)) == 0) red[tid / WAVE] = ss;
   }
+  __syncthreads();
+  if (d >= a.dv || tid >= 256) return;
+  const float inv = a.factor / sqrtf(((red[0] + red[1]) + (red[2] + red[3])) / a.vdim + a.eps);
+  write_gated(g, a, row / a.heads, head, d, o * inv);
 }
 
 // ---------------------------------------------------------- simple kernel
@@ -862,7 +860,7 @@ static void allow_lds(K kernel, size_t lds) {
 template <int KIND, int MAPS, int RC, int VB, int QB>
 static void launch_tiles(dim3 grid, const torch::Tensor& q, const torch::Tensor& cache, GatedOut g, float* po,
                          float* pml, const int* tiles, PagedRows b, AttnShape a, int n_splits) {
-  constexpr int KT = MAPS * RC * 32 + VB * 16 <= 256 ? 64 : 32;
+  constexpr int KT = MAPS * RC * 32 + VB * 16 <= 512 ? 64 : 32;
   static_assert(PAGE % KT == 0, "a tile lies in one page");
   const size_t lds = 2 * KT * (MAPS * RC * 32 + VB * 16 + 2 * TPAD) * 2;
   allow_lds(&paged_attn_kernel<KIND, MAPS, RC, VB, QB, KT>, lds);
@@ -957,7 +955,7 @@ static void run_attention(const torch::Tensor& q, const torch::Tensor& cache, co
 #undef PA
   HIP_CHECK_LAST();
   if (parts) {
-    paged_attn_combine<KIND, MAPS><<<t * a.heads, 128, 0, stream>>>(po, pml, g, a, t * a.heads, n_splits);
+    paged_attn_combine<KIND, MAPS><<<t * a.heads, COMBINE_THREADS(MAPS), 0, stream>>>(po, pml, g, a, t * a.heads, n_splits);
     HIP_CHECK_LAST();
   }
 }
